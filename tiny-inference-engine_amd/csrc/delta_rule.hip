@@ -7,8 +7,8 @@
 //
 // Gated delta rule, per value head with state S `[key_dim][value_dim]` (float32, in the sequence's slot):
 //   S <- diag(g) S ;  u = beta (v - S^T k) ;  S <- S + k u^T ;  o = S^T q
-// with q and k unit vectors (q also times key_dim^(-1/2)), beta in (0, 1) and one decay in (0, 1) per head and
-// key channel. `delta_prepare` makes q, k, v, beta and g of every token of a step, in parallel over tokens;
+// with q and k unit vectors (q also times key_dim^(-1/2)), beta in (0, 1) and decays in (0, 1): one per head and
+// key channel, or one per head. `delta_prepare` makes q, k, v, beta and g of every token of a step, in parallel over tokens;
 // `gated_delta_scan` walks each sequence's tokens in order.
 #include "common.h"
 
@@ -127,14 +127,15 @@ extern "C" int tie_conv_state_update(const float* u, int row, int taps, float* s
 
 // ---------------------------------------------------------------- what the delta rule takes of a token
 // Row t of `u`: [q (G d) | k (G d) | v (H e) | b (H)], the first C = 2 G d + H e columns convolved, then silu.
-// Row t of `a`: the decay's argument (H d), `a_row` apart. out row: [q^ | k^ | v | g (H d) | beta (H)]:
+// Row t of `a`: the decay's argument (H da), `a_row` apart, da = d or 1 (one decay a head). out row: [q^ | k^ | v |
+// g (H da) | beta (H)] and, with one decay a head, the decays' logarithms (H) behind:
 //   q^, k^ unit vectors per head (x / sqrt(sum x^2 + 1e-6)), q^ also times d^(-1/2); beta = sigmoid(b);
 //   g = exp(-exp(A_log[head]) * softplus(a + dt_bias)).
 __global__ void delta_prepare_kernel(const float* __restrict__ u, int row, const float* __restrict__ w, int taps,
                                      const float* __restrict__ state, const int* __restrict__ state_slots,
                                      const int* __restrict__ seq_of_row, const int* __restrict__ query_start,
                                      const float* __restrict__ a, int a_row, const float* __restrict__ A_log,
-                                     const float* __restrict__ dt_bias, int G, int H, int d, int e,
+                                     const float* __restrict__ dt_bias, int G, int H, int d, int e, int da,
                                      float* __restrict__ out, int out_row) {
   extern __shared__ float vals[];
   const int t = blockIdx.x;
@@ -146,10 +147,13 @@ __global__ void delta_prepare_kernel(const float* __restrict__ u, int row, const
   // three workgroups a row: q and k with their unit norms, v, and beta with the decays
   if (blockIdx.y == 2) {
     const float* b = u + static_cast<size_t>(t) * row + C;
-    for (int h = threadIdx.x; h < H; h += blockDim.x) o[C + H * d + h] = sigmoid_f(b[h]);
+    for (int h = threadIdx.x; h < H; h += blockDim.x) o[C + H * da + h] = sigmoid_f(b[h]);
     const float* ar = a + static_cast<size_t>(t) * a_row;
-    for (int c = threadIdx.x; c < H * d; c += blockDim.x)
-      o[C + c] = expf(-expf(A_log[c / d]) * softplus_f(ar[c] + dt_bias[c]));
+    for (int c = threadIdx.x; c < H * da; c += blockDim.x) {
+      const float log_g = -expf(A_log[c / da]) * softplus_f(ar[c] + dt_bias[c]);
+      o[C + c] = expf(log_g);
+      if (da == 1) o[C + 2 * H + c] = log_g;
+    }
     return;
   }
   const int lo = blockIdx.y == 0 ? 0 : 2 * G * d, hi = blockIdx.y == 0 ? 2 * G * d : C;
@@ -176,14 +180,15 @@ __global__ void delta_prepare_kernel(const float* __restrict__ u, int row, const
 extern "C" int tie_delta_prepare(const float* u, int row, const float* w, int taps, const float* state,
                                  const int* state_slots, const int* seq_of_row, const int* query_start,
                                  const float* a, int a_row, const float* A_log, const float* dt_bias, int T, int G,
-                                 int H, int d, int e, float* out, int out_row, hipStream_t stream) {
+                                 int H, int d, int e, int head_decay, float* out, int out_row, hipStream_t stream) {
   const int C = 2 * G * d + H * e;
+  const int da = head_decay ? 1 : d;
   if (T <= 0 || G <= 0 || H <= 0 || d <= 0 || e <= 0 || taps < 1 || taps > CONV_MAX_TAPS || row < C + H ||
-      out_row < C + H + H * d || a_row < H * d || static_cast<size_t>(C) * 4 > 65536 || (taps > 1 && !state))
+      out_row < C + H + (head_decay ? 2 * H : H * d) || a_row < H * da || static_cast<size_t>(C) * 4 > 65536 || (taps > 1 && !state))
     return TIE_BAD_ARGUMENT;
   const int threads = C >= 2048 ? 1024 : (C >= 1024 ? 512 : 256);
   delta_prepare_kernel<<<dim3(T, 3), threads, static_cast<size_t>(C) * sizeof(float), stream>>>(
-      u, row, w, taps, state, state_slots, seq_of_row, query_start, a, a_row, A_log, dt_bias, G, H, d, e, out,
+      u, row, w, taps, state, state_slots, seq_of_row, query_start, a, a_row, A_log, dt_bias, G, H, d, e, da, out,
       out_row);
   return tie_launch_status();
 }
@@ -194,7 +199,8 @@ extern "C" int tie_delta_prepare(const float* u, int row, const float* w, int ta
 // beyond key_dim stay zero), so the two sums over key rows (S^T k, S^T q) meet inside eight neighbouring lanes,
 // through three lane permutations each and without a barrier. The DELTA_WAVES waves of a workgroup take columns
 // side by side and share the token's k, q and g in LDS, staged NT tokens at a time (the next ones are on their way
-// from memory meanwhile, four words a load where the row's layout allows), every p's rows four words behind the
+// from memory meanwhile, four words a load where the row's layout allows; one decay a head travels with the values
+// instead), every p's rows four words behind the
 // last one's so that the eight addresses of one read fall into different banks; the lanes of one p read the same
 // words. A token's words are in registers before the token before it is done.
 #define DELTA_COLS 8
@@ -214,10 +220,10 @@ struct DeltaRowPlan {
   int k_at, q_at, g_at, v_at, b_at, first_col, d, e, t1, row;
 };
 
-// k, q and g of the tokens tb .. tb + NT - 1 of the head (padded to DP rows) into registers, W words a load:
-// entry (x * DELTA_THREADS + thread) * W of [token][k, q, g][row]. Every load is issued whether it counts or not
+// k, q and g (VECS 3; 2: without g) of the tokens tb .. tb + NT - 1 of the head (padded to DP rows) into registers, W
+// words a load: entry (x * DELTA_THREADS + thread) * W of [token][k, q, g][row]. Every load is issued whether it counts or not
 // (from an address that exists), so that none waits for a branch.
-template <int DP, int NT, int W, int PER>
+template <int DP, int NT, int VECS, int W, int PER>
 __device__ __forceinline__ void delta_fetch(const float* __restrict__ tok, const DeltaRowPlan pl, int tb,
                                             float (&stage)[PER][W]) {
   const float* first = tok + static_cast<size_t>(tb) * pl.row;
@@ -225,7 +231,7 @@ __device__ __forceinline__ void delta_fetch(const float* __restrict__ tok, const
 #pragma unroll
   for (int x = 0; x < PER; ++x) {
     const int idx = (x * DELTA_THREADS + static_cast<int>(threadIdx.x)) * W;
-    const int tk = idx / (3 * DP), rest = idx % (3 * DP), which = rest / DP, i = rest % DP;
+    const int tk = idx / (VECS * DP), rest = idx % (VECS * DP), which = rest / DP, i = rest % DP;
     const float* r = first + static_cast<size_t>(min(tk, left - 1)) * pl.row +
                      (which == 0 ? pl.k_at : (which == 1 ? pl.q_at : pl.g_at));
     const float pad = which == 2 ? 1.f : 0.f;      // padding rows: no key, no query, no decay
@@ -240,8 +246,9 @@ __device__ __forceinline__ void delta_fetch(const float* __restrict__ tok, const
   }
 }
 
-// The values of the wave's columns and beta of the same tokens: entry j * 64 + lane of [token][columns, beta].
-template <int NT, int VB>
+// The values of the wave's columns and beta (EXTRA 2: and the head's decay) of the same tokens: entry j * 64 + lane of
+// [token][columns, beta, decay].
+template <int NT, int EXTRA, int VB>
 __device__ __forceinline__ void delta_fetch_values(const float* __restrict__ tok, const DeltaRowPlan pl, int tb,
                                                    int lane, float (&stage_vb)[VB]) {
   const float* first = tok + static_cast<size_t>(tb) * pl.row;
@@ -249,24 +256,25 @@ __device__ __forceinline__ void delta_fetch_values(const float* __restrict__ tok
 #pragma unroll
   for (int j = 0; j < VB; ++j) {
     const int idx = j * TIE_WAVE + lane;
-    const int tk = idx / (DELTA_COLS + 1), x = idx % (DELTA_COLS + 1);
+    const int tk = idx / (DELTA_COLS + EXTRA), x = idx % (DELTA_COLS + EXTRA);
     const float* r = first + static_cast<size_t>(min(tk, left - 1)) * pl.row;
-    const float v = r[x == DELTA_COLS ? pl.b_at : pl.v_at + min(pl.first_col + x, pl.e - 1)];
-    stage_vb[j] = (tk < NT && tk < left && (x == DELTA_COLS || pl.first_col + x < pl.e)) ? v : 0.f;
+    const float v = r[x == DELTA_COLS ? pl.b_at : (x > DELTA_COLS ? pl.g_at : pl.v_at + min(pl.first_col + x, pl.e - 1))];
+    stage_vb[j] = (tk < NT && tk < left && (x >= DELTA_COLS || pl.first_col + x < pl.e)) ? v : 0.f;
   }
 }
 
-// One token through the lane's rows: S <- g S; u = beta (v - S^T k); S <- S + k u; returns S^T q.
-template <int R>
+// One token through the lane's rows: S <- g S; u = beta (v - S^T k); S <- S + k u; returns S^T q. GR = R: a decay a
+// row; GR = 1: one for all of them.
+template <int R, int GR>
 __device__ __forceinline__ float delta_token(float (&S)[R], const float (&kk)[R], const float (&qq)[R],
-                                             const float (&gg)[R], float v, float beta) {
+                                             const float (&gg)[GR], float v, float beta) {
   float dot0 = 0.f, dot1 = 0.f, dot2 = 0.f, dot3 = 0.f;
 #pragma unroll
   for (int r = 0; r < R; r += 4) {
-    S[r] *= gg[r];
-    S[r + 1] *= gg[r + 1];
-    S[r + 2] *= gg[r + 2];
-    S[r + 3] *= gg[r + 3];
+    S[r] *= gg[r % GR];
+    S[r + 1] *= gg[(r + 1) % GR];
+    S[r + 2] *= gg[(r + 2) % GR];
+    S[r + 3] *= gg[(r + 3) % GR];
     dot0 = fmaf(S[r], kk[r], dot0);
     dot1 = fmaf(S[r + 1], kk[r + 1], dot1);
     dot2 = fmaf(S[r + 2], kk[r + 2], dot2);
@@ -301,7 +309,7 @@ struct DeltaScanMode {
   int outputs;   // outputs are written
 };
 
-template <int R, int W>
+template <int R, int W, bool HEAD_DECAY>
 __global__ __launch_bounds__(DELTA_THREADS) void gated_delta_scan_kernel(
     const float* __restrict__ tok, int row, float* __restrict__ out, int out_row, float* __restrict__ state,
     const int* __restrict__ query_start, const int* __restrict__ state_slots, int G, int H, int d, int e,
@@ -309,10 +317,13 @@ __global__ __launch_bounds__(DELTA_THREADS) void gated_delta_scan_kernel(
   constexpr int DP = R * DELTA_PARTS;                 // padded key rows
   constexpr int RP = R + 4;                           // words from one p's rows to the next one's in LDS
   constexpr int NT = 4 * DELTA_THREADS / DP;          // tokens staged at a time: 4 to 32
-  constexpr int PER = NT * 3 * DP / (DELTA_THREADS * W);
-  constexpr int VB = (NT * (DELTA_COLS + 1) + TIE_WAVE - 1) / TIE_WAVE;
-  __shared__ __attribute__((aligned(16))) float kqg[NT * 3 * DELTA_PARTS * RP];   // [token][k, q, g][p][row]
-  __shared__ float vbs[DELTA_WAVES][NT * (DELTA_COLS + 1)];     // a wave: [token][the values of its columns, beta]
+  constexpr int VECS = HEAD_DECAY ? 2 : 3;            // k, q and, with a decay a key channel, g
+  constexpr int GR = HEAD_DECAY ? 1 : R;
+  constexpr int VW = DELTA_COLS + (HEAD_DECAY ? 2 : 1);
+  constexpr int PER = NT * VECS * DP / (DELTA_THREADS * W);
+  constexpr int VB = (NT * VW + TIE_WAVE - 1) / TIE_WAVE;
+  __shared__ __attribute__((aligned(16))) float kqg[NT * VECS * DELTA_PARTS * RP];   // [token][k, q, g][p][row]
+  __shared__ float vbs[DELTA_WAVES][NT * VW];     // a wave: [token][the values of its columns, beta, one decay]
   const int item = blockIdx.x / H, head = blockIdx.x % H;
   const int kv = head / (H / G);
   const int wave = threadIdx.x / TIE_WAVE, lane = threadIdx.x % TIE_WAVE;
@@ -340,26 +351,29 @@ __global__ __launch_bounds__(DELTA_THREADS) void gated_delta_scan_kernel(
   pl.q_at = kv * d;
   pl.k_at = G * d + kv * d;
   pl.v_at = 2 * G * d + head * e;
-  pl.g_at = 2 * G * d + H * e + head * d;
-  pl.b_at = 2 * G * d + H * e + H * d + head;
+  pl.g_at = 2 * G * d + H * e + (HEAD_DECAY ? head : head * d);
+  pl.b_at = 2 * G * d + H * e + (HEAD_DECAY ? H : H * d) + head;
   pl.first_col = first_col;
   pl.d = d, pl.e = e, pl.t1 = t1, pl.row = row;
   float* vb = vbs[wave];
   const bool writes = mode.outputs && p == 0 && col < e;
   float stage[PER][W], stage_vb[VB];
-  delta_fetch<DP, NT, W, PER>(tok, pl, t0, stage);
-  delta_fetch_values<NT, VB>(tok, pl, t0, lane, stage_vb);
-  float ka[R], qa[R], ga[R], kb[R], qb[R], gb[R];
-  auto read = [&](int j, float (&kk)[R], float (&qq)[R], float (&gg)[R]) {     // token j of the staged ones
-    const float* at = kqg + (j * 3 * DELTA_PARTS + p) * RP;
+  delta_fetch<DP, NT, VECS, W, PER>(tok, pl, t0, stage);
+  delta_fetch_values<NT, VW - DELTA_COLS, VB>(tok, pl, t0, lane, stage_vb);
+  float ka[R], qa[R], ga[GR], kb[R], qb[R], gb[GR];
+  auto read = [&](int j, float (&kk)[R], float (&qq)[R], float (&gg)[GR]) {     // token j of the staged ones
+    const float* at = kqg + (j * VECS * DELTA_PARTS + p) * RP;
+    if constexpr (HEAD_DECAY) gg[0] = vb[j * VW + DELTA_COLS + 1];
 #pragma unroll
     for (int r = 0; r < R; r += 4) {
       const float4 k4 = *reinterpret_cast<const float4*>(at + r);
       const float4 q4 = *reinterpret_cast<const float4*>(at + DELTA_PARTS * RP + r);
-      const float4 g4 = *reinterpret_cast<const float4*>(at + 2 * DELTA_PARTS * RP + r);
       kk[r] = k4.x, kk[r + 1] = k4.y, kk[r + 2] = k4.z, kk[r + 3] = k4.w;
       qq[r] = q4.x, qq[r + 1] = q4.y, qq[r + 2] = q4.z, qq[r + 3] = q4.w;
-      gg[r] = g4.x, gg[r + 1] = g4.y, gg[r + 2] = g4.z, gg[r + 3] = g4.w;
+      if constexpr (!HEAD_DECAY) {
+        const float4 g4 = *reinterpret_cast<const float4*>(at + 2 * DELTA_PARTS * RP + r);
+        gg[r] = g4.x, gg[r + 1] = g4.y, gg[r + 2] = g4.z, gg[r + 3] = g4.w;
+      }
     }
   };
   for (int tb = t0; tb < t1; tb += NT) {
@@ -378,19 +392,19 @@ __global__ __launch_bounds__(DELTA_THREADS) void gated_delta_scan_kernel(
 #pragma unroll
     for (int j = 0; j < VB; ++j) {
       const int idx = j * TIE_WAVE + lane;
-      if (idx < NT * (DELTA_COLS + 1)) vb[idx] = stage_vb[j];
+      if (idx < NT * VW) vb[idx] = stage_vb[j];
     }
     __syncthreads();
     if (tb + NT < t1) {
-      delta_fetch<DP, NT, W, PER>(tok, pl, tb + NT, stage);
-      delta_fetch_values<NT, VB>(tok, pl, tb + NT, lane, stage_vb);
+      delta_fetch<DP, NT, VECS, W, PER>(tok, pl, tb + NT, stage);
+      delta_fetch_values<NT, VW - DELTA_COLS, VB>(tok, pl, tb + NT, lane, stage_vb);
     }
     const int count = min(NT, t1 - tb);
     float* o = out + static_cast<size_t>(tb) * out_row + head * e + col;
     if constexpr (R > 16) {   // too many rows a lane for two tokens' words in registers
       for (int j = 0; j < count; ++j) {
         read(j, ka, qa, ga);
-        const float sum = delta_token<R>(S, ka, qa, ga, vb[j * (DELTA_COLS + 1) + c], vb[j * (DELTA_COLS + 1) + DELTA_COLS]);
+        const float sum = delta_token<R, GR>(S, ka, qa, ga, vb[j * VW + c], vb[j * VW + DELTA_COLS]);
         if (writes) o[static_cast<size_t>(j) * out_row] = sum;
       }
       continue;
@@ -398,12 +412,11 @@ __global__ __launch_bounds__(DELTA_THREADS) void gated_delta_scan_kernel(
     read(0, ka, qa, ga);
     for (int j = 0; j < count; j += 2) {
       if (j + 1 < count) read(j + 1, kb, qb, gb);
-      const float first = delta_token<R>(S, ka, qa, ga, vb[j * (DELTA_COLS + 1) + c], vb[j * (DELTA_COLS + 1) + DELTA_COLS]);
+      const float first = delta_token<R, GR>(S, ka, qa, ga, vb[j * VW + c], vb[j * VW + DELTA_COLS]);
       if (writes) o[static_cast<size_t>(j) * out_row] = first;
       if (j + 1 < count) {
         if (j + 2 < count) read(j + 2, ka, qa, ga);
-        const float second = delta_token<R>(S, kb, qb, gb, vb[(j + 1) * (DELTA_COLS + 1) + c],
-                                            vb[(j + 1) * (DELTA_COLS + 1) + DELTA_COLS]);
+        const float second = delta_token<R, GR>(S, kb, qb, gb, vb[(j + 1) * VW + c], vb[(j + 1) * VW + DELTA_COLS]);
         if (writes) o[static_cast<size_t>(j + 1) * out_row] = second;
       }
     }
@@ -518,37 +531,39 @@ __global__ __launch_bounds__(COMBINE_THREADS) void gated_delta_combine_kernel(
 
 // tok: rows of delta_prepare; out: float32 [T][>= H e]; state: [slots][H][d][e].
 static int launch_delta_scan(const float* tok, int row, float* out, int out_row, float* state, const int* query_start,
-                             const int* state_slots, int num_items, int G, int H, int d, int e, DeltaScanMode mode,
-                             hipStream_t stream) {
+                             const int* state_slots, int num_items, int G, int H, int d, int e, int head_decay,
+                             DeltaScanMode mode, hipStream_t stream) {
   constexpr int wg_cols = DELTA_WAVES * DELTA_COLS;
   const dim3 grid(num_items * H, (mode.columns + wg_cols - 1) / wg_cols);
   if (grid.y > 65535) return TIE_BAD_ARGUMENT;
   // four words a load where every head's k, q and g start at a multiple of four words of an aligned row
   const bool wide = d % 4 == 0 && (H * e) % 4 == 0 && row % 4 == 0 && reinterpret_cast<uintptr_t>(tok) % 16 == 0;
-#define SCAN(R)                                                                                                    \
-  do {                                                                                                             \
-    if (wide)                                                                                                      \
-      gated_delta_scan_kernel<R, 4><<<grid, DELTA_THREADS, 0, stream>>>(tok, row, out, out_row, state, query_start, \
-                                                                        state_slots, G, H, d, e, mode);             \
-    else                                                                                                           \
-      gated_delta_scan_kernel<R, 1><<<grid, DELTA_THREADS, 0, stream>>>(tok, row, out, out_row, state, query_start, \
-                                                                        state_slots, G, H, d, e, mode);             \
+#define SCAN_AS(R, W, HD)                                                                                     \
+  gated_delta_scan_kernel<R, W, HD><<<grid, DELTA_THREADS, 0, stream>>>(tok, row, out, out_row, state, query_start, \
+                                                                        state_slots, G, H, d, e, mode)
+#define SCAN(R)                                          \
+  do {                                                   \
+    if (wide && head_decay) SCAN_AS(R, 4, true);         \
+    else if (wide) SCAN_AS(R, 4, false);                 \
+    else if (head_decay) SCAN_AS(R, 1, true);            \
+    else SCAN_AS(R, 1, false);                           \
   } while (0)
   if (d <= 32) SCAN(4);
   else if (d <= 64) SCAN(8);
   else if (d <= 128) SCAN(16);
   else SCAN(32);
 #undef SCAN
+#undef SCAN_AS
   return tie_launch_status();
 }
 
 extern "C" int tie_gated_delta_scan(const float* tok, int row, float* out, int out_row, float* state,
                                     const int* query_start, const int* state_slots, int num_seqs, int G, int H, int d,
-                                    int e, hipStream_t stream) {
+                                    int e, int head_decay, hipStream_t stream) {
   if (num_seqs <= 0 || G <= 0 || H <= 0 || H % G || d <= 0 || d > 256 || e <= 0 || out_row < H * e ||
-      row < 2 * G * d + H * e + H + H * d)
+      row < 2 * G * d + H * e + H + (head_decay ? H : H * d))
     return TIE_BAD_ARGUMENT;
-  return launch_delta_scan(tok, row, out, out_row, state, query_start, state_slots, num_seqs, G, H, d, e,
+  return launch_delta_scan(tok, row, out, out_row, state, query_start, state_slots, num_seqs, G, H, d, e, head_decay,
                            DeltaScanMode{nullptr, e, 0, 1, 1}, stream);
 }
 
@@ -563,7 +578,7 @@ extern "C" int tie_gated_delta_scan_chunked(const float* tok, int row, float* ou
   if (num_seqs <= 0 || count <= 0 || G <= 0 || H <= 0 || H % G || d <= 0 || d > 256 || e <= 0 || out_row < H * e ||
       row < 2 * G * d + H * e + H + H * d || !items || !first_chunk || !ends || !starts)
     return TIE_BAD_ARGUMENT;
-  int rc = launch_delta_scan(tok, row, out, out_row, ends, nullptr, nullptr, count, G, H, d, e,
+  int rc = launch_delta_scan(tok, row, out, out_row, ends, nullptr, nullptr, count, G, H, d, e, 0,
                              DeltaScanMode{items, e + d, 1, 1, 0}, stream);
   if (rc != TIE_OK) return rc;
   const dim3 grid(num_seqs * H, (e + COMBINE_COLS - 1) / COMBINE_COLS);
@@ -575,15 +590,16 @@ extern "C" int tie_gated_delta_scan_chunked(const float* tok, int row, float* ou
                                                                      d, e, jt);
   rc = tie_launch_status();
   if (rc != TIE_OK) return rc;
-  return launch_delta_scan(tok, row, out, out_row, starts, nullptr, nullptr, count, G, H, d, e,
+  return launch_delta_scan(tok, row, out, out_row, starts, nullptr, nullptr, count, G, H, d, e, 0,
                            DeltaScanMode{items, e, 0, 0, 1}, stream);
 }
 
 // ---------------------------------------------------------------- the norm of the heads' outputs, gated
-// out = o / rms(o over each group of `group` columns) * w[column in group] * sigmoid(gate), a wave a group.
+// out = o / rms(o over each group of `group` columns) * w[column in group] * sigmoid(gate) (or * silu(gate)), a wave a
+// group.
 template <typename TO>
 __global__ void grouped_gated_rms_norm_kernel(const float* __restrict__ o, int o_row, const float* __restrict__ w,
-                                              float eps, const float* __restrict__ gate, int gate_row,
+                                              float eps, const float* __restrict__ gate, int gate_row, int silu_gate,
                                               TO* __restrict__ out, int groups, int group) {
   const int lane = threadIdx.x & (TIE_WAVE - 1);
   const int g = blockIdx.y * (blockDim.x / TIE_WAVE) + threadIdx.x / TIE_WAVE;
@@ -595,22 +611,23 @@ __global__ void grouped_gated_rms_norm_kernel(const float* __restrict__ o, int o
   for (int c = lane; c < group; c += TIE_WAVE) ss = fmaf(r[c], r[c], ss);
   const float inv = 1.0f / sqrtf(wave_sum(ss) / static_cast<float>(group) + eps);
   TO* d = out + (t * groups + g) * group;
-  for (int c = lane; c < group; c += TIE_WAVE) store_from_float(d + c, (r[c] * inv) * w[c] * sigmoid_f(gt[c]));
+  for (int c = lane; c < group; c += TIE_WAVE)
+    store_from_float(d + c, (r[c] * inv) * w[c] * (silu_gate ? silu_f(gt[c]) : sigmoid_f(gt[c])));
 }
 
 extern "C" int tie_grouped_gated_rms_norm(const float* o, int o_row, const float* w, float eps, const float* gate,
-                                          int gate_row, void* out, int out_dtype, int T, int groups, int group,
-                                          hipStream_t stream) {
+                                          int gate_row, int silu_gate, void* out, int out_dtype, int T, int groups,
+                                          int group, hipStream_t stream) {
   if (T <= 0 || groups <= 0 || group <= 0 || o_row < groups * group || gate_row < groups * group)
     return TIE_BAD_ARGUMENT;
   const int waves = groups >= 4 ? 4 : groups;
   const dim3 grid(T, (groups + waves - 1) / waves);
   if (out_dtype == TIE_F32)
-    grouped_gated_rms_norm_kernel<float><<<grid, waves * TIE_WAVE, 0, stream>>>(o, o_row, w, eps, gate, gate_row,
-                                                                                static_cast<float*>(out), groups, group);
+    grouped_gated_rms_norm_kernel<float><<<grid, waves * TIE_WAVE, 0, stream>>>(
+        o, o_row, w, eps, gate, gate_row, silu_gate, static_cast<float*>(out), groups, group);
   else if (out_dtype == TIE_BF16)
     grouped_gated_rms_norm_kernel<bf16_t><<<grid, waves * TIE_WAVE, 0, stream>>>(
-        o, o_row, w, eps, gate, gate_row, static_cast<bf16_t*>(out), groups, group);
+        o, o_row, w, eps, gate, gate_row, silu_gate, static_cast<bf16_t*>(out), groups, group);
   else
     return TIE_BAD_ARGUMENT;
   return tie_launch_status();

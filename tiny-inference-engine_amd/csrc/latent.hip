@@ -126,7 +126,8 @@ extern "C" int tie_rms_norm_columns(const float* x, int x_row, const float* w, f
 }
 
 // ---------------------------------------------------------------- a matrix of its own for every head
-// out[t][h][n] = sum_k x[t][h][k] * w[h][n][k]   (n < N, k < K; float32 sums), optionally times sigmoid(gate[t][h][n]).
+// out[t][h][n] = sum_k x[t][h][k] * w[h][n][k]   (n < N, k < K; float32 sums), optionally times sigmoid(gate[t][h][n])
+// or, with gate_col 0, by one gate a head, sigmoid(gate[t][h]).
 // x rows `x_row` apart with heads `x_head` apart, out likewise; w is [H][N][K] row-major. A workgroup of 256
 // threads takes a tile of 64 rows x 64 columns of one head through LDS in steps of 16 along K; a thread 4 x 4.
 #define HL_TILE 64
@@ -136,7 +137,7 @@ template <typename TX, typename TW, typename TO>
 __global__ __launch_bounds__(256) void head_linear_kernel(const TX* __restrict__ x, int x_row, int x_head,
                                                           const TW* __restrict__ w, TO* __restrict__ out, int out_row,
                                                           int out_head, const float* __restrict__ gate, int gate_row,
-                                                          int gate_head, int T, int N, int K) {
+                                                          int gate_head, int gate_col, int T, int N, int K) {
   __shared__ float xs[HL_K][HL_TILE + 4];
   __shared__ float ws[HL_K][HL_TILE + 4];
   const int h = blockIdx.z;
@@ -173,7 +174,7 @@ __global__ __launch_bounds__(256) void head_linear_kernel(const TX* __restrict__
       const int n = n0 + tx * 4 + j;
       if (n >= N) continue;
       float v = acc[i][j];
-      if (gate) v *= sigmoid_f(gate[static_cast<size_t>(t) * gate_row + h * gate_head + n]);
+      if (gate) v *= sigmoid_f(gate[static_cast<size_t>(t) * gate_row + h * gate_head + n * gate_col]);
       store_from_float(out + static_cast<size_t>(t) * out_row + h * out_head + n, v);
     }
   }
@@ -196,7 +197,8 @@ __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const bf16_t* __r
                                                                const bf16_t* __restrict__ w, TO* __restrict__ out,
                                                                int out_row, int out_head,
                                                                const float* __restrict__ gate, int gate_row,
-                                                               int gate_head, int T, int N, int K, int whole) {
+                                                               int gate_head, int gate_col, int T, int N, int K,
+                                                               int whole) {
   const int h = blockIdx.z;
   const int wave = threadIdx.x / TIE_WAVE, lane = threadIdx.x % TIE_WAVE;
   const int t0 = (ALONG_T ? blockIdx.x * 4 + wave : blockIdx.x) * 16;
@@ -235,14 +237,16 @@ __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const bf16_t* __r
   // a lane holds row t0 + lane % 16 and, of every tile, the four columns from (lane / 16) * 4 on
   const int t = t0 + r;
   if (t >= T) return;
+  float one = 1.f;           // a gate for the whole head is asked for once
+  if (gate && gate_col == 0) one = sigmoid_f(gate[static_cast<size_t>(t) * gate_row + h * gate_head]);
 #pragma unroll
   for (int i = 0; i < NTILES; ++i) {
     const int n = n0 + i * 16 + kb * 4;
     if (n >= N) continue;
     TO* o = out + static_cast<size_t>(t) * out_row + h * out_head + n;
-    const float* g = gate ? gate + static_cast<size_t>(t) * gate_row + h * gate_head + n : nullptr;
+    const float* g = gate && gate_col ? gate + static_cast<size_t>(t) * gate_row + h * gate_head + n : nullptr;
     if (whole) {           // n + 3 < N, and four columns are one aligned word of out (and of gate)
-      float y[4] = {acc[i][0], acc[i][1], acc[i][2], acc[i][3]};
+      float y[4] = {acc[i][0] * one, acc[i][1] * one, acc[i][2] * one, acc[i][3] * one};
       if (g) {
         const float4 g4 = *reinterpret_cast<const float4*>(g);
         y[0] *= sigmoid_f(g4.x), y[1] *= sigmoid_f(g4.y), y[2] *= sigmoid_f(g4.z), y[3] *= sigmoid_f(g4.w);
@@ -260,7 +264,7 @@ __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const bf16_t* __r
 #pragma unroll
     for (int v = 0; v < 4; ++v) {
       if (n + v >= N) continue;
-      float y = acc[i][v];
+      float y = acc[i][v] * one;
       if (g) y *= sigmoid_f(g[v]);
       store_from_float(o + v, y);
     }
@@ -271,43 +275,45 @@ __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const bf16_t* __r
 
 template <typename TO>
 static void launch_head_linear_mfma(const bf16_t* x, int x_row, int x_head, const bf16_t* w, TO* out, int out_row,
-                                    int out_head, const float* gate, int gate_row, int gate_head, int T, int H, int N,
-                                    int K, hipStream_t stream) {
+                                    int out_head, const float* gate, int gate_row, int gate_head, int gate_col, int T,
+                                    int H, int N, int K, hipStream_t stream) {
   // four columns a store (and a gate load): sizes in steps of four from aligned addresses
   const int whole = N % 4 == 0 && out_row % 4 == 0 && out_head % 4 == 0 &&
                     reinterpret_cast<uintptr_t>(out) % (4 * sizeof(TO)) == 0 &&
-                    (!gate || (gate_row % 4 == 0 && gate_head % 4 == 0 && reinterpret_cast<uintptr_t>(gate) % 16 == 0));
+                    (!gate || !gate_col || (gate_row % 4 == 0 && gate_head % 4 == 0 && reinterpret_cast<uintptr_t>(gate) % 16 == 0));
   if (T <= HL_FEW_ROWS) {
     const dim3 grid((T + 15) / 16, (N + 63) / 64, H);
     head_linear_mfma_kernel<TO, 1, false><<<grid, 256, 0, stream>>>(x, x_row, x_head, w, out, out_row, out_head, gate,
-                                                                    gate_row, gate_head, T, N, K, whole);
+                                                                    gate_row, gate_head, gate_col, T, N, K, whole);
   } else {
     const dim3 grid((T + 63) / 64, (N + 63) / 64, H);
     head_linear_mfma_kernel<TO, 4, true><<<grid, 256, 0, stream>>>(x, x_row, x_head, w, out, out_row, out_head, gate,
-                                                                   gate_row, gate_head, T, N, K, whole);
+                                                                   gate_row, gate_head, gate_col, T, N, K, whole);
   }
 }
 
 extern "C" int tie_head_linear(const void* x, int x_dtype, int x_row, int x_head, const void* w, int w_dtype, void* out,
                                int out_dtype, int out_row, int out_head, const float* gate, int gate_row,
-                               int gate_head, int T, int H, int N, int K, hipStream_t stream) {
+                               int gate_head, int gate_col, int T, int H, int N, int K, hipStream_t stream) {
   if (T <= 0 || H <= 0 || N <= 0 || K <= 0 || H > 65535 || (T + 15) / 16 > 65535 * 4) return TIE_BAD_ARGUMENT;
   if (x_dtype == TIE_BF16 && w_dtype == TIE_BF16 && (out_dtype == TIE_BF16 || out_dtype == TIE_F32) && K % 8 == 0 &&
       x_row % 8 == 0 && x_head % 8 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 &&
       reinterpret_cast<uintptr_t>(w) % 16 == 0) {
     if (out_dtype == TIE_BF16)
       launch_head_linear_mfma(static_cast<const bf16_t*>(x), x_row, x_head, static_cast<const bf16_t*>(w),
-                              static_cast<bf16_t*>(out), out_row, out_head, gate, gate_row, gate_head, T, H, N, K, stream);
+                              static_cast<bf16_t*>(out), out_row, out_head, gate, gate_row, gate_head, gate_col, T, H, N,
+                              K, stream);
     else
       launch_head_linear_mfma(static_cast<const bf16_t*>(x), x_row, x_head, static_cast<const bf16_t*>(w),
-                              static_cast<float*>(out), out_row, out_head, gate, gate_row, gate_head, T, H, N, K, stream);
+                              static_cast<float*>(out), out_row, out_head, gate, gate_row, gate_head, gate_col, T, H, N,
+                              K, stream);
     return tie_launch_status();
   }
   const dim3 grid((T + HL_TILE - 1) / HL_TILE, (N + HL_TILE - 1) / HL_TILE, H);
 #define HL(TX, TW, TO)                                                                                              \
   head_linear_kernel<TX, TW, TO><<<grid, 256, 0, stream>>>(static_cast<const TX*>(x), x_row, x_head,               \
                                                            static_cast<const TW*>(w), static_cast<TO*>(out), out_row, \
-                                                           out_head, gate, gate_row, gate_head, T, N, K)
+                                                           out_head, gate, gate_row, gate_head, gate_col, T, N, K)
   if (x_dtype == TIE_F32 && w_dtype == TIE_F32 && out_dtype == TIE_F32) HL(float, float, float);
   else if (x_dtype == TIE_BF16 && w_dtype == TIE_BF16 && out_dtype == TIE_BF16) HL(bf16_t, bf16_t, bf16_t);
   else if (x_dtype == TIE_BF16 && w_dtype == TIE_BF16 && out_dtype == TIE_F32) HL(bf16_t, bf16_t, float);

@@ -5,7 +5,9 @@
 //              the choice looks at s + correction: experts form `groups` equal groups of neighbours, a group scores
 //              its best member (or the sum of its `group_top` best), only members of the `keep` best groups stay
 //              eligible (the others count as -inf), and the `top` best of those are chosen, ties to the lower index;
-//              the weights are s at the chosen, as they are or divided by their sum (+ an eps), times a factor.
+//              the weights are s at the chosen, as they are or divided by their sum (+ an eps), times a factor. Or s
+//              are the logits themselves and the weights the softmax over the chosen ones alone. A bias may be added
+//              to the logits first.
 //              `shared` further slots a row name the experts E, E + 1, ... (experts every row uses: a shared expert,
 //              cut into pieces of the routed experts' size), all with the weight sigmoid(logits[E]), one more
 //              column of the router's product.
@@ -14,8 +16,9 @@
 //              without weights, which the caller treats as it likes), and the list of row tiles (expert, first
 //              place) the products run over. Integer counters only; which place a slot gets inside its expert's
 //              range depends on timing, but no result does: a row's sums are formed the same way at every place.
-//   products   act[place] = silu(x[row] Wg_e^T) * (x[row] Wu_e^T), or relu(x[row] Wu_e^T)^2 for experts without a
-//              gate, and   parts[place] = act[place] Wd_e^T,
+//   products   act[place] = silu(x[row] Wg_e^T) * (x[row] Wu_e^T), or with sums cut off at a limit
+//              g sigmoid(slope g) (u + shift), g = min(x[row] Wg_e^T, limit), u = clamp(x[row] Wu_e^T, -limit, limit),
+//              or relu(x[row] Wu_e^T)^2 for experts without a gate, and   parts[place] = act[place] Wd_e^T,
 //              one workgroup a (row tile of one expert, column tile). The generic kernels multiply and add in
 //              float32 on the vector units for any sizes and float32 / bfloat16 operands (the true 32-bit path);
 //              the bfloat16 kernels run the same tiles on the matrix cores.
@@ -43,9 +46,14 @@ __device__ __forceinline__ void wave_argmax(float& v, int& i) {   // ties: the l
   }
 }
 
+#define SCORE_SOFTMAX 0
+#define SCORE_SIGMOID 1
+#define SCORE_LOGIT 2        // chosen by the logits, weighted by the softmax over the chosen ones
+
 __global__ __launch_bounds__(TIE_WAVE) void moe_route_kernel(const float* __restrict__ logits, int row,
+                                                             const float* __restrict__ bias,
                                                              const float* __restrict__ correction, int E, int groups,
-                                                             int keep, int top, int sigmoid_scores, int group_top,
+                                                             int keep, int top, int scoring, int group_top,
                                                              int renormalize, float renorm_eps, float weight_scale,
                                                              int shared, int* __restrict__ ids,
                                                              float* __restrict__ weights) {
@@ -56,20 +64,22 @@ __global__ __launch_bounds__(TIE_WAVE) void moe_route_kernel(const float* __rest
   const int lane = threadIdx.x;
   const size_t t = blockIdx.x;
   const float* z = logits + t * row;
+  auto logit = [&](int e) { return bias != nullptr ? z[e] + bias[e] : z[e]; };
   const int slots = top + shared;          // of a row: the chosen, then the experts every row uses
-  if (sigmoid_scores) {
+  if (scoring != SCORE_SOFTMAX) {
     for (int e = lane; e < E; e += TIE_WAVE) {
-      const float s = 1.0f / (1.0f + expf(-z[e]));
+      const float l = logit(e);
+      const float s = scoring == SCORE_SIGMOID ? 1.0f / (1.0f + expf(-l)) : l;
       score[e] = s;
       choice[e] = s + (correction != nullptr ? correction[e] : 0.f);
     }
   } else {
     float m = -INFINITY;
-    for (int e = lane; e < E; e += TIE_WAVE) m = fmaxf(m, z[e]);
+    for (int e = lane; e < E; e += TIE_WAVE) m = fmaxf(m, logit(e));
     m = wave_max(m);
     float sum = 0.f;
     for (int e = lane; e < E; e += TIE_WAVE) {
-      const float p = expf(z[e] - m);
+      const float p = expf(logit(e) - m);
       score[e] = p;
       sum += p;
     }
@@ -138,14 +148,22 @@ __global__ __launch_bounds__(TIE_WAVE) void moe_route_kernel(const float* __rest
     if (bi >= E) bi = 0;               // fewer eligible experts than `top`: a configuration's fault, not a fault here
     if (lane == 0) {
       ids[t * slots + k] = bi;
-      weights[t * slots + k] = bv == -INFINITY ? 0.f : score[bi];
+      weights[t * slots + k] = bv == -INFINITY ? (scoring == SCORE_LOGIT ? -INFINITY : 0.f) : score[bi];
       choice[bi] = -INFINITY;
     }
     __syncthreads();
   }
   if (lane == 0) {
     float* w = weights + t * slots;
-    if (renormalize) {
+    if (scoring == SCORE_LOGIT) {             // the softmax over the chosen logits alone
+      float m = -INFINITY, sum = 0.f;
+      for (int k = 0; k < top; ++k) m = fmaxf(m, w[k]);
+      for (int k = 0; k < top; ++k) {
+        w[k] = expf(w[k] - m);
+        sum += w[k];
+      }
+      for (int k = 0; k < top; ++k) w[k] = w[k] / sum * weight_scale;
+    } else if (renormalize) {
       float sum = 0.f;
       for (int k = 0; k < top; ++k) sum += w[k];
       sum += renorm_eps;
@@ -164,16 +182,16 @@ __global__ __launch_bounds__(TIE_WAVE) void moe_route_kernel(const float* __rest
 }
 
 // logits [T][row] float32 with row >= E (+ 1 with shared slots: column E is the gate of the experts every row uses);
-// ids and weights [T][top + shared].
-extern "C" int tie_moe_route(const float* logits, int row, const float* correction, int T, int E, int groups, int keep,
-                             int top, int sigmoid_scores, int group_top, int renormalize, float renorm_eps,
+// bias and correction [E] or null; ids and weights [T][top + shared].
+extern "C" int tie_moe_route(const float* logits, int row, const float* bias, const float* correction, int T, int E,
+                             int groups, int keep, int top, int scoring, int group_top, int renormalize, float renorm_eps,
                              float weight_scale, int shared, int* ids, float* weights, hipStream_t stream) {
   if (T <= 0 || E <= 0 || E > MOE_MAX_EXPERTS || groups <= 0 || E % groups != 0 || keep <= 0 || keep > groups ||
       top <= 0 || top > E || group_top <= 0 || group_top > MOE_MAX_GROUP_TOP || shared < 0 ||
-      row < E + (shared > 0 ? 1 : 0))
+      row < E + (shared > 0 ? 1 : 0) || scoring < SCORE_SOFTMAX || scoring > SCORE_LOGIT)
     return TIE_BAD_ARGUMENT;
   const size_t lds = sizeof(float) * (2 * static_cast<size_t>(E) + groups);
-  moe_route_kernel<<<T, TIE_WAVE, lds, stream>>>(logits, row, correction, E, groups, keep, top, sigmoid_scores,
+  moe_route_kernel<<<T, TIE_WAVE, lds, stream>>>(logits, row, bias, correction, E, groups, keep, top, scoring,
                                                  group_top, renormalize, renorm_eps, weight_scale, shared, ids,
                                                  weights);
   return tie_launch_status();
@@ -248,8 +266,19 @@ extern "C" int tie_moe_align(const int* ids, int slots, int real, int tile_rows,
 
 __device__ __forceinline__ float silu_f(float g) { return g / (1.0f + expf(-g)); }
 
+// What a gated expert makes of its gate's and up's sums.
+struct GateParams {
+  float limit, slope, shift;      // MODE 3 only
+};
+
+__device__ __forceinline__ float clipped_gate_f(float a, float b, GateParams p) {
+  const float g = fminf(a, p.limit), u = fminf(fmaxf(b, -p.limit), p.limit);
+  return g / (1.0f + expf(-p.slope * g)) * (u + p.shift);
+}
+
 // MODE 1 (gated): x rows are gathered (row = slot_at[place] / top), w_a and w_b are the gate and up weights
-// [real][N][K], out[place][c] = silu(a) * b. MODE 2 (experts without a gate): rows gathered likewise, w_a the up
+// [real][N][K], out[place][c] = silu(a) * b. MODE 3 (gated, sums cut off at a limit): the same rows and weights,
+// out[place][c] = clipped_gate(a, b). MODE 2 (experts without a gate): rows gathered likewise, w_a the up
 // weight, out[place][c] = relu(a)^2. MODE 0: x rows are the places themselves (act [slots][K]), w_a is the down
 // weight and out[place][c] = a.
 __device__ __forceinline__ float relu_squared_f(float a) { const float r = fmaxf(a, 0.f); return r * r; }
@@ -258,8 +287,8 @@ template <typename TX, typename TW, typename TO, int MODE>
 __global__ __launch_bounds__(256) void moe_gemm_generic_kernel(
     const TX* __restrict__ x, const TW* __restrict__ w_a, const TW* __restrict__ w_b, TO* __restrict__ out,
     const int* __restrict__ offsets, const int* __restrict__ slot_at, const int* __restrict__ tiles,
-    const int* __restrict__ num_tiles, int top, int N, int K) {
-  constexpr bool GATED = MODE == 1;
+    const int* __restrict__ num_tiles, int top, int N, int K, GateParams gp) {
+  constexpr bool GATED = MODE == 1 || MODE == 3;
   constexpr bool GATHER = MODE != 0;
   const int tile = blockIdx.x;
   if (tile >= *num_tiles) return;
@@ -325,8 +354,10 @@ __global__ __launch_bounds__(256) void moe_gemm_generic_kernel(
     for (int j = 0; j < 4; ++j) {
       const int c = col0 + tx * 4 + j;
       if (c >= N) continue;
-      const float v = GATED ? silu_f(acc_a[i][j]) * acc_b[i][j]
-                            : (MODE == 2 ? relu_squared_f(acc_a[i][j]) : acc_a[i][j]);
+      const float v = MODE == 1   ? silu_f(acc_a[i][j]) * acc_b[i][j]
+                      : MODE == 3 ? clipped_gate_f(acc_a[i][j], acc_b[i][j], gp)
+                      : MODE == 2 ? relu_squared_f(acc_a[i][j])
+                                  : acc_a[i][j];
       store_from_float(out + static_cast<size_t>(place0 + r) * N + c, v);
     }
   }
@@ -335,23 +366,27 @@ __global__ __launch_bounds__(256) void moe_gemm_generic_kernel(
 extern "C" int tie_moe_generic_tile_rows() { return GR; }
 
 // gated = 1: out [slots][N] of out_dtype = silu(x Wa^T) * (x Wb^T) over gathered rows of x [T][K];
+// gated = 3: the same with clipped_gate (limit, slope, shift);
 // gated = 2: out [slots][N] of out_dtype = relu(x Wa^T)^2 over gathered rows of x [T][K];
 // gated = 0: out [slots][N] = x Wa^T over x [slots][K]. Weights [real][N][K].
 extern "C" int tie_moe_gemm_generic(const void* x, int x_dtype, const void* w_a, const void* w_b, int w_dtype, void* out,
                                     int out_dtype, int gated, const int* offsets, const int* slot_at, const int* tiles,
-                                    const int* num_tiles, int max_tiles, int top, int N, int K, hipStream_t stream) {
-  if (max_tiles <= 0 || top <= 0 || N <= 0 || K <= 0 || gated < 0 || gated > 2 || (gated == 1 && w_b == nullptr))
+                                    const int* num_tiles, int max_tiles, int top, int N, int K, float limit, float slope,
+                                    float shift, hipStream_t stream) {
+  if (max_tiles <= 0 || top <= 0 || N <= 0 || K <= 0 || gated < 0 || gated > 3 || (gated % 2 == 1 && w_b == nullptr))
     return TIE_BAD_ARGUMENT;
+  const GateParams gp{limit, slope, shift};
   if ((x_dtype | w_dtype | out_dtype) & ~1) return TIE_BAD_ARGUMENT;
   const dim3 grid(max_tiles, (N + GC - 1) / GC);
   if (grid.y > 65535) return TIE_BAD_ARGUMENT;
 #define LAUNCH_G(TX, TW, TO, G)                                                                                    \
   moe_gemm_generic_kernel<TX, TW, TO, G><<<grid, 256, 0, stream>>>(                                                \
       static_cast<const TX*>(x), static_cast<const TW*>(w_a), static_cast<const TW*>(w_b), static_cast<TO*>(out), \
-      offsets, slot_at, tiles, num_tiles, top, N, K)
+      offsets, slot_at, tiles, num_tiles, top, N, K, gp)
 #define LAUNCH(TX, TW, TO)                    \
   {                                           \
     if (gated == 1) LAUNCH_G(TX, TW, TO, 1);  \
+    else if (gated == 3) LAUNCH_G(TX, TW, TO, 3); \
     else if (gated == 2) LAUNCH_G(TX, TW, TO, 2); \
     else LAUNCH_G(TX, TW, TO, 0);             \
   }
@@ -399,9 +434,9 @@ template <int MT, int NT, int MODE>
 __global__ __launch_bounds__(256) void moe_gemm_bf16_kernel(
     const bf16_t* __restrict__ x, const bf16_t* __restrict__ w_a, const bf16_t* __restrict__ w_b,
     void* __restrict__ out, const int* __restrict__ offsets, const int* __restrict__ slot_at,
-    const int* __restrict__ tiles, const int* __restrict__ num_tiles, int top, int N, int K) {
+    const int* __restrict__ tiles, const int* __restrict__ num_tiles, int top, int N, int K, GateParams gp) {
   static_assert(MT == 1 || MT == 4 || MT == 8, "one x tile a wave, or MT / 4 loaded by each of the four waves");
-  constexpr bool GATED = MODE == 1;       // two weights, silu(a) * b
+  constexpr bool GATED = MODE == 1 || MODE == 3;       // two weights, silu(a) * b or clipped_gate(a, b)
   constexpr bool GATHER = MODE != 0;      // rows of x gathered by slot; the activations go out as bfloat16
   constexpr int OWN = MT == 1 ? 1 : MT / 4;                  // x fragments this wave loads a k-block
   const int tile = blockIdx.x;
@@ -519,8 +554,10 @@ __global__ __launch_bounds__(256) void moe_gemm_bf16_kernel(
       float v[4];
 #pragma unroll
       for (int i = 0; i < 4; ++i)
-        v[i] = GATED ? silu_f(acc_a[mt][nt][i]) * acc_b[mt][nt][i]
-                     : (MODE == 2 ? relu_squared_f(acc_a[mt][nt][i]) : acc_a[mt][nt][i]);
+        v[i] = MODE == 1   ? silu_f(acc_a[mt][nt][i]) * acc_b[mt][nt][i]
+               : MODE == 3 ? clipped_gate_f(acc_a[mt][nt][i], acc_b[mt][nt][i], gp)
+               : MODE == 2 ? relu_squared_f(acc_a[mt][nt][i])
+                           : acc_a[mt][nt][i];
       if (GATHER) {
         bf16_t* o = static_cast<bf16_t*>(out) + at;
         if (c + 3 < N && N % 4 == 0) {
@@ -549,30 +586,33 @@ extern "C" int tie_moe_bf16_tile_rows(int slots, int real) {
 }
 
 // bfloat16 x and weights; gated = 1: out bfloat16 [slots][N] = silu(x Wa^T) * (x Wb^T) over gathered rows of x;
+// gated = 3: the same with clipped_gate (limit, slope, shift);
 // gated = 2: out bfloat16 [slots][N] = relu(x Wa^T)^2 over gathered rows of x;
 // gated = 0: out float32 [slots][N] = x Wa^T over x [slots][K]. tile_rows (16, 64 or 128) as given to tie_moe_align.
 extern "C" int tie_moe_gemm_bf16(const void* x, const void* w_a, const void* w_b, void* out, int gated,
                                  const int* offsets, const int* slot_at, const int* tiles, const int* num_tiles,
-                                 int max_tiles, int tile_rows, int top, int N, int K, hipStream_t stream) {
-  if (max_tiles <= 0 || top <= 0 || N <= 0 || K <= 0 || K % 8 != 0 || gated < 0 || gated > 2 ||
-      (gated == 1 && w_b == nullptr) || (tile_rows != 16 && tile_rows != 64 && tile_rows != 128) || reinterpret_cast<uintptr_t>(x) % 16 != 0 ||
+                                 int max_tiles, int tile_rows, int top, int N, int K, float limit, float slope,
+                                 float shift, hipStream_t stream) {
+  if (max_tiles <= 0 || top <= 0 || N <= 0 || K <= 0 || K % 8 != 0 || gated < 0 || gated > 3 ||
+      (gated % 2 == 1 && w_b == nullptr) || (tile_rows != 16 && tile_rows != 64 && tile_rows != 128) || reinterpret_cast<uintptr_t>(x) % 16 != 0 ||
       reinterpret_cast<uintptr_t>(w_a) % 16 != 0 || reinterpret_cast<uintptr_t>(w_b) % 16 != 0 ||
       reinterpret_cast<uintptr_t>(out) % 16 != 0)
     return TIE_BAD_ARGUMENT;
-  const int columns = tile_rows == 16 ? 16 : (tile_rows == 128 && gated == 1 ? 128 : 256);   // of a workgroup
+  const int columns = tile_rows == 16 ? 16 : (tile_rows == 128 && gated % 2 == 1 ? 128 : 256);   // of a workgroup
+  const GateParams gp{limit, slope, shift};
   const dim3 grid(max_tiles, (N + columns - 1) / columns);
   if (grid.y > 65535) return TIE_BAD_ARGUMENT;
 #define LAUNCH_B(MT, NT, G)                                                                                  \
   moe_gemm_bf16_kernel<MT, NT, G><<<grid, 256, 0, stream>>>(static_cast<const bf16_t*>(x),                   \
                                                             static_cast<const bf16_t*>(w_a),                 \
                                                             static_cast<const bf16_t*>(w_b), out, offsets,   \
-                                                            slot_at, tiles, num_tiles, top, N, K)
+                                                            slot_at, tiles, num_tiles, top, N, K, gp)
   if (tile_rows == 128) {
-    if (gated == 1) LAUNCH_B(8, 2, 1); else if (gated == 2) LAUNCH_B(8, 4, 2); else LAUNCH_B(8, 4, 0);
+    if (gated == 1) LAUNCH_B(8, 2, 1); else if (gated == 3) LAUNCH_B(8, 2, 3); else if (gated == 2) LAUNCH_B(8, 4, 2); else LAUNCH_B(8, 4, 0);
   } else if (tile_rows == 64) {
-    if (gated == 1) LAUNCH_B(4, 4, 1); else if (gated == 2) LAUNCH_B(4, 4, 2); else LAUNCH_B(4, 4, 0);
+    if (gated == 1) LAUNCH_B(4, 4, 1); else if (gated == 3) LAUNCH_B(4, 4, 3); else if (gated == 2) LAUNCH_B(4, 4, 2); else LAUNCH_B(4, 4, 0);
   } else {
-    if (gated == 1) LAUNCH_B(1, 1, 1); else if (gated == 2) LAUNCH_B(1, 1, 2); else LAUNCH_B(1, 1, 0);
+    if (gated == 1) LAUNCH_B(1, 1, 1); else if (gated == 3) LAUNCH_B(1, 1, 3); else if (gated == 2) LAUNCH_B(1, 1, 2); else LAUNCH_B(1, 1, 0);
   }
 #undef LAUNCH_B
   return tie_launch_status();

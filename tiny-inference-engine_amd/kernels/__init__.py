@@ -62,6 +62,7 @@ _SOURCES = {
     "delta_rule": ("tie_delta_rule", "delta_rule.hip"),
     "latent": ("tie_latent", "latent.hip"),
     "pointwise": ("tie_pointwise", "pointwise.hip"),
+    "residual": ("tie_residual", "residual.hip"),
 }
 # libraries compiled once per head size: key -> (file stem prefix, source)
 _PER_HEAD_DIM = {
@@ -109,16 +110,16 @@ _SIGNATURES = {
         "tie_argmax_static": [_c_void, _c_void, _c_void, _c_int, _c_int, _c_void],
     },
     "moe": {
-        "tie_moe_route": [_c_void, _c_int, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
-                          _c_float, _c_float, _c_int, _c_void, _c_void, _c_void],
+        "tie_moe_route": [_c_void, _c_int, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
+                          _c_int, _c_float, _c_float, _c_int, _c_void, _c_void, _c_void],
         "tie_moe_max_tiles": [_c_int, _c_int, _c_int],
         "tie_moe_align": [_c_void, _c_int, _c_int, _c_int, _c_void, _c_void, _c_void, _c_void, _c_int, _c_void, _c_void],
         "tie_moe_generic_tile_rows": [],
         "tie_moe_gemm_generic": [_c_void, _c_int, _c_void, _c_void, _c_int, _c_void, _c_int, _c_int, _c_void, _c_void,
-                                 _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_void],
+                                 _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_void],
         "tie_moe_bf16_tile_rows": [_c_int, _c_int],
         "tie_moe_gemm_bf16": [_c_void, _c_void, _c_void, _c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_int,
-                              _c_int, _c_int, _c_int, _c_int, _c_void],
+                              _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_void],
         "tie_moe_combine": [_c_void, _c_void, _c_void, _c_void, _c_int, _c_void, _c_int, _c_int, _c_int, _c_int, _c_void],
     },
     "gemm_generic": {
@@ -147,18 +148,23 @@ _SIGNATURES = {
                          _c_int, _c_void, _c_void, _c_float, _c_float, _c_float, _c_void, _c_int, _c_void],
         "tie_conv_state_update": [_c_void, _c_int, _c_int, _c_void, _c_void, _c_void, _c_int, _c_int, _c_void],
         "tie_delta_prepare": [_c_void, _c_int, _c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_void, _c_int,
-                              _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void, _c_int, _c_void],
+                              _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void, _c_int, _c_void],
         "tie_gated_delta_scan": [_c_void, _c_int, _c_void, _c_int, _c_void, _c_void, _c_void, _c_int, _c_int, _c_int,
-                                 _c_int, _c_int, _c_void],
+                                 _c_int, _c_int, _c_int, _c_void],
         "tie_gated_delta_scan_chunked": [_c_void, _c_int, _c_void, _c_int, _c_void, _c_void, _c_int, _c_void, _c_void,
                                          _c_int, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_void],
-        "tie_grouped_gated_rms_norm": [_c_void, _c_int, _c_void, _c_float, _c_void, _c_int, _c_void, _c_int, _c_int,
-                                       _c_int, _c_int, _c_void],
+        "tie_grouped_gated_rms_norm": [_c_void, _c_int, _c_void, _c_float, _c_void, _c_int, _c_int, _c_void, _c_int,
+                                       _c_int, _c_int, _c_int, _c_void],
     },
     "pointwise": {
         "tie_dynamic_tanh": [_c_void, _c_void, _c_long, _c_int, _c_void, _c_void, _c_void, _c_void, _c_int, _c_void,
                              _c_int, _c_int, _c_int, _c_void],
         "tie_token_gate": [_c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_void, _c_int, _c_int, _c_int, _c_void],
+    },
+    "residual": {
+        "tie_add_results": [_c_void, _c_float, _c_void, _c_long, _c_int, _c_void, _c_long, _c_int, _c_void, _c_void,
+                            _c_void, _c_void, _c_int, _c_int, _c_void, _c_float, _c_int, _c_void, _c_int, _c_int,
+                            _c_int, _c_void],
     },
     "latent": {
         "tie_rms_norm_columns": [_c_void, _c_int, _c_void, _c_float, _c_void, _c_int, _c_int, _c_int, _c_void],
@@ -166,7 +172,7 @@ _SIGNATURES = {
                                _c_int, _c_int, _c_int, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
                                _c_int, _c_void],
         "tie_head_linear": [_c_void, _c_int, _c_int, _c_int, _c_void, _c_int, _c_void, _c_int, _c_int, _c_int, _c_void,
-                            _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void],
+                            _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void],
     },
     "skinny_gemm_bf16": {
         "tie_skinny_gemm_splits": [_c_int, _c_int],
@@ -1778,12 +1784,15 @@ MOE_MAX_EXPERTS = 1024       # MOE_MAX_EXPERTS of csrc/moe.hip
 
 
 MOE_MAX_GROUP_TOP = 8         # MOE_MAX_GROUP_TOP of csrc/moe.hip
+MOE_SCORINGS = {"softmax": 0, "sigmoid": 1, "softmax_chosen": 2}     # SCORE_* of csrc/moe.hip
 
 
 def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], groups: int, keep: int, top: int,
               ids: torch.Tensor, weights: torch.Tensor, scoring: str = "softmax", group_top: int = 1,
-              renormalize: bool = False, renorm_eps: float = 0.0, weight_scale: float = 1.0, shared: int = 0) -> None:
-    """The router's choice for every row of float32 ``logits [T, E]`` (``[T, E + 1]`` with ``shared``).
+              renormalize: bool = False, renorm_eps: float = 0.0, weight_scale: float = 1.0, shared: int = 0,
+              bias: Optional[torch.Tensor] = None) -> None:
+    """The router's choice for every row of float32 ``logits [T, E]`` (``[T, E + 1]`` with ``shared``), to which
+    ``bias`` (float32 ``[E]``) is added first where there is one.
 
     ``s = softmax(logits)`` over the experts, or with ``scoring`` ``"sigmoid"`` ``sigmoid(logits)`` expert by expert;
     the choice looks at ``s + correction``: the experts form ``groups`` equal groups of neighbours, a group scores
@@ -1791,7 +1800,8 @@ def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], groups: 
     eligible, and the ``top`` best of those are chosen (ties to the lower index) into ``ids`` int32; ``weights``
     float32 are ``s`` at the chosen, with ``renormalize`` divided by their sum + ``renorm_eps``, times
     ``weight_scale``. ``shared`` n: both arrays are ``[T, top + n]``, the last n slots of a row name the experts
-    ``E .. E + n - 1`` (experts every row uses) with the weight ``sigmoid(logits[:, E])``.
+    ``E .. E + n - 1`` (experts every row uses) with the weight ``sigmoid(logits[:, E])``. ``scoring``
+    ``"softmax_chosen"``: ``s`` are the logits themselves and the weights the softmax over the chosen ones alone.
     """
     _f32(logits, "router logits")
     T, row = logits.shape
@@ -1803,14 +1813,16 @@ def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], groups: 
     _f32(weights, "routing weights", (T, slots))
     if tuple(ids.shape) != (T, slots):
         raise InvalidArgument(f"chosen experts {list(ids.shape)} do not fit {[T, slots]}")
-    if scoring not in ("softmax", "sigmoid"):
-        raise InvalidArgument(f"router scoring '{scoring}' (supported: softmax, sigmoid)")
+    if bias is not None:
+        _f32(bias, "the logits' bias", (E,))
+    if scoring not in MOE_SCORINGS:
+        raise InvalidArgument(f"router scoring '{scoring}' (supported: {', '.join(MOE_SCORINGS)})")
     if not 0 < E <= MOE_MAX_EXPERTS or groups <= 0 or E % groups or not 0 < keep <= groups or not 0 < top <= E or \
             not 0 < group_top <= MOE_MAX_GROUP_TOP or shared < 0:
         raise InvalidArgument(f"moe_route: {E} experts (at most {MOE_MAX_EXPERTS}) in {groups} groups scored by their "
                               f"{group_top} best, {keep} kept, top {top}")
-    _call(_lib("moe").tie_moe_route, "moe_route", logits.data_ptr(), row, _ptr(correction), T, E, groups, keep, top,
-          int(scoring == "sigmoid"), int(group_top), int(bool(renormalize)), float(renorm_eps), float(weight_scale),
+    _call(_lib("moe").tie_moe_route, "moe_route", logits.data_ptr(), row, _ptr(bias), _ptr(correction), T, E, groups,
+          keep, top, MOE_SCORINGS[scoring], int(group_top), int(bool(renormalize)), float(renorm_eps), float(weight_scale),
           int(shared), ids.data_ptr(), weights.data_ptr(), _stream())
 
 
@@ -1875,14 +1887,19 @@ def _moe_weights(w: torch.Tensor, real: int, name: str):
 
 
 def moe_gate_up(x: torch.Tensor, w_gate: Optional[torch.Tensor], w_up: torch.Tensor, rows: ExpertRows,
-                act: torch.Tensor) -> None:
+                act: torch.Tensor, clipped: Optional[tuple] = None) -> None:
     """``act[place] = silu(x[row] Wg_e^T) * (x[row] Wu_e^T)`` for every sorted slot: ``x [T, K]``, weights
     ``[real, F, K]``. Without gate weights (``w_gate`` None) the experts have no gate and the activation is the square
-    of relu: ``act[place] = relu(x[row] Wu_e^T)^2``."""
+    of relu: ``act[place] = relu(x[row] Wu_e^T)^2``. ``clipped`` ``(limit, slope, shift)`` (with gate weights): the sums
+    are cut off first, ``g = min(gate sum, limit)``, ``u = clamp(up sum, -limit, limit)``, and the activation is
+    ``g sigmoid(slope g) (u + shift)``."""
     _gpu(x, "the experts' input rows")
     _gpu(act, "the experts' activations")
     F_, K = _moe_weights(w_up, rows.real, "up weights")
-    mode = 2 if w_gate is None else 1
+    mode = 2 if w_gate is None else (1 if clipped is None else 3)
+    if clipped is not None and (w_gate is None or not clipped[0] > 0):
+        raise InvalidArgument(f"clipped sums need a gate and a positive limit, got {clipped}")
+    gate_params = tuple(float(v) for v in clipped) if clipped is not None else (0.0, 0.0, 0.0)
     if w_gate is not None and (tuple(w_up.shape) != tuple(w_gate.shape) or w_up.dtype != w_gate.dtype or
                                not w_gate.is_contiguous() or not w_gate.is_cuda):
         raise InvalidArgument("gate and up weights must be alike")
@@ -1893,13 +1910,13 @@ def moe_gate_up(x: torch.Tensor, w_gate: Optional[torch.Tensor], w_up: torch.Ten
         _call(_lib("moe").tie_moe_gemm_bf16, "moe_gate_up", x.data_ptr(), first.data_ptr(),
               w_up.data_ptr() if w_gate is not None else None,
               act.data_ptr(), mode, rows.offsets.data_ptr(), rows.slot_at.data_ptr(), rows.tiles.data_ptr(),
-              rows.num_tiles.data_ptr(), rows.max_tiles, rows.tile_rows, rows.top, F_, K, _stream())
+              rows.num_tiles.data_ptr(), rows.max_tiles, rows.tile_rows, rows.top, F_, K, *gate_params, _stream())
         return
     _call(_lib("moe").tie_moe_gemm_generic, "moe_gate_up", x.data_ptr(), _code(x, "rows"), first.data_ptr(),
           w_up.data_ptr() if w_gate is not None else None, _code(first, "expert weights"), act.data_ptr(),
           _code(act, "activations"), mode,
           rows.offsets.data_ptr(), rows.slot_at.data_ptr(), rows.tiles.data_ptr(), rows.num_tiles.data_ptr(),
-          rows.max_tiles, rows.top, F_, K, _stream())
+          rows.max_tiles, rows.top, F_, K, *gate_params, _stream())
 
 
 def moe_down(act: torch.Tensor, w_down: torch.Tensor, rows: ExpertRows, parts: torch.Tensor) -> None:
@@ -1912,12 +1929,12 @@ def moe_down(act: torch.Tensor, w_down: torch.Tensor, rows: ExpertRows, parts: t
     if _moe_on_matrix_cores(rows, act, w_down, parts, False):
         _call(_lib("moe").tie_moe_gemm_bf16, "moe_down", act.data_ptr(), w_down.data_ptr(), None, parts.data_ptr(), 0,
               rows.offsets.data_ptr(), rows.slot_at.data_ptr(), rows.tiles.data_ptr(), rows.num_tiles.data_ptr(),
-              rows.max_tiles, rows.tile_rows, rows.top, N, F_, _stream())
+              rows.max_tiles, rows.tile_rows, rows.top, N, F_, 0.0, 0.0, 0.0, _stream())
         return
     _call(_lib("moe").tie_moe_gemm_generic, "moe_down", act.data_ptr(), _code(act, "activations"), w_down.data_ptr(),
           None, _code(w_down, "down weights"), parts.data_ptr(), F32, 0, rows.offsets.data_ptr(),
           rows.slot_at.data_ptr(), rows.tiles.data_ptr(), rows.num_tiles.data_ptr(), rows.max_tiles, rows.top, N, F_,
-          _stream())
+          0.0, 0.0, 0.0, _stream())
 
 
 def moe_combine(routed: RoutedParts, out: torch.Tensor, accumulate: bool = False) -> None:
@@ -2013,6 +2030,56 @@ def layer_norm(x: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.Ten
         return
     _call(_lib("hyper").tie_layer_norm, "layer_norm", x.data_ptr(), _code(x, "layer norm input"), weight.data_ptr(),
           float(eps), out.data_ptr(), _code(out, "layer norm output"), _ptr(rows), count, n, _stream())
+
+
+def add_results(x: torch.Tensor, results, scale: float = 1.0, norm: Optional[tuple] = None) -> None:
+    """``x += scale * (the sum of results)`` for the results of sub-layers that ran side by side, one pass over the
+    float32 stream ``x [T, n]``. ``results``: up to two of float32 rows ``[T, n]`` or planes of partial sums
+    ``[P, T, n]`` (added in plane order) and at most one ``RoutedParts``. ``norm`` ``(kind, weight, eps, out)``: also
+    ``out = norm(x)`` of the updated rows, ``kind`` "layer_norm" or "rms_norm"."""
+    _f32(x, "the stream")
+    T, n = x.shape
+    dense, routed = [], None
+    for y in results:
+        if isinstance(y, RoutedParts):
+            if routed is not None:
+                raise InvalidArgument("add_results takes one routed feed-forward's parts")
+            routed = y
+            continue
+        _f32(y, "a sub-layer's result")
+        if y.dim() not in (2, 3) or tuple(y.shape[-2:]) != (T, n):
+            raise InvalidArgument(f"add_results: a result {list(y.shape)} does not fit the stream {[T, n]}")
+        dense.append(y)
+    if len(dense) > 2 or n > ROW_IN_LDS_MAX:
+        raise InvalidArgument(f"add_results takes two results besides a routed one, of rows of at most {ROW_IN_LDS_MAX}")
+    parts = where = weights = self_rows = None
+    self_code, top = F32, 1
+    if routed is not None:
+        parts, where, weights, self_rows = routed.parts, routed.where, routed.weights, routed.self_rows
+        top = where.shape[1]
+        _f32(parts, "the experts' results")
+        _i32(where, "places", T * top)
+        _f32(weights, "routing weights", (T, top))
+        _gpu(self_rows, "the feed-forward's input rows")
+        if parts.shape[-1] != n or tuple(self_rows.shape) != (T, n):
+            raise InvalidArgument("add_results: the routed parts do not fit the stream")
+        self_code = _code(self_rows, "the feed-forward's input rows")
+    kind, weight, eps, out = norm if norm is not None else ("layer_norm", None, 0.0, None)
+    if norm is not None:
+        if _NORM_KINDS.get(kind) not in (0, 1):
+            raise InvalidArgument(f"add_results norms with 'layer_norm' or 'rms_norm', not '{kind}'")
+        _f32(weight, "norm weight", (n,))
+        _gpu(out, "normed rows")
+        if tuple(out.shape) != (T, n):
+            raise InvalidArgument(f"add_results: normed rows {list(out.shape)} do not fit {[T, n]}")
+    if T == 0:
+        return
+    dense += [None] * (2 - len(dense))
+    args = [v for y in dense for v in (_ptr(y), T * n if y is not None else 0,
+                                       0 if y is None else (y.shape[0] if y.dim() == 3 else 1))]
+    _call(_lib("residual").tie_add_results, "add_results", x.data_ptr(), float(scale), *args, _ptr(parts), _ptr(where),
+          _ptr(weights), _ptr(self_rows), self_code, top, _ptr(weight), float(eps), _NORM_KINDS[kind], _ptr(out),
+          _code(out, "normed rows") if out is not None else F32, T, n, _stream())
 
 
 def hyper_connection(streams: torch.Tensor, x: Optional[torch.Tensor] = None, from_x: bool = False, fold: bool = False,
@@ -2124,25 +2191,35 @@ def conv_state_update(u: torch.Tensor, taps: int, state: torch.Tensor, batch, ch
           _stream())
 
 
+def delta_row(kv_heads: int, heads: int, key_dim: int, value_dim: int, head_decay: bool = False) -> int:
+    """Columns of a row of ``delta_prepare``: q, k, v, the decays, beta; with one decay a head their logarithms too, and
+    the row rounded up to four words."""
+    base = 2 * kv_heads * key_dim + heads * value_dim + heads
+    return -(-(base + 2 * heads) // 4) * 4 if head_decay else base + heads * key_dim
+
+
 def delta_prepare(u: torch.Tensor, weight: torch.Tensor, taps: int, state: Optional[torch.Tensor], batch,
                   a: torch.Tensor, A_log: torch.Tensor, dt_bias: torch.Tensor, kv_heads: int, heads: int, key_dim: int,
-                  value_dim: int, out: torch.Tensor) -> None:
+                  value_dim: int, out: torch.Tensor, head_decay: bool = False) -> None:
     """What the gated delta rule takes of every token, from the projections' float32 sums.
 
     ``u`` rows ``[q (G d) | k (G d) | v (H e) | b (H)]``: q, k, v through the short convolution and silu, q and k
     made unit vectors per head (q also times ``d ** -0.5``), ``beta = sigmoid(b)``; ``a`` rows ``[H d]``: the decays
-    ``exp(-exp(A_log[head]) * softplus(a + dt_bias))``. ``out`` rows: ``[q | k | v | decay | beta]`` float32."""
+    ``exp(-exp(A_log[head]) * softplus(a + dt_bias))``. ``out`` rows: ``[q | k | v | decay | beta]`` float32, of
+    ``delta_row(...)`` columns. ``head_decay``: one decay a head (``a`` rows and ``dt_bias`` of ``[H]``); the decays'
+    logarithms follow ``beta``."""
     G, H, d, e = kv_heads, heads, key_dim, value_dim
     C = 2 * G * d + H * e
+    decays = H if head_decay else H * d
     _gpu_strided(u, "projected rows")
     _gpu_strided(a, "decay rows")
     T = u.shape[0]
-    if u.dtype != torch.float32 or u.shape[1] < C + H or a.dtype != torch.float32 or tuple(a.shape) != (T, H * d):
+    if u.dtype != torch.float32 or u.shape[1] < C + H or a.dtype != torch.float32 or tuple(a.shape) != (T, decays):
         raise InvalidArgument(f"projected rows {list(u.shape)} / decay rows {list(a.shape)} do not fit the heads")
     _f32(weight, "convolution weights", (C, taps))
     _f32(A_log, "A_log", (H,))
-    _f32(dt_bias, "dt_bias", (H * d,))
-    _f32(out, "delta rule rows", (T, C + H + H * d))
+    _f32(dt_bias, "dt_bias", (decays,))
+    _f32(out, "delta rule rows", (T, delta_row(G, H, d, e, head_decay)))
     if not 1 <= taps <= CONV_MAX_TAPS or C > ROW_IN_LDS_MAX:
         raise InvalidArgument(f"a convolution of {taps} taps over {C} channels exceeds what the kernel takes")
     if taps > 1:
@@ -2153,8 +2230,8 @@ def delta_prepare(u: torch.Tensor, weight: torch.Tensor, taps: int, state: Optio
         return
     _call(_lib("delta_rule").tie_delta_prepare, "delta_prepare", u.data_ptr(), u.stride(0), weight.data_ptr(), taps,
           _ptr(state), batch.state_slots.data_ptr(), batch.seq_of_row.data_ptr(), batch.query_start.data_ptr(),
-          a.data_ptr(), a.stride(0), A_log.data_ptr(), dt_bias.data_ptr(), T, G, H, d, e, out.data_ptr(),
-          out.stride(0), _stream())
+          a.data_ptr(), a.stride(0), A_log.data_ptr(), dt_bias.data_ptr(), T, G, H, d, e, int(head_decay),
+          out.data_ptr(), out.stride(0), _stream())
 
 
 DELTA_CHUNK_ROWS = 256                 # rows of a chunk of the gated delta rule's chunked walk
@@ -2163,7 +2240,8 @@ DELTA_CHUNK_SCRATCH_MAX = 1 << 30      # bytes of chunk states above which a ste
 
 
 def gated_delta_scan(tok: torch.Tensor, out: torch.Tensor, state: torch.Tensor, batch, kv_heads: int, heads: int,
-                     key_dim: int, value_dim: int, chunks: Optional[ScanChunks] = None, scratch=None) -> None:
+                     key_dim: int, value_dim: int, chunks: Optional[ScanChunks] = None, scratch=None,
+                     head_decay: bool = False) -> None:
     """The gated delta rule, token by token through each sequence's state ``[slots, H, d, e]`` (float32):
     ``S <- decay * S`` row by row; ``u = beta * (v - S^T k)``; ``S <- S + k u^T``; ``o = S^T q``. ``tok``: the rows of
     ``delta_prepare``; ``out`` float32 ``[T, H e]``.
@@ -2176,7 +2254,7 @@ def gated_delta_scan(tok: torch.Tensor, out: torch.Tensor, state: torch.Tensor, 
     outputs. The same values up to rounding."""
     G, H, d, e = kv_heads, heads, key_dim, value_dim
     T = tok.shape[0]
-    _f32(tok, "delta rule rows", (T, 2 * G * d + H * e + H + H * d))
+    _f32(tok, "delta rule rows", (T, delta_row(G, H, d, e, head_decay)))
     _f32(out, "delta rule output", (T, H * e))
     _f32(state, "delta rule state")
     if tuple(state.shape[1:]) != (H, d, e) or H % G or d > DELTA_RULE_MAX_DIM:
@@ -2184,7 +2262,7 @@ def gated_delta_scan(tok: torch.Tensor, out: torch.Tensor, state: torch.Tensor, 
                               f"{DELTA_RULE_MAX_DIM}, {G} key heads)")
     if batch.num_seqs == 0:
         return
-    if chunks is not None and chunks.count * H * d * (e + d) * 4 <= DELTA_CHUNK_SCRATCH_MAX:
+    if chunks is not None and not head_decay and chunks.count * H * d * (e + d) * 4 <= DELTA_CHUNK_SCRATCH_MAX:
         ends = scratch("delta_rule.chunk_ends", (chunks.count, H, d, e + d), torch.float32)
         starts = scratch("delta_rule.chunk_starts", (chunks.count, H, d, e), torch.float32)
         _call(_lib("delta_rule").tie_gated_delta_scan_chunked, "gated_delta_scan_chunked", tok.data_ptr(),
@@ -2194,12 +2272,13 @@ def gated_delta_scan(tok: torch.Tensor, out: torch.Tensor, state: torch.Tensor, 
         return
     _call(_lib("delta_rule").tie_gated_delta_scan, "gated_delta_scan", tok.data_ptr(), tok.stride(0), out.data_ptr(),
           out.stride(0), state.data_ptr(), batch.query_start.data_ptr(), batch.state_slots.data_ptr(), batch.num_seqs,
-          G, H, d, e, _stream())
+          G, H, d, e, int(head_decay), _stream())
 
 
 def grouped_gated_rms_norm(o: torch.Tensor, weight: torch.Tensor, eps: float, gate: torch.Tensor, out: torch.Tensor,
-                           groups: int) -> None:
-    """out = o / rms(o over each of ``groups`` equal groups of columns) * weight[column in its group] * sigmoid(gate).
+                           groups: int, activation: str = "sigmoid") -> None:
+    """out = o / rms(o over each of ``groups`` equal groups of columns) * weight[column in its group] * act(gate),
+    ``activation`` "sigmoid" or "silu".
     ``o`` float32 ``[T, n]``, ``gate`` float32 rows of n (a view whose rows may lie further apart)."""
     _f32(o, "gated norm input")
     T, n = o.shape
@@ -2212,10 +2291,12 @@ def grouped_gated_rms_norm(o: torch.Tensor, weight: torch.Tensor, eps: float, ga
     _gpu(out, "gated norm output")
     if tuple(out.shape) != (T, n):
         raise InvalidArgument(f"gated norm output {list(out.shape)} does not match input {[T, n]}")
+    if activation not in ("sigmoid", "silu"):
+        raise InvalidArgument(f"the gate's activation is 'sigmoid' or 'silu', not '{activation}'")
     if T == 0:
         return
     _call(_lib("delta_rule").tie_grouped_gated_rms_norm, "grouped_gated_rms_norm", o.data_ptr(), o.stride(0),
-          weight.data_ptr(), float(eps), gate.data_ptr(), gate.stride(0), out.data_ptr(),
+          weight.data_ptr(), float(eps), gate.data_ptr(), gate.stride(0), int(activation == "silu"), out.data_ptr(),
           _code(out, "gated norm output"), T, groups, n // groups, _stream())
 
 
@@ -2291,7 +2372,7 @@ def rms_norm_columns(x: torch.Tensor, weight: torch.Tensor, eps: float, out: tor
 def head_linear(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, gate: Optional[torch.Tensor] = None) -> None:
     """``out[t, h] = w[h] @ x[t, h]`` for every head: ``x`` ``[T, H, K]``, ``w`` ``[H, N, K]``, ``out`` ``[T, H, N]``
     (views whose rows and heads may lie further apart; the last dimension is dense), float32 sums; with ``gate``
-    (float32 ``[T, H, N]`` view) the result is multiplied by ``sigmoid(gate)``."""
+    (float32 ``[T, H, N]`` view, or ``[T, H, 1]``: one gate a head) the result is multiplied by ``sigmoid(gate)``."""
     for t, name in ((x, "head inputs"), (out, "head outputs")):
         if not isinstance(t, torch.Tensor) or not t.is_cuda:
             raise KernelUnavailable(f"{name} must be a tensor on a GPU: the engine's kernels have no CPU fallback")
@@ -2305,11 +2386,12 @@ def head_linear(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, gate: Optio
     if gate is not None:
         if not gate.is_cuda or gate.dim() != 3:
             raise InvalidArgument("head gates must be a [rows, heads, width] tensor on the GPU")
-        if gate.dtype != torch.float32 or tuple(gate.shape) != (T, H, N) or gate.stride(2) != 1:
+        if gate.dtype != torch.float32 or tuple(gate.shape) not in ((T, H, N), (T, H, 1)) or \
+                (gate.shape[2] > 1 and gate.stride(2) != 1):
             raise InvalidArgument(f"head gates {list(gate.shape)} {gate.dtype} do not fit float32 {[T, H, N]}")
     if T == 0:
         return
     _call(_lib("latent").tie_head_linear, "head_linear", x.data_ptr(), _code(x, "head inputs"), x.stride(0), x.stride(1),
           w.data_ptr(), _code(w, "head matrices"), out.data_ptr(), _code(out, "head outputs"), out.stride(0),
           out.stride(1), _ptr(gate), gate.stride(0) if gate is not None else 0,
-          gate.stride(1) if gate is not None else 0, T, H, N, K, _stream())
+          gate.stride(1) if gate is not None else 0, int(gate is None or gate.shape[2] == N), T, H, N, K, _stream())

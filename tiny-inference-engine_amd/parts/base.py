@@ -319,6 +319,9 @@ class Norm(Part):
     # True: forward() takes ``lazy=True`` and may then return rows without their 1 / rms, registered with
     # ``ctx.set_row_scale``: only for a consumer that applies it (``takes_row_scale``; see ``Block.normed``).
     leaves_row_scale = False
+    # True: forward() takes ``results`` = (sub-layers' results, scale), adds them to x in its own pass and norms the sum.
+    adds_results = False
+    reads_either_type = False   # True: forward() also reads bfloat16 rows (an embedding table's, gathered by ``rows``)
 
     def forward(self, ctx: StepContext, x: torch.Tensor, rows: Optional[torch.Tensor] = None,
                 out_name: str = "norm.out", out_dtype: torch.dtype = None) -> torch.Tensor:
@@ -378,7 +381,9 @@ class Block(Part):
 
     @staticmethod
     def normed(ctx: StepContext, norm, x: torch.Tensor, consumer=None) -> torch.Tensor:
-        if not norm.adds_owed:
+        if norm.adds_owed:
+            ctx.run_late()
+        else:
             ctx.settle()
         if getattr(norm, "leaves_row_scale", False) and getattr(consumer, "takes_row_scale", False):
             return norm.forward(ctx, x, lazy=True)

@@ -17,6 +17,11 @@ layers share), ``g = gelu_tanh(W_gate x) * e`` from the stream itself (no norm b
 ``x += y / sqrt(mean(y^2) + eps) * w``. Parameters: ``hidden``, ``dim``, ``vocab``, ``table`` (tensor name),
 ``table_columns``, ``first``, ``eps``, ``names`` (``gate``, ``proj``, ``norm``).
 
+``parallel_residual`` runs both sub-layers side by side: with ``h = pre(x)``, one norm, ``x += scale * (mixer(h) +
+feed_forward(h))``. What a layer adds is left with the step and rides in the next layer's first pass over the stream,
+which adds the sub-layers' results (rows, planes of partial sums, a routed feed-forward's parts not yet combined) and
+norms the sum in one kernel. Parameters: ``hidden``, ``scale``.
+
 ``hyper_connections`` keeps ``streams`` copies of the residual instead of one. All start as the embedding's rows.
 Sub-layer q of a layer (its mixer, then its feed-forward) has three small tensors ``in`` ``[streams]``, ``out``
 ``[streams]`` and ``mix`` ``[streams, streams]`` (from, to): it reads ``u = sum_s in[s] x_s``, computes
@@ -178,6 +183,55 @@ class SandwichNormBlock(Block):
         missing = [n for n in needed if n not in layer.norms]
         if missing:
             raise InvalidArgument(f"a sandwich_norm block needs the norms {', '.join(needed)}; missing {', '.join(missing)}")
+
+
+@register_part("block", "parallel_residual")
+class ParallelResidualBlock(Block):
+    capturable = True
+    replayable = True      # what is left for the next layer names scratch memory only, the same for every layer
+    NORMS = ("pre",)
+
+    def __init__(self, params):
+        super().__init__(params)
+        self.hidden = int(params["hidden"])
+        self.scale = float(params.get("scale", 1.0))
+
+    @classmethod
+    def check_layer(cls, layer) -> None:
+        if layer.mixer is None and layer.feed_forward is None:
+            raise InvalidArgument("a parallel_residual block needs a mixer, a feed-forward or both")
+        if "pre" not in layer.norms:
+            raise InvalidArgument("a parallel_residual block needs the norm 'pre'")
+
+    @staticmethod
+    def _result(ctx: StepContext, part, run, name: str):
+        """A sub-layer's result: float32 rows, planes of partial sums or a routed feed-forward's parts."""
+        if getattr(part, "returns_result", False):
+            return run(None)
+        zeros = ctx.scratch(name, (ctx.num_tokens, part.hidden), torch.float32)
+        zeros.zero_()
+        run(zeros)
+        ctx.settle()
+        return zeros
+
+    def forward(self, ctx: StepContext, x: torch.Tensor, layer, cache) -> None:
+        norm = layer.norms["pre"]
+        key = ("parallel_residual.add", x.shape[0], self.hidden, self.scale)
+        left = ctx.take_late(key) if norm.adds_results else None
+        if left is not None:
+            h = norm.forward(ctx, x, results=left)
+        else:
+            h = self.normed(ctx, norm, x)
+        results = []
+        if layer.mixer is not None:
+            results.append(self._result(ctx, layer.mixer, lambda residual: layer.mixer.forward(ctx, h, cache, residual),
+                                        "block.mixer_result"))
+        if layer.feed_forward is not None:
+            results.append(self._result(ctx, layer.feed_forward,
+                                        lambda residual: layer.feed_forward.forward(ctx, h, residual),
+                                        "block.feed_forward_result"))
+        # settle() (the model's end, a hook, another kind of block) adds them without a norm behind
+        ctx.leave_late(key, lambda left: kernels.add_results(x, *left), (results, self.scale))
 
 
 @register_part("block", "hyper_connections")

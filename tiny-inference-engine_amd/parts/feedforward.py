@@ -31,6 +31,10 @@ result is the weighted sum of the chosen experts' results. Parameters: ``hidden`
 For designs that have them: ``scoring`` ``sigmoid`` (scores are ``sigmoid(logits)`` expert by expert);
 ``group_top`` n (a group scores the sum of its n best members instead of its best); ``renormalize`` True (the
 weights are the chosen scores divided by their sum + ``renorm_eps``); ``weight_scale`` (a factor on the weights);
+``scoring`` ``softmax_chosen`` (the choice looks at the logits, to which the vector ``router_bias`` is added where it is
+named, and the weights are the softmax over the chosen logits alone); ``expert_activation`` ``clipped_gate`` with
+``activation_params`` (limit, slope, shift), ``g = min(gate_e h, limit)``, ``u = clamp(up_e h, -limit, limit)``,
+``down_e(g sigmoid(slope g) (u + shift))``;
 ``expert_activation`` ``relu_squared`` with no ``gate`` names (experts without a gate, ``down_e(relu(up_e h)^2)``);
 ``shared`` ``{"intermediate", "up", "down", "gate_logit"}`` (and ``"gate"`` for gated experts): one more expert of the
 same form that every row uses, its result multiplied by ``sigmoid(w_gate_logit . h)``, one number a row. It runs as
@@ -181,8 +185,8 @@ class RoutedExperts(FeedForward):
         self.groups = int(params.get("groups") or 1)
         self.keep_groups = int(params.get("keep_groups") or self.groups)
         self.scoring = params.get("scoring") or "softmax"
-        if self.scoring not in ("softmax", "sigmoid"):
-            raise UnsupportedError(f"router scoring '{self.scoring}' (supported: softmax, sigmoid)")
+        if self.scoring not in kernels.MOE_SCORINGS:
+            raise UnsupportedError(f"router scoring '{self.scoring}' (supported: {', '.join(kernels.MOE_SCORINGS)})")
         self.group_top = int(params.get("group_top") or 1)
         self.renormalize = bool(params.get("renormalize"))
         self.renorm_eps = float(params.get("renorm_eps") or 0.0)
@@ -190,9 +194,16 @@ class RoutedExperts(FeedForward):
         names = params["names"]
         self.gated = bool(names.get("gate"))
         self.activation = params.get("expert_activation") or ("silu" if self.gated else "relu_squared")
-        if (self.gated and self.activation != "silu") or (not self.gated and self.activation != "relu_squared"):
+        if self.activation not in (("silu", "clipped_gate") if self.gated else ("relu_squared",)):
             raise UnsupportedError(f"experts {'with' if self.gated else 'without'} a gate and the activation "
-                                   f"'{self.activation}' (supported: silu with a gate, relu_squared without)")
+                                   f"'{self.activation}' (supported: silu and clipped_gate with a gate, relu_squared "
+                                   f"without)")
+        self.clipped = None
+        if self.activation == "clipped_gate":
+            p = params["activation_params"]
+            self.clipped = tuple(float(p[k]) for k in ("limit", "slope", "shift"))
+            if not self.clipped[0] > 0:
+                raise InvalidArgument(f"the limit of an expert's sums must be positive, got {self.clipped[0]}")
         if self.experts <= 0 or self.identity < 0 or self.outputs > kernels.MOE_MAX_EXPERTS:
             raise InvalidArgument(f"a routed feed-forward takes 1 to {kernels.MOE_MAX_EXPERTS} experts, got "
                                   f"{self.experts} + {self.identity}")
@@ -219,6 +230,7 @@ class RoutedExperts(FeedForward):
             router_names, router_sizes = [names["router"]], [self.outputs]
         self.router = Linear(router_names, router_sizes, self.hidden)
         self.correction: torch.Tensor = None
+        self.router_bias: torch.Tensor = None
         self.gate: torch.Tensor = None        # [experts (+ shared pieces), intermediate, hidden]
         self.up: torch.Tensor = None
         self.down: torch.Tensor = None        # [experts (+ shared pieces), hidden, intermediate]
@@ -227,6 +239,8 @@ class RoutedExperts(FeedForward):
         specs = self.router.tensors()
         if self.names.get("correction"):
             specs.append(TensorSpec(self.names["correction"], (self.outputs,), "vector", ("normal", 0.02)))
+        if self.names.get("router_bias"):
+            specs.append(TensorSpec(self.names["router_bias"], (self.outputs,), "vector", ("normal", 0.02)))
         inner = ("gate", "up") if self.gated else ("up",)
         for e in range(self.experts):
             for key in inner:
@@ -242,6 +256,8 @@ class RoutedExperts(FeedForward):
         self.router.load(fetch)
         if self.names.get("correction"):
             self.correction = fetch(self.names["correction"], "vector")
+        if self.names.get("router_bias"):
+            self.router_bias = fetch(self.names["router_bias"], "vector")
         F_, pieces = self.intermediate, self.shared_pieces
 
         def stack(key, inner_rows: bool):
@@ -272,11 +288,12 @@ class RoutedExperts(FeedForward):
         weights = ctx.scratch("moe.weights", (T, slots), torch.float32)
         kernels.moe_route(logits, self.correction, self.groups, self.keep_groups, self.top, ids, weights,
                           scoring=self.scoring, group_top=self.group_top, renormalize=self.renormalize,
-                          renorm_eps=self.renorm_eps, weight_scale=self.weight_scale, shared=self.shared_pieces)
+                          renorm_eps=self.renorm_eps, weight_scale=self.weight_scale, shared=self.shared_pieces,
+                          bias=self.router_bias)
         tile_rows = kernels.moe_tile_rows(h.dtype, self.up.dtype, self.hidden, self.intermediate, T * slots, real)
         rows = kernels.moe_align(ids, real, tile_rows, ctx.scratch)
         act = ctx.scratch("moe.act", (T * slots, self.intermediate))
-        kernels.moe_gate_up(h, self.gate, self.up, rows, act)
+        kernels.moe_gate_up(h, self.gate, self.up, rows, act, clipped=self.clipped)
         parts = ctx.scratch("moe.parts", (T * slots, self.hidden), torch.float32)
         kernels.moe_down(act, self.down, rows, parts)
         routed = kernels.RoutedParts(parts, rows.where, weights, h)

@@ -7,7 +7,8 @@
     head h:  key = [Wuk[h] c | rotated part],  value = Wuv[h] c
              score = (q_unrotated . Wuk[h] c + q_rotated . k_rotated) * scale
     softmax over the window (or all keys), with exp(sink[h]) as one more term of the denominator where sinks exist
-    y = Wo (heads side by side * sigmoid(Wg h))            (the gate only where ``g`` is named)
+    y = Wo (heads side by side * sigmoid(Wg h))            (the gate only where ``g`` is named; ``gate_per`` "head":
+                          one gate a head instead of one a value)
 
 What is cached is c and the rotated key part, nothing per head. The scores need no key per head either:
 ``q_unrotated . Wuk[h] c = (Wuk[h]^T q_unrotated) . c``, so the query's unrotated part goes through ``Wuk[h]^T`` once
@@ -19,7 +20,7 @@ kernels are the ones every other attention here uses. Prompt portions and decode
 Parameters: ``hidden``, ``num_heads``, ``head_dim`` (unrotated), ``rope_dim``, ``value_dim``, ``kv_rank``, ``scale``,
 ``window`` (None: all keys), ``sink`` (tensor name or None), ``eps``, ``position`` (a PartSpec of the position family
 that describes a rotation table over ``rope_dim``), ``names`` (``q``, ``dkv``, ``dkv_norm``, ``uk``, ``uv``, ``o`` and
-optionally ``g``; with ``q_rank`` ``dq``, ``dq_norm`` and ``uq`` instead of ``q``), ``output_scale`` (a factor on the
+optionally ``g``, with ``gate_per`` "value" (the default) or "head"; with ``q_rank`` ``dq``, ``dq_norm`` and ``uq`` instead of ``q``), ``output_scale`` (a factor on the
 result, folded into the latent-to-value matrices).
 """
 
@@ -39,6 +40,7 @@ from .linear import Linear
 @register_part("mixer", "latent_attention")
 class LatentAttention(Mixer):
     capturable = True
+    replayable = True      # what a step shares between layers (angles, work lists) is made by the first and kept
     returns_result = True
 
     def __init__(self, params):
@@ -64,11 +66,15 @@ class LatentAttention(Mixer):
         self.q_width = H * (self.dim + self.rope_dim)
         self.latent_width = self.kv_rank + self.rope_dim
         self.gated = bool(names.get("g"))
+        self.gate_per = params.get("gate_per") or "value"
+        if self.gate_per not in ("value", "head"):
+            raise InvalidArgument(f"a latent attention is gated per 'value' or per 'head', not '{self.gate_per}'")
+        self.gate_width = 0 if not self.gated else (H if self.gate_per == "head" else H * self.value_dim)
         self.q_rank = int(params.get("q_rank") or 0)
         first, first_width = (names["dq"], self.q_rank) if self.q_rank else (names["q"], self.q_width)
         self.first_width = first_width
         inputs = [first, names["dkv"]] + ([names["g"]] if self.gated else [])
-        sizes = [first_width, self.latent_width] + ([H * self.value_dim] if self.gated else [])
+        sizes = [first_width, self.latent_width] + ([self.gate_width] if self.gated else [])
         self.inputs = Linear(inputs, sizes, self.hidden)
         self.q_up = Linear([names["uq"]], [self.q_width], self.q_rank) if self.q_rank else None
         self.q_norm: torch.Tensor = None
@@ -147,7 +153,7 @@ class LatentAttention(Mixer):
         kernels.paged_attention(q_latent, cache.k_cache, cache.v_cache, attn, step, ctx.batch, H, self.scale,
                                 self.window, scratch=ctx.scratch, sinks=self.sinks)
         heads = ctx.scratch("latent.heads", (T, H * self.value_dim))
-        gate = proj[:, self.first_width + self.latent_width:].unflatten(1, (H, self.value_dim)) if self.gated else None
+        gate = proj[:, self.first_width + self.latent_width:].unflatten(1, (H, self.gate_width // H)) if self.gated else None
         kernels.head_linear(attn.view(T, H, D)[:, :, :self.kv_rank], self.uv, heads.view(T, H, self.value_dim), gate)
         if residual is not None:
             self.out(heads, residual, accumulate=True, ctx=ctx)

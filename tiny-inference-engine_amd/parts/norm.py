@@ -34,6 +34,7 @@ class RMSNorm(Norm):
     replayable = True
     adds_owed = True
     leaves_row_scale = True
+    reads_either_type = True
 
     def __init__(self, params):
         super().__init__(params)
@@ -97,6 +98,8 @@ class RMSNorm(Norm):
 class LayerNorm(Norm):
     capturable = True
     replayable = True
+    adds_results = True
+    reads_either_type = True
 
     def __init__(self, params):
         super().__init__(params)
@@ -112,11 +115,15 @@ class LayerNorm(Norm):
         self.weight = fetch(self.weight_name, "vector")
 
     def forward(self, ctx: StepContext, x: torch.Tensor, rows: Optional[torch.Tensor] = None,
-                out_name: str = "norm.out", out_dtype: torch.dtype = None) -> torch.Tensor:
+                out_name: str = "norm.out", out_dtype: torch.dtype = None, results=None) -> torch.Tensor:
+        """``results`` (without ``rows``): ``(sub-layers' results, scale)`` that are added to ``x`` in the same pass."""
         count = x.shape[0] if rows is None else rows.numel()
         out = ctx.scratch(out_name, (count, self.dim), out_dtype or ctx.act_dtype)
         ctx.set_row_scale(out, None)
-        kernels.layer_norm(x, self.weight, self.eps, out, rows)
+        if results is not None:
+            kernels.add_results(x, *results, norm=("layer_norm", self.weight, self.eps, out))
+        else:
+            kernels.layer_norm(x, self.weight, self.eps, out, rows)
         return out
 
 

@@ -24,7 +24,10 @@ token's); its last ``taps - 1`` inputs are a second state of the mixer, so it de
 projections (``a1``/``a2``, ``g1``/``g2``) run as one product each: the second over the block-diagonal of the two
 matrices. Everything behind the products is float32. Parameters: ``hidden``, ``heads``, ``kv_heads``, ``key_dim``,
 ``value_dim``, ``conv``, ``eps``, ``names`` (``q``, ``k``, ``v``, ``b``, ``a1``, ``a2``, ``g1``, ``g2``, ``o``, ``A_log``,
-``dt_bias``, ``norm``, ``q_conv``, ``k_conv``, ``v_conv``), ``low_rank`` (the inner size of the two-step projections
+``dt_bias``, ``norm``, ``q_conv``, ``k_conv``, ``v_conv``; ``a`` instead of ``a1`` and ``a2`` and ``g`` instead of ``g1``
+and ``g2`` where one matrix makes the decay's argument or the gate: it is then part of the first product), ``decay``
+"channel" (the default, as above) or "head" (``Wa h`` and ``dt_bias`` have one entry a head, and S is multiplied by one
+number), ``gate_activation`` "sigmoid" (the default) or "silu", ``low_rank`` (the inner size of the two-step projections
 where random weights are made; a file's tensors say their own), ``output_scale`` (a factor on the result, folded into the
 norm's weight).
 
@@ -170,6 +173,7 @@ class MinGru(Mixer):
 @register_part("mixer", "gated_delta_rule")
 class GatedDeltaRule(Mixer):
     capturable = True
+    replayable = True        # the chunks of a long step are listed once and kept
     returns_result = True
 
     def __init__(self, params):
@@ -183,19 +187,30 @@ class GatedDeltaRule(Mixer):
         self.eps = float(params["eps"])
         self.output_scale = float(params.get("output_scale", 1.0))
         self.low_rank = int(params.get("low_rank") or 16)        # for random weights only: a file's own size counts
+        self.decay = params.get("decay") or "channel"
+        self.gate_activation = params.get("gate_activation") or "sigmoid"
         if self.heads % self.kv_heads:
             raise InvalidArgument(f"{self.heads} value heads are no multiple of {self.kv_heads} query/key heads")
         if self.key_dim > kernels.DELTA_RULE_MAX_DIM:
             raise InvalidArgument(f"a key size of {self.key_dim} exceeds {kernels.DELTA_RULE_MAX_DIM}")
         if not 1 <= self.taps <= kernels.CONV_MAX_TAPS:
             raise InvalidArgument(f"a convolution of {self.taps} taps: 1 to {kernels.CONV_MAX_TAPS} are supported")
+        if self.decay not in ("channel", "head"):
+            raise InvalidArgument(f"a delta rule decays per 'channel' or per 'head', not '{self.decay}'")
+        if self.gate_activation not in ("sigmoid", "silu"):
+            raise InvalidArgument(f"the output gate is 'sigmoid' or 'silu', not '{self.gate_activation}'")
         n = self.names = dict(params["names"])
+        self.head_decay = self.decay == "head"
         self.qk_width, self.v_width = self.kv_heads * self.key_dim, self.heads * self.value_dim
-        self.decay_width = self.heads * self.key_dim
+        self.decay_width = self.heads if self.head_decay else self.heads * self.key_dim
         self.channels = 2 * self.qk_width + self.v_width          # what the convolution runs over
-        self.inputs = Linear([n["q"], n["k"], n["v"], n["b"]],
-                             [self.qk_width, self.qk_width, self.v_width, self.heads], self.hidden)
-        self.low_ranks = None                                      # (rank of a1, rank of g1): from the stored shapes
+        # The decay's argument and the gate come from one matrix each, part of the first product, or from two in a row.
+        self.direct = [(key, width) for key, width in (("a", self.decay_width), ("g", self.v_width)) if n.get(key)]
+        self.two_step = [(key, width) for key, width in (("a", self.decay_width), ("g", self.v_width)) if not n.get(key)]
+        self.inputs = Linear([n["q"], n["k"], n["v"], n["b"]] + [n[key] for key, _ in self.direct],
+                             [self.qk_width, self.qk_width, self.v_width, self.heads] + [w for _, w in self.direct],
+                             self.hidden)
+        self.low_ranks = None                                      # the two-step projections' inner sizes, as stored
         self.low: Linear = None
         self.second: Linear = None
         self.out = Linear([n["o"]], [self.hidden], self.v_width)
@@ -210,11 +225,10 @@ class GatedDeltaRule(Mixer):
     def tensors(self) -> List[TensorSpec]:
         n = self.names
         specs = self.inputs.tensors() + self.out.tensors()
-        # The inner size of the two-step projections is whatever the file holds (None: any).
-        specs += [TensorSpec(n["a1"], (None, self.hidden), "matrix", ("normal", 0.02), free_dims=(self.low_rank,)),
-                  TensorSpec(n["a2"], (self.decay_width, None), "matrix", ("normal", 0.1), free_dims=(self.low_rank,)),
-                  TensorSpec(n["g1"], (None, self.hidden), "matrix", ("normal", 0.02), free_dims=(self.low_rank,)),
-                  TensorSpec(n["g2"], (self.v_width, None), "matrix", ("normal", 0.1), free_dims=(self.low_rank,))]
+        # The inner size of a two-step projection is whatever the file holds (None: any).
+        for key, width in self.two_step:
+            specs += [TensorSpec(n[key + "1"], (None, self.hidden), "matrix", ("normal", 0.02), free_dims=(self.low_rank,)),
+                      TensorSpec(n[key + "2"], (width, None), "matrix", ("normal", 0.1), free_dims=(self.low_rank,))]
         specs += [TensorSpec(n["A_log"], (self.heads,), "vector", ("normal", 0.5)),
                   TensorSpec(n["dt_bias"], (self.decay_width,), "vector", ("normal", 0.5)),
                   TensorSpec(n["norm"], (self.value_dim,), "vector", ("one_plus_uniform", 0.1))]
@@ -226,18 +240,23 @@ class GatedDeltaRule(Mixer):
         n = self.names
         self.inputs.load(fetch)
         self.out.load(fetch)
-        a1, a2, g1, g2 = (fetch(n[k], "matrix") for k in ("a1", "a2", "g1", "g2"))
-        ra, rg = a1.shape[0], g1.shape[0]
-        if a2.shape[1] != ra or g2.shape[1] != rg:
-            raise InvalidArgument(f"{n['a2']} / {n['g2']} do not take what {n['a1']} / {n['g1']} give")
-        self.low_ranks = (ra, rg)
-        self.low = Linear([n["a1"], n["g1"]], [ra, rg], self.hidden)
-        self.low.set_weight(torch.cat([a1, g1], dim=0).contiguous())
-        both = a2.new_zeros((self.decay_width + self.v_width, ra + rg))
-        both[:self.decay_width, :ra] = a2
-        both[self.decay_width:, ra:] = g2
-        self.second = Linear(["(a2 | g2)"], [self.decay_width + self.v_width], ra + rg)
-        self.second.set_weight(both)
+        if self.two_step:
+            firsts = [fetch(n[key + "1"], "matrix") for key, _ in self.two_step]
+            seconds = [fetch(n[key + "2"], "matrix") for key, _ in self.two_step]
+            self.low_ranks = tuple(f.shape[0] for f in firsts)
+            for (key, _), rank, w in zip(self.two_step, self.low_ranks, seconds):
+                if w.shape[1] != rank:
+                    raise InvalidArgument(f"{n[key + '2']} does not take what {n[key + '1']} gives")
+            self.low = Linear([n[key + "1"] for key, _ in self.two_step], list(self.low_ranks), self.hidden)
+            self.low.set_weight(torch.cat(firsts, dim=0).contiguous())
+            total = sum(width for _, width in self.two_step)
+            both = seconds[0].new_zeros((total, sum(self.low_ranks)))       # the second steps, side by side
+            row = col = 0
+            for (_, width), rank, w in zip(self.two_step, self.low_ranks, seconds):
+                both[row:row + width, col:col + rank] = w
+                row, col = row + width, col + rank
+            self.second = Linear(["(second steps)"], [total], sum(self.low_ranks))
+            self.second.set_weight(both)
         self.conv_weight = torch.cat([fetch(n[k], "vector").to(torch.float32).reshape(-1, self.taps)
                                       for k in ("q_conv", "k_conv", "v_conv")]).contiguous()
         self.A_log = fetch(n["A_log"], "vector").to(torch.float32).contiguous()
@@ -249,21 +268,32 @@ class GatedDeltaRule(Mixer):
         state, conv_state = (cache[0], cache[1].state) if isinstance(cache, tuple) else (cache, None)
         proj = ctx.scratch("delta_rule.proj", (T, self.inputs.total_out), torch.float32)
         self.inputs(h, proj, ctx=ctx)
-        low = ctx.scratch("delta_rule.low", (T, sum(self.low_ranks)))
-        self.low(h, low, ctx=ctx)
-        second = ctx.scratch("delta_rule.second", (T, self.decay_width + self.v_width), torch.float32)
-        self.second(low, second)
-        tok = ctx.scratch("delta_rule.tokens", (T, self.channels + self.heads + self.decay_width), torch.float32)
-        kernels.delta_prepare(proj, self.conv_weight, self.taps, conv_state, ctx.batch, second[:, :self.decay_width],
-                              self.A_log, self.dt_bias, self.kv_heads, self.heads, self.key_dim, self.value_dim, tok)
+        columns, at = {}, self.channels + self.heads
+        for key, width in self.direct:
+            columns[key] = proj[:, at:at + width]
+            at += width
+        if self.two_step:
+            low = ctx.scratch("delta_rule.low", (T, sum(self.low_ranks)))
+            self.low(h, low, ctx=ctx)
+            second = ctx.scratch("delta_rule.second", (T, self.second.total_out), torch.float32)
+            self.second(low, second)
+            at = 0
+            for key, width in self.two_step:
+                columns[key] = second[:, at:at + width]
+                at += width
+        sizes = (self.kv_heads, self.heads, self.key_dim, self.value_dim)
+        tok = ctx.scratch("delta_rule.tokens", (T, kernels.delta_row(*sizes, self.head_decay)), torch.float32)
+        kernels.delta_prepare(proj, self.conv_weight, self.taps, conv_state, ctx.batch, columns["a"], self.A_log,
+                              self.dt_bias, *sizes, tok, head_decay=self.head_decay)
         if conv_state is not None and state.writes:
             kernels.conv_state_update(proj, self.taps, conv_state, ctx.batch, self.channels)
         o = ctx.scratch("delta_rule.o", (T, self.v_width), torch.float32)
         chunks = None
         if max(ctx.batch.host_new_tokens) >= kernels.DELTA_CHUNKS_FROM:      # such steps are never recorded
             chunks = kernels.scan_chunks(ctx.batch, ctx.device, rows=kernels.DELTA_CHUNK_ROWS)
-        kernels.gated_delta_scan(tok, o, state.state, ctx.batch, self.kv_heads, self.heads, self.key_dim,
-                                 self.value_dim, chunks=chunks, scratch=ctx.scratch)
+        kernels.gated_delta_scan(tok, o, state.state, ctx.batch, *sizes, chunks=chunks, scratch=ctx.scratch,
+                                 head_decay=self.head_decay)
         gated = ctx.scratch("delta_rule.gated", (T, self.v_width))
-        kernels.grouped_gated_rms_norm(o, self.norm_weight, self.eps, second[:, self.decay_width:], gated, self.heads)
+        kernels.grouped_gated_rms_norm(o, self.norm_weight, self.eps, columns["g"], gated, self.heads,
+                                       activation=self.gate_activation)
         return _finish(ctx, self.out, gated, residual, "delta_rule.result")
