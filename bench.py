@@ -4,7 +4,7 @@
     python bench.py --shape 32b                 the same measurements at the Qwen3-32B sizes
     python bench.py --sweep [--shape 32b]       decode at contexts 4096 / 16384 / 32768 x batch 1 / 8 / 32, a line a point
     python bench.py --workload stress           64 requests through the scheduler at the Qwen3-1.7B sizes
-    python bench.py --workload minerax          another design beside Qwen3 at equal sizes (also duzozen, topapel, zovudra): prefill, decode
+    python bench.py --workload minerax          another design beside Qwen3 at equal sizes (also duzozen, topapel, vipalorn, zovudra): prefill, decode
 
 Prints ONE JSON line. A "step" is one decode step of the engine (schedule, build the batch, run
 the model, sample greedily) at the default batch of 8 with every sequence near the benchmark
@@ -190,11 +190,42 @@ def qwen3_beside_zovudra(size):
                 intermediate_size=size["ff"], vocab_size=size["vocab"])
 
 
+# ``--workload vipalorn``: the Vipalorn design at sizes that resemble a real model's layers, beside Qwen3 with the same
+# stream, as many heads of the same size and a gated feed-forward as wide as the experts a token uses together. Layers
+# repeat (three with the gated delta rule, one with latent attention over all earlier keys); every layer routes to
+# experts beside its mixer. The cached latent and its rotated key part together are one head of 256.
+VIPALORN_SIZES = {
+    "2k": {"width": 2048, "heads": 16, "kv_heads": 4, "dim": 128, "rot_dim": 64, "kv_rank": 192, "delta_heads": 16,
+           "delta_kv_heads": 8, "delta_dim": 128, "experts": 32, "expert_ff": 768, "top": 4, "layers": 8, "vocab": 32000,
+           "context": 4096},
+    "4k": {"width": 4096, "heads": 32, "kv_heads": 8, "dim": 128, "rot_dim": 64, "kv_rank": 192, "delta_heads": 32,
+           "delta_kv_heads": 16, "delta_dim": 128, "experts": 64, "expert_ff": 1536, "top": 4, "layers": 4, "vocab": 32000,
+           "context": 8192},
+}
+
+
+def vipalorn_config(size):
+    moe = {"kind": "moe", "expert": {"ff": size["expert_ff"], "limit": 7.0},
+           "router": {"experts": size["experts"], "top": size["top"]}}
+    delta = {"type": "delta", "mlp": moe,
+             "mixer": {"heads": size["delta_heads"], "kv_heads": size["delta_kv_heads"], "dim": size["delta_dim"],
+                       "vdim": size["delta_dim"], "conv": 4}}
+    latent = {"type": "latent_attention", "mlp": moe,
+              "mixer": {"heads": size["heads"], "dim": size["dim"], "rot_dim": size["rot_dim"], "vdim": size["dim"],
+                        "kv_rank": size["kv_rank"], "scale": (size["dim"] + size["rot_dim"]) ** -0.5,
+                        "rot": {"dims": size["rot_dim"], "base": 10000.0}}}
+    pattern = [delta, delta, delta, latent]
+    return {"architecture": "Vipalorn", "vocab": size["vocab"], "width": size["width"], "norm": {"eps": 1e-6},
+            "residual_mult": 0.5, "logit_scale": 2.0,
+            "layers": [pattern[i % len(pattern)] for i in range(size["layers"])]}
+
+
 # design -> (sizes, its config at a size, Qwen3 at that size, the context a decode step may reach)
 DESIGNS = {
     "duzozen": (DUZOZEN_SIZES, duzozen_config, qwen3_beside, lambda size: 2 * size["window"]),
     "topapel": (TOPAPEL_SIZES, topapel_config, qwen3_beside_topapel, lambda size: 2 * size["chunk"]),
     "minerax": (MINERAX_SIZES, minerax_config, qwen3_beside_minerax, lambda size: 4 * size["window"]),
+    "vipalorn": (VIPALORN_SIZES, vipalorn_config, qwen3_beside, lambda size: size["context"]),
     "zovudra": (ZOVUDRA_SIZES, zovudra_config, qwen3_beside_zovudra, lambda size: 4 * size["window"]),
 }
 BLOCK_SIZE = 16
@@ -454,14 +485,14 @@ def main():
     parser.add_argument("--layers", type=int, default=0, help="run fewer layers than the shape has (0 = all)")
     parser.add_argument("--shape", choices=sorted(SHAPES), default=None,
                         help="layer sizes: 8b (default), 32b, or 1.7b (the default of --workload stress)")
-    parser.add_argument("--workload", choices=["decode", "stress", "long-prompt", "duzozen", "topapel", "minerax", "zovudra"], default="decode",
+    parser.add_argument("--workload", choices=["decode", "stress", "long-prompt", "duzozen", "topapel", "minerax", "vipalorn", "zovudra"], default="decode",
                         help="decode: the headline measurement; stress: many requests through a small cache; "
-                             "long-prompt: one long prompt in portions; duzozen, topapel, minerax, zovudra: that design beside Qwen3 at "
-                             "equal sizes (--sizes), prefill and decode")
+                             "long-prompt: one long prompt in portions; duzozen, topapel, minerax, vipalorn, zovudra: that design "
+                             "beside Qwen3 at equal sizes (--sizes), prefill and decode")
     parser.add_argument("--design-models", default="design,qwen3",
-                        help="duzozen, topapel, minerax: which of the two models to run (design: the workload's own; or its name)")
-    parser.add_argument("--design-batches", default="1,8,64", help="duzozen, topapel, minerax: the decode batch sizes to time")
-    parser.add_argument("--sizes", default="2k,4k", help="duzozen, topapel, minerax: the sizes to run, of " + ", ".join(sorted(DUZOZEN_SIZES)))
+                        help="a design's workload: which of the two models to run (design: the workload's own; or its name)")
+    parser.add_argument("--design-batches", default="1,8,64", help="a design's workload: the decode batch sizes to time")
+    parser.add_argument("--sizes", default="2k,4k", help="a design's workload: the sizes to run, of " + ", ".join(sorted(DUZOZEN_SIZES)))
     parser.add_argument("--prompt-tokens", type=int, default=8192, help="long-prompt: tokens of the prompt")
     parser.add_argument("--portion", type=int, default=512, help="long-prompt and stress: tokens of a prompt portion (stress: also the token budget of a step)")
     parser.add_argument("--requests", type=int, default=64, help="stress: concurrent requests")

@@ -1,0 +1,735 @@
+"""Vipalorn on the GPU against the plain implementation: each mechanism's kernel alone, then whole models under
+every way of cutting the work, in float32 (tight) and bfloat16, and greedy generation through the engine."""
+
+import copy
+import json
+import subprocess
+import sys
+from types import SimpleNamespace
+
+import numpy as np
+import pytest
+import torch
+
+import plain_vipalorn as plain
+import trace_helpers as th
+from vipalorn_fixtures import BLOCK_SIZE, CONFIGS, load_plain, write_model
+
+pytestmark = pytest.mark.gpu
+F64 = torch.float64
+
+
+def rnd(*shape, seed=0, scale=1.0):
+    g = torch.Generator().manual_seed(seed)
+    return torch.randn(*shape, generator=g, dtype=torch.float32) * scale
+
+
+def close(got, want, rel, what=""):
+    got, want = got.detach().cpu().to(F64), want.detach().cpu().to(F64)
+    assert torch.isfinite(got).all(), f"{what}: non-finite values"
+    err = float((got - want).abs().max() / want.abs().max().clamp_min(1e-30))
+    assert err <= rel, f"{what}: relative error {err:.3e} > {rel:.0e}"
+
+
+def i32(values):
+    return torch.tensor(values, dtype=torch.int32, device="cuda")
+
+
+def scratch_memory(fill=float("nan")):
+    """Scratch as the kernels are handed it: what nobody wrote is not zero."""
+    held = {}
+
+    def get(name, shape, dtype=torch.float32):
+        key = (name, tuple(shape), dtype)
+        if key not in held:
+            t = torch.empty(tuple(shape), dtype=dtype, device="cuda")
+            if dtype.is_floating_point:
+                t.fill_(fill)
+            held[key] = t
+        return held[key]
+
+    return get
+
+
+# ------------------------------------------------------------------------------------------- kernels alone
+@pytest.mark.parametrize("n", [30, 64, 101, 352, 2048, 5000, 9004])
+def test_adding_side_by_side_results_and_norming_the_sum(n):
+    from tie_amd import kernels
+
+    T, top, scale = 7, 5, 0.37
+    x, rows, planes = rnd(T, n, seed=n), rnd(T, n, seed=1), rnd(6, T, n, seed=2)
+    parts, h = rnd(T * top, n, seed=3), rnd(T, n, seed=4)
+    where = torch.randperm(T * top, generator=torch.Generator().manual_seed(5)).view(T, top).to(torch.int32)
+    where[2, 1] = where[6, 4] = -1                               # experts that returned their input
+    weights = torch.rand(T, top, generator=torch.Generator().manual_seed(6))
+    w = 1 + 0.2 * rnd(n, seed=7)
+    picked = torch.where((where >= 0)[..., None], parts[where.long().clamp_min(0)], h[:, None, :])
+    routed_sum = (weights[..., None].to(F64) * picked.to(F64)).sum(1)
+    routed = kernels.RoutedParts(parts.cuda(), where.cuda(), weights.cuda(), h.cuda())
+    cases = [([rows.cuda()], rows.to(F64)), ([planes.cuda(), routed], planes.to(F64).sum(0) + routed_sum),
+             ([routed], routed_sum), ([planes.cuda(), rows.cuda()], planes.to(F64).sum(0) + rows.to(F64))]
+    for results, added in cases:
+        want = x.to(F64) + scale * added
+        xd = x.clone().cuda()
+        kernels.add_results(xd, results, scale)
+        close(xd, want, 1e-6, "the stream")
+        for kind, norm in (("layer_norm", plain.layer_norm), ("rms_norm", plain.rms_norm)):
+            for dtype, tolerance in ((torch.float32, 3e-6), (torch.bfloat16, 8e-3)):
+                xd, out = x.clone().cuda(), torch.empty(T, n, dtype=dtype, device="cuda")
+                kernels.add_results(xd, results, scale, norm=(kind, w.cuda(), 1e-5, out))
+                close(xd, want, 1e-6, "the stream beside a norm")
+                close(out, norm(want, w.to(F64), 1e-5), tolerance, f"{kind} of the sum, {dtype}")
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("scale", [1.0, 0.25])
+def test_an_embedding_with_a_norm(dtype, scale):
+    from tie_amd.parts.base import PartSpec, build_part
+
+    table, w = rnd(50, 44, seed=1, scale=0.05).to(dtype), 1 + 0.3 * rnd(44, seed=2)
+    part = build_part("embedding", PartSpec("token_embedding", {
+        "vocab": 50, "hidden": 44, "weight": "embed", "scale": scale,
+        "norm": PartSpec("layer_norm", {"dim": 44, "eps": 1e-3, "weight": "embed.norm"})}))
+    assert {s.name for s in part.all_tensors()} == {"embed", "embed.norm"}
+    part.load_all(lambda name, role: table.cuda() if name == "embed" else w.cuda(), "float32", "cuda")
+    get = scratch_memory()
+    ctx = SimpleNamespace(scratch=lambda name, shape, dt=None: get(name, shape, dt or torch.float32), act_dtype=dtype,
+                          set_row_scale=lambda *a: None)
+    tokens = [3, 49, 0, 3, 17]
+    x = part.forward(ctx, i32(tokens))
+    assert x.dtype == torch.float32
+    close(x, plain.layer_norm(table.to(F64)[tokens] * scale, w.to(F64), 1e-3), 3e-6, "normed embedding")
+
+
+@pytest.mark.parametrize("T", [1, 11, 200])
+@pytest.mark.parametrize("H,K,N", [(3, 28, 24), (8, 64, 64), (20, 48, 8), (2, 100, 7), (4, 192, 72)])
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+def test_a_matrix_per_head_with_one_gate_a_head(H, K, N, dtype, T):
+    from tie_amd import kernels
+
+    x, w = rnd(T, H, K, seed=1).to(dtype), rnd(H, N, K, seed=2, scale=0.3).to(dtype)
+    wide = rnd(T, 5 + H + 3, seed=3, scale=2.0).cuda()                 # the gates are columns of wider rows
+    gate = wide[:, 5:5 + H].unflatten(1, (H, 1))
+    out = torch.empty(T, H, N, dtype=dtype, device="cuda")
+    kernels.head_linear(x.cuda(), w.cuda(), out, gate)
+    want = torch.einsum("thk,hnk->thn", x.to(F64), w.to(F64)) * torch.sigmoid(gate.cpu().to(F64))
+    close(out, want, 1e-5 if dtype == torch.float32 else 8e-3, "gated per head")
+
+
+@pytest.mark.parametrize("E,top", [(1, 1), (5, 5), (7, 2), (64, 6), (100, 8), (200, 1)])
+def test_a_router_weighted_over_the_chosen_alone(E, top):
+    from tie_amd import kernels
+
+    T = 60
+    z, bias = rnd(T, E, seed=E, scale=2.0), rnd(E, seed=1)
+    ids, w = torch.empty(T, top, dtype=torch.int32, device="cuda"), torch.empty(T, top, device="cuda")
+    kernels.moe_route(z.cuda(), None, 1, 1, top, ids, w, scoring="softmax_chosen", bias=bias.cuda())
+    chosen, weights = plain.route((z + bias).to(F64), top)
+    assert torch.equal(ids.cpu().long(), chosen), "the chosen experts, the largest first"
+    close(w, weights, 2e-6, "weights")
+    # logits far below or above zero neither vanish nor overflow, and close ones stay apart
+    far = torch.tensor([[-300.0, -301.0, -299.5, -400.0], [400.0, 401.0, 400.5, 0.0], [7.0, 7.0, 7.000001, 7.0]])
+    ids, w = torch.empty(3, 2, dtype=torch.int32, device="cuda"), torch.empty(3, 2, device="cuda")
+    kernels.moe_route(far.cuda(), None, 1, 1, 2, ids, w, scoring="softmax_chosen")
+    chosen, weights = plain.route(far.to(F64), 2)
+    assert torch.equal(ids.cpu().long(), chosen) and chosen.tolist() == [[2, 0], [1, 2], [2, 0]]
+    close(w, weights, 2e-6, "weights of far logits")
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("T,E,top,F_,K", [(3, 4, 2, 24, 64), (70, 3, 2, 16, 40), (300, 5, 1, 72, 96), (700, 4, 3, 64, 128),
+                                          (200, 2, 2, 9, 100)])
+@pytest.mark.parametrize("limit", [0.4, 1000.0])
+def test_experts_whose_sums_are_cut_off(T, E, top, F_, K, limit, dtype):
+    """A limit most sums meet and one none does; the float32 kernels and the matrix-core ones in all tile sizes."""
+    from tie_amd import kernels
+
+    h = rnd(T, K, seed=1)
+    gate, up, down = rnd(E, F_, K, seed=2, scale=0.2), rnd(E, F_, K, seed=3, scale=0.2), rnd(E, K, F_, seed=4, scale=0.3)
+    h, gate, up, down = (t.to(dtype) for t in (h, gate, up, down))
+    g = torch.Generator().manual_seed(4)
+    ids = torch.stack([torch.randperm(E, generator=g)[:top] for _ in range(T)]).to(torch.int32)
+    weights = torch.rand(T, top, generator=g)
+    want = torch.zeros(T, K, dtype=F64)
+    for e in range(E):
+        y = plain.expert(h.to(F64), gate[e].to(F64), up[e].to(F64), down[e].to(F64), limit)
+        want += y * (weights.to(F64) * (ids == e)).sum(1, keepdim=True)
+    get = scratch_memory()
+    tile = kernels.moe_tile_rows(dtype, dtype, K, F_, T * top, E)
+    rows = kernels.moe_align(ids.cuda(), E, tile, get)
+    act = get("act", (T * top, F_), dtype)
+    kernels.moe_gate_up(h.cuda(), gate.cuda(), up.cuda(), rows, act, clipped=(limit, 1.702, 1.0))
+    parts = get("parts", (T * top, K))
+    kernels.moe_down(act, down.cuda(), rows, parts)
+    out = torch.zeros(T, K, device="cuda")
+    kernels.moe_combine(kernels.RoutedParts(parts, rows.where, weights.cuda(), h.cuda()), out)
+    close(out, want, 1e-5 if dtype == torch.float32 else 2e-2, f"experts in tiles of {tile}")
+
+
+@pytest.mark.parametrize("activation", ["silu", "sigmoid"])
+def test_the_gated_norm_of_the_heads_outputs(activation):
+    from tie_amd import kernels
+
+    T, H, e = 9, 3, 70
+    o, w, wide = rnd(T, H * e, seed=1), 1 + 0.2 * rnd(e, seed=2), rnd(T, H * e + 11, seed=3, scale=2.0).cuda()
+    gate = wide[:, 11:]
+    out = torch.empty(T, H * e, device="cuda")
+    kernels.grouped_gated_rms_norm(o.cuda(), w.cuda(), 1e-3, gate, out, H, activation=activation)
+    g = gate.cpu().to(F64)
+    act = torch.nn.functional.silu(g) if activation == "silu" else torch.sigmoid(g)
+    close(out, plain.rms_norm(o.to(F64).view(T, H, e), w.to(F64), 1e-3).view(T, -1) * act, 3e-6, "gated norm")
+
+
+def delta_inputs(G, H, d, e, T, seed, decay_spread, repeat_keys=False):
+    """What the rule takes of T tokens: unit queries and keys, values, beta and the decays' logarithms."""
+    q, k = rnd(T, G, d, seed=seed).to(F64), rnd(T, G, d, seed=seed + 1).to(F64)
+    if repeat_keys:                # keys that hardly differ from their neighbours: the corrections nearly cancel
+        k = k[:1] + 0.05 * k
+    q, k = plain.unit(q) * d ** -0.5, plain.unit(k)
+    beta = torch.sigmoid(2.0 * rnd(T, H, seed=seed + 3))
+    log_g = -torch.exp(decay_spread * rnd(T, H, seed=seed + 4)) * torch.nn.functional.softplus(rnd(T, H, seed=seed + 5))
+    return q.float(), k.float(), rnd(T, H, e, seed=seed + 2), beta, log_g
+
+
+@pytest.mark.parametrize("chunks", [False, True])
+@pytest.mark.parametrize("G,H,d,e,lens,spread,repeat", [
+    (2, 4, 32, 64, [1, 64, 65, 130, 7], 0.5, False), (1, 1, 16, 16, [200], 1.0, True), (3, 3, 20, 9, [70, 3], 2.0, False),
+    (1, 2, 128, 128, [300], -2.0, True), (2, 2, 128, 80, [128, 1], 0.0, False), (1, 1, 256, 48, [150], -1.0, False),
+    (1, 2, 100, 33, [190], 3.0, True), (1, 3, 7, 5, [63, 2], 1.0, False)])
+def test_the_delta_rule_with_one_decay_a_head(G, H, d, e, lens, spread, repeat, chunks):
+    """Token by token and in chunks of matrix products, from states that are not zero in slots out of order; weak and
+    very strong decays, keys that repeat themselves, the first rows of a chunk and its last, ragged ones and whole."""
+    from tie_amd import kernels
+
+    T, S = sum(lens), len(lens)
+    q, k, v, beta, log_g = delta_inputs(G, H, d, e, T, 10, spread, repeat)
+    C = 2 * G * d + H * e
+    tok = torch.full((T, kernels.delta_row(G, H, d, e, True)), float("nan"))
+    tok[:, :C] = torch.cat([q.reshape(T, -1), k.reshape(T, -1), v.reshape(T, -1)], dim=1)
+    tok[:, C:C + 3 * H] = torch.cat([torch.exp(log_g), beta, log_g], dim=1)
+    state = rnd(S + 3, H, d, e, seed=9)
+    slots = torch.randperm(S + 3, generator=torch.Generator().manual_seed(1))[:S]
+    starts = [sum(lens[:i]) for i in range(S + 1)]
+    want, want_state = torch.zeros(T, H, e, dtype=F64), state.to(F64).clone()
+    for s in range(S):
+        a, b = starts[s], starts[s + 1]
+        for h in range(H):
+            kv = h // (H // G)
+            want[a:b, h], want_state[slots[s], h] = plain.delta_rule_scan(
+                q[a:b, kv].to(F64), k[a:b, kv].to(F64), v[a:b, h].to(F64), beta[a:b, h].to(F64),
+                torch.exp(log_g[a:b, h].to(F64)), state[slots[s], h].to(F64))
+    batch = SimpleNamespace(num_seqs=S, query_start=i32(starts), state_slots=i32(slots.tolist()), host_new_tokens=lens, memo={})
+    listed = kernels.scan_chunks(batch, "cuda", rows=kernels.DELTA_HEAD_CHUNK_ROWS, force=True) if chunks else None
+    on_gpu, out = state.cuda(), torch.full((T, H * e), float("nan"), device="cuda")
+    kernels.gated_delta_scan(tok.cuda(), out, on_gpu, batch, G, H, d, e, chunks=listed, scratch=scratch_memory(), head_decay=True)
+    close(out, want.view(T, -1), 3e-6, "outputs")
+    close(on_gpu, want_state, 1e-6, "states")
+
+
+def test_heads_in_several_passes_where_the_chunks_memory_is_short(monkeypatch):
+    from tie_amd import kernels
+
+    G, H, d, e, T = 2, 6, 24, 20, 150
+    q, k, v, beta, log_g = delta_inputs(G, H, d, e, T, 3, 0.5)
+    C = 2 * G * d + H * e
+    tok = torch.zeros(T, kernels.delta_row(G, H, d, e, True))
+    tok[:, :C] = torch.cat([q.reshape(T, -1), k.reshape(T, -1), v.reshape(T, -1)], dim=1)
+    tok[:, C:C + 3 * H] = torch.cat([torch.exp(log_g), beta, log_g], dim=1)
+    batch = SimpleNamespace(num_seqs=1, query_start=i32([0, T]), state_slots=i32([0]), host_new_tokens=[T], memo={})
+    listed = kernels.scan_chunks(batch, "cuda", rows=kernels.DELTA_HEAD_CHUNK_ROWS, force=True)
+    results = []
+    for limit in (kernels.DELTA_CHUNK_SCRATCH_MAX, 700_000, 1):              # all heads, several and one at a time
+        monkeypatch.setattr(kernels, "DELTA_CHUNK_SCRATCH_MAX", limit)
+        out, state = torch.empty(T, H * e, device="cuda"), rnd(1, H, d, e, seed=7).cuda()
+        kernels.gated_delta_scan(tok.cuda(), out, state, batch, G, H, d, e, chunks=listed, scratch=scratch_memory(), head_decay=True)
+        results.append((out.cpu(), state.cpu()))
+    for out, state in results[1:]:
+        assert torch.equal(out, results[0][0]) and torch.equal(state, results[0][1])
+
+
+@pytest.mark.parametrize("G,H,d,e,taps", [(2, 4, 8, 24, 3), (1, 1, 64, 16, 4), (3, 3, 20, 9, 1), (1, 4, 128, 128, 8)])
+def test_what_the_delta_rule_takes_of_a_token(G, H, d, e, taps):
+    """Convolution, silu, unit vectors, beta, decays and their logarithms, over steps shorter than the taps."""
+    from tie_amd import kernels
+
+    T, C = 40, 2 * G * d + H * e
+    u, a = rnd(T, C + H + 5, seed=1), rnd(T, H, seed=2, scale=2.0)
+    w, A_log, dt = rnd(C, taps, seed=3, scale=0.5), rnd(H, seed=4), rnd(H, seed=5)
+    y = torch.nn.functional.silu(plain.short_convolution(u[:, :C].to(F64), w.to(F64)))
+    q = plain.unit(y[:, :G * d].view(T, G, d)) * d ** -0.5
+    k = plain.unit(y[:, G * d:2 * G * d].view(T, G, d))
+    log_g = -torch.exp(A_log.to(F64)) * torch.nn.functional.softplus(a.to(F64) + dt.to(F64))
+    want = torch.cat([q.view(T, -1), k.view(T, -1), y[:, 2 * G * d:], torch.exp(log_g),
+                      torch.sigmoid(u[:, C:C + H].to(F64)), log_g], dim=1)
+    state = torch.zeros(3, max(taps - 1, 1), C, device="cuda")
+    got, at = [], 0
+    for n in (1, 2, 1, 13, 3, 20):
+        batch = SimpleNamespace(num_seqs=1, query_start=i32([0, n]), state_slots=i32([1]), seq_of_row=i32([0] * n))
+        ud = u[at:at + n].cuda()
+        tok = torch.zeros(n, kernels.delta_row(G, H, d, e, True), device="cuda")
+        kernels.delta_prepare(ud, w.cuda(), taps, state if taps > 1 else None, batch, a[at:at + n].cuda(), A_log.cuda(),
+                              dt.cuda(), G, H, d, e, tok, head_decay=True)
+        if taps > 1:
+            kernels.conv_state_update(ud, taps, state, batch, C)
+        got.append(tok[:, :C + 3 * H].cpu())
+        at += n
+    got = torch.cat(got)
+    for name, lo, hi in (("q", 0, G * d), ("k", G * d, 2 * G * d), ("v", 2 * G * d, C), ("decay", C, C + H),
+                         ("beta", C + H, C + 2 * H), ("log decay", C + 2 * H, C + 3 * H)):
+        close(got[:, lo:hi], want[:, lo:hi], 5e-6, name)
+
+
+# ------------------------------------------------------------------------------------------- whole models
+LENGTHS = {"A": [1, 23, 210, 37, 5], "B": [170, 2, 41, 90], "C": [33, 150, 8], "D": [12, 260, 3, 21, 9],
+           "E": [150, 1, 66, 97], "F": [3, 140, 64, 20]}
+TOLERANCE = {"float32": 2e-5, "bfloat16": 3e-2}        # of the largest logit; the queries are drawn wide
+
+
+@pytest.fixture(scope="module")
+def folders(tmp_path_factory):
+    out = {}
+    for name, config in CONFIGS.items():
+        for dtype in ("float32", "bfloat16"):
+            folder = tmp_path_factory.mktemp(f"vipalorn_{name}_{dtype}")
+            out[name, dtype] = write_model(folder, config, seed=61 + len(out), dtype=dtype)
+    return out
+
+
+def reference(folder, config, requests, streams=None):
+    weights = load_plain(folder)
+    out = {}
+    for rid, toks in requests.items():
+        logits, behind = plain.forward(config, weights, toks)
+        out[rid] = logits.float()
+        if streams is not None:
+            streams[rid] = behind
+    return out
+
+
+def worst_error(got, want):
+    worst = 0.0
+    for rid, ref in want.items():
+        mine = torch.stack([got[rid][p] for p in range(ref.shape[0])])
+        worst = max(worst, float(((mine - ref).abs().amax(dim=1) / ref.abs().max()).max()))
+    return worst
+
+
+def check(got, want, tolerance, label):
+    worst = 0.0
+    for rid, ref in want.items():
+        rows = got[rid]
+        assert sorted(rows) == list(range(ref.shape[0])), f"{label}: request {rid} misses positions"
+        mine = torch.stack([rows[p] for p in range(ref.shape[0])])
+        assert torch.isfinite(mine).all(), f"{label}: request {rid} has non-finite logits"
+        err = (mine - ref).abs().amax(dim=1) / ref.abs().max()
+        bad = int(torch.argmax((err > tolerance).float())) if bool((err > tolerance).any()) else -1
+        assert bad < 0, (f"{label}: request {rid} first differs at position {bad} "
+                         f"(relative error {float(err[bad]):.3e}, allowed {tolerance:.0e})")
+        worst = max(worst, float(err.max()))
+    print(f"[observed] {label}: {worst:.3e}")
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("name", sorted(CONFIGS))
+def test_every_way_of_cutting_the_work(folders, name, dtype):
+    from tie_amd.engine.replay import TraceReplayer
+
+    folder, config = folders[name, dtype], CONFIGS[name]
+    requests = th.make_requests(config["vocab"], LENGTHS[name], seed=5)
+    want = reference(folder, config, requests)
+    bs = BLOCK_SIZE[name]
+    biggest = max(th.round64(len(t)) for t in requests.values())
+
+    def replayer(max_tokens):
+        return TraceReplayer.from_folder(folder, dtype, max_tokens, block_size=bs, state_slots=4)
+
+    results = {"whole": th.collect(replayer(biggest), th.whole(requests)),
+               "prefill+decode": th.collect(replayer(biggest), th.prefill_then_decode(requests, tail=40)),
+               "portions": th.collect(replayer(biggest), th.portions(requests)),
+               "long portions": th.collect(replayer(biggest), th.portions(requests, sizes=(131, 2, 129))),
+               "portions of two": th.collect(replayer(biggest), th.portions(requests, sizes=(2,))),
+               "token by token": th.collect(replayer(biggest), th.portions(requests, sizes=(1,)))}
+    for label, seed, sizes in (("mixed", 3, (13, 7, 2, 5, 3, 2, 9)), ("mixed, long portions", 4, (130, 2, 5))):
+        steps, peak = th.mixed(requests, max_live=4, seed=seed, sizes=sizes)
+        assert max(len(s["entries"]) for s in steps) >= 3
+        rep = replayer(peak)
+        results[label] = th.collect(rep, steps)
+        assert rep.cache.all_free()                                   # every page and slot came back
+    for label, got in results.items():
+        check(got, want, TOLERANCE[dtype], f"{name}/{dtype}/{label}")
+    if dtype == "float32":       # the ways of cutting agree with each other beyond what they owe the plain one
+        for label in results:
+            for rid in requests:
+                a = torch.stack([results["whole"][rid][p] for p in range(len(requests[rid]))])
+                b = torch.stack([results[label][rid][p] for p in range(len(requests[rid]))])
+                assert float((a - b).abs().max() / a.abs().max()) < 1e-5, f"{name}: whole vs {label}, request {rid}"
+
+
+def random_config(seed):
+    """A model of random layers and sizes: every choice the reader knows is drawn, present or absent."""
+    import random
+
+    rng = random.Random(seed)
+    pick = rng.choice
+    width = pick([40, 64, 72, 96, 128])
+
+    def mixer():
+        if rng.random() < 0.5:
+            kv = pick([1, 2, 3])
+            dim = pick([8, 12, 16, 32, 48, 64])
+            m = {"heads": kv * pick([1, 2, 4]), "dim": dim}
+            if rng.random() < 0.8:
+                m.update(kv_heads=kv, vdim=pick([dim, 8, 20, 64]), conv=pick([1, 2, 3, 4, 6]))
+            return {"type": "delta", "mixer": m}
+        r = pick([4, 8, 16, 32])
+        m = {"heads": pick([1, 2, 5, 8, 18]), "dim": pick([8, 16, 24, 40]), "rot_dim": r, "vdim": pick([8, 16, 24, 56]),
+             "kv_rank": pick([12, 16, 40, 64]), "scale": rng.uniform(0.1, 0.3),
+             "rot": {"dims": pick([r, r, r // 2]), "base": pick([50.0, 1000.0, 10000.0, 500000.0])}}
+        return {"type": "latent_attention", "mixer": m}
+
+    def mlp():
+        if rng.random() < 0.2:
+            return None
+        experts = pick([1, 2, 4, 7, 10])
+        return {"kind": "moe", "expert": {"ff": pick([8, 16, 24, 40, 9]), "limit": pick([0.3, 1.0, 2.5, 7.0])},
+                "router": {"experts": experts, "top": rng.randint(1, min(experts, 5))}}
+
+    config = {"architecture": "Vipalorn", "vocab": pick([50, 97, 200]), "width": width,
+              "norm": {"eps": pick([1e-6, 1e-5, 1e-4])},
+              "layers": [{**mixer(), "mlp": mlp()} for _ in range(rng.randint(1, 5))]}
+    if rng.random() < 0.7:
+        config["residual_mult"] = pick([0.25, 0.6, 1.5])
+    if rng.random() < 0.7:
+        config["logit_scale"] = pick([0.1, 2.0, 5.0])
+    return config, pick([4, 8, 16, 32])
+
+
+@pytest.mark.parametrize("dtype,seed", [("float32", s) for s in range(12)] + [("bfloat16", s) for s in (1, 4, 7, 10)])
+def test_models_of_random_layers_and_sizes(tmp_path, seed, dtype):
+    from tie_amd.engine.replay import TraceReplayer
+
+    config, bs = random_config(seed)
+    folder = write_model(tmp_path / "model", config, seed=100 + seed, dtype=dtype)
+    requests = th.make_requests(config["vocab"], [155, 3, 41, 1, 58], seed=seed)
+    want = reference(folder, config, requests)
+    biggest = max(th.round64(len(t)) for t in requests.values())
+    results = {"whole": th.collect(TraceReplayer.from_folder(folder, dtype, biggest, block_size=bs), th.whole(requests)),
+               "prefill+decode": th.collect(TraceReplayer.from_folder(folder, dtype, biggest, block_size=bs),
+                                            th.prefill_then_decode(requests, tail=35))}
+    steps, peak = th.mixed(requests, max_live=4, seed=seed)
+    rep = TraceReplayer.from_folder(folder, dtype, max(peak, bs), block_size=bs)
+    results["mixed"] = th.collect(rep, steps)
+    assert rep.cache.all_free()
+    for label, got in results.items():
+        check(got, want, TOLERANCE[dtype], f"random model {seed}/{dtype}/{label}: {json.dumps(config)}")
+
+
+@pytest.mark.parametrize("name", sorted(CONFIGS))
+def test_the_stream_after_every_layer(folders, name):
+    from tie_amd.engine.replay import TraceReplayer
+
+    folder, config = folders[name, "float32"], CONFIGS[name]
+    requests = th.make_requests(config["vocab"], [29], seed=8)
+    streams = {}
+    reference(folder, config, requests, streams)
+    rep = TraceReplayer.from_folder(folder, "float32", 64, block_size=BLOCK_SIZE[name])
+    seen = []
+    rep.model.layer_hook = lambda index, x: seen.append(x.detach().double().cpu().clone())
+    th.collect(rep, th.whole(requests))
+    assert len(seen) == len(config["layers"])
+    for i, (mine, ref) in enumerate(zip(seen, streams["r0"])):
+        close(mine, ref, 1e-5, f"{name}: the stream after layer {i}")
+
+
+def test_layers_of_one_shape_run_from_one_launch_list(folders):
+    """The five delta-rule layers of D: what a layer leaves for the next one's first pass carries over."""
+    from tie_amd.engine.replay import TraceReplayer
+
+    folder, config = folders["D", "float32"], CONFIGS["D"]
+    requests = th.make_requests(config["vocab"], [150, 47], seed=18)
+    want = reference(folder, config, requests)
+    got = []
+    for replay in (True, False):
+        rep = TraceReplayer.from_folder(folder, "float32", 256, block_size=16)
+        rep.model.replay_layers = replay
+        got.append(th.collect(rep, th.whole(requests)))
+        assert rep.model.layers_replayed == (4 if replay else 0)          # two of five in each of two steps
+        check(got[-1], want, TOLERANCE["float32"], f"launch lists {replay}")
+    for rid, toks in requests.items():
+        assert all(torch.equal(got[0][rid][p], got[1][rid][p]) for p in range(len(toks)))
+
+
+def test_a_fault_of_one_position_or_one_term_would_show(folders):
+    """The engine agrees with the plain model, and the plain model with one mechanism slightly off does not agree
+    with the engine by a wide margin."""
+    from tie_amd.engine.replay import TraceReplayer
+
+    folder, config = folders["A", "float32"], CONFIGS["A"]
+    requests = th.make_requests(config["vocab"], [48, 31], seed=21)
+    got = th.collect(TraceReplayer.from_folder(folder, "float32", 128, block_size=BLOCK_SIZE["A"]),
+                     th.prefill_then_decode(requests, tail=20))
+    weights = load_plain(folder)
+    assert worst_error(got, reference(folder, config, requests)) < TOLERANCE["float32"]
+
+    def off(label, config_change=None, weight_change=None):
+        cfg, w = copy.deepcopy(config), dict(weights)
+        if config_change:
+            config_change(cfg)
+        if weight_change:
+            weight_change(w)
+        err = worst_error(got, {rid: plain.forward(cfg, w, toks)[0].float() for rid, toks in requests.items()})
+        print(f"[observed] {label}: {err:.3e}")
+        assert err > 100 * TOLERANCE["float32"], f"{label} does not show in the logits ({err:.3e})"
+
+    layer = lambda c, i: c["layers"][i]                                              # noqa: E731
+    off("a factor on the stream", lambda c: c.update(residual_mult=0.71))
+    off("logits left unscaled", lambda c: c.pop("logit_scale"))
+    off("the whole rotated part turned", lambda c: layer(c, 0)["mixer"]["rot"].update(dims=8))
+    off("another base", lambda c: layer(c, 0)["mixer"]["rot"].update(base=120.0))
+    off("another scale", lambda c: layer(c, 3)["mixer"].update(scale=0.26))
+    off("one expert fewer", lambda c: layer(c, 0)["mlp"]["router"].update(top=1))
+    off("one expert more", lambda c: layer(c, 4)["mlp"]["router"].update(top=2))
+    off("a higher limit", lambda c: layer(c, 1)["mlp"]["expert"].update(limit=2.0))
+    off("no experts", lambda c: layer(c, 4).update(mlp=None))
+    off("an embedding norm off", None, lambda w: w.__setitem__("embed.norm", torch.roll(w["embed.norm"], 1)))
+    off("a router without its bias", None, lambda w: w.__setitem__("l0.mlp.router.b", w["l0.mlp.router.b"] * 0))
+    off("gates of the wrong heads", None, lambda w: w.__setitem__("l0.mix.g", torch.roll(w["l0.mix.g"], 1, 0)))
+    off("a convolution that forgets its oldest input", None,
+        lambda w: w.__setitem__("l1.mix.k.conv", torch.cat([w["l1.mix.k.conv"][:, :1] * 0, w["l1.mix.k.conv"][:, 1:]], 1)))
+    off("no decay", None, lambda w: w.__setitem__("l1.mix.A_log", w["l1.mix.A_log"] - 30.0))
+    off("decays of the wrong heads", None, lambda w: w.__setitem__("l2.mix.a", torch.roll(w["l2.mix.a"], 1, 0)))
+    off("step sizes of the wrong heads", None, lambda w: w.__setitem__("l2.mix.b", torch.roll(w["l2.mix.b"], 1, 0)))
+    # value heads interleaved over the key heads instead of in blocks
+    order = torch.tensor([0, 2, 1, 3])
+    off("the wrong key head", None, lambda w: w.update(
+        {"l1.mix.v": w["l1.mix.v"].view(4, 24, -1)[order].reshape(96, -1),
+         "l1.mix.v.conv": w["l1.mix.v.conv"].view(4, 24, -1)[order].reshape(96, -1)}))
+
+
+def far_model(tmp_path):
+    """One latent-attention layer in which token 49 in a prompt alone answers the query of token 48, wherever it
+    stands: the rotated parts are zero, so that the distance does not count."""
+    config = {"architecture": "Vipalorn", "vocab": 50, "width": 32, "norm": {"eps": 1e-5},
+              "layers": [{"type": "latent_attention", "mlp": None,
+                          "mixer": {"heads": 2, "dim": 16, "rot_dim": 4, "vdim": 8, "kv_rank": 20, "scale": 1.0,
+                                    "rot": {"dims": 4, "base": 100.0}}}]}
+
+    def point(tensors):
+        w = {k: v.to(F64) for k, v in tensors.items()}
+        rows = plain.layer_norm(plain.layer_norm(w["embed"], w["embed.norm"], 1e-5), w["l0.norm1"], 1e-5)
+        latent = plain.rms_norm(rows[49] @ w["l0.mix.dkv"][:20].T, w["l0.mix.dkv.norm"], 1e-5)
+        keys = (w["l0.mix.uk"] @ latent).view(2, 16)
+        q = torch.zeros(2, 20, 32, dtype=F64)
+        q[:, :16] = 40.0 * (keys / (keys * keys).sum(-1, keepdim=True))[:, :, None] * rows[48] / (rows[48] @ rows[48])
+        tensors["l0.mix.q"] = q.view(40, 32).float()
+        tensors["l0.mix.dkv"][20:] = 0.0
+        tensors["l0.mix.uv"] *= 5.0
+
+    folder = write_model(tmp_path / "far", config, seed=77, dtype="float32", change=point)
+    return config, folder
+
+
+def test_a_far_key_decides_a_token(tmp_path):
+    """The answering key at the first position, on both sides of pages' borders, far back and just before the query;
+    asked for by a decoded token, by the last token of a whole prompt and at the end and the start of a portion."""
+    from tie_amd.engine.replay import TraceReplayer
+
+    config, folder = far_model(tmp_path)
+    weights = load_plain(folder)
+    base = torch.randint(0, 48, (400,), generator=torch.Generator().manual_seed(3)).tolist()
+    base[-1] = 48
+    for place in (0, 1, 15, 16, 47, 48, 200, 255, 256, 383, 384, 397, 398):
+        tokens = list(base)
+        tokens[place] = 49
+        full = plain.forward(config, weights, tokens)[0][-1].float()
+        without = plain.forward(config, weights, base)[0][-1].float()
+        assert float((without - full).abs().max() / full.abs().max()) > 0.05, f"the key at {place} does not decide"
+        rep = TraceReplayer.from_folder(folder, "float32", 448, block_size=16)
+        for cuts in ([400], [399, 400], [384, 400], [100, 398, 400], [16, 17, 300, 399, 400]):
+            steps, at = [], 0
+            for cut in cuts:
+                steps.append({"step": len(steps), "entries": [{"id": "a", "tokens": tokens[at:cut],
+                                                               "want": [cut - at - 1] if cut == 400 else []}],
+                              "end": ["a"] if cut == 400 else []})
+                at = cut
+            for step in steps:
+                logits = rep.run_step(step)
+            err = float((logits.float().cpu()[0] - full).abs().max() / full.abs().max())
+            assert err < TOLERANCE["float32"], f"key at {place}, cut at {cuts}: {err:.3e}"
+        assert rep.cache.all_free()
+
+
+def test_a_state_remembers_the_first_token_through_every_cut(tmp_path):
+    """One delta-rule layer that hardly decays: the last token's logits still know the first token, through long
+    decoding and chunk borders; a state lost at any cut would show."""
+    from tie_amd.engine.replay import TraceReplayer
+
+    config = {"architecture": "Vipalorn", "vocab": 60, "width": 48, "norm": {"eps": 1e-5}, "residual_mult": 2.0,
+              "layers": [{"type": "delta", "mlp": None,
+                          "mixer": {"heads": 2, "kv_heads": 1, "dim": 64, "vdim": 24, "conv": 3}}]}
+
+    def remember(tensors):
+        tensors["l0.mix.A_log"].fill_(-12.0)
+        tensors["l0.mix.b"] *= 3.0
+
+    folder = write_model(tmp_path / "state", config, seed=5, dtype="float32", change=remember)
+    weights = load_plain(folder)
+    tokens = torch.randint(1, 60, (330,), generator=torch.Generator().manual_seed(8)).tolist()
+    full = plain.forward(config, weights, tokens)[0].float()
+    other = plain.forward(config, weights, [(tokens[0] + 7) % 60] + tokens[1:])[0].float()
+    assert float((other[-1] - full[-1]).abs().max() / full.abs().max()) > 30 * TOLERANCE["float32"]
+    want = {"a": full}
+    for sizes in ((330,), (64,), (63, 1), (129, 2), (65, 130), (128, 1), (2, 150), (1,)):
+        rep = TraceReplayer.from_folder(folder, "float32", 384, block_size=16)
+        got = th.collect(rep, th.portions({"a": tokens}, sizes=sizes))
+        check(got, want, TOLERANCE["float32"], f"portions of {sizes}")
+
+
+def test_long_decoding_with_pages_and_slots_used_again(folders):
+    """Two requests decode 150 tokens each side by side, then others run in the pages and slots they left."""
+    from tie_amd.engine.replay import TraceReplayer
+
+    for dtype in ("float32", "bfloat16"):
+        folder, config = folders["A", dtype], CONFIGS["A"]
+        requests = th.make_requests(config["vocab"], [170, 165, 60, 140], seed=9)
+        want = reference(folder, config, requests)
+        steps = [{"step": 0, "entries": [{"id": r, "tokens": requests[r][:20 - i], "want": list(range(20 - i))}
+                                        for i, r in enumerate(("r0", "r1"))], "end": []}]
+        at = {"r0": 20, "r1": 19}
+        while at:
+            entries = [{"id": r, "tokens": [requests[r][p]], "want": [0]} for r, p in at.items()]
+            at = {r: p + 1 for r, p in at.items()}
+            ended = [r for r, p in at.items() if p == len(requests[r])]
+            steps.append({"step": len(steps), "entries": entries, "end": ended})
+            for r in ended:
+                del at[r]
+        for r in ("r2", "r3"):
+            steps.append({"step": len(steps), "entries": [{"id": r, "tokens": requests[r], "want": list(range(len(requests[r])))}],
+                          "end": [r]})
+        rep = TraceReplayer.from_folder(folder, dtype, 384, block_size=4, state_slots=2)
+        got = th.collect(rep, steps)
+        assert rep.cache.all_free()
+        check(got, want, TOLERANCE[dtype], f"long decoding, {dtype}")
+
+
+def test_state_slots_are_cleared_when_they_are_used_again(folders):
+    """Six requests through two state slots, one after another and side by side: every request starts from a zero
+    state and a zero convolution, whatever the slot held."""
+    from tie_amd.engine.replay import TraceReplayer
+
+    folder, config = folders["F", "float32"], CONFIGS["F"]
+    requests = th.make_requests(config["vocab"], [19, 30, 1, 135, 7, 22], seed=30)
+    want = reference(folder, config, requests)
+    steps, peak = th.mixed(requests, max_live=2, seed=6)
+    rep = TraceReplayer.from_folder(folder, "float32", peak, block_size=BLOCK_SIZE["F"], state_slots=2)
+    got = th.collect(rep, steps)
+    assert rep.cache.all_free()
+    check(got, want, TOLERANCE["float32"], "slots used again")
+
+
+def test_a_batch_gives_what_each_request_gives_alone(folders):
+    """Unequal requests in one step, a long portion (its recurrence in chunks) beside single decoded tokens."""
+    from tie_amd.engine.replay import TraceReplayer
+
+    folder, config = folders["D", "float32"], CONFIGS["D"]
+    requests = th.make_requests(config["vocab"], [200, 40, 3, 90], seed=33)
+    want = reference(folder, config, requests)
+    rep = TraceReplayer.from_folder(folder, "float32", 512, block_size=16)
+    cuts = {"r0": [0, 20, 180, 199, 200], "r1": [0, 38, 39, 40, 40], "r2": [0, 1, 2, 3, 3], "r3": [0, 2, 3, 60, 90]}
+    steps = []
+    for i in range(4):
+        entries = [{"id": r, "tokens": requests[r][c[i]:c[i + 1]], "want": list(range(c[i + 1] - c[i]))}
+                   for r, c in cuts.items() if c[i + 1] > c[i]]
+        steps.append({"step": i, "entries": entries, "end": [r for r, c in cuts.items()
+                                                             if c[i] < len(requests[r]) == c[i + 1]]})
+    check(th.collect(rep, steps), want, TOLERANCE["float32"], "a batch of unequal requests")
+    assert rep.cache.all_free()
+
+
+@pytest.mark.parametrize("name", ["A", "B", "D"])
+def test_decode_steps_replayed_from_recordings_give_the_eager_logits(folders, name):
+    """bfloat16 decode-only steps are recorded into HIP graphs and replayed; every replay against the eager engine."""
+    from tie_amd.engine.replay import TraceReplayer
+
+    folder, config = folders[name, "bfloat16"], CONFIGS[name]
+    requests = th.make_requests(config["vocab"], [50, 41, 47], seed=10)
+    steps, peak = th.mixed(requests, max_live=3, seed=4, tail=30)
+    eager = TraceReplayer.from_folder(folder, "bfloat16", peak, block_size=BLOCK_SIZE[name], use_graphs=False)
+    recorded = TraceReplayer.from_folder(folder, "bfloat16", peak, block_size=BLOCK_SIZE[name])
+    assert recorded.runner.use_graphs
+    a, b = th.collect(eager, steps), th.collect(recorded, steps)
+    assert recorded.runner.graph_replays > 10
+    for rid, toks in requests.items():
+        for p in range(len(toks)):
+            assert torch.equal(a[rid][p], b[rid][p]), f"request {rid}, position {p}"
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("name", ["A", "B", "E"])
+def test_greedy_generation_through_the_engine(folders, name, dtype):
+    """The engine's own entry point and scheduler: several requests at once, prompts in portions, a small pool."""
+    import tie_amd
+
+    folder, config = folders[name, dtype], CONFIGS[name]
+    weights = load_plain(folder)
+    prompts = list(th.make_requests(config["vocab"], [7, 19, 3, 30], seed=12).values())
+    new = 10
+    engine = tie_amd.create_engine(folder, dtype=dtype, kv_blocks=64, block_size=BLOCK_SIZE[name], max_seqs=3,
+                                   max_tokens_per_step=16, prefill_chunk=8)
+    ids = [engine.add_request(p, tie_amd.SamplingParams(max_tokens=new)) for p in prompts]
+    while engine.has_work():
+        engine.step()
+    for sid, prompt in zip(ids, prompts):
+        generated = list(engine.sequence(sid).generated)
+        assert len(generated) == new
+        tokens = list(prompt)
+        for i, token in enumerate(generated):       # every generated token is the plain model's best, or ties it
+            logits = plain.forward(config, weights, tokens)[0][-1]
+            best = float(logits.max())
+            margin = 1e-4 * float(logits.abs().max()) if dtype == "float32" else 0.05 * float(logits.abs().max())
+            assert float(logits[token]) >= best - margin, f"request {sid}: token {i} is not the plain model's choice"
+            tokens.append(token)
+
+
+def test_the_command_line_generates_the_plain_models_tokens(folders):
+    from conftest import ROOT
+
+    folder, config = folders["A", "float32"], CONFIGS["A"]
+    weights = load_plain(folder)
+    prompt = list(th.make_requests(config["vocab"], [11], seed=14).values())[0]
+    tokens = list(prompt)
+    for _ in range(6):
+        tokens.append(int(plain.forward(config, weights, tokens)[0][-1].argmax()))
+    proc = subprocess.run([sys.executable, str(ROOT / "bin" / "tie"), "generate", "-m", folder, "-p",
+                           ",".join(map(str, prompt)), "--temp", "0", "--max-tokens", "6", "--dtype", "float32",
+                           "--kv-mem", "16M"], capture_output=True, text=True, timeout=600)
+    assert proc.returncode == 0, proc.stderr[-2000:]
+    assert [int(t) for t in proc.stdout.split()] == tokens[len(prompt):]
+
+
+def test_the_trace_program_runs_the_design(folders, tmp_path):
+    """JSON lines in, .f32 files and 'done' lines out; four slots, pages used again."""
+    from conftest import ROOT
+
+    folder, config = folders["B", "float32"], CONFIGS["B"]
+    requests = th.make_requests(config["vocab"], [23, 140, 9, 31, 17], seed=2)
+    steps, peak = th.mixed(requests, max_live=4, seed=1)
+    out = tmp_path / "out"
+    proc = subprocess.run([sys.executable, str(ROOT / "bin" / "trace_run"), "--model", folder, "--dtype", "float32",
+                           "--out", str(out), "--max-tokens", str(peak)],
+                          input="".join(json.dumps(s) + "\n" for s in steps), capture_output=True, text=True, timeout=600)
+    assert proc.returncode == 0, proc.stderr[-2000:]
+    assert [line for line in proc.stdout.splitlines() if line.startswith("done")] == [f"done {s['step']}" for s in steps]
+    want = reference(folder, config, requests)
+    position = {}
+    for s in steps:
+        data = np.fromfile(out / f"{s['step']}.f32", dtype="<f4").reshape(-1, config["vocab"])
+        r = 0
+        for e in s["entries"]:
+            start = position.get(e["id"], 0)
+            for w in e["want"]:
+                ref = want[e["id"]][start + w]
+                assert float(np.abs(data[r] - ref.numpy()).max() / ref.abs().max()) < TOLERANCE["float32"]
+                r += 1
+            position[e["id"]] = start + len(e["tokens"])
+        assert r == data.shape[0]

@@ -60,6 +60,7 @@ _SOURCES = {
     "recurrent": ("tie_recurrent", "recurrent.hip"),
     "hyper": ("tie_hyper", "hyper.hip"),
     "delta_rule": ("tie_delta_rule", "delta_rule.hip"),
+    "delta_chunks": ("tie_delta_chunks", "delta_chunks.hip"),
     "latent": ("tie_latent", "latent.hip"),
     "pointwise": ("tie_pointwise", "pointwise.hip"),
     "residual": ("tie_residual", "residual.hip"),
@@ -155,6 +156,12 @@ _SIGNATURES = {
                                          _c_int, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_void],
         "tie_grouped_gated_rms_norm": [_c_void, _c_int, _c_void, _c_float, _c_void, _c_int, _c_int, _c_void, _c_int,
                                        _c_int, _c_int, _c_int, _c_void],
+    },
+    "delta_chunks": {
+        "tie_delta_chunk_rows": [],
+        "tie_delta_chunk_floats": [_c_int, _c_int],
+        "tie_delta_chunks": [_c_void, _c_int, _c_void, _c_int, _c_void, _c_void, _c_int, _c_void, _c_void, _c_int,
+                             _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void],
     },
     "pointwise": {
         "tie_dynamic_tanh": [_c_void, _c_void, _c_long, _c_int, _c_void, _c_void, _c_void, _c_void, _c_int, _c_void,
@@ -2237,6 +2244,19 @@ def delta_prepare(u: torch.Tensor, weight: torch.Tensor, taps: int, state: Optio
 DELTA_CHUNK_ROWS = 256                 # rows of a chunk of the gated delta rule's chunked walk
 DELTA_CHUNKS_FROM = 1024               # a step's longest portion from which the rule runs in chunks (three launches)
 DELTA_CHUNK_SCRATCH_MAX = 1 << 30      # bytes of chunk states above which a step walks its sequences whole
+# With one decay a head a chunk's products are matrix products (csrc/delta_chunks.hip): shorter chunks, and from shorter
+# portions on. Above the scratch limit the heads run in several passes.
+DELTA_HEAD_CHUNK_ROWS = 64             # DC_ROWS of csrc/delta_chunks.hip
+DELTA_HEAD_CHUNKS_FROM = 128
+
+
+def delta_chunks(batch, device, head_decay: bool = False) -> Optional[ScanChunks]:
+    """The chunks in which a step's gated delta rules run, or None where every sequence is walked in one go (steps of
+    short portions; steps with chunks are never recorded)."""
+    longest = max(batch.host_new_tokens)
+    if head_decay:
+        return scan_chunks(batch, device, rows=DELTA_HEAD_CHUNK_ROWS, force=True) if longest >= DELTA_HEAD_CHUNKS_FROM else None
+    return scan_chunks(batch, device, rows=DELTA_CHUNK_ROWS) if longest >= DELTA_CHUNKS_FROM else None
 
 
 def gated_delta_scan(tok: torch.Tensor, out: torch.Tensor, state: torch.Tensor, batch, kv_heads: int, heads: int,
@@ -2251,7 +2271,8 @@ def gated_delta_scan(tok: torch.Tensor, out: torch.Tensor, state: torch.Tensor, 
     ``S_t = (I - beta k k^T) diag(decay) S_(t-1) + beta k v^T``, so a chunk is ``S_end = P S_start + L``: every chunk
     walks from a zero state with ``d`` more columns that start as the identity and take no values (they end as
     ``P``), the chunks' states are combined in order, and every chunk walks again from its true start, with
-    outputs. The same values up to rounding."""
+    outputs. The same values up to rounding. With ``head_decay`` (one decay a head) a chunk of up to
+    ``DELTA_HEAD_CHUNK_ROWS`` rows is solved as matrix products instead of token by token."""
     G, H, d, e = kv_heads, heads, key_dim, value_dim
     T = tok.shape[0]
     _f32(tok, "delta rule rows", (T, delta_row(G, H, d, e, head_decay)))
@@ -2262,7 +2283,19 @@ def gated_delta_scan(tok: torch.Tensor, out: torch.Tensor, state: torch.Tensor, 
                               f"{DELTA_RULE_MAX_DIM}, {G} key heads)")
     if batch.num_seqs == 0:
         return
-    if chunks is not None and not head_decay and chunks.count * H * d * (e + d) * 4 <= DELTA_CHUNK_SCRATCH_MAX:
+    if chunks is not None and head_decay:
+        if chunks.longest > DELTA_HEAD_CHUNK_ROWS:
+            raise InvalidArgument(f"a chunk of {chunks.longest} rows exceeds {DELTA_HEAD_CHUNK_ROWS}")
+        floats = int(_lib("delta_chunks").tie_delta_chunk_floats(d, e))
+        at_once = max(1, min(H, DELTA_CHUNK_SCRATCH_MAX // (chunks.count * floats * 4)))
+        memory = scratch("delta_rule.chunk_memory", (chunks.count * at_once * floats,), torch.float32)
+        for head0 in range(0, H, at_once):
+            _call(_lib("delta_chunks").tie_delta_chunks, "delta_chunks", tok.data_ptr(), tok.stride(0), out.data_ptr(),
+                  out.stride(0), state.data_ptr(), batch.state_slots.data_ptr(), batch.num_seqs,
+                  chunks.items.data_ptr(), chunks.first_item.data_ptr(), chunks.count, memory.data_ptr(), G, H, d, e,
+                  head0, min(at_once, H - head0), _stream())
+        return
+    if chunks is not None and chunks.count * H * d * (e + d) * 4 <= DELTA_CHUNK_SCRATCH_MAX:
         ends = scratch("delta_rule.chunk_ends", (chunks.count, H, d, e + d), torch.float32)
         starts = scratch("delta_rule.chunk_starts", (chunks.count, H, d, e), torch.float32)
         _call(_lib("delta_rule").tie_gated_delta_scan_chunked, "gated_delta_scan_chunked", tok.data_ptr(),

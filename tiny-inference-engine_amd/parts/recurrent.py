@@ -288,9 +288,7 @@ class GatedDeltaRule(Mixer):
         if conv_state is not None and state.writes:
             kernels.conv_state_update(proj, self.taps, conv_state, ctx.batch, self.channels)
         o = ctx.scratch("delta_rule.o", (T, self.v_width), torch.float32)
-        chunks = None
-        if max(ctx.batch.host_new_tokens) >= kernels.DELTA_CHUNKS_FROM:      # such steps are never recorded
-            chunks = kernels.scan_chunks(ctx.batch, ctx.device, rows=kernels.DELTA_CHUNK_ROWS)
+        chunks = kernels.delta_chunks(ctx.batch, ctx.device, self.head_decay)
         kernels.gated_delta_scan(tok, o, state.state, ctx.batch, *sizes, chunks=chunks, scratch=ctx.scratch,
                                  head_decay=self.head_decay)
         gated = ctx.scratch("delta_rule.gated", (T, self.v_width))
