@@ -166,6 +166,40 @@ def test_experts_whose_sums_are_cut_off(T, E, top, F_, K, limit, dtype):
     close(out, want, 1e-5 if dtype == torch.float32 else 2e-2, f"experts in tiles of {tile}")
 
 
+@pytest.mark.parametrize("tile", [16, 64, 128, 256])
+@pytest.mark.parametrize("kind", ["silu", "relu_squared", "clipped"])
+@pytest.mark.parametrize("T,E,top,F_,K", [(3, 4, 2, 96, 128), (90, 3, 2, 128, 96), (600, 5, 1, 160, 224), (400, 40, 3, 96, 352)])
+def test_experts_over_packed_weights(T, E, top, F_, K, kind, tile):
+    """All tile sizes, also those the sizes would not choose: ragged tiles, columns in no step of a tile's, experts that
+    nobody chose, one that gets most rows; every activation an expert can have."""
+    from tie_amd import kernels
+
+    bf = torch.bfloat16
+    h, down = rnd(T, K, seed=1).to(bf), rnd(E, K, F_, seed=4, scale=0.2).to(bf)
+    gate, up = rnd(E, F_, K, seed=2, scale=0.1).to(bf), rnd(E, F_, K, seed=3, scale=0.1).to(bf)
+    g = torch.Generator().manual_seed(4)
+    ids = torch.stack([torch.randperm(E - 1, generator=g)[:top] for _ in range(T)]).to(torch.int32)       # the last: nobody's
+    ids[: T // 2, 0] = 0
+    ids[: T // 2, 1:] = (ids[: T // 2, 1:] % (E - 2)) + 1
+    weights = torch.rand(T, top, generator=g)
+    want = torch.zeros(T, K, dtype=F64)
+    for e in range(E):
+        a, b = h.to(F64) @ gate[e].to(F64).T, h.to(F64) @ up[e].to(F64).T
+        act = {"silu": lambda: torch.nn.functional.silu(a) * b, "relu_squared": lambda: torch.relu(b) ** 2,
+               "clipped": lambda: plain.clipped_gate(a, b, 0.6)}[kind]()
+        want += (act @ down[e].to(F64).T) * (weights.to(F64) * (ids == e)).sum(1, keepdim=True)
+    up_packed, down_packed = kernels.pack_experts(None if kind == "relu_squared" else gate.cuda(), up.cuda(), down.cuda())
+    get = scratch_memory()
+    rows = kernels.moe_align(ids.cuda(), E, tile, get)
+    act = get("act", (T * top, F_), bf)
+    kernels.moe_gate_up(h.cuda(), None, up_packed, rows, act, clipped=(0.6, 1.702, 1.0) if kind == "clipped" else None)
+    parts = get("parts", (T * top, K))
+    kernels.moe_down(act, down_packed, rows, parts)
+    out = torch.zeros(T, K, device="cuda")
+    kernels.moe_combine(kernels.RoutedParts(parts, rows.where, weights.cuda(), h.cuda()), out)
+    close(out, want, 2e-2, f"packed experts in tiles of {tile}")
+
+
 @pytest.mark.parametrize("activation", ["silu", "sigmoid"])
 def test_the_gated_norm_of_the_heads_outputs(activation):
     from tie_amd import kernels
@@ -662,6 +696,24 @@ def test_decode_steps_replayed_from_recordings_give_the_eager_logits(folders, na
     for rid, toks in requests.items():
         for p in range(len(toks)):
             assert torch.equal(a[rid][p], b[rid][p]), f"request {rid}, position {p}"
+
+
+@pytest.mark.parametrize("graphs", [False, True])
+def test_sub_layers_on_two_streams_give_what_one_stream_gives(folders, monkeypatch, graphs):
+    from tie_amd.engine.replay import TraceReplayer
+    from tie_amd.parts.block import ParallelResidualBlock
+
+    for name in ("A", "B", "D"):
+        folder, config = folders[name, "bfloat16"], CONFIGS[name]
+        requests = th.make_requests(config["vocab"], [150, 41, 47], seed=10)
+        steps, peak = th.mixed(requests, max_live=3, seed=4, tail=25, sizes=(130, 7))
+        got = []
+        for side_by_side in (True, False):
+            monkeypatch.setattr(ParallelResidualBlock, "SIDE_BY_SIDE", side_by_side)
+            rep = TraceReplayer.from_folder(folder, "bfloat16", peak, block_size=BLOCK_SIZE[name], use_graphs=graphs)
+            got.append(th.collect(rep, steps))
+        for rid, toks in requests.items():
+            assert all(torch.equal(got[0][rid][p], got[1][rid][p]) for p in range(len(toks))), f"{name}, request {rid}"
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])

@@ -2,7 +2,8 @@
 
 A mixes both mixers, latent attention whose cached head (28 + 8) is padded to 48 and whose rotation covers part of the
 rotated dimensions, grouped delta-rule heads with three taps, layers with and without experts. B has twenty latent
-heads (more than one wave of the matrix-core decode kernel takes), one expert chosen of one, delta-rule keys wider
+heads (more than one wave of the matrix-core decode kernel takes), one expert chosen of one, experts of the sizes
+whose matrices are packed, delta-rule keys wider
 than their values and ungrouped. C has sizes in no step of 8, convolutions of one tap (no state beside the matrix), all
 experts chosen, three value heads on one key head. D is five delta-rule layers of one shape in a row, with keys and
 values of different sizes in the matrix-core steps, no factors on the stream or the logits. E is attention alone:
@@ -45,8 +46,8 @@ B = {
     "architecture": "Vipalorn", "vocab": 211, "width": 96, "norm": {"eps": 1e-6}, "residual_mult": 1.25,
     "logit_scale": 3.0,
     "layers": [
-        {**_delta(2, 2, 40, 16, 2), "mlp": _moe(1, 1, 72, 2.0)},
-        {**_latent(20, 16, 16, 8, 48, 0.15, 777.0), "mlp": _moe(16, 4, 32, 1.0)},
+        {**_delta(2, 2, 40, 16, 2), "mlp": _moe(1, 1, 96, 2.0)},
+        {**_latent(20, 16, 16, 8, 48, 0.15, 777.0), "mlp": _moe(16, 4, 128, 1.0)},
         {**_latent(4, 32, 32, 24, 64, 0.1, 250.0), "mlp": None},
     ],
 }

@@ -25,7 +25,7 @@
 //
 // Nothing here reads the step on the host: the tile list and its length live on the device, the grid is sized
 // for the most tiles T * top slots can make and workgroups beyond the list leave at once.
-#include "common.h"
+#include "expert_activation.h"
 
 #include <math.h>
 
@@ -264,24 +264,12 @@ extern "C" int tie_moe_align(const int* ids, int slots, int real, int tile_rows,
 #define GC 64
 #define GK 16
 
-__device__ __forceinline__ float silu_f(float g) { return g / (1.0f + expf(-g)); }
-
-// What a gated expert makes of its gate's and up's sums.
-struct GateParams {
-  float limit, slope, shift;      // MODE 3 only
-};
-
-__device__ __forceinline__ float clipped_gate_f(float a, float b, GateParams p) {
-  const float g = fminf(a, p.limit), u = fminf(fmaxf(b, -p.limit), p.limit);
-  return g / (1.0f + expf(-p.slope * g)) * (u + p.shift);
-}
 
 // MODE 1 (gated): x rows are gathered (row = slot_at[place] / top), w_a and w_b are the gate and up weights
 // [real][N][K], out[place][c] = silu(a) * b. MODE 3 (gated, sums cut off at a limit): the same rows and weights,
 // out[place][c] = clipped_gate(a, b). MODE 2 (experts without a gate): rows gathered likewise, w_a the up
 // weight, out[place][c] = relu(a)^2. MODE 0: x rows are the places themselves (act [slots][K]), w_a is the down
 // weight and out[place][c] = a.
-__device__ __forceinline__ float relu_squared_f(float a) { const float r = fmaxf(a, 0.f); return r * r; }
 
 template <typename TX, typename TW, typename TO, int MODE>
 __global__ __launch_bounds__(256) void moe_gemm_generic_kernel(

@@ -57,6 +57,7 @@ _SOURCES = {
     "sample_filtered": ("tie_sample_filtered", "sample_filtered.hip"),
     "machine_peaks": ("tie_machine_peaks", "machine_peaks.hip"),
     "moe": ("tie_moe", "moe.hip"),
+    "moe_packed": ("tie_moe_packed", "moe_packed.hip"),
     "recurrent": ("tie_recurrent", "recurrent.hip"),
     "hyper": ("tie_hyper", "hyper.hip"),
     "delta_rule": ("tie_delta_rule", "delta_rule.hip"),
@@ -122,6 +123,11 @@ _SIGNATURES = {
         "tie_moe_gemm_bf16": [_c_void, _c_void, _c_void, _c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_int,
                               _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_void],
         "tie_moe_combine": [_c_void, _c_void, _c_void, _c_void, _c_int, _c_void, _c_int, _c_int, _c_int, _c_int, _c_void],
+    },
+    "moe_packed": {
+        "tie_moe_packed_tile_rows": [_c_int, _c_int, _c_int],
+        "tie_moe_gemm_packed": [_c_void, _c_int, _c_void, _c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_int,
+                                _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_void],
     },
     "gemm_generic": {
         "tie_gemm_generic": [_c_void, _c_int, _c_void, _c_int, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int,
@@ -302,6 +308,17 @@ def _call(fn, what: str, *args) -> None:
     if _recording is not None:
         _recording.append((fn, args, what))
     _check(status, what)
+
+
+def _order_streams(waiting: torch.cuda.Stream, first: torch.cuda.Stream) -> int:
+    waiting.wait_stream(first)
+    return 0
+
+
+def order_streams(waiting: torch.cuda.Stream, first: torch.cuda.Stream) -> None:
+    """What is launched on ``waiting`` from now on runs behind everything launched on ``first`` so far. Noted like a
+    launch, so that layers run from a launch list keep their order; a recorded step gets a fork or a join."""
+    _call(_order_streams, "order_streams", waiting, first)
 
 
 def replay_call(fn, what: str, args) -> None:
@@ -1833,6 +1850,21 @@ def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], groups: 
           int(shared), ids.data_ptr(), weights.data_ptr(), _stream())
 
 
+def pack_experts(w_gate: Optional[torch.Tensor], w_up: torch.Tensor, w_down: torch.Tensor):
+    """The experts' matrices as the packed products take them: ``(up, down)``, each one ``PackedWeight`` of all experts'
+    matrices one behind the other (``[real * N, K]``), gate and up rows interleaved in blocks of 8; or None where the
+    sizes or types do not fit (bfloat16; the stream and the experts' inner size in steps of 32 and at least 96)."""
+    real, F_, K = w_up.shape
+    if not all(t.dtype == torch.bfloat16 and t.is_cuda for t in (w_up, w_down)) or (w_gate is not None and
+                                                                                  w_gate.dtype != torch.bfloat16) or \
+            K % 32 or F_ % 32 or min(K, F_) < 96 or max(K, F_) > (1 << 20):
+        return None
+    first = w_up.reshape(real * F_, K)
+    if w_gate is not None:
+        first = interleave_gate_up(w_gate.reshape(real * F_, K), first)
+    return pack_weight(first), pack_weight(w_down.reshape(real * K, F_))
+
+
 class ExpertRows:
     """The (row, choice) slots of a step sorted by expert, on the device: see ``moe_align``."""
 
@@ -1840,10 +1872,12 @@ class ExpertRows:
 
 
 def moe_tile_rows(x_dtype: torch.dtype, w_dtype: torch.dtype, hidden: int, intermediate: int, slots: int,
-                  real: int) -> int:
+                  real: int, packed: bool = False) -> int:
     """Rows of a row tile of the experts' products, which also says which kernels run them: 16, 64 or 128 (by the rows an
     expert gets on average) for the matrix-core kernels, which take bfloat16 rows and weights whose inner sizes
     are multiples of 8; the float32 kernels' tile otherwise."""
+    if packed:                 # weights of ``pack_experts``
+        return int(_lib("moe_packed").tie_moe_packed_tile_rows(slots, real, intermediate))
     lib = _lib("moe")
     if x_dtype == torch.bfloat16 and w_dtype == torch.bfloat16 and hidden % 8 == 0 and intermediate % 8 == 0:
         return int(lib.tie_moe_bf16_tile_rows(slots, real))
@@ -1893,13 +1927,39 @@ def _moe_weights(w: torch.Tensor, real: int, name: str):
     return w.shape[1], w.shape[2]
 
 
+def _moe_packed(x: torch.Tensor, w: PackedWeight, out: torch.Tensor, mode: int, rows: ExpertRows, gate_params, what: str,
+                columns: int = 0) -> None:
+    """One product of the experts over packed weights (see csrc/moe_packed.hip)."""
+    _gpu(x, "the experts' rows")
+    _gpu(out, "the experts' results")
+    total, K = w.shape
+    N = total // rows.real
+    width = N // 2 if mode in (1, 3) else N
+    if x.dtype != torch.bfloat16 or x.dim() != 2 or x.shape[1] != K or total % rows.real or N % 16 or \
+            x.shape[0] * (rows.top if mode else 1) != rows.slots or tuple(out.shape) != (rows.slots, width) or \
+            out.dtype != (torch.bfloat16 if mode else torch.float32):
+        raise InvalidArgument(f"{what}: rows {list(x.shape)} {x.dtype}, results {list(out.shape)} {out.dtype}, packed "
+                              f"weights {list(w.shape)} of {rows.real} experts")
+    _call(_lib("moe_packed").tie_moe_gemm_packed, what, x.data_ptr(), x.shape[0], w.data_ptr(), out.data_ptr(), mode,
+          rows.offsets.data_ptr(), rows.slot_at.data_ptr(), rows.tiles.data_ptr(), rows.num_tiles.data_ptr(),
+          rows.max_tiles, rows.tile_rows, int(columns), rows.top, N, K, *gate_params, _stream())
+
+
 def moe_gate_up(x: torch.Tensor, w_gate: Optional[torch.Tensor], w_up: torch.Tensor, rows: ExpertRows,
                 act: torch.Tensor, clipped: Optional[tuple] = None) -> None:
     """``act[place] = silu(x[row] Wg_e^T) * (x[row] Wu_e^T)`` for every sorted slot: ``x [T, K]``, weights
     ``[real, F, K]``. Without gate weights (``w_gate`` None) the experts have no gate and the activation is the square
     of relu: ``act[place] = relu(x[row] Wu_e^T)^2``. ``clipped`` ``(limit, slope, shift)`` (with gate weights): the sums
     are cut off first, ``g = min(gate sum, limit)``, ``u = clamp(up sum, -limit, limit)``, and the activation is
-    ``g sigmoid(slope g) (u + shift)``."""
+    ``g sigmoid(slope g) (u + shift)``. ``w_up`` may be the packed first matrices of ``pack_experts`` (gate weights then
+    None; whether they hold gates follows from their rows)."""
+    if isinstance(w_up, PackedWeight):
+        gated = w_up.shape[0] == 2 * rows.real * act.shape[1]
+        if clipped is not None and (not gated or not clipped[0] > 0):
+            raise InvalidArgument(f"clipped sums need a gate and a positive limit, got {clipped}")
+        _moe_packed(x, w_up, act, (1 if clipped is None else 3) if gated else 2, rows,
+                    tuple(float(v) for v in clipped) if clipped is not None else (0.0, 0.0, 0.0), "moe_gate_up")
+        return
     _gpu(x, "the experts' input rows")
     _gpu(act, "the experts' activations")
     F_, K = _moe_weights(w_up, rows.real, "up weights")
@@ -1927,7 +1987,11 @@ def moe_gate_up(x: torch.Tensor, w_gate: Optional[torch.Tensor], w_up: torch.Ten
 
 
 def moe_down(act: torch.Tensor, w_down: torch.Tensor, rows: ExpertRows, parts: torch.Tensor) -> None:
-    """``parts[place] = act[place] Wd_e^T`` (float32 ``[slots, N]``) for every sorted slot; weights ``[real, N, F]``."""
+    """``parts[place] = act[place] Wd_e^T`` (float32 ``[slots, N]``) for every sorted slot; weights ``[real, N, F]`` or the
+    packed ones of ``pack_experts``."""
+    if isinstance(w_down, PackedWeight):
+        _moe_packed(act, w_down, parts, 0, rows, (0.0, 0.0, 0.0), "moe_down")
+        return
     _gpu(act, "the experts' activations")
     _f32(parts, "the experts' results")
     N, F_ = _moe_weights(w_down, rows.real, "down weights")

@@ -139,6 +139,7 @@ class Workspace:
         self.device = device
         self._buffers: Dict[Any, torch.Tensor] = {}
         self._views: Dict[Any, torch.Tensor] = {}     # (name, dtype, shape) -> view: a layer asks again every step
+        self._side_stream: Optional[torch.cuda.Stream] = None
         self.generation = 0   # grows whenever a buffer is replaced: recorded steps are then stale
 
     def get(self, name: str, shape, dtype: torch.dtype) -> torch.Tensor:
@@ -160,6 +161,13 @@ class Workspace:
             self._views.clear()
         view = self._views[(name, dtype, shape)] = buf[:numel].view(*shape)
         return view
+
+    def side_stream(self) -> torch.cuda.Stream:
+        """One more stream beside the one the step runs on (of the same priority), for launches that need not wait for
+        the step's other launches; the same one for every layer and step."""
+        if self._side_stream is None:
+            self._side_stream = torch.cuda.Stream(self.device)
+        return self._side_stream
 
     def nbytes(self) -> int:
         return sum(b.numel() * b.element_size() for b in self._buffers.values())

@@ -20,7 +20,10 @@ layers share), ``g = gelu_tanh(W_gate x) * e`` from the stream itself (no norm b
 ``parallel_residual`` runs both sub-layers side by side: with ``h = pre(x)``, one norm, ``x += scale * (mixer(h) +
 feed_forward(h))``. What a layer adds is left with the step and rides in the next layer's first pass over the stream,
 which adds the sub-layers' results (rows, planes of partial sums, a routed feed-forward's parts not yet combined) and
-norms the sum in one kernel. Parameters: ``hidden``, ``scale``.
+norms the sum in one kernel. Neither sub-layer waits for the other: the feed-forward is launched on a second stream
+that forks behind the norm and joins before the results are added, so that in a decode step (a chain of short kernels
+each, in a recorded step two branches of the graph) the two chains' latencies overlap. Parameters: ``hidden``,
+``scale``.
 
 ``hyper_connections`` keeps ``streams`` copies of the residual instead of one. All start as the embedding's rows.
 Sub-layer q of a layer (its mixer, then its feed-forward) has three small tensors ``in`` ``[streams]``, ``out``
@@ -189,6 +192,7 @@ class SandwichNormBlock(Block):
 class ParallelResidualBlock(Block):
     capturable = True
     replayable = True      # what is left for the next layer names scratch memory only, the same for every layer
+    SIDE_BY_SIDE = True
     NORMS = ("pre",)
 
     def __init__(self, params):
@@ -222,14 +226,25 @@ class ParallelResidualBlock(Block):
             h = norm.forward(ctx, x, results=left)
         else:
             h = self.normed(ctx, norm, x)
-        results = []
-        if layer.mixer is not None:
-            results.append(self._result(ctx, layer.mixer, lambda residual: layer.mixer.forward(ctx, h, cache, residual),
-                                        "block.mixer_result"))
-        if layer.feed_forward is not None:
-            results.append(self._result(ctx, layer.feed_forward,
-                                        lambda residual: layer.feed_forward.forward(ctx, h, residual),
-                                        "block.feed_forward_result"))
+        def run_mixer():
+            return self._result(ctx, layer.mixer, lambda residual: layer.mixer.forward(ctx, h, cache, residual),
+                                "block.mixer_result")
+
+        def run_feed_forward():
+            return self._result(ctx, layer.feed_forward, lambda residual: layer.feed_forward.forward(ctx, h, residual),
+                                "block.feed_forward_result")
+
+        both = layer.mixer is not None and layer.feed_forward is not None
+        if both and self.SIDE_BY_SIDE and getattr(layer.feed_forward, "returns_result", False):
+            here, side = torch.cuda.current_stream(ctx.device), ctx.workspace.side_stream()
+            kernels.order_streams(side, here)
+            with torch.cuda.stream(side):
+                beside = run_feed_forward()
+            results = [run_mixer(), beside]
+            kernels.order_streams(here, side)
+        else:
+            results = [run() for part, run in ((layer.mixer, run_mixer), (layer.feed_forward, run_feed_forward))
+                       if part is not None]
         # settle() (the model's end, a hook, another kind of block) adds them without a norm behind
         ctx.leave_late(key, lambda left: kernels.add_results(x, *left), (results, self.scale))
 

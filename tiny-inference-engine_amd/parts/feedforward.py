@@ -231,8 +231,8 @@ class RoutedExperts(FeedForward):
         self.router = Linear(router_names, router_sizes, self.hidden)
         self.correction: torch.Tensor = None
         self.router_bias: torch.Tensor = None
-        self.gate: torch.Tensor = None        # [experts (+ shared pieces), intermediate, hidden]
-        self.up: torch.Tensor = None
+        self.gate: torch.Tensor = None        # [experts (+ shared pieces), intermediate, hidden]; in packed blocks
+        self.up: torch.Tensor = None          # (``kernels.pack_experts``) where the sizes fit, gate and up as one
         self.down: torch.Tensor = None        # [experts (+ shared pieces), hidden, intermediate]
 
     def tensors(self) -> List[TensorSpec]:
@@ -278,6 +278,9 @@ class RoutedExperts(FeedForward):
 
         self.gate = stack("gate", True) if self.gated else None
         self.up, self.down = stack("up", True), stack("down", False)
+        packed = kernels.pack_experts(self.gate, self.up, self.down)
+        if packed is not None:        # the products then read these alone
+            self.gate, (self.up, self.down) = None, packed
 
     def forward(self, ctx: StepContext, h: torch.Tensor, residual: Optional[torch.Tensor]):
         T = h.shape[0]
@@ -290,7 +293,8 @@ class RoutedExperts(FeedForward):
                           scoring=self.scoring, group_top=self.group_top, renormalize=self.renormalize,
                           renorm_eps=self.renorm_eps, weight_scale=self.weight_scale, shared=self.shared_pieces,
                           bias=self.router_bias)
-        tile_rows = kernels.moe_tile_rows(h.dtype, self.up.dtype, self.hidden, self.intermediate, T * slots, real)
+        tile_rows = kernels.moe_tile_rows(h.dtype, self.up.dtype, self.hidden, self.intermediate, T * slots, real,
+                                          packed=isinstance(self.up, kernels.PackedWeight))
         rows = kernels.moe_align(ids, real, tile_rows, ctx.scratch)
         act = ctx.scratch("moe.act", (T * slots, self.intermediate))
         kernels.moe_gate_up(h, self.gate, self.up, rows, act, clipped=self.clipped)
