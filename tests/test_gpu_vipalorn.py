@@ -698,6 +698,8 @@ def test_decode_steps_replayed_from_recordings_give_the_eager_logits(folders, na
             assert torch.equal(a[rid][p], b[rid][p]), f"request {rid}, position {p}"
 
 
+@pytest.mark.skip(reason="two streams in one step are switched off: a run with them ended in a segmentation fault of the "
+                         "host process whose cause is not known")
 @pytest.mark.parametrize("graphs", [False, True])
 def test_sub_layers_on_two_streams_give_what_one_stream_gives(folders, monkeypatch, graphs):
     from tie_amd.engine.replay import TraceReplayer
