@@ -61,6 +61,14 @@ class ModelRunner:
         self._recorded: Dict[Tuple, _RecordedStep] = {}
         self.graph_replays = 0
 
+    def __del__(self):
+        # A replay may still run (a step queued ahead that nobody read): it ends before its recording goes.
+        try:
+            if self._recorded:
+                torch.cuda.synchronize(self.device)
+        except Exception:          # the interpreter is shutting down, or the constructor failed early
+            pass
+
     def _forward(self, batch: StepBatch) -> Optional[torch.Tensor]:
         ctx = StepContext(batch, self.model.mode, self.device, self.workspace, self.cache, self.model.cache_plan)
         return self.model.forward(ctx)
