@@ -136,6 +136,35 @@ def test_a_router_weighted_over_the_chosen_alone(E, top):
     close(w, weights, 2e-6, "weights of far logits")
 
 
+@pytest.mark.parametrize("scoring,groups,keep,shared", [("softmax_chosen", 1, 1, 0), ("softmax", 3, 2, 0), ("sigmoid", 4, 2, 2)])
+@pytest.mark.parametrize("T,E,top", [(1, 12, 2), (8, 24, 3), (64, 252, 6), (17, 60, 4), (65, 12, 2)])
+def test_routing_and_sorting_in_one_launch(T, E, top, scoring, groups, keep, shared):
+    """Few rows go through one launch; the same choices, weights and sorted slots as through the two."""
+    from tie_amd import kernels
+
+    wide = rnd(T, E + 9, seed=E + T, scale=2.0).cuda()
+    logits = wide[:, 3:3 + E + (1 if shared else 0)]                   # columns of wider rows
+    bias, correction = rnd(E, seed=1).cuda(), rnd(E, seed=2, scale=0.1).cuda()
+    if scoring == "softmax_chosen":
+        correction = None
+    kw = dict(scoring=scoring, group_top=2, renormalize=scoring == "sigmoid", renorm_eps=1e-9, weight_scale=1.5,
+              shared=shared, bias=bias)
+    slots, real, tile = top + shared, E + shared, 16
+    ids, w = torch.full((T, slots), -7, dtype=torch.int32, device="cuda"), torch.zeros(T, slots, device="cuda")
+    kernels.moe_route(logits, correction, groups, keep, top, ids, w, **kw)
+    ids2, w2, get = torch.empty_like(ids), torch.empty_like(w), scratch_memory()
+    rows = kernels.moe_route_align(logits, correction, groups, keep, top, ids2, w2, real, tile, get, **kw)
+    assert torch.equal(ids, ids2) and torch.equal(w, w2)
+    where, slot_at, offsets = rows.where.cpu().view(-1), rows.slot_at.cpu(), rows.offsets.cpu()
+    flat = ids.cpu().view(-1)
+    assert sorted(where.tolist()) == list(range(T * slots)), "every slot has a place of its own"
+    assert all(int(slot_at[int(where[i])]) == i for i in range(T * slots))
+    assert all(int(offsets[flat[i]]) <= int(where[i]) < int(offsets[flat[i] + 1]) for i in range(T * slots))
+    counts = torch.bincount(flat.long(), minlength=real)
+    tiles = rows.tiles.cpu()[: int(rows.num_tiles)].tolist()
+    assert tiles == [[e, int(offsets[e]) + r] for e in range(real) for r in range(0, int(counts[e]), tile)]
+
+
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("T,E,top,F_,K", [(3, 4, 2, 24, 64), (70, 3, 2, 16, 40), (300, 5, 1, 72, 96), (700, 4, 3, 64, 128),
                                           (200, 2, 2, 9, 100)])
@@ -281,6 +310,38 @@ def test_heads_in_several_passes_where_the_chunks_memory_is_short(monkeypatch):
         assert torch.equal(out, results[0][0]) and torch.equal(state, results[0][1])
 
 
+@pytest.mark.parametrize("head_decay", [True, False])
+@pytest.mark.parametrize("lens", [[300], [1, 130, 2, 40, 16, 15, 1, 64], [127, 129]])
+@pytest.mark.parametrize("G,H,d,e,taps", [(2, 4, 8, 24, 3), (1, 1, 64, 16, 4), (2, 2, 100, 50, 2), (1, 2, 200, 300, 4), (1, 2, 16, 8, 6)])
+def test_what_the_delta_rule_takes_of_many_tokens(G, H, d, e, taps, lens, head_decay):
+    """Steps of many rows, sequences of which go on from a state; borders between sequences anywhere among the rows."""
+    from tie_amd import kernels
+
+    T, S, C, A = sum(lens), len(lens), 2 * G * d + H * e, H if head_decay else H * d
+    u, a, past = rnd(T, C + H + 3, seed=1), rnd(T, A, seed=2, scale=2.0), rnd(S + 2, taps - 1, C, seed=6)
+    w, A_log, dt = rnd(C, taps, seed=3, scale=0.5), rnd(H, seed=4), rnd(A, seed=5)
+    slots = torch.randperm(S + 2, generator=torch.Generator().manual_seed(2))[:S].tolist()
+    starts = [sum(lens[:i]) for i in range(S + 1)]
+    conv = [plain.short_convolution(torch.cat([past[slots[s]], u[starts[s]:starts[s + 1], :C]]).to(F64), w.to(F64))[taps - 1:]
+            for s in range(S)]
+    y = torch.nn.functional.silu(torch.cat(conv))
+    q = plain.unit(y[:, :G * d].view(T, G, d)) * d ** -0.5
+    k = plain.unit(y[:, G * d:2 * G * d].view(T, G, d))
+    log_g = -torch.exp(A_log.to(F64)).repeat_interleave(A // H) * torch.nn.functional.softplus(a.to(F64) + dt.to(F64))
+    want = [q.view(T, -1), k.view(T, -1), y[:, 2 * G * d:], torch.exp(log_g), torch.sigmoid(u[:, C:C + H].to(F64))]
+    if head_decay:
+        want.append(log_g)
+    batch = SimpleNamespace(num_seqs=S, query_start=i32(starts), state_slots=i32(slots),
+                            seq_of_row=i32([s for s, n in enumerate(lens) for _ in range(n)]))
+    tok = torch.full((T, kernels.delta_row(G, H, d, e, head_decay)), float("nan"), device="cuda")
+    kernels.delta_prepare(u.cuda(), w.cuda(), taps, past.cuda(), batch, a.cuda(), A_log.cuda(), dt.cuda(), G, H, d, e, tok,
+                          head_decay=head_decay)
+    at = 0
+    for name, part in zip(("q", "k", "v", "decay", "beta", "log decay"), want):
+        close(tok[:, at:at + part.shape[1]], part, 5e-6, name)
+        at += part.shape[1]
+
+
 @pytest.mark.parametrize("G,H,d,e,taps", [(2, 4, 8, 24, 3), (1, 1, 64, 16, 4), (3, 3, 20, 9, 1), (1, 4, 128, 128, 8)])
 def test_what_the_delta_rule_takes_of_a_token(G, H, d, e, taps):
     """Convolution, silu, unit vectors, beta, decays and their logarithms, over steps shorter than the taps."""
@@ -307,6 +368,19 @@ def test_what_the_delta_rule_takes_of_a_token(G, H, d, e, taps):
             kernels.conv_state_update(ud, taps, state, batch, C)
         got.append(tok[:, :C + 3 * H].cpu())
         at += n
+    if taps > 1:         # single rows of two sequences: the kernel brings the convolutions' states up to date itself
+        twin = state.clone()
+        for n in range(3):
+            ud = rnd(2, C + H, seed=20 + n).cuda()
+            batch = SimpleNamespace(num_seqs=2, query_start=i32([0, 1, 2]), state_slots=i32([2, 1]), seq_of_row=i32([0, 1]))
+            rows = []
+            for shift, st in ((True, state), (False, twin)):
+                tok = torch.zeros(2, kernels.delta_row(G, H, d, e, True), device="cuda")
+                kernels.delta_prepare(ud, w.cuda(), taps, st, batch, a[:2].cuda(), A_log.cuda(), dt.cuda(), G, H, d, e, tok,
+                                      head_decay=True, shift_state=shift)
+                rows.append(tok)
+            kernels.conv_state_update(ud, taps, twin, batch, C)
+            assert torch.equal(state, twin) and torch.equal(rows[0], rows[1])
     got = torch.cat(got)
     for name, lo, hi in (("q", 0, G * d), ("k", G * d, 2 * G * d), ("v", 2 * G * d, C), ("decay", C, C + H),
                          ("beta", C + H, C + 2 * H), ("log decay", C + 2 * H, C + 3 * H)):

@@ -18,6 +18,22 @@ __device__ __forceinline__ float silu_f(float x) { return x / (1.0f + expf(-x));
 __device__ __forceinline__ float sigmoid_f(float x) { return 1.0f / (1.0f + expf(-x)); }
 __device__ __forceinline__ float softplus_f(float x) { return x > 20.f ? x : log1pf(expf(x)); }
 
+// The same for a sequence's only row of a step, whose channel c no other thread reads: the state takes the row's input.
+__device__ __forceinline__ float conv_and_shift(float u, const float* __restrict__ w, float* hist, int taps, int C, int c) {
+  float past[CONV_MAX_TAPS - 1];
+#pragma unroll
+  for (int j = 0; j < CONV_MAX_TAPS - 1; ++j)
+    if (j < taps - 1) past[j] = hist[static_cast<size_t>(j) * C + c];
+  float y = 0.f;
+#pragma unroll
+  for (int j = 0; j < CONV_MAX_TAPS - 1; ++j)
+    if (j < taps - 1) y = fmaf(w[c * taps + j], past[j], y);
+#pragma unroll
+  for (int j = 0; j < CONV_MAX_TAPS - 1; ++j)
+    if (j < taps - 1) hist[static_cast<size_t>(j) * C + c] = j + 1 < taps - 1 ? past[j + 1 < CONV_MAX_TAPS - 1 ? j + 1 : j] : u;
+  return fmaf(w[c * taps + taps - 1], u, y);
+}
+
 // The convolution's sum for row t (of the sequence that starts at row `start`), channel c of the C convolved
 // columns, whose inputs are columns of `u` rows `row` apart.
 __device__ __forceinline__ float conv_at(const float* __restrict__ u, size_t row, const float* __restrict__ w,
@@ -131,8 +147,11 @@ extern "C" int tie_conv_state_update(const float* u, int row, int taps, float* s
 // g (H da) | beta (H)] and, with one decay a head, the decays' logarithms (H) behind:
 //   q^, k^ unit vectors per head (x / sqrt(sum x^2 + 1e-6)), q^ also times d^(-1/2); beta = sigmoid(b);
 //   g = exp(-exp(A_log[head]) * softplus(a + dt_bias)).
+// SHIFT: every sequence has one row, and the convolution's state is brought up to date here (`shifted` is the state;
+// otherwise `state`, which is only read).
+template <bool SHIFT>
 __global__ void delta_prepare_kernel(const float* __restrict__ u, int row, const float* __restrict__ w, int taps,
-                                     const float* __restrict__ state, const int* __restrict__ state_slots,
+                                     const float* __restrict__ state, float* shifted, const int* __restrict__ state_slots,
                                      const int* __restrict__ seq_of_row, const int* __restrict__ query_start,
                                      const float* __restrict__ a, int a_row, const float* __restrict__ A_log,
                                      const float* __restrict__ dt_bias, int G, int H, int d, int e, int da,
@@ -142,7 +161,7 @@ __global__ void delta_prepare_kernel(const float* __restrict__ u, int row, const
   const int s = seq_of_row[t];
   const int start = query_start[s];
   const int C = 2 * G * d + H * e;
-  const float* hist = state + static_cast<size_t>(state_slots[s]) * (taps - 1) * C;
+  const size_t slot_at = static_cast<size_t>(state_slots[s]) * (taps - 1) * C;
   float* o = out + static_cast<size_t>(t) * out_row;
   // three workgroups a row: q and k with their unit norms, v, and beta with the decays
   if (blockIdx.y == 2) {
@@ -158,8 +177,9 @@ __global__ void delta_prepare_kernel(const float* __restrict__ u, int row, const
   }
   const int lo = blockIdx.y == 0 ? 0 : 2 * G * d, hi = blockIdx.y == 0 ? 2 * G * d : C;
   for (int c = lo + threadIdx.x; c < hi; c += blockDim.x) {
-    const float y = taps > 1 ? conv_at(u, row, w, hist, taps, C, t, start, c)
-                             : w[c] * u[static_cast<size_t>(t) * row + c];
+    const float y = taps == 1 ? w[c] * u[static_cast<size_t>(t) * row + c]
+                    : SHIFT   ? conv_and_shift(u[static_cast<size_t>(t) * row + c], w, shifted + slot_at, taps, C, c)
+                              : conv_at(u, row, w, state + slot_at, taps, C, t, start, c);
     if (blockIdx.y == 0) vals[c] = silu_f(y);
     else o[c] = silu_f(y);
   }
@@ -177,7 +197,99 @@ __global__ void delta_prepare_kernel(const float* __restrict__ u, int row, const
   }
 }
 
-extern "C" int tie_delta_prepare(const float* u, int row, const float* w, int taps, const float* state,
+// The same for many rows: a wave takes the channels of one q or k head, or 64 PER channels of v, and walks
+// DELTA_WALK_ROWS rows with the convolution's window in registers, so that an input is read once instead of once a tap;
+// lane l holds channels l, l + 64, ... A unit behind the last one makes beta and the decays.
+#define DELTA_WALK_ROWS 16
+#define DELTA_WALK_WAVES 4
+
+template <int PER, int TAPS>
+__global__ __launch_bounds__(DELTA_WALK_WAVES* TIE_WAVE) void delta_prepare_walk_kernel(
+    const float* __restrict__ u, int row, const float* __restrict__ w, const float* __restrict__ state,
+    const int* __restrict__ state_slots, const int* __restrict__ seq_of_row, const int* __restrict__ query_start,
+    const float* __restrict__ a, int a_row, const float* __restrict__ A_log, const float* __restrict__ dt_bias, int T,
+    int G, int H, int d, int e, int da, float* __restrict__ out, int out_row, int units) {
+  const int unit = blockIdx.x * DELTA_WALK_WAVES + threadIdx.x / TIE_WAVE, lane = threadIdx.x % TIE_WAVE;
+  if (unit >= units) return;                       // the whole wave; there is no barrier below
+  const int first = blockIdx.y * DELTA_WALK_ROWS, rows = min(DELTA_WALK_ROWS, T - first);
+  const int C = 2 * G * d + H * e;
+  if (unit == units - 1) {
+    const int width = H * da;
+    for (int i = lane; i < rows * width; i += TIE_WAVE) {
+      const int t = first + i / width, c = i % width;
+      float* o = out + static_cast<size_t>(t) * out_row;
+      const float log_g = -expf(A_log[c / da]) * softplus_f(a[static_cast<size_t>(t) * a_row + c] + dt_bias[c]);
+      o[C + c] = expf(log_g);
+      if (da == 1) o[C + 2 * H + c] = log_g;
+    }
+    for (int i = lane; i < rows * H; i += TIE_WAVE) {
+      const int t = first + i / H, h = i % H;
+      out[static_cast<size_t>(t) * out_row + C + H * da + h] = sigmoid_f(u[static_cast<size_t>(t) * row + C + h]);
+    }
+    return;
+  }
+  const bool head = unit < 2 * G;                  // a q or k head: a unit vector
+  const int c0 = head ? unit * d : 2 * G * d + (unit - 2 * G) * TIE_WAVE * PER;
+  const int width = head ? d : min(TIE_WAVE * PER, C - c0);
+  const float scale = unit < G ? 1.0f / sqrtf(static_cast<float>(d)) : 1.0f;
+  int ch[PER];
+  float wt[TAPS][PER], win[TAPS][PER];             // win: the inputs of rows t - TAPS + 1 .. t
+#pragma unroll
+  for (int p = 0; p < PER; ++p) {
+    ch[p] = c0 + min(lane + p * TIE_WAVE, width - 1);
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) wt[j][p] = w[ch[p] * TAPS + j];
+  }
+  int start = 0, left = 0;                         // the first row of t's sequence, rows left in it
+  constexpr int AHEAD = 4;                         // rows asked for before they are needed
+  float ahead[AHEAD][PER];
+#pragma unroll
+  for (int r = 0; r < AHEAD; ++r)
+#pragma unroll
+    for (int p = 0; p < PER; ++p) ahead[r][p] = u[static_cast<size_t>(first + min(r, rows - 1)) * row + ch[p]];
+  for (int r = 0; r < rows; ++r) {
+    const int t = first + r;
+    if (left == 0) {                               // a sequence begins here, or this wave's rows do
+      const int s = seq_of_row[t];
+      start = query_start[s];
+      left = query_start[s + 1] - t;
+      const float* hist = state + static_cast<size_t>(state_slots[s]) * (TAPS - 1) * C;
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) {
+        const int src = t - (TAPS - 1) + j;
+        const float* from = src >= start ? u + static_cast<size_t>(src) * row
+                                         : hist + static_cast<size_t>(src - start + TAPS - 1) * C;
+#pragma unroll
+        for (int p = 0; p < PER; ++p) win[j][p] = from[ch[p]];
+      }
+    }
+    --left;
+    float y[PER], ss = 0.f;
+#pragma unroll
+    for (int p = 0; p < PER; ++p) {
+      win[TAPS - 1][p] = ahead[0][p];
+#pragma unroll
+      for (int j = 0; j + 1 < AHEAD; ++j) ahead[j][p] = ahead[j + 1][p];
+      ahead[AHEAD - 1][p] = u[static_cast<size_t>(first + min(r + AHEAD, rows - 1)) * row + ch[p]];
+      float v = 0.f;
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) v = fmaf(wt[j][p], win[j][p], v);
+      y[p] = silu_f(v);
+      if (lane + p * TIE_WAVE < width) ss = fmaf(y[p], y[p], ss);
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) win[j][p] = win[j + 1][p];
+    }
+    const float f = head ? 1.0f / sqrtf(wave_sum(ss) + 1e-6f) * scale : 1.0f;
+    float* o = out + static_cast<size_t>(t) * out_row;
+#pragma unroll
+    for (int p = 0; p < PER; ++p)
+      if (lane + p * TIE_WAVE < width) o[ch[p]] = y[p] * f;
+  }
+}
+
+#define DELTA_WALK_FROM 128       // rows of a step from which the walk runs
+
+extern "C" int tie_delta_prepare(const float* u, int row, const float* w, int taps, float* state, int shift,
                                  const int* state_slots, const int* seq_of_row, const int* query_start,
                                  const float* a, int a_row, const float* A_log, const float* dt_bias, int T, int G,
                                  int H, int d, int e, int head_decay, float* out, int out_row, hipStream_t stream) {
@@ -186,10 +298,33 @@ extern "C" int tie_delta_prepare(const float* u, int row, const float* w, int ta
   if (T <= 0 || G <= 0 || H <= 0 || d <= 0 || e <= 0 || taps < 1 || taps > CONV_MAX_TAPS || row < C + H ||
       out_row < C + H + (head_decay ? 2 * H : H * d) || a_row < H * da || static_cast<size_t>(C) * 4 > 65536 || (taps > 1 && !state))
     return TIE_BAD_ARGUMENT;
+  if (T >= DELTA_WALK_FROM && !shift && taps >= 2 && taps <= 4 && d <= 4 * TIE_WAVE) {
+    const int per = d <= TIE_WAVE ? 1 : (d <= 2 * TIE_WAVE ? 2 : 4);
+    const int units = 2 * G + (H * e + TIE_WAVE * per - 1) / (TIE_WAVE * per) + 1;
+    const dim3 grid((units + DELTA_WALK_WAVES - 1) / DELTA_WALK_WAVES, (T + DELTA_WALK_ROWS - 1) / DELTA_WALK_ROWS);
+#define WALK(PER, TAPS)                                                                                            \
+  delta_prepare_walk_kernel<PER, TAPS><<<grid, DELTA_WALK_WAVES * TIE_WAVE, 0, stream>>>(                           \
+      u, row, w, state, state_slots, seq_of_row, query_start, a, a_row, A_log, dt_bias, T, G, H, d, e, da, out, out_row, \
+      units)
+#define WALKS(PER)                                                                             \
+  {                                                                                            \
+    if (taps == 2) WALK(PER, 2); else if (taps == 3) WALK(PER, 3); else WALK(PER, 4);          \
+  }
+    if (per == 1) WALKS(1) else if (per == 2) WALKS(2) else WALKS(4)
+#undef WALKS
+#undef WALK
+    return tie_launch_status();
+  }
   const int threads = C >= 2048 ? 1024 : (C >= 1024 ? 512 : 256);
-  delta_prepare_kernel<<<dim3(T, 3), threads, static_cast<size_t>(C) * sizeof(float), stream>>>(
-      u, row, w, taps, state, state_slots, seq_of_row, query_start, a, a_row, A_log, dt_bias, G, H, d, e, da, out,
-      out_row);
+  const size_t lds = static_cast<size_t>(C) * sizeof(float);
+  if (shift && taps > 1)
+    delta_prepare_kernel<true><<<dim3(T, 3), threads, lds, stream>>>(u, row, w, taps, nullptr, state, state_slots,
+                                                                     seq_of_row, query_start, a, a_row, A_log, dt_bias,
+                                                                     G, H, d, e, da, out, out_row);
+  else
+    delta_prepare_kernel<false><<<dim3(T, 3), threads, lds, stream>>>(u, row, w, taps, state, nullptr, state_slots,
+                                                                      seq_of_row, query_start, a, a_row, A_log, dt_bias,
+                                                                      G, H, d, e, da, out, out_row);
   return tie_launch_status();
 }
 

@@ -50,19 +50,35 @@ __device__ __forceinline__ void wave_argmax(float& v, int& i) {   // ties: the l
 #define SCORE_SIGMOID 1
 #define SCORE_LOGIT 2        // chosen by the logits, weighted by the softmax over the chosen ones
 
-__global__ __launch_bounds__(TIE_WAVE) void moe_route_kernel(const float* __restrict__ logits, int row,
-                                                             const float* __restrict__ bias,
-                                                             const float* __restrict__ correction, int E, int groups,
-                                                             int keep, int top, int scoring, int group_top,
-                                                             int renormalize, float renorm_eps, float weight_scale,
-                                                             int shared, int* __restrict__ ids,
-                                                             float* __restrict__ weights) {
-  extern __shared__ float lds[];
+struct RouteParams {
+  const float* logits;     // rows `row` apart
+  int row;
+  const float* bias;       // [E] or null
+  const float* correction; // [E] or null
+  int E, groups, keep, top, scoring, group_top, renormalize;
+  float renorm_eps, weight_scale;
+  int shared;
+  int* ids;                // [T][top + shared]
+  float* weights;          // [T][top + shared]
+};
+
+// Between a wave's writes to its LDS and its reads: its LDS instructions run in order, the compiler must keep it.
+__device__ __forceinline__ void wave_order() {
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+}
+
+// One row by one wave, whose LDS holds 2 E + groups floats; the choice also goes to ids_lds where that is given.
+__device__ void route_row(const RouteParams& p, float* lds, size_t t, int lane, int* ids_lds) {
+  const float *logits = p.logits, *bias = p.bias, *correction = p.correction;
+  const int row = p.row, E = p.E, groups = p.groups, keep = p.keep, top = p.top, scoring = p.scoring;
+  const int group_top = p.group_top, renormalize = p.renormalize, shared = p.shared;
+  const float renorm_eps = p.renorm_eps, weight_scale = p.weight_scale;
+  int* ids = p.ids;
+  float* weights = p.weights;
   float* score = lds;              // [E]
   float* choice = score + E;       // [E]
   float* group_score = choice + E; // [groups]
-  const int lane = threadIdx.x;
-  const size_t t = blockIdx.x;
   const float* z = logits + t * row;
   auto logit = [&](int e) { return bias != nullptr ? z[e] + bias[e] : z[e]; };
   const int slots = top + shared;          // of a row: the chosen, then the experts every row uses
@@ -90,7 +106,7 @@ __global__ __launch_bounds__(TIE_WAVE) void moe_route_kernel(const float* __rest
       choice[e] = s + (correction != nullptr ? correction[e] : 0.f);
     }
   }
-  __syncthreads();
+  wave_order();
   const int size = E / groups;
   if (groups > 1 && keep < groups) {
     for (int g = lane; g < groups; g += TIE_WAVE) {
@@ -114,7 +130,7 @@ __global__ __launch_bounds__(TIE_WAVE) void moe_route_kernel(const float* __rest
       }
       group_score[g] = total;
     }
-    __syncthreads();
+    wave_order();
     // the `keep` best groups get +inf as their mark, one at a time
     for (int k = 0; k < keep; ++k) {
       float bv = -INFINITY;
@@ -128,11 +144,11 @@ __global__ __launch_bounds__(TIE_WAVE) void moe_route_kernel(const float* __rest
       }
       wave_argmax(bv, bi);
       if (lane == 0 && bi < groups) group_score[bi] = INFINITY;
-      __syncthreads();
+      wave_order();
     }
     for (int e = lane; e < E; e += TIE_WAVE)
       if (group_score[e / size] != INFINITY) choice[e] = -INFINITY;
-    __syncthreads();
+    wave_order();
   }
   for (int k = 0; k < top; ++k) {
     float bv = -INFINITY;
@@ -148,10 +164,11 @@ __global__ __launch_bounds__(TIE_WAVE) void moe_route_kernel(const float* __rest
     if (bi >= E) bi = 0;               // fewer eligible experts than `top`: a configuration's fault, not a fault here
     if (lane == 0) {
       ids[t * slots + k] = bi;
+      if (ids_lds != nullptr) ids_lds[t * slots + k] = bi;
       weights[t * slots + k] = bv == -INFINITY ? (scoring == SCORE_LOGIT ? -INFINITY : 0.f) : score[bi];
       choice[bi] = -INFINITY;
     }
-    __syncthreads();
+    wave_order();
   }
   if (lane == 0) {
     float* w = weights + t * slots;
@@ -175,10 +192,16 @@ __global__ __launch_bounds__(TIE_WAVE) void moe_route_kernel(const float* __rest
       const float g = 1.0f / (1.0f + expf(-z[E]));
       for (int k = 0; k < shared; ++k) {
         ids[t * slots + top + k] = E + k;
+        if (ids_lds != nullptr) ids_lds[t * slots + top + k] = E + k;
         w[top + k] = g;
       }
     }
   }
+}
+
+__global__ __launch_bounds__(TIE_WAVE) void moe_route_kernel(RouteParams p) {
+  extern __shared__ float lds[];
+  route_row(p, lds, blockIdx.x, threadIdx.x, nullptr);
 }
 
 // logits [T][row] float32 with row >= E (+ 1 with shared slots: column E is the gate of the experts every row uses);
@@ -191,22 +214,26 @@ extern "C" int tie_moe_route(const float* logits, int row, const float* bias, co
       row < E + (shared > 0 ? 1 : 0) || scoring < SCORE_SOFTMAX || scoring > SCORE_LOGIT)
     return TIE_BAD_ARGUMENT;
   const size_t lds = sizeof(float) * (2 * static_cast<size_t>(E) + groups);
-  moe_route_kernel<<<T, TIE_WAVE, lds, stream>>>(logits, row, bias, correction, E, groups, keep, top, scoring,
-                                                 group_top, renormalize, renorm_eps, weight_scale, shared, ids,
-                                                 weights);
+  moe_route_kernel<<<T, TIE_WAVE, lds, stream>>>(RouteParams{logits, row, bias, correction, E, groups, keep, top, scoring,
+                                                             group_top, renormalize, renorm_eps, weight_scale, shared,
+                                                             ids, weights});
   return tie_launch_status();
 }
 
 // ------------------------------------------------------------------ align
 #define ALIGN_THREADS 1024
 
-__global__ __launch_bounds__(ALIGN_THREADS) void moe_align_kernel(const int* __restrict__ ids, int slots, int real,
-                                                                  int tile_rows, int* __restrict__ offsets,
-                                                                  int* __restrict__ slot_at, int* __restrict__ where,
-                                                                  int* __restrict__ tiles, int max_tiles,
-                                                                  int* __restrict__ num_tiles) {
-  __shared__ int count[MOE_MAX_EXPERTS];
-  __shared__ int cursor[MOE_MAX_EXPERTS];
+struct AlignOut {
+  int* offsets;
+  int* slot_at;
+  int* where;
+  int* tiles;
+  int max_tiles;
+  int* num_tiles;
+};
+
+// The whole workgroup; `count` and `cursor` are LDS of `real` integers each, ids may lie anywhere.
+__device__ void align_slots(const int* ids, int slots, int real, int tile_rows, int* count, int* cursor, AlignOut o) {
   const int tid = threadIdx.x;
   for (int e = tid; e < real; e += ALIGN_THREADS) count[e] = 0;
   __syncthreads();
@@ -218,28 +245,53 @@ __global__ __launch_bounds__(ALIGN_THREADS) void moe_align_kernel(const int* __r
   if (tid == 0) {
     int at = 0, n = 0;
     for (int e = 0; e < real; ++e) {
-      offsets[e] = at;
+      o.offsets[e] = at;
       cursor[e] = at;
-      for (int r = 0; r < count[e] && n < max_tiles; r += tile_rows, ++n) {
-        tiles[2 * n] = e;
-        tiles[2 * n + 1] = at + r;
+      for (int r = 0; r < count[e] && n < o.max_tiles; r += tile_rows, ++n) {
+        o.tiles[2 * n] = e;
+        o.tiles[2 * n + 1] = at + r;
       }
       at += count[e];
     }
-    offsets[real] = at;
-    *num_tiles = n;
+    o.offsets[real] = at;
+    *o.num_tiles = n;
   }
   __syncthreads();
   for (int s = tid; s < slots; s += ALIGN_THREADS) {
     const int e = ids[s];
     if (e >= 0 && e < real) {
       const int place = atomicAdd(&cursor[e], 1);
-      slot_at[place] = s;
-      where[s] = place;
+      o.slot_at[place] = s;
+      o.where[s] = place;
     } else {
-      where[s] = -1;
+      o.where[s] = -1;
     }
   }
+}
+
+__global__ __launch_bounds__(ALIGN_THREADS) void moe_align_kernel(const int* __restrict__ ids, int slots, int real,
+                                                                  int tile_rows, AlignOut o) {
+  __shared__ int count[MOE_MAX_EXPERTS];
+  __shared__ int cursor[MOE_MAX_EXPERTS];
+  align_slots(ids, slots, real, tile_rows, count, cursor, o);
+}
+
+// Both for a step of few rows, in one workgroup: a wave a row at a time, then the sort over the choices in LDS.
+#define MOE_FEW_ROWS 64
+#define MOE_FEW_EXPERTS 256
+#define MOE_FEW_SLOTS 1024
+
+__global__ __launch_bounds__(ALIGN_THREADS) void moe_route_align_kernel(RouteParams p, int T, int real, int tile_rows,
+                                                                        AlignOut o) {
+  extern __shared__ float lds[];                       // 2 E + groups floats a wave
+  __shared__ int ids[MOE_FEW_SLOTS];
+  __shared__ int count[MOE_FEW_EXPERTS + MOE_MAX_GROUP_TOP];
+  __shared__ int cursor[MOE_FEW_EXPERTS + MOE_MAX_GROUP_TOP];
+  const int wave = threadIdx.x / TIE_WAVE, lane = threadIdx.x % TIE_WAVE;
+  for (int t = wave; t < T; t += ALIGN_THREADS / TIE_WAVE)
+    route_row(p, lds + wave * (2 * p.E + p.groups), t, lane, ids);
+  __syncthreads();
+  align_slots(ids, T * (p.top + p.shared), real, tile_rows, count, cursor, o);
 }
 
 // The most row tiles `slots` slots over `real` experts can make: every expert's last tile may be ragged.
@@ -253,8 +305,28 @@ extern "C" int tie_moe_align(const int* ids, int slots, int real, int tile_rows,
   if (slots <= 0 || real <= 0 || real > MOE_MAX_EXPERTS || tile_rows <= 0 ||
       max_tiles < tie_moe_max_tiles(slots, real, tile_rows))
     return TIE_BAD_ARGUMENT;
-  moe_align_kernel<<<1, ALIGN_THREADS, 0, stream>>>(ids, slots, real, tile_rows, offsets, slot_at, where, tiles,
-                                                    max_tiles, num_tiles);
+  moe_align_kernel<<<1, ALIGN_THREADS, 0, stream>>>(ids, slots, real, tile_rows,
+                                                    AlignOut{offsets, slot_at, where, tiles, max_tiles, num_tiles});
+  return tie_launch_status();
+}
+
+// tie_moe_route and tie_moe_align in one launch: T <= 64, E <= 256, T (top + shared) <= 1024.
+extern "C" int tie_moe_route_align(const float* logits, int row, const float* bias, const float* correction, int T, int E,
+                                   int groups, int keep, int top, int scoring, int group_top, int renormalize,
+                                   float renorm_eps, float weight_scale, int shared, int* ids, float* weights, int real,
+                                   int tile_rows, int* offsets, int* slot_at, int* where, int* tiles, int max_tiles,
+                                   int* num_tiles, hipStream_t stream) {
+  if (T <= 0 || T > MOE_FEW_ROWS || E <= 0 || E > MOE_FEW_EXPERTS || groups <= 0 || E % groups != 0 || keep <= 0 ||
+      keep > groups || top <= 0 || top > E || group_top <= 0 || group_top > MOE_MAX_GROUP_TOP || shared < 0 ||
+      row < E + (shared > 0 ? 1 : 0) || scoring < SCORE_SOFTMAX || scoring > SCORE_LOGIT ||
+      T * (top + shared) > MOE_FEW_SLOTS || real <= 0 || real > MOE_FEW_EXPERTS + MOE_MAX_GROUP_TOP || tile_rows <= 0 ||
+      max_tiles < tie_moe_max_tiles(T * (top + shared), real, tile_rows))
+    return TIE_BAD_ARGUMENT;
+  const size_t lds = sizeof(float) * (2 * static_cast<size_t>(E) + groups) * (ALIGN_THREADS / TIE_WAVE);
+  moe_route_align_kernel<<<1, ALIGN_THREADS, lds, stream>>>(
+      RouteParams{logits, row, bias, correction, E, groups, keep, top, scoring, group_top, renormalize, renorm_eps,
+                  weight_scale, shared, ids, weights},
+      T, real, tile_rows, AlignOut{offsets, slot_at, where, tiles, max_tiles, num_tiles});
   return tie_launch_status();
 }
 

@@ -114,6 +114,9 @@ _SIGNATURES = {
     "moe": {
         "tie_moe_route": [_c_void, _c_int, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
                           _c_int, _c_float, _c_float, _c_int, _c_void, _c_void, _c_void],
+        "tie_moe_route_align": [_c_void, _c_int, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
+                                _c_int, _c_float, _c_float, _c_int, _c_void, _c_void, _c_int, _c_int, _c_void, _c_void,
+                                _c_void, _c_void, _c_int, _c_void, _c_void],
         "tie_moe_max_tiles": [_c_int, _c_int, _c_int],
         "tie_moe_align": [_c_void, _c_int, _c_int, _c_int, _c_void, _c_void, _c_void, _c_void, _c_int, _c_void, _c_void],
         "tie_moe_generic_tile_rows": [],
@@ -154,7 +157,7 @@ _SIGNATURES = {
         "tie_conv_qkv": [_c_void, _c_int, _c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_int, _c_int, _c_int,
                          _c_int, _c_void, _c_void, _c_float, _c_float, _c_float, _c_void, _c_int, _c_void],
         "tie_conv_state_update": [_c_void, _c_int, _c_int, _c_void, _c_void, _c_void, _c_int, _c_int, _c_void],
-        "tie_delta_prepare": [_c_void, _c_int, _c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_void, _c_int,
+        "tie_delta_prepare": [_c_void, _c_int, _c_void, _c_int, _c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_int,
                               _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void, _c_int, _c_void],
         "tie_gated_delta_scan": [_c_void, _c_int, _c_void, _c_int, _c_void, _c_void, _c_void, _c_int, _c_int, _c_int,
                                  _c_int, _c_int, _c_int, _c_void],
@@ -1811,6 +1814,48 @@ MOE_MAX_GROUP_TOP = 8         # MOE_MAX_GROUP_TOP of csrc/moe.hip
 MOE_SCORINGS = {"softmax": 0, "sigmoid": 1, "softmax_chosen": 2}     # SCORE_* of csrc/moe.hip
 
 
+def _check_router(logits: torch.Tensor, top: int, shared: int):
+    _gpu_strided(logits, "router logits")
+    if logits.dtype != torch.float32:
+        raise InvalidArgument(f"router logits must be float32, got {logits.dtype}")
+    return logits.shape[0], logits.shape[1] - (1 if shared else 0), top + shared
+
+
+# Up to here one workgroup routes all rows of a step and sorts their slots in the same launch (MOE_FEW_* of csrc/moe.hip).
+MOE_FEW_ROWS, MOE_FEW_EXPERTS, MOE_FEW_SLOTS = 64, 256, 1024
+
+
+def moe_route_align(logits: torch.Tensor, correction: Optional[torch.Tensor], groups: int, keep: int, top: int,
+                    ids: torch.Tensor, weights: torch.Tensor, real: int, tile_rows: int, scratch, scoring: str = "softmax",
+                    group_top: int = 1, renormalize: bool = False, renorm_eps: float = 0.0, weight_scale: float = 1.0,
+                    shared: int = 0, bias: Optional[torch.Tensor] = None) -> "ExpertRows":
+    """``moe_route`` and then ``moe_align``; in steps of few rows as one launch."""
+    T, E, slots = _check_router(logits, top, shared)
+    few = T <= MOE_FEW_ROWS and E <= MOE_FEW_EXPERTS and T * slots <= MOE_FEW_SLOTS and \
+        0 < real <= MOE_FEW_EXPERTS + MOE_MAX_GROUP_TOP
+    if not few or T == 0:
+        moe_route(logits, correction, groups, keep, top, ids, weights, scoring, group_top, renormalize, renorm_eps,
+                  weight_scale, shared, bias)
+        return moe_align(ids, real, tile_rows, scratch)
+    if correction is not None:
+        _f32(correction, "the choice's correction", (E,))
+    if bias is not None:
+        _f32(bias, "the logits' bias", (E,))
+    _i32(ids, "chosen experts")
+    _f32(weights, "routing weights", (T, slots))
+    if tuple(ids.shape) != (T, slots) or scoring not in MOE_SCORINGS or groups <= 0 or E % groups or \
+            not 0 < keep <= groups or not 0 < top <= E or not 0 < group_top <= MOE_MAX_GROUP_TOP or shared < 0:
+        raise InvalidArgument(f"moe_route_align: {E} experts in {groups} groups scored by their {group_top} best, {keep} "
+                              f"kept, top {top}, scoring '{scoring}', chosen {list(ids.shape)}")
+    rows = _expert_rows(T, slots, real, tile_rows, scratch)
+    _call(_lib("moe").tie_moe_route_align, "moe_route_align", logits.data_ptr(), logits.stride(0), _ptr(bias),
+          _ptr(correction), T, E, groups, keep, top, MOE_SCORINGS[scoring], int(group_top), int(bool(renormalize)),
+          float(renorm_eps), float(weight_scale), int(shared), ids.data_ptr(), weights.data_ptr(), real, tile_rows,
+          rows.offsets.data_ptr(), rows.slot_at.data_ptr(), rows.where.data_ptr(), rows.tiles.data_ptr(),
+          rows.max_tiles, rows.num_tiles.data_ptr(), _stream())
+    return rows
+
+
 def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], groups: int, keep: int, top: int,
               ids: torch.Tensor, weights: torch.Tensor, scoring: str = "softmax", group_top: int = 1,
               renormalize: bool = False, renorm_eps: float = 0.0, weight_scale: float = 1.0, shared: int = 0,
@@ -1827,10 +1872,7 @@ def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], groups: 
     ``E .. E + n - 1`` (experts every row uses) with the weight ``sigmoid(logits[:, E])``. ``scoring``
     ``"softmax_chosen"``: ``s`` are the logits themselves and the weights the softmax over the chosen ones alone.
     """
-    _f32(logits, "router logits")
-    T, row = logits.shape
-    E = row - (1 if shared else 0)
-    slots = top + shared
+    T, E, slots = _check_router(logits, top, shared)
     if correction is not None:
         _f32(correction, "the choice's correction", (E,))
     _i32(ids, "chosen experts")
@@ -1845,7 +1887,9 @@ def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], groups: 
             not 0 < group_top <= MOE_MAX_GROUP_TOP or shared < 0:
         raise InvalidArgument(f"moe_route: {E} experts (at most {MOE_MAX_EXPERTS}) in {groups} groups scored by their "
                               f"{group_top} best, {keep} kept, top {top}")
-    _call(_lib("moe").tie_moe_route, "moe_route", logits.data_ptr(), row, _ptr(bias), _ptr(correction), T, E, groups,
+    if T == 0:
+        return
+    _call(_lib("moe").tie_moe_route, "moe_route", logits.data_ptr(), logits.stride(0), _ptr(bias), _ptr(correction), T, E, groups,
           keep, top, MOE_SCORINGS[scoring], int(group_top), int(bool(renormalize)), float(renorm_eps), float(weight_scale),
           int(shared), ids.data_ptr(), weights.data_ptr(), _stream())
 
@@ -1903,9 +1947,17 @@ def moe_align(ids: torch.Tensor, real: int, tile_rows: int, scratch) -> ExpertRo
     """
     _i32(ids, "chosen experts")
     T, top = ids.shape
-    slots = T * top
     if not 0 < real <= MOE_MAX_EXPERTS:
         raise InvalidArgument(f"moe_align takes 1 to {MOE_MAX_EXPERTS} experts, got {real}")
+    rows = _expert_rows(T, top, real, tile_rows, scratch)
+    _call(_lib("moe").tie_moe_align, "moe_align", ids.data_ptr(), rows.slots, real, tile_rows, rows.offsets.data_ptr(),
+          rows.slot_at.data_ptr(), rows.where.data_ptr(), rows.tiles.data_ptr(), rows.max_tiles,
+          rows.num_tiles.data_ptr(), _stream())
+    return rows
+
+
+def _expert_rows(T: int, top: int, real: int, tile_rows: int, scratch) -> "ExpertRows":
+    slots = T * top
     rows = ExpertRows()
     rows.slots, rows.top, rows.real, rows.tile_rows = slots, top, real, tile_rows
     rows.max_tiles = slots // tile_rows + min(real, slots)
@@ -1914,9 +1966,6 @@ def moe_align(ids: torch.Tensor, real: int, tile_rows: int, scratch) -> ExpertRo
     rows.where = scratch("moe.where", (T, top), torch.int32)
     rows.tiles = scratch("moe.tiles", (rows.max_tiles, 2), torch.int32)
     rows.num_tiles = scratch("moe.num_tiles", (1,), torch.int32)
-    _call(_lib("moe").tie_moe_align, "moe_align", ids.data_ptr(), slots, real, tile_rows, rows.offsets.data_ptr(),
-          rows.slot_at.data_ptr(), rows.where.data_ptr(), rows.tiles.data_ptr(), rows.max_tiles,
-          rows.num_tiles.data_ptr(), _stream())
     return rows
 
 
@@ -2271,14 +2320,15 @@ def delta_row(kv_heads: int, heads: int, key_dim: int, value_dim: int, head_deca
 
 def delta_prepare(u: torch.Tensor, weight: torch.Tensor, taps: int, state: Optional[torch.Tensor], batch,
                   a: torch.Tensor, A_log: torch.Tensor, dt_bias: torch.Tensor, kv_heads: int, heads: int, key_dim: int,
-                  value_dim: int, out: torch.Tensor, head_decay: bool = False) -> None:
+                  value_dim: int, out: torch.Tensor, head_decay: bool = False, shift_state: bool = False) -> None:
     """What the gated delta rule takes of every token, from the projections' float32 sums.
 
     ``u`` rows ``[q (G d) | k (G d) | v (H e) | b (H)]``: q, k, v through the short convolution and silu, q and k
     made unit vectors per head (q also times ``d ** -0.5``), ``beta = sigmoid(b)``; ``a`` rows ``[H d]``: the decays
     ``exp(-exp(A_log[head]) * softplus(a + dt_bias))``. ``out`` rows: ``[q | k | v | decay | beta]`` float32, of
     ``delta_row(...)`` columns. ``head_decay``: one decay a head (``a`` rows and ``dt_bias`` of ``[H]``); the decays'
-    logarithms follow ``beta``."""
+    logarithms follow ``beta``. ``shift_state`` (a step of one row a sequence): the convolution's state takes the rows'
+    inputs in the same launch, instead of ``conv_state_update`` behind it."""
     G, H, d, e = kv_heads, heads, key_dim, value_dim
     C = 2 * G * d + H * e
     decays = H if head_decay else H * d
@@ -2297,10 +2347,12 @@ def delta_prepare(u: torch.Tensor, weight: torch.Tensor, taps: int, state: Optio
         _f32(state, "convolution state")
         if tuple(state.shape[1:]) != (taps - 1, C):
             raise InvalidArgument(f"convolution state {list(state.shape)} does not fit {[taps - 1, C]} a slot")
+    if shift_state and T != batch.num_seqs:
+        raise InvalidArgument(f"a step of {T} rows for {batch.num_seqs} sequences cannot shift the states as it goes")
     if T == 0:
         return
     _call(_lib("delta_rule").tie_delta_prepare, "delta_prepare", u.data_ptr(), u.stride(0), weight.data_ptr(), taps,
-          _ptr(state), batch.state_slots.data_ptr(), batch.seq_of_row.data_ptr(), batch.query_start.data_ptr(),
+          _ptr(state), int(shift_state), batch.state_slots.data_ptr(), batch.seq_of_row.data_ptr(), batch.query_start.data_ptr(),
           a.data_ptr(), a.stride(0), A_log.data_ptr(), dt_bias.data_ptr(), T, G, H, d, e, int(head_decay),
           out.data_ptr(), out.stride(0), _stream())
 

@@ -161,6 +161,8 @@ class Model:
 
         for part in self._all_parts():
             part.load_all(fetch, mode, device)
+        for layer in self.layers:
+            layer.block.layer_loaded(layer)
         self.mode = mode
         self.device = device
         self._find_layers_alike()

@@ -121,6 +121,11 @@ class Part:
         for child in self.children():
             child.load_all(fetch, mode, device)
 
+    def first_product(self):
+        """The Linear of the first product the part forms from its input rows through ``StepContext.product``, if it has
+        one that a block may form together with another part's (``Block.join_first_products``)."""
+        return None
+
     def all_capturable(self) -> bool:
         return bool(self.capturable) and all(child.all_capturable() for child in self.children())
 
@@ -188,6 +193,7 @@ class StepContext:
         self._owed = None                  # (target, planes): target += planes[0] + planes[1] + ... is still to be done
         self._pending = None               # (target, linear, x): target += x @ linear.weight^T is still to be launched
         self._late = None                  # (key, run, payload): a block's last pass, left for the next block to merge
+        self._given: Dict[int, torch.Tensor] = {}   # id of a Linear -> its product's columns (give_product)
         self._row_scales: Dict[int, Any] = {}   # address of rows that lack their norm's 1 / rms -> kernels.RowScale
 
     @property
@@ -247,6 +253,20 @@ class StepContext:
             target, linear, x = self._pending
             self._pending = None
             linear.add_to(self, x, target)
+
+    # A block may form the first products of several parts over the same rows as one; a part then finds its columns here.
+    def give_product(self, linear, columns: torch.Tensor) -> None:
+        self._given[id(linear)] = columns
+
+    def product(self, linear, x: torch.Tensor, name: str) -> torch.Tensor:
+        """float32 ``x @ linear.weight^T``: the columns a block left for this product, or the product run now into the
+        scratch rows ``name``."""
+        given = self._given.pop(id(linear), None) if self._given else None
+        if given is not None:
+            return given
+        out = self.scratch(name, (x.shape[0], linear.total_out), torch.float32)
+        linear(x, out, ctx=self)
+        return out
 
     # Rows that a norm left without their 1 / rms (kernels.RowScale): the products formed from them apply it.
     def set_row_scale(self, rows: torch.Tensor, scale) -> None:
@@ -386,6 +406,9 @@ class Block(Part):
     ``parts.Linear`` with the step context, or asks ``ctx.row_scale_of`` itself), a norm that can may hand it the
     rows without their 1 / rms.
     """
+
+    def layer_loaded(self, layer) -> None:
+        """Called once when all parts of the layer hold their weights."""
 
     @staticmethod
     def normed(ctx: StepContext, norm, x: torch.Tensor, consumer=None) -> torch.Tensor:

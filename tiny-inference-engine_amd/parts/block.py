@@ -20,7 +20,8 @@ layers share), ``g = gelu_tanh(W_gate x) * e`` from the stream itself (no norm b
 ``parallel_residual`` runs both sub-layers side by side: with ``h = pre(x)``, one norm, ``x += scale * (mixer(h) +
 feed_forward(h))``. What a layer adds is left with the step and rides in the next layer's first pass over the stream,
 which adds the sub-layers' results (rows, planes of partial sums, a routed feed-forward's parts not yet combined) and
-norms the sum in one kernel. Neither sub-layer needs the other's result; with ``SIDE_BY_SIDE`` the feed-forward is
+norms the sum in one kernel. The first products of mixer and feed-forward (a router's) read the same rows and run as
+one, over their weights side by side. Neither sub-layer needs the other's result; with ``SIDE_BY_SIDE`` the feed-forward is
 launched on a second stream that forks behind the norm and joins before the results are added (in a recorded step: two
 branches of the graph). Parameters: ``hidden``, ``scale``.
 
@@ -200,6 +201,11 @@ class ParallelResidualBlock(Block):
         super().__init__(params)
         self.hidden = int(params["hidden"])
         self.scale = float(params.get("scale", 1.0))
+        self.first = None             # the sub-layers' first products as one Linear
+
+    def layer_loaded(self, layer) -> None:
+        linears = [part.first_product() for part in (layer.mixer, layer.feed_forward) if part is not None]
+        self.first = Linear.joined(linears) if len(linears) == 2 and None not in linears else None
 
     @classmethod
     def check_layer(cls, layer) -> None:
@@ -227,6 +233,15 @@ class ParallelResidualBlock(Block):
             h = norm.forward(ctx, x, results=left)
         else:
             h = self.normed(ctx, norm, x)
+        if self.first is not None:
+            both = ctx.scratch("block.first_products", (x.shape[0], self.first.total_out), torch.float32)
+            self.first(h, both, ctx=ctx)
+            at = 0
+            for part in (layer.mixer, layer.feed_forward):
+                linear = part.first_product()
+                ctx.give_product(linear, both[:, at:at + linear.total_out])
+                at += linear.total_out
+
         def run_mixer():
             return self._result(ctx, layer.mixer, lambda residual: layer.mixer.forward(ctx, h, cache, residual),
                                 "block.mixer_result")

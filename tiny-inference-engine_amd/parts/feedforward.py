@@ -282,20 +282,21 @@ class RoutedExperts(FeedForward):
         if packed is not None:        # the products then read these alone
             self.gate, (self.up, self.down) = None, packed
 
+    def first_product(self):
+        return self.router
+
     def forward(self, ctx: StepContext, h: torch.Tensor, residual: Optional[torch.Tensor]):
         T = h.shape[0]
         slots, real = self.top + self.shared_pieces, self.experts + self.shared_pieces
-        logits = ctx.scratch("moe.logits", (T, self.router.total_out), torch.float32)
-        self.router(h, logits, ctx=ctx)
+        logits = ctx.product(self.router, h, "moe.logits")
         ids = ctx.scratch("moe.ids", (T, slots), torch.int32)
         weights = ctx.scratch("moe.weights", (T, slots), torch.float32)
-        kernels.moe_route(logits, self.correction, self.groups, self.keep_groups, self.top, ids, weights,
-                          scoring=self.scoring, group_top=self.group_top, renormalize=self.renormalize,
-                          renorm_eps=self.renorm_eps, weight_scale=self.weight_scale, shared=self.shared_pieces,
-                          bias=self.router_bias)
         tile_rows = kernels.moe_tile_rows(h.dtype, self.up.dtype, self.hidden, self.intermediate, T * slots, real,
                                           packed=isinstance(self.up, kernels.PackedWeight))
-        rows = kernels.moe_align(ids, real, tile_rows, ctx.scratch)
+        rows = kernels.moe_route_align(logits, self.correction, self.groups, self.keep_groups, self.top, ids, weights, real,
+                                       tile_rows, ctx.scratch, scoring=self.scoring, group_top=self.group_top,
+                                       renormalize=self.renormalize, renorm_eps=self.renorm_eps,
+                                       weight_scale=self.weight_scale, shared=self.shared_pieces, bias=self.router_bias)
         act = ctx.scratch("moe.act", (T * slots, self.intermediate))
         kernels.moe_gate_up(h, self.gate, self.up, rows, act, clipped=self.clipped)
         parts = ctx.scratch("moe.parts", (T * slots, self.hidden), torch.float32)

@@ -94,6 +94,9 @@ class LatentAttention(Mixer):
     def children(self) -> List[Part]:
         return [self.position]
 
+    def first_product(self):
+        return self.inputs
+
     def cache_need(self):
         return PagedKV(1, self.cache_dim, self.window)
 
@@ -129,8 +132,7 @@ class LatentAttention(Mixer):
 
     def forward(self, ctx: StepContext, h: torch.Tensor, cache, residual: Optional[torch.Tensor]):
         T, H, D = h.shape[0], self.num_heads, self.cache_dim
-        proj = ctx.scratch("latent.proj", (T, self.inputs.total_out), torch.float32)
-        self.inputs(h, proj, ctx=ctx)
+        proj = ctx.product(self.inputs, h, "latent.proj")
         q_plain = ctx.scratch("latent.q_plain", (T, H * self.dim))
         q_latent = ctx.scratch("latent.q", (T, H * D))
         step = cache.step

@@ -65,6 +65,26 @@ class Linear:
             parts = [p.to(torch.float32) for p in parts]
         self.set_weight(torch.cat(parts, dim=0).contiguous())
 
+    @classmethod
+    def joined(cls, linears: Sequence["Linear"]) -> Optional["Linear"]:
+        """One projection whose columns are those of ``linears`` side by side, which give up their own weights; None
+        where they differ in input size or type, or one has a bias. Rows of zeros fill it up to a whole block of 16."""
+        weights = [l.weight for l in linears]
+        if any(l.bias is not None or l.weight is None for l in linears) or len({w.dtype for w in weights}) > 1 or \
+                len({l.in_features for l in linears}) > 1:
+            return None
+        rows = [w.unpacked() if isinstance(w, kernels.PackedWeight) else w for w in weights]
+        total = sum(w.shape[0] for w in rows)
+        fill = -total % 16
+        if fill:
+            rows.append(rows[0].new_zeros((fill, rows[0].shape[1])))
+        both = cls([n for l in linears for n in l.names] + (["(zeros)"] if fill else []),
+                   [o for l in linears for o in l.out_features] + ([fill] if fill else []), linears[0].in_features)
+        both.set_weight(torch.cat(rows, dim=0).contiguous())
+        for l in linears:
+            l.weight = None
+        return both
+
     def set_weight(self, w: torch.Tensor) -> None:
         """Keeps ``w`` (``[out, in]``), in the matrix cores' blocked layout where the bfloat16 products can read that."""
         self.weight = kernels.pack_weight(w) if kernels.packable(w) else w

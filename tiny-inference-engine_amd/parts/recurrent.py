@@ -216,6 +216,9 @@ class GatedDeltaRule(Mixer):
         self.out = Linear([n["o"]], [self.hidden], self.v_width)
         self.conv_weight = self.A_log = self.dt_bias = self.norm_weight = None
 
+    def first_product(self):
+        return self.inputs
+
     def cache_need(self):
         state = FixedState((self.heads, self.key_dim, self.value_dim))
         if self.taps > 1:
@@ -266,8 +269,7 @@ class GatedDeltaRule(Mixer):
     def forward(self, ctx: StepContext, h: torch.Tensor, cache, residual: Optional[torch.Tensor]):
         T = h.shape[0]
         state, conv_state = (cache[0], cache[1].state) if isinstance(cache, tuple) else (cache, None)
-        proj = ctx.scratch("delta_rule.proj", (T, self.inputs.total_out), torch.float32)
-        self.inputs(h, proj, ctx=ctx)
+        proj = ctx.product(self.inputs, h, "delta_rule.proj")
         columns, at = {}, self.channels + self.heads
         for key, width in self.direct:
             columns[key] = proj[:, at:at + width]
@@ -283,9 +285,10 @@ class GatedDeltaRule(Mixer):
                 at += width
         sizes = (self.kv_heads, self.heads, self.key_dim, self.value_dim)
         tok = ctx.scratch("delta_rule.tokens", (T, kernels.delta_row(*sizes, self.head_decay)), torch.float32)
+        shift = conv_state is not None and state.writes and ctx.batch.all_decode
         kernels.delta_prepare(proj, self.conv_weight, self.taps, conv_state, ctx.batch, columns["a"], self.A_log,
-                              self.dt_bias, *sizes, tok, head_decay=self.head_decay)
-        if conv_state is not None and state.writes:
+                              self.dt_bias, *sizes, tok, head_decay=self.head_decay, shift_state=shift)
+        if conv_state is not None and state.writes and not shift:
             kernels.conv_state_update(proj, self.taps, conv_state, ctx.batch, self.channels)
         o = ctx.scratch("delta_rule.o", (T, self.v_width), torch.float32)
         chunks = kernels.delta_chunks(ctx.batch, ctx.device, self.head_decay)
