@@ -21,6 +21,12 @@
 // B[slot][n = lane % 16] and receives C[4 (lane / 16) + r][lane % 16]. The four slots of instruction i of a block of 16
 // along K stand for its elements 4 slot + i: so four consecutive floats of a row feed four instructions, and an
 // accumulator block is the next product's B operand as it stands.
+//
+// What one launch leaves for the next lies in memory in blocks of 16 x 16 elements, 1 KB, in the order in which the reader's
+// lanes take them (four consecutive words a lane): a load or a store of a wave is then 1 KB of consecutive memory. A block
+// read as an A operand holds element (m, k) at word 4 (16 (k / 4) + m) + k % 4, a block in accumulator layout (read as a B
+// operand) element (k, n) at word 4 (16 (k / 4) + n) + k % 4. (Row-major, with 64 bytes of 16 rows a load, the states
+// kernel took 101 us of a 2048-token prompt of 16 heads.)
 #include "common.h"
 
 #define DC_ROWS 64                 // tokens of a chunk at most
@@ -63,23 +69,26 @@ struct DeltaChunks {
   int head0, heads;        // the heads of this launch
   int ep;                  // e rounded up to 16
   int D;                   // d rounded up as the chunks' memory is
-  float* u;                // [..][64][ep]: U0, then U
-  float* w;                // [..][64][D]
-  float* kt;               // [..][D][64]
-  float* p;                // [..][64][64]
-  float* decay;            // [..][64]: e^(b_i)
-  float* s0;               // [..][D][ep]
+  float* u;                // [ep / 16][4] blocks: U0, then U
+  float* w;                // [4][D / 16] blocks (A)
+  float* kt;               // [D / 16][4] blocks (A): K~ transposed
+  float* q;                // [4][D / 16] blocks (A): e^(b_i) q_i
+  float* p;                // [4][4] blocks (A), those above the diagonal unused
+  float* s0;               // [ep / 16][D / 16] blocks: the state before the chunk
+  float* decay;            // [1]: e^(b_end)
 };
 
 // WIDE: q and k of every head start on 16-byte addresses and d is a multiple of 4.
 template <bool WIDE>
 __global__ __launch_bounds__(DC_THREADS) void delta_chunk_prepare_kernel(DeltaChunks g) {
+  extern __shared__ __attribute__((aligned(16))) float keys[];             // [64][D + 4]: the chunk's keys
   __shared__ __attribute__((aligned(16))) float A[DC_ROWS * DC_AR];
   __shared__ __attribute__((aligned(16))) float inv[4][16 * DC_TR];        // (I + A_rr)^-1 of the diagonal blocks
   __shared__ double b[DC_ROWS];
   __shared__ __attribute__((aligned(16))) float beta[DC_ROWS];             // all three are 0 behind the chunk's end:
   __shared__ __attribute__((aligned(16))) float beta_eb[DC_ROWS];          // beta_i e^(b_i)
   __shared__ __attribute__((aligned(16))) float to_end[DC_ROWS];           // e^(b_end - b_i)
+  __shared__ float eb[DC_ROWS];                                            // e^(b_i)
   const int item = blockIdx.x / g.heads, head = g.head0 + blockIdx.x % g.heads;
   const int kv = head / (g.H / g.G);
   const int t0 = g.items[3 * item + 1], n = g.items[3 * item + 2] - t0;
@@ -98,39 +107,45 @@ __global__ __launch_bounds__(DC_THREADS) void delta_chunk_prepare_kernel(DeltaCh
       const double before = __shfl_up(sum, off, TIE_WAVE);
       if (lane >= off) sum += before;
     }
-    const float eb = expf(static_cast<float>(sum));
+    const float e_b = expf(static_cast<float>(sum));
     const double end = __shfl(sum, TIE_WAVE - 1, TIE_WAVE);
     b[lane] = sum;
     beta[lane] = bt;
-    beta_eb[lane] = bt * eb;
+    beta_eb[lane] = bt * e_b;
+    eb[lane] = e_b;
     to_end[lane] = lane < n ? expf(static_cast<float>(end - sum)) : 0.f;
-    g.decay[entry * DC_ROWS + lane] = eb;
+    if (lane == TIE_WAVE - 1) g.decay[entry] = e_b;
   }
+  const int kr = g.D + 4, quads = g.D / 4, blocks = g.D / 16;
+  for (int i = threadIdx.x; i < DC_ROWS * quads; i += DC_THREADS) {      // rows behind the chunk's end: the last one's
+    const int t = i / quads, c = (i % quads) * 4;
+    *reinterpret_cast<float4*>(keys + t * kr + c) =
+        dc_load4<WIDE>(rows + static_cast<size_t>(min(t, n - 1)) * g.row + k_at, c, g.d);
+  }
+  __syncthreads();
   // rows 16 tile .. of K K^T and Q K^T; which wave has the longest rows turns with the workgroup
   const int tile = (wave + blockIdx.x) & 3;
   dc_floatx4 kk[4], qk[4];
 #pragma unroll
   for (int nt = 0; nt < 4; ++nt) kk[nt] = qk[nt] = dc_floatx4{0.f, 0.f, 0.f, 0.f};
-  const float* own = rows + static_cast<size_t>(min(tile * 16 + r16, n - 1)) * g.row;
-  const float* key[4];
-#pragma unroll
-  for (int nt = 0; nt < 4; ++nt) key[nt] = rows + static_cast<size_t>(min(nt * 16 + r16, n - 1)) * g.row + k_at;
+  const float* own = rows + static_cast<size_t>(min(tile * 16 + r16, n - 1)) * g.row + q_at;
+  const float own_eb = eb[tile * 16 + r16];
+  float* qe = g.q + (entry * 4 + tile) * blocks * 256 + lane * 4;
 #pragma unroll 2
-  for (int k0 = 0; k0 < g.D; k0 += 16) {
-    const int i0 = k0 + quad * 4;
-    const float4 ka = dc_load4<WIDE>(own + k_at, i0, g.d), qa = dc_load4<WIDE>(own + q_at, i0, g.d);
-    float4 kb[4];
-#pragma unroll
-    for (int nt = 0; nt < 4; ++nt) kb[nt] = dc_load4<WIDE>(key[nt], i0, g.d);
+  for (int kb = 0; kb < blocks; ++kb) {
+    const int i0 = kb * 16 + quad * 4;
+    const float4 qa = dc_load4<WIDE>(own, i0, g.d);
+    const float4 ka = *reinterpret_cast<const float4*>(keys + (tile * 16 + r16) * kr + i0);
+    *reinterpret_cast<float4*>(qe + kb * 256) = make_float4(qa.x * own_eb, qa.y * own_eb, qa.z * own_eb, qa.w * own_eb);
 #pragma unroll
     for (int nt = 0; nt < 4; ++nt) {
       if (nt > tile) continue;
-      const dc_floatx4 kv4 = {kb[nt].x, kb[nt].y, kb[nt].z, kb[nt].w};
+      const float4 v = *reinterpret_cast<const float4*>(keys + (nt * 16 + r16) * kr + i0);
+      const dc_floatx4 kv4 = {v.x, v.y, v.z, v.w};
       kk[nt] = dc_mfma4(ka, kv4, kk[nt]);
       qk[nt] = dc_mfma4(qa, kv4, qk[nt]);
     }
   }
-  __syncthreads();
   float* pe = g.p + entry * DC_ROWS * DC_ROWS;
 #pragma unroll
   for (int nt = 0; nt < 4; ++nt) {
@@ -141,7 +156,7 @@ __global__ __launch_bounds__(DC_THREADS) void delta_chunk_prepare_kernel(DeltaCh
       const bool in = i < n && j <= i;
       const float f = in ? expf(static_cast<float>(b[i] - b[j])) : 0.f;
       A[i * DC_AR + j] = in && j < i ? beta[i] * f * kk[nt][r] : 0.f;
-      pe[i * DC_ROWS + j] = in ? f * qk[nt][r] : 0.f;
+      pe[(tile * 4 + nt) * 256 + (r16 / 4) * 64 + (quad * 4 + r) * 4 + r16 % 4] = in ? f * qk[nt][r] : 0.f;
     }
   }
   __syncthreads();
@@ -182,20 +197,22 @@ __global__ __launch_bounds__(DC_THREADS) void delta_chunk_prepare_kernel(DeltaCh
     const bool is_k = nt * 16 >= g.ep;
     const int c = nt * 16 - (is_k ? g.ep : 0) + r16;
     const bool live = c < (is_k ? g.d : g.e);
-    const float* src = rows + (is_k ? k_at : v_at) + (live ? c : 0);
+    const float* src = rows + v_at + (live ? c : 0);
     const float* factor = is_k ? beta_eb : beta;
     dc_floatx4 x[4];
 #pragma unroll
     for (int r = 0; r < 4; ++r)
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
-        x[r][i] = src[static_cast<size_t>(min(r * 16 + quad * 4 + i, n - 1)) * g.row];
+      for (int i = 0; i < 4; ++i) {
+        const int t = r * 16 + quad * 4 + i;
+        x[r][i] = is_k ? keys[t * kr + c] : src[static_cast<size_t>(min(t, n - 1)) * g.row];
+      }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       if (!live) x[r] = dc_floatx4{0.f, 0.f, 0.f, 0.f};
       if (is_k) {
         const float4 f = *reinterpret_cast<const float4*>(to_end + r * 16 + quad * 4);
-        *reinterpret_cast<float4*>(g.kt + (entry * g.D + c) * DC_ROWS + r * 16 + quad * 4) =
+        *reinterpret_cast<float4*>(g.kt + ((entry * blocks + c / 16) * 4 + r) * 256 + lane * 4) =
             make_float4(x[r][0] * f.x, x[r][1] * f.y, x[r][2] * f.z, x[r][3] * f.w);
       }
       const float4 f = *reinterpret_cast<const float4*>(factor + r * 16 + quad * 4);
@@ -207,12 +224,17 @@ __global__ __launch_bounds__(DC_THREADS) void delta_chunk_prepare_kernel(DeltaCh
       for (int s = 0; s < r; ++s) x[r] = dc_mfma4(off[r][s], x[s], x[r]);
       x[r] = dc_mfma4(diag[r], x[r], dc_floatx4{0.f, 0.f, 0.f, 0.f});
     }
-    float* dst = is_k ? g.w + entry * DC_ROWS * g.D + c : g.u + entry * DC_ROWS * g.ep + c;
-    const int step = is_k ? g.D : g.ep;
 #pragma unroll
-    for (int r = 0; r < 4; ++r)
+    for (int r = 0; r < 4; ++r) {
+      if (is_k) {
+        float* dst = g.w + ((entry * 4 + r) * blocks + c / 16) * 256 + (r16 / 4) * 64 + r16 % 4;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) dst[(r * 16 + quad * 4 + i) * step] = x[r][i];
+        for (int i = 0; i < 4; ++i) dst[(quad * 4 + i) * 4] = x[r][i];
+      } else {
+        *reinterpret_cast<float4*>(g.u + ((entry * (g.ep / 16) + nt) * 4 + r) * 256 + lane * 4) =
+            make_float4(x[r][0], x[r][1], x[r][2], x[r][3]);
+      }
+    }
   }
 }
 
@@ -221,26 +243,24 @@ template <int TD>
 struct DeltaChunkOperands {
   float4 w[4][TD];         // [row block of the chunk][block of the wave's key rows]
   float4 k[TD][4];         // [block of the wave's key rows][row block of the chunk]
-  float u0[4];
+  float4 u0;
   float decay;
 };
 
 template <int D, int TD>
-__device__ __forceinline__ void delta_chunk_fetch(const DeltaChunks& g, size_t entry, int wave, int r16, int quad, int col,
+__device__ __forceinline__ void delta_chunk_fetch(const DeltaChunks& g, size_t entry, int wave, int lane, int slab,
                                                   DeltaChunkOperands<TD>& o) {
-  const float* w = g.w + entry * DC_ROWS * D + wave * (D / 4) + quad * 4;
-  const float* kt = g.kt + (entry * D + wave * (D / 4)) * DC_ROWS + quad * 4;
-  const float* u = g.u + (entry * DC_ROWS + wave * 16 + quad * 4) * g.ep + col;
+  const float* w = g.w + (entry * 4 * (D / 16) + wave * TD) * 256 + lane * 4;
+  const float* kt = g.kt + (entry * (D / 16) + wave * TD) * 4 * 256 + lane * 4;
 #pragma unroll
   for (int m = 0; m < 4; ++m)
 #pragma unroll
     for (int t = 0; t < TD; ++t) {
-      o.w[m][t] = *reinterpret_cast<const float4*>(w + (m * 16 + r16) * D + t * 16);
-      o.k[t][m] = *reinterpret_cast<const float4*>(kt + (t * 16 + r16) * DC_ROWS + m * 16);
+      o.w[m][t] = *reinterpret_cast<const float4*>(w + (m * (D / 16) + t) * 256);
+      o.k[t][m] = *reinterpret_cast<const float4*>(kt + (t * 4 + m) * 256);
     }
-#pragma unroll
-  for (int r = 0; r < 4; ++r) o.u0[r] = u[r * g.ep];
-  o.decay = g.decay[entry * DC_ROWS + DC_ROWS - 1];
+  o.u0 = *reinterpret_cast<const float4*>(g.u + ((entry * (g.ep / 16) + slab) * 4 + wave) * 256 + lane * 4);
+  o.decay = g.decay[entry];
 }
 
 // The four waves share the key rows: wave w holds rows [w D / 4, (w + 1) D / 4) of the 16 columns of S in accumulator
@@ -274,17 +294,16 @@ __global__ __launch_bounds__(DC_THREADS, 1) void delta_chunk_states_kernel(Delta
   DeltaChunkOperands<TD> even, odd;
   auto step = [&](int c, DeltaChunkOperands<TD>& now, DeltaChunkOperands<TD>& next) {
     const size_t entry = static_cast<size_t>(c) * g.heads + local;
-    delta_chunk_fetch<D, TD>(g, static_cast<size_t>(min(c + 1, c1 - 1)) * g.heads + local, wave, r16, quad, col, next);
-    float* s0 = g.s0 + (entry * D + row0) * g.ep + col;
+    delta_chunk_fetch<D, TD>(g, static_cast<size_t>(min(c + 1, c1 - 1)) * g.heads + local, wave, lane, slab, next);
+    __builtin_amdgcn_sched_barrier(0);           // the loads stay ahead of the chunk's products
+    float* s0 = g.s0 + ((entry * (g.ep / 16) + slab) * (D / 16) + wave * TD) * 256 + lane * 4;
 #pragma unroll
-    for (int t = 0; t < TD; ++t)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) s0[(16 * t + r) * g.ep] = S[t][r];
+    for (int t = 0; t < TD; ++t) *reinterpret_cast<dc_floatx4*>(s0 + t * 256) = S[t];
     dc_floatx4 acc[4];                         // W S - U0, of the wave's key rows
 #pragma unroll
     for (int m = 0; m < 4; ++m) {
       const bool mine = m == wave;
-      acc[m] = dc_floatx4{mine ? -now.u0[0] : 0.f, mine ? -now.u0[1] : 0.f, mine ? -now.u0[2] : 0.f, mine ? -now.u0[3] : 0.f};
+      acc[m] = dc_floatx4{mine ? -now.u0.x : 0.f, mine ? -now.u0.y : 0.f, mine ? -now.u0.z : 0.f, mine ? -now.u0.w : 0.f};
     }
 #pragma unroll
     for (int t = 0; t < TD; ++t) {
@@ -305,10 +324,8 @@ __global__ __launch_bounds__(DC_THREADS, 1) void delta_chunk_states_kernel(Delta
 #pragma unroll
     for (int m = 0; m < 4; ++m)
       U[m] = -((buf[0][m][lane] + buf[1][m][lane]) + (buf[2][m][lane] + buf[3][m][lane]));
-    float* u = g.u + (entry * DC_ROWS + wave * 16 + quad * 4) * g.ep + col;
-    const dc_floatx4 mine = wave == 0 ? U[0] : (wave == 1 ? U[1] : (wave == 2 ? U[2] : U[3]));
-#pragma unroll
-    for (int r = 0; r < 4; ++r) u[r * g.ep] = mine[r];
+    *reinterpret_cast<dc_floatx4*>(g.u + ((entry * (g.ep / 16) + slab) * 4 + wave) * 256 + lane * 4) =
+        wave == 0 ? U[0] : (wave == 1 ? U[1] : (wave == 2 ? U[2] : U[3]));
 #pragma unroll
     for (int t = 0; t < TD; ++t)
 #pragma unroll
@@ -325,7 +342,7 @@ __global__ __launch_bounds__(DC_THREADS, 1) void delta_chunk_states_kernel(Delta
       for (int t = 0; t < TD; ++t) S[t] = dc_mfma(now.k[t][m].w, U[m][3], S[t]);
     }
   };
-  delta_chunk_fetch<D, TD>(g, static_cast<size_t>(c0) * g.heads + local, wave, r16, quad, col, even);
+  delta_chunk_fetch<D, TD>(g, static_cast<size_t>(c0) * g.heads + local, wave, lane, slab, even);
   for (int c = c0; c < c1; c += 2) {
     step(c, even, odd);
     if (c + 1 >= c1) break;
@@ -340,32 +357,26 @@ __global__ __launch_bounds__(DC_THREADS, 1) void delta_chunk_states_kernel(Delta
     }
 }
 
-template <bool WIDE>
 __global__ __launch_bounds__(DC_THREADS) void delta_chunk_outputs_kernel(DeltaChunks g, float* __restrict__ out,
                                                                          int out_row) {
   const int item = blockIdx.x / g.heads, head = g.head0 + blockIdx.x % g.heads;
-  const int kv = head / (g.H / g.G);
   const int t0 = g.items[3 * item + 1], n = g.items[3 * item + 2] - t0;
   const size_t entry = blockIdx.x;
-  const int lane = threadIdx.x % TIE_WAVE, wave = __builtin_amdgcn_readfirstlane(threadIdx.x / TIE_WAVE), r16 = lane & 15, quad = lane >> 4;
-  const int col = (blockIdx.y * 4 + wave) * 16 + r16;
-  if ((blockIdx.y * 4 + wave) * 16 >= g.ep) return;                    // the whole wave; there is no barrier below
-  const float* q[4];
-#pragma unroll
-  for (int m = 0; m < 4; ++m)
-    q[m] = g.tok + static_cast<size_t>(t0 + min(m * 16 + r16, n - 1)) * g.row + kv * g.d;
-  const float* s0 = g.s0 + (entry * g.D + quad * 4) * g.ep + col;
+  const int lane = threadIdx.x % TIE_WAVE, wave = __builtin_amdgcn_readfirstlane(threadIdx.x / TIE_WAVE);
+  const int r16 = lane & 15, quad = lane >> 4;
+  const int slab = blockIdx.y * 4 + wave, slabs = g.ep / 16, blocks = g.D / 16;
+  if (slab >= slabs) return;                                           // the whole wave; there is no barrier below
+  const float* q = g.q + entry * 4 * blocks * 256 + lane * 4;
+  const float* s0 = g.s0 + (entry * slabs + slab) * blocks * 256 + lane * 4;
   dc_floatx4 acc[4];
 #pragma unroll
   for (int m = 0; m < 4; ++m) acc[m] = dc_floatx4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll 2
-  for (int k0 = 0; k0 < g.D; k0 += 16) {
+  for (int kb = 0; kb < blocks; ++kb) {
+    const dc_floatx4 v = *reinterpret_cast<const dc_floatx4*>(s0 + kb * 256);
     float4 a[4];
-    float v[4];
 #pragma unroll
-    for (int r = 0; r < 4; ++r) v[r] = s0[(k0 + r) * g.ep];
-#pragma unroll
-    for (int m = 0; m < 4; ++m) a[m] = dc_load4<WIDE>(q[m], k0 + quad * 4, g.d);
+    for (int m = 0; m < 4; ++m) a[m] = *reinterpret_cast<const float4*>(q + (m * blocks + kb) * 256);
 #pragma unroll
     for (int m = 0; m < 4; ++m) acc[m] = dc_mfma(a[m].x, v[0], acc[m]);
 #pragma unroll
@@ -375,27 +386,15 @@ __global__ __launch_bounds__(DC_THREADS) void delta_chunk_outputs_kernel(DeltaCh
 #pragma unroll
     for (int m = 0; m < 4; ++m) acc[m] = dc_mfma(a[m].w, v[3], acc[m]);
   }
-#pragma unroll
-  for (int m = 0; m < 4; ++m) {
-    const float4 eb = *reinterpret_cast<const float4*>(g.decay + entry * DC_ROWS + m * 16 + quad * 4);
-    acc[m][0] *= eb.x, acc[m][1] *= eb.y, acc[m][2] *= eb.z, acc[m][3] *= eb.w;
-  }
-  const float* pe = g.p + (entry * DC_ROWS + r16) * DC_ROWS + quad * 4;
-  const float* u = g.u + (entry * DC_ROWS + quad * 4) * g.ep + col;
+  const float* pe = g.p + entry * DC_ROWS * DC_ROWS + lane * 4;
+  const float* u = g.u + (entry * slabs + slab) * 4 * 256 + lane * 4;
 #pragma unroll
   for (int jt = 0; jt < 4; ++jt) {
-    float v[4];
+    const dc_floatx4 v = *reinterpret_cast<const dc_floatx4*>(u + jt * 256);
 #pragma unroll
-    for (int r = 0; r < 4; ++r) v[r] = u[(jt * 16 + r) * g.ep];
-#pragma unroll
-    for (int m = jt; m < 4; ++m) {
-      const float4 a = *reinterpret_cast<const float4*>(pe + m * 16 * DC_ROWS + jt * 16);
-      acc[m] = dc_mfma(a.x, v[0], acc[m]);
-      acc[m] = dc_mfma(a.y, v[1], acc[m]);
-      acc[m] = dc_mfma(a.z, v[2], acc[m]);
-      acc[m] = dc_mfma(a.w, v[3], acc[m]);
-    }
+    for (int m = jt; m < 4; ++m) acc[m] = dc_mfma4(*reinterpret_cast<const float4*>(pe + (m * 4 + jt) * 256), v, acc[m]);
   }
+  const int col = slab * 16 + r16;
   if (col >= g.e) return;
 #pragma unroll
   for (int m = 0; m < 4; ++m)
@@ -412,7 +411,7 @@ extern "C" int tie_delta_chunk_dim(int d) { return d <= 64 ? 64 : (d <= 128 ? 12
 // Floats of the memory of one (chunk, head).
 extern "C" int tie_delta_chunk_floats(int d, int e) {
   const int D = tie_delta_chunk_dim(d), ep = (e + 15) / 16 * 16;
-  return DC_ROWS * ep + 2 * DC_ROWS * D + DC_ROWS * DC_ROWS + DC_ROWS + D * ep;
+  return DC_ROWS * ep + 3 * DC_ROWS * D + DC_ROWS * DC_ROWS + 4 + D * ep;
 }
 
 // tok: rows of delta_prepare with one decay a head; out float32 [T][>= H e]; state [slots][H][d][e]; items [count][3]
@@ -434,12 +433,24 @@ extern "C" int tie_delta_chunks(const float* tok, int row, float* out, int out_r
   g.u = memory;
   g.w = g.u + entries * DC_ROWS * ep;
   g.kt = g.w + entries * DC_ROWS * g.D;
-  g.p = g.kt + entries * DC_ROWS * g.D;
-  g.decay = g.p + entries * DC_ROWS * DC_ROWS;
-  g.s0 = g.decay + entries * DC_ROWS;
+  g.q = g.kt + entries * DC_ROWS * g.D;
+  g.p = g.q + entries * DC_ROWS * g.D;
+  g.s0 = g.p + entries * DC_ROWS * DC_ROWS;
+  g.decay = g.s0 + entries * g.D * ep;
   const bool wide = d % 4 == 0 && row % 4 == 0 && reinterpret_cast<uintptr_t>(tok) % 16 == 0;
-  if (wide) delta_chunk_prepare_kernel<true><<<static_cast<unsigned>(entries), DC_THREADS, 0, stream>>>(g);
-  else delta_chunk_prepare_kernel<false><<<static_cast<unsigned>(entries), DC_THREADS, 0, stream>>>(g);
+  const size_t lds = sizeof(float) * DC_ROWS * (g.D + 4);
+  static bool raised = false;
+  if (!raised) {             // with the rest of its LDS the keys of 256 dimensions exceed the 64 KB of an ordinary launch
+    for (const void* kernel : {reinterpret_cast<const void*>(&delta_chunk_prepare_kernel<true>),
+                               reinterpret_cast<const void*>(&delta_chunk_prepare_kernel<false>)}) {
+      const hipError_t err = hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize,
+                                                 static_cast<int>(sizeof(float) * DC_ROWS * (256 + 4)));
+      if (err != hipSuccess) return static_cast<int>(err);
+    }
+    raised = true;
+  }
+  if (wide) delta_chunk_prepare_kernel<true><<<static_cast<unsigned>(entries), DC_THREADS, lds, stream>>>(g);
+  else delta_chunk_prepare_kernel<false><<<static_cast<unsigned>(entries), DC_THREADS, lds, stream>>>(g);
   int rc = tie_launch_status();
   if (rc != TIE_OK) return rc;
   const int pairs = num_seqs * heads;
@@ -452,7 +463,6 @@ extern "C" int tie_delta_chunks(const float* tok, int row, float* out, int out_r
   rc = tie_launch_status();
   if (rc != TIE_OK) return rc;
   const dim3 grid(static_cast<unsigned>(entries), (ep + 63) / 64);
-  if (wide) delta_chunk_outputs_kernel<true><<<grid, DC_THREADS, 0, stream>>>(g, out, out_row);
-  else delta_chunk_outputs_kernel<false><<<grid, DC_THREADS, 0, stream>>>(g, out, out_row);
+  delta_chunk_outputs_kernel<<<grid, DC_THREADS, 0, stream>>>(g, out, out_row);
   return tie_launch_status();
 }

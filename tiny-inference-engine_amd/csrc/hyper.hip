@@ -39,6 +39,66 @@ __global__ void layer_norm_kernel(const TX* __restrict__ x, const float* __restr
   for (int c = threadIdx.x; c < n; c += blockDim.x) store_from_float(o + c, ((row[c] - mean) * inv) * w[c]);
 }
 
+// The same for rows in steps of four columns: a thread holds V x four columns in registers, every load under way first.
+template <typename T>
+__device__ __forceinline__ float4 load_four(const T* p);
+template <>
+__device__ __forceinline__ float4 load_four<float>(const float* p) { return *reinterpret_cast<const float4*>(p); }
+template <>
+__device__ __forceinline__ float4 load_four<bf16_t>(const bf16_t* p) {
+  const uint2 v = *reinterpret_cast<const uint2*>(p);
+  return make_float4(__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xffff0000u), __uint_as_float(v.y << 16),
+                     __uint_as_float(v.y & 0xffff0000u));
+}
+
+template <typename TX, typename TO, int V>
+__global__ void layer_norm_row_kernel(const TX* __restrict__ x, const float* __restrict__ w, float eps,
+                                      TO* __restrict__ out, const int* __restrict__ rows, int n) {
+  __shared__ float scratch[16];
+  const TX* r = x + (rows ? static_cast<size_t>(rows[blockIdx.x]) : blockIdx.x) * n;
+  float4 v[V], wt[V];
+  float sum = 0.f;
+#pragma unroll
+  for (int j = 0; j < V; ++j) {
+    const int c = (threadIdx.x + j * blockDim.x) * 4;
+    v[j] = c < n ? load_four(r + c) : make_float4(0.f, 0.f, 0.f, 0.f);
+    wt[j] = c < n ? load_four(w + c) : make_float4(0.f, 0.f, 0.f, 0.f);
+  }
+#pragma unroll
+  for (int j = 0; j < V; ++j) sum += (v[j].x + v[j].y) + (v[j].z + v[j].w);
+  const float mean = block_sum(sum, scratch) / static_cast<float>(n);
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < V; ++j) {
+    if ((threadIdx.x + j * blockDim.x) * 4 >= n) continue;
+    const float a = v[j].x - mean, b = v[j].y - mean, c = v[j].z - mean, d = v[j].w - mean;
+    ss += (a * a + b * b) + (c * c + d * d);
+  }
+  const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / static_cast<float>(n) + eps);
+  TO* o = out + static_cast<size_t>(blockIdx.x) * n;
+#pragma unroll
+  for (int j = 0; j < V; ++j) {
+    const int c = (threadIdx.x + j * blockDim.x) * 4;
+    if (c >= n) continue;
+    const float a = ((v[j].x - mean) * inv) * wt[j].x, b = ((v[j].y - mean) * inv) * wt[j].y;
+    const float e = ((v[j].z - mean) * inv) * wt[j].z, f = ((v[j].w - mean) * inv) * wt[j].w;
+    if constexpr (sizeof(TO) == 2) *reinterpret_cast<uint2*>(o + c) = make_uint2(pack_bf16x2(a, b), pack_bf16x2(e, f));
+    else *reinterpret_cast<float4*>(o + c) = make_float4(a, b, e, f);
+  }
+}
+
+template <typename TX, typename TO>
+static void launch_layer_norm_row(const TX* x, const float* w, float eps, TO* out, const int* rows, int count, int n,
+                                  hipStream_t stream) {
+  const int quads = n / 4;
+  if (quads <= 1024)
+    layer_norm_row_kernel<TX, TO, 1><<<count, (quads + TIE_WAVE - 1) / TIE_WAVE * TIE_WAVE, 0, stream>>>(x, w, eps, out, rows, n);
+  else if (quads <= 2048)
+    layer_norm_row_kernel<TX, TO, 2><<<count, 1024, 0, stream>>>(x, w, eps, out, rows, n);
+  else
+    layer_norm_row_kernel<TX, TO, 4><<<count, 1024, 0, stream>>>(x, w, eps, out, rows, n);
+}
+
 static int row_threads(int n) { return n >= 4096 ? 512 : (n >= 1024 ? 256 : (n >= 256 ? 128 : 64)); }
 
 extern "C" int tie_layer_norm(const void* x, int x_dtype, const float* w, float eps, void* out, int out_dtype,
@@ -46,9 +106,16 @@ extern "C" int tie_layer_norm(const void* x, int x_dtype, const float* w, float 
   if (count <= 0 || n <= 0 || static_cast<size_t>(n) * 4 > 65536) return TIE_BAD_ARGUMENT;
   const int threads = row_threads(n);
   const size_t lds = static_cast<size_t>(n) * sizeof(float);
-#define LN(TX, TO)                                                                                      \
-  layer_norm_kernel<TX, TO><<<count, threads, lds, stream>>>(static_cast<const TX*>(x), w, eps,         \
-                                                             static_cast<TO*>(out), rows, n)
+  const bool in_fours = n % 4 == 0 && reinterpret_cast<uintptr_t>(x) % 16 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0 &&
+                        reinterpret_cast<uintptr_t>(out) % 16 == 0;
+#define LN(TX, TO)                                                                                               \
+  do {                                                                                                           \
+    if (in_fours)                                                                                                \
+      launch_layer_norm_row(static_cast<const TX*>(x), w, eps, static_cast<TO*>(out), rows, count, n, stream);   \
+    else                                                                                                         \
+      layer_norm_kernel<TX, TO><<<count, threads, lds, stream>>>(static_cast<const TX*>(x), w, eps,              \
+                                                                 static_cast<TO*>(out), rows, n);                \
+  } while (0)
   if (x_dtype == TIE_F32 && out_dtype == TIE_F32) LN(float, float);
   else if (x_dtype == TIE_F32 && out_dtype == TIE_BF16) LN(float, bf16_t);
   else if (x_dtype == TIE_BF16 && out_dtype == TIE_BF16) LN(bf16_t, bf16_t);

@@ -68,8 +68,90 @@ __device__ __forceinline__ void wave_order() {
   __builtin_amdgcn_wave_barrier();
 }
 
+// One row by one wave without groups and with up to 64 PER experts: lane l holds the experts l, l + 64, ..., counts how
+// many stand before each of its own (ties to the lower index), and writes those that `top` or fewer stand before.
+template <int PER>
+__device__ void route_row_ranked(const RouteParams& p, size_t t, int lane, int* ids_lds) {
+  const float* z = p.logits + t * p.row;
+  const int E = p.E, top = p.top, slots = top + p.shared;
+  float score[PER], choice[PER];
+  float m = -INFINITY;
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int e = lane + i * TIE_WAVE;
+    score[i] = e < E ? z[e] + (p.bias != nullptr ? p.bias[e] : 0.f) : -INFINITY;
+    m = fmaxf(m, score[i]);
+  }
+  if (p.scoring == SCORE_SIGMOID) {
+#pragma unroll
+    for (int i = 0; i < PER; ++i) score[i] = 1.0f / (1.0f + expf(-score[i]));
+  } else if (p.scoring == SCORE_SOFTMAX) {
+    m = wave_max(m);
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      score[i] = expf(score[i] - m);
+      sum += score[i];
+    }
+    sum = wave_sum(sum);
+#pragma unroll
+    for (int i = 0; i < PER; ++i) score[i] /= sum;
+  }
+  int before[PER];
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int e = lane + i * TIE_WAVE;
+    choice[i] = e < E ? score[i] + (p.correction != nullptr ? p.correction[e] : 0.f) : -INFINITY;
+    before[i] = 0;
+  }
+#pragma unroll
+  for (int ib = 0; ib < PER; ++ib) {
+    const int count = min(TIE_WAVE, E - ib * TIE_WAVE);
+    for (int lb = 0; lb < count; ++lb) {
+      const float v = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, choice[ib]), lb));
+      const int b = ib * TIE_WAVE + lb;
+#pragma unroll
+      for (int i = 0; i < PER; ++i) before[i] += (v > choice[i] || (v == choice[i] && b < lane + i * TIE_WAVE)) ? 1 : 0;
+    }
+  }
+  bool chosen[PER];
+  float best = -INFINITY, sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    chosen[i] = lane + i * TIE_WAVE < E && before[i] < top;
+    if (chosen[i]) best = fmaxf(best, score[i]);
+  }
+  if (p.scoring == SCORE_LOGIT) {             // the softmax over the chosen logits alone
+    best = wave_max(best);
+#pragma unroll
+    for (int i = 0; i < PER; ++i) score[i] = expf(score[i] - best);
+  }
+  if (p.scoring == SCORE_LOGIT || p.renormalize) {
+#pragma unroll
+    for (int i = 0; i < PER; ++i) sum += chosen[i] ? score[i] : 0.f;
+    sum = wave_sum(sum) + (p.scoring == SCORE_LOGIT ? 0.f : p.renorm_eps);
+#pragma unroll
+    for (int i = 0; i < PER; ++i) score[i] /= sum;
+  }
+  auto put = [&](int slot, int e, float w) {
+    p.ids[t * slots + slot] = e;
+    p.weights[t * slots + slot] = w;
+    if (ids_lds != nullptr) ids_lds[t * slots + slot] = e;
+  };
+#pragma unroll
+  for (int i = 0; i < PER; ++i)
+    if (chosen[i]) put(before[i], lane + i * TIE_WAVE, score[i] * p.weight_scale);
+  if (lane < p.shared) put(top + lane, E + lane, 1.0f / (1.0f + expf(-z[E])));
+}
+
 // One row by one wave, whose LDS holds 2 E + groups floats; the choice also goes to ids_lds where that is given.
 __device__ void route_row(const RouteParams& p, float* lds, size_t t, int lane, int* ids_lds) {
+  if ((p.groups == 1 || p.keep == p.groups) && p.E <= 4 * TIE_WAVE && p.shared <= TIE_WAVE) {
+    if (p.E <= TIE_WAVE) route_row_ranked<1>(p, t, lane, ids_lds);
+    else if (p.E <= 2 * TIE_WAVE) route_row_ranked<2>(p, t, lane, ids_lds);
+    else route_row_ranked<4>(p, t, lane, ids_lds);
+    return;
+  }
   const float *logits = p.logits, *bias = p.bias, *correction = p.correction;
   const int row = p.row, E = p.E, groups = p.groups, keep = p.keep, top = p.top, scoring = p.scoring;
   const int group_top = p.group_top, renormalize = p.renormalize, shared = p.shared;
@@ -242,19 +324,34 @@ __device__ void align_slots(const int* ids, int slots, int real, int tile_rows, 
     if (e >= 0 && e < real) atomicAdd(&count[e], 1);
   }
   __syncthreads();
-  if (tid == 0) {
-    int at = 0, n = 0;
-    for (int e = 0; e < real; ++e) {
-      o.offsets[e] = at;
-      cursor[e] = at;
-      for (int r = 0; r < count[e] && n < o.max_tiles; r += tile_rows, ++n) {
-        o.tiles[2 * n] = e;
-        o.tiles[2 * n + 1] = at + r;
+  if (tid < TIE_WAVE) {                       // a lane an expert, 64 at a time: running sums of slots and of tiles
+    int slots_before = 0, tiles_before = 0;
+    for (int base = 0; base < real; base += TIE_WAVE) {
+      const int e = base + tid;
+      const int c = e < real ? count[e] : 0, n = (c + tile_rows - 1) / tile_rows;
+      int c_sum = c, n_sum = n;
+#pragma unroll
+      for (int off = 1; off < TIE_WAVE; off *= 2) {
+        const int c_up = __shfl_up(c_sum, off, TIE_WAVE), n_up = __shfl_up(n_sum, off, TIE_WAVE);
+        if (tid >= off) c_sum += c_up, n_sum += n_up;
       }
-      at += count[e];
+      const int at = slots_before + c_sum - c;
+      int tile = tiles_before + n_sum - n;
+      if (e < real) {
+        o.offsets[e] = at;
+        cursor[e] = at;
+        for (int r = 0; r < c && tile < o.max_tiles; r += tile_rows, ++tile) {
+          o.tiles[2 * tile] = e;
+          o.tiles[2 * tile + 1] = at + r;
+        }
+      }
+      slots_before += __shfl(c_sum, TIE_WAVE - 1, TIE_WAVE);
+      tiles_before += __shfl(n_sum, TIE_WAVE - 1, TIE_WAVE);
     }
-    o.offsets[real] = at;
-    *o.num_tiles = n;
+    if (tid == 0) {
+      o.offsets[real] = slots_before;
+      *o.num_tiles = min(tiles_before, o.max_tiles);
+    }
   }
   __syncthreads();
   for (int s = tid; s < slots; s += ALIGN_THREADS) {

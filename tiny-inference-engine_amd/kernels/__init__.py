@@ -2363,7 +2363,7 @@ DELTA_CHUNK_SCRATCH_MAX = 1 << 30      # bytes of chunk states above which a ste
 # With one decay a head a chunk's products are matrix products (csrc/delta_chunks.hip): shorter chunks, and from shorter
 # portions on. Above the scratch limit the heads run in several passes.
 DELTA_HEAD_CHUNK_ROWS = 64             # DC_ROWS of csrc/delta_chunks.hip
-DELTA_HEAD_CHUNKS_FROM = 128
+DELTA_HEAD_CHUNKS_FROM = 96
 
 
 def delta_chunks(batch, device, head_decay: bool = False) -> Optional[ScanChunks]:
