@@ -199,7 +199,7 @@ __global__ void delta_prepare_kernel(const float* __restrict__ u, int row, const
 
 // The same for many rows: a wave takes the channels of one q or k head, or 64 PER channels of v, and walks
 // DELTA_WALK_ROWS rows with the convolution's window in registers, so that an input is read once instead of once a tap;
-// lane l holds channels l, l + 64, ... A unit behind the last one makes beta and the decays.
+// lane l holds channels l, l + 64, ... The units behind them make the decays, 64 PER columns each, the first of them beta too.
 #define DELTA_WALK_ROWS 16
 #define DELTA_WALK_WAVES 4
 
@@ -213,15 +213,17 @@ __global__ __launch_bounds__(DELTA_WALK_WAVES* TIE_WAVE) void delta_prepare_walk
   if (unit >= units) return;                       // the whole wave; there is no barrier below
   const int first = blockIdx.y * DELTA_WALK_ROWS, rows = min(DELTA_WALK_ROWS, T - first);
   const int C = 2 * G * d + H * e;
-  if (unit == units - 1) {
-    const int width = H * da;
+  const int decays = 2 * G + (H * e + TIE_WAVE * PER - 1) / (TIE_WAVE * PER);        // the first unit of the decays
+  if (unit >= decays) {
+    const int lo = (unit - decays) * TIE_WAVE * PER, width = min(TIE_WAVE * PER, H * da - lo);
     for (int i = lane; i < rows * width; i += TIE_WAVE) {
-      const int t = first + i / width, c = i % width;
+      const int t = first + i / width, c = lo + i % width;
       float* o = out + static_cast<size_t>(t) * out_row;
       const float log_g = -expf(A_log[c / da]) * softplus_f(a[static_cast<size_t>(t) * a_row + c] + dt_bias[c]);
       o[C + c] = expf(log_g);
       if (da == 1) o[C + 2 * H + c] = log_g;
     }
+    if (unit > decays) return;
     for (int i = lane; i < rows * H; i += TIE_WAVE) {
       const int t = first + i / H, h = i % H;
       out[static_cast<size_t>(t) * out_row + C + H * da + h] = sigmoid_f(u[static_cast<size_t>(t) * row + C + h]);
@@ -300,7 +302,8 @@ extern "C" int tie_delta_prepare(const float* u, int row, const float* w, int ta
     return TIE_BAD_ARGUMENT;
   if (T >= DELTA_WALK_FROM && !shift && taps >= 2 && taps <= 4 && d <= 4 * TIE_WAVE) {
     const int per = d <= TIE_WAVE ? 1 : (d <= 2 * TIE_WAVE ? 2 : 4);
-    const int units = 2 * G + (H * e + TIE_WAVE * per - 1) / (TIE_WAVE * per) + 1;
+    const int per_unit = TIE_WAVE * per;
+    const int units = 2 * G + (H * e + per_unit - 1) / per_unit + (H * da + per_unit - 1) / per_unit;
     const dim3 grid((units + DELTA_WALK_WAVES - 1) / DELTA_WALK_WAVES, (T + DELTA_WALK_ROWS - 1) / DELTA_WALK_ROWS);
 #define WALK(PER, TAPS)                                                                                            \
   delta_prepare_walk_kernel<PER, TAPS><<<grid, DELTA_WALK_WAVES * TIE_WAVE, 0, stream>>>(                           \
