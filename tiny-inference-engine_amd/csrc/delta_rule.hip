@@ -734,10 +734,10 @@ extern "C" int tie_gated_delta_scan_chunked(const float* tok, int row, float* ou
 
 // ---------------------------------------------------------------- the norm of the heads' outputs, gated
 // out = o / rms(o over each group of `group` columns) * w[column in group] * sigmoid(gate) (or * silu(gate)), a wave a
-// group.
+// group; the weights of neighbouring groups lie w_group apart (0: one weight for all groups), w null: all 1.
 template <typename TO>
 __global__ void grouped_gated_rms_norm_kernel(const float* __restrict__ o, int o_row, const float* __restrict__ w,
-                                              float eps, const float* __restrict__ gate, int gate_row, int silu_gate,
+                                              int w_group, float eps, const float* __restrict__ gate, int gate_row, int silu_gate,
                                               TO* __restrict__ out, int groups, int group) {
   const int lane = threadIdx.x & (TIE_WAVE - 1);
   const int g = blockIdx.y * (blockDim.x / TIE_WAVE) + threadIdx.x / TIE_WAVE;
@@ -750,10 +750,10 @@ __global__ void grouped_gated_rms_norm_kernel(const float* __restrict__ o, int o
   const float inv = 1.0f / sqrtf(wave_sum(ss) / static_cast<float>(group) + eps);
   TO* d = out + (t * groups + g) * group;
   for (int c = lane; c < group; c += TIE_WAVE)
-    store_from_float(d + c, (r[c] * inv) * w[c] * (silu_gate ? silu_f(gt[c]) : sigmoid_f(gt[c])));
+    store_from_float(d + c, (r[c] * inv) * (w ? w[static_cast<size_t>(g) * w_group + c] : 1.f) * (silu_gate ? silu_f(gt[c]) : sigmoid_f(gt[c])));
 }
 
-extern "C" int tie_grouped_gated_rms_norm(const float* o, int o_row, const float* w, float eps, const float* gate,
+extern "C" int tie_grouped_gated_rms_norm(const float* o, int o_row, const float* w, int w_group, float eps, const float* gate,
                                           int gate_row, int silu_gate, void* out, int out_dtype, int T, int groups,
                                           int group, hipStream_t stream) {
   if (T <= 0 || groups <= 0 || group <= 0 || o_row < groups * group || gate_row < groups * group)
@@ -762,10 +762,10 @@ extern "C" int tie_grouped_gated_rms_norm(const float* o, int o_row, const float
   const dim3 grid(T, (groups + waves - 1) / waves);
   if (out_dtype == TIE_F32)
     grouped_gated_rms_norm_kernel<float><<<grid, waves * TIE_WAVE, 0, stream>>>(
-        o, o_row, w, eps, gate, gate_row, silu_gate, static_cast<float*>(out), groups, group);
+        o, o_row, w, w_group, eps, gate, gate_row, silu_gate, static_cast<float*>(out), groups, group);
   else if (out_dtype == TIE_BF16)
     grouped_gated_rms_norm_kernel<bf16_t><<<grid, waves * TIE_WAVE, 0, stream>>>(
-        o, o_row, w, eps, gate, gate_row, silu_gate, static_cast<bf16_t*>(out), groups, group);
+        o, o_row, w, w_group, eps, gate, gate_row, silu_gate, static_cast<bf16_t*>(out), groups, group);
   else
     return TIE_BAD_ARGUMENT;
   return tie_launch_status();

@@ -857,7 +857,7 @@ extern "C" int tie_qk_norm_rope_kv_write(const void* qkv, int in_dtype, void* q_
 struct RoutedParts {
   const float* parts;     // [slots][n] float32, or null: y is planes
   const int* where;       // [R][top]
-  const float* weights;   // [R][top]
+  const float* weights;   // [R][top], or null: all 1
   const void* self;       // [R][n] rows of self_dtype
   int self_dtype;
   int top;
@@ -870,7 +870,7 @@ __device__ __forceinline__ float routed_value(const RoutedParts& rp, size_t r, i
     const float part = at >= 0 ? rp.parts[static_cast<size_t>(at) * n + i]
                        : (rp.self_dtype == TIE_F32 ? static_cast<const float*>(rp.self)[r * n + i]
                                                    : bf16_to_float(static_cast<const bf16_t*>(rp.self)[r * n + i]));
-    y = fmaf(rp.weights[r * rp.top + k], part, y);
+    y = fmaf(rp.weights ? rp.weights[r * rp.top + k] : 1.f, part, y);
   }
   return y;
 }
@@ -971,7 +971,7 @@ extern "C" int tie_norm_add_norm(const float* y, long plane_stride, int count, c
     return TIE_BAD_ARGUMENT;
   if (parts == nullptr && (y == nullptr || count < 1 || (count > 1 && plane_stride < static_cast<long>(R) * n)))
     return TIE_BAD_ARGUMENT;
-  if (parts != nullptr && (where == nullptr || weights == nullptr || self == nullptr || top < 1 ||
+  if (parts != nullptr && (where == nullptr || self == nullptr || top < 1 ||
                            (self_dtype != TIE_F32 && self_dtype != TIE_BF16)))
     return TIE_BAD_ARGUMENT;
   if (w_next != nullptr && out_dtype != TIE_F32 && out_dtype != TIE_BF16) return TIE_BAD_ARGUMENT;
@@ -1011,26 +1011,35 @@ extern "C" int tie_norm_add_norm(const float* y, long plane_stride, int count, c
 }
 
 // --------------------------------------------------------------------- gelu
-// out = 0.5 z (1 + erf(z / sqrt 2)), the exact form, in float32.
-template <typename TX, typename TO>
+// out = 0.5 z (1 + erf(z / sqrt 2)), the exact form, or the tanh form, in float32.
+template <typename TX, typename TO, bool TANH>
 __global__ void gelu_kernel(const TX* __restrict__ x, TO* __restrict__ out, size_t count) {
   const size_t i = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
   if (i >= count) return;
   const float z = load_as_float(x + i);
-  store_from_float(out + i, 0.5f * z * (1.0f + erff(z * 0.70710678118654752440f)));
+  if (TANH) store_from_float(out + i, sizeof(TO) == 2 ? gelu_tanh_fast(z) : gelu_tanh_exact(z));
+  else store_from_float(out + i, 0.5f * z * (1.0f + erff(z * 0.70710678118654752440f)));
 }
 
-extern "C" int tie_gelu(const void* x, int in_dtype, void* out, int out_dtype, long long count, hipStream_t stream) {
+extern "C" int tie_gelu(const void* x, int in_dtype, void* out, int out_dtype, long long count, int tanh_form,
+                        hipStream_t stream) {
   if (count <= 0 || count > 0x7fffffffLL * 256) return TIE_BAD_ARGUMENT;
   const unsigned blocks = static_cast<unsigned>((count + 255) / 256);
-#define LAUNCH(TX, TO) \
-  gelu_kernel<TX, TO><<<blocks, 256, 0, stream>>>(static_cast<const TX*>(x), static_cast<TO*>(out), static_cast<size_t>(count))
-  if (in_dtype == TIE_F32 && out_dtype == TIE_F32) LAUNCH(float, float);
-  else if (in_dtype == TIE_F32 && out_dtype == TIE_BF16) LAUNCH(float, bf16_t);
-  else if (in_dtype == TIE_BF16 && out_dtype == TIE_BF16) LAUNCH(bf16_t, bf16_t);
-  else if (in_dtype == TIE_BF16 && out_dtype == TIE_F32) LAUNCH(bf16_t, float);
+#define LAUNCH_F(TX, TO, TANH)                                                                            \
+  gelu_kernel<TX, TO, TANH><<<blocks, 256, 0, stream>>>(static_cast<const TX*>(x), static_cast<TO*>(out), \
+                                                        static_cast<size_t>(count))
+#define LAUNCH(TX, TO)                   \
+  {                                      \
+    if (tanh_form) LAUNCH_F(TX, TO, true); \
+    else LAUNCH_F(TX, TO, false);        \
+  }
+  if (in_dtype == TIE_F32 && out_dtype == TIE_F32) LAUNCH(float, float)
+  else if (in_dtype == TIE_F32 && out_dtype == TIE_BF16) LAUNCH(float, bf16_t)
+  else if (in_dtype == TIE_BF16 && out_dtype == TIE_BF16) LAUNCH(bf16_t, bf16_t)
+  else if (in_dtype == TIE_BF16 && out_dtype == TIE_F32) LAUNCH(bf16_t, float)
   else return TIE_BAD_ARGUMENT;
 #undef LAUNCH
+#undef LAUNCH_F
   return tie_launch_status();
 }
 

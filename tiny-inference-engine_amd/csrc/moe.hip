@@ -10,7 +10,7 @@
 //              to the logits first.
 //              `shared` further slots a row name the experts E, E + 1, ... (experts every row uses: a shared expert,
 //              cut into pieces of the routed experts' size), all with the weight sigmoid(logits[E]), one more
-//              column of the router's product.
+//              column of the router's product, or with the weight 1.
 //   align      the T * top (row, choice) slots sorted by expert: offsets[e] .. offsets[e + 1] are the places of
 //              expert e's slots, slot_at[place] = slot, where[slot] = place (-1 for a choice >= `real`: an expert
 //              without weights, which the caller treats as it likes), and the list of row tiles (expert, first
@@ -57,7 +57,7 @@ struct RouteParams {
   const float* correction; // [E] or null
   int E, groups, keep, top, scoring, group_top, renormalize;
   float renorm_eps, weight_scale;
-  int shared;
+  int shared, shared_gated;
   int* ids;                // [T][top + shared]
   float* weights;          // [T][top + shared]
 };
@@ -141,7 +141,7 @@ __device__ void route_row_ranked(const RouteParams& p, size_t t, int lane, int* 
 #pragma unroll
   for (int i = 0; i < PER; ++i)
     if (chosen[i]) put(before[i], lane + i * TIE_WAVE, score[i] * p.weight_scale);
-  if (lane < p.shared) put(top + lane, E + lane, 1.0f / (1.0f + expf(-z[E])));
+  if (lane < p.shared) put(top + lane, E + lane, p.shared_gated ? 1.0f / (1.0f + expf(-z[E])) : 1.0f);
 }
 
 // One row by one wave, whose LDS holds 2 E + groups floats; the choice also goes to ids_lds where that is given.
@@ -271,7 +271,7 @@ __device__ void route_row(const RouteParams& p, float* lds, size_t t, int lane, 
       for (int k = 0; k < top; ++k) w[k] *= weight_scale;
     }
     if (shared > 0) {
-      const float g = 1.0f / (1.0f + expf(-z[E]));
+      const float g = p.shared_gated ? 1.0f / (1.0f + expf(-z[E])) : 1.0f;
       for (int k = 0; k < shared; ++k) {
         ids[t * slots + top + k] = E + k;
         if (ids_lds != nullptr) ids_lds[t * slots + top + k] = E + k;
@@ -290,15 +290,16 @@ __global__ __launch_bounds__(TIE_WAVE) void moe_route_kernel(RouteParams p) {
 // bias and correction [E] or null; ids and weights [T][top + shared].
 extern "C" int tie_moe_route(const float* logits, int row, const float* bias, const float* correction, int T, int E,
                              int groups, int keep, int top, int scoring, int group_top, int renormalize, float renorm_eps,
-                             float weight_scale, int shared, int* ids, float* weights, hipStream_t stream) {
+                             float weight_scale, int shared, int shared_gated, int* ids, float* weights,
+                             hipStream_t stream) {
   if (T <= 0 || E <= 0 || E > MOE_MAX_EXPERTS || groups <= 0 || E % groups != 0 || keep <= 0 || keep > groups ||
       top <= 0 || top > E || group_top <= 0 || group_top > MOE_MAX_GROUP_TOP || shared < 0 ||
-      row < E + (shared > 0 ? 1 : 0) || scoring < SCORE_SOFTMAX || scoring > SCORE_LOGIT)
+      row < E + (shared > 0 && shared_gated ? 1 : 0) || scoring < SCORE_SOFTMAX || scoring > SCORE_LOGIT)
     return TIE_BAD_ARGUMENT;
   const size_t lds = sizeof(float) * (2 * static_cast<size_t>(E) + groups);
   moe_route_kernel<<<T, TIE_WAVE, lds, stream>>>(RouteParams{logits, row, bias, correction, E, groups, keep, top, scoring,
                                                              group_top, renormalize, renorm_eps, weight_scale, shared,
-                                                             ids, weights});
+                                                             shared_gated, ids, weights});
   return tie_launch_status();
 }
 
@@ -410,19 +411,19 @@ extern "C" int tie_moe_align(const int* ids, int slots, int real, int tile_rows,
 // tie_moe_route and tie_moe_align in one launch: T <= 64, E <= 256, T (top + shared) <= 1024.
 extern "C" int tie_moe_route_align(const float* logits, int row, const float* bias, const float* correction, int T, int E,
                                    int groups, int keep, int top, int scoring, int group_top, int renormalize,
-                                   float renorm_eps, float weight_scale, int shared, int* ids, float* weights, int real,
+                                   float renorm_eps, float weight_scale, int shared, int shared_gated, int* ids, float* weights, int real,
                                    int tile_rows, int* offsets, int* slot_at, int* where, int* tiles, int max_tiles,
                                    int* num_tiles, hipStream_t stream) {
   if (T <= 0 || T > MOE_FEW_ROWS || E <= 0 || E > MOE_FEW_EXPERTS || groups <= 0 || E % groups != 0 || keep <= 0 ||
       keep > groups || top <= 0 || top > E || group_top <= 0 || group_top > MOE_MAX_GROUP_TOP || shared < 0 ||
-      row < E + (shared > 0 ? 1 : 0) || scoring < SCORE_SOFTMAX || scoring > SCORE_LOGIT ||
+      row < E + (shared > 0 && shared_gated ? 1 : 0) || scoring < SCORE_SOFTMAX || scoring > SCORE_LOGIT ||
       T * (top + shared) > MOE_FEW_SLOTS || real <= 0 || real > MOE_FEW_EXPERTS + MOE_MAX_GROUP_TOP || tile_rows <= 0 ||
       max_tiles < tie_moe_max_tiles(T * (top + shared), real, tile_rows))
     return TIE_BAD_ARGUMENT;
   const size_t lds = sizeof(float) * (2 * static_cast<size_t>(E) + groups) * (ALIGN_THREADS / TIE_WAVE);
   moe_route_align_kernel<<<1, ALIGN_THREADS, lds, stream>>>(
       RouteParams{logits, row, bias, correction, E, groups, keep, top, scoring, group_top, renormalize, renorm_eps,
-                  weight_scale, shared, ids, weights},
+                  weight_scale, shared, shared_gated, ids, weights},
       T, real, tile_rows, AlignOut{offsets, slot_at, where, tiles, max_tiles, num_tiles});
   return tie_launch_status();
 }
@@ -437,7 +438,8 @@ extern "C" int tie_moe_route_align(const float* logits, int row, const float* bi
 // MODE 1 (gated): x rows are gathered (row = slot_at[place] / top), w_a and w_b are the gate and up weights
 // [real][N][K], out[place][c] = silu(a) * b. MODE 3 (gated, sums cut off at a limit): the same rows and weights,
 // out[place][c] = clipped_gate(a, b). MODE 2 (experts without a gate): rows gathered likewise, w_a the up
-// weight, out[place][c] = relu(a)^2. MODE 0: x rows are the places themselves (act [slots][K]), w_a is the down
+// weight, out[place][c] = relu(a)^2. MODE 4 (gated, the expert's input times its slot's weight w): as MODE 1 with
+// out[place][c] = silu(w a) * (w b). MODE 0: x rows are the places themselves (act [slots][K]), w_a is the down
 // weight and out[place][c] = a.
 
 template <typename TX, typename TW, typename TO, int MODE>
@@ -445,7 +447,7 @@ __global__ __launch_bounds__(256) void moe_gemm_generic_kernel(
     const TX* __restrict__ x, const TW* __restrict__ w_a, const TW* __restrict__ w_b, TO* __restrict__ out,
     const int* __restrict__ offsets, const int* __restrict__ slot_at, const int* __restrict__ tiles,
     const int* __restrict__ num_tiles, int top, int N, int K, GateParams gp) {
-  constexpr bool GATED = MODE == 1 || MODE == 3;
+  constexpr bool GATED = MODE == 1 || MODE == 3 || MODE == 4;
   constexpr bool GATHER = MODE != 0;
   const int tile = blockIdx.x;
   if (tile >= *num_tiles) return;
@@ -507,11 +509,13 @@ __global__ __launch_bounds__(256) void moe_gemm_generic_kernel(
   for (int i = 0; i < 2; ++i) {
     const int r = ty * 2 + i;
     if (r >= rows) continue;
+    const float w = MODE == 4 ? gp.slot_weights[slot_at[place0 + r]] : 1.f;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int c = col0 + tx * 4 + j;
       if (c >= N) continue;
-      const float v = MODE == 1   ? silu_f(acc_a[i][j]) * acc_b[i][j]
+      const float v = MODE == 4   ? silu_f(w * acc_a[i][j]) * (w * acc_b[i][j])
+                      : MODE == 1 ? silu_f(acc_a[i][j]) * acc_b[i][j]
                       : MODE == 3 ? clipped_gate_f(acc_a[i][j], acc_b[i][j], gp)
                       : MODE == 2 ? relu_squared_f(acc_a[i][j])
                                   : acc_a[i][j];
@@ -525,14 +529,16 @@ extern "C" int tie_moe_generic_tile_rows() { return GR; }
 // gated = 1: out [slots][N] of out_dtype = silu(x Wa^T) * (x Wb^T) over gathered rows of x [T][K];
 // gated = 3: the same with clipped_gate (limit, slope, shift);
 // gated = 2: out [slots][N] of out_dtype = relu(x Wa^T)^2 over gathered rows of x [T][K];
+// gated = 4: as 1 with the sums times slot_weights [slots] first;
 // gated = 0: out [slots][N] = x Wa^T over x [slots][K]. Weights [real][N][K].
 extern "C" int tie_moe_gemm_generic(const void* x, int x_dtype, const void* w_a, const void* w_b, int w_dtype, void* out,
                                     int out_dtype, int gated, const int* offsets, const int* slot_at, const int* tiles,
                                     const int* num_tiles, int max_tiles, int top, int N, int K, float limit, float slope,
-                                    float shift, hipStream_t stream) {
-  if (max_tiles <= 0 || top <= 0 || N <= 0 || K <= 0 || gated < 0 || gated > 3 || (gated % 2 == 1 && w_b == nullptr))
+                                    float shift, const float* slot_weights, hipStream_t stream) {
+  if (max_tiles <= 0 || top <= 0 || N <= 0 || K <= 0 || gated < 0 || gated > 4 ||
+      ((gated % 2 == 1 || gated == 4) && w_b == nullptr) || (gated == 4 && slot_weights == nullptr))
     return TIE_BAD_ARGUMENT;
-  const GateParams gp{limit, slope, shift};
+  const GateParams gp{limit, slope, shift, slot_weights};
   if ((x_dtype | w_dtype | out_dtype) & ~1) return TIE_BAD_ARGUMENT;
   const dim3 grid(max_tiles, (N + GC - 1) / GC);
   if (grid.y > 65535) return TIE_BAD_ARGUMENT;
@@ -544,6 +550,7 @@ extern "C" int tie_moe_gemm_generic(const void* x, int x_dtype, const void* w_a,
   {                                           \
     if (gated == 1) LAUNCH_G(TX, TW, TO, 1);  \
     else if (gated == 3) LAUNCH_G(TX, TW, TO, 3); \
+    else if (gated == 4) LAUNCH_G(TX, TW, TO, 4); \
     else if (gated == 2) LAUNCH_G(TX, TW, TO, 2); \
     else LAUNCH_G(TX, TW, TO, 0);             \
   }
@@ -593,7 +600,7 @@ __global__ __launch_bounds__(256) void moe_gemm_bf16_kernel(
     void* __restrict__ out, const int* __restrict__ offsets, const int* __restrict__ slot_at,
     const int* __restrict__ tiles, const int* __restrict__ num_tiles, int top, int N, int K, GateParams gp) {
   static_assert(MT == 1 || MT == 4 || MT == 8, "one x tile a wave, or MT / 4 loaded by each of the four waves");
-  constexpr bool GATED = MODE == 1 || MODE == 3;       // two weights, silu(a) * b or clipped_gate(a, b)
+  constexpr bool GATED = MODE == 1 || MODE == 3 || MODE == 4;       // two weights, silu(a) * b or clipped_gate(a, b)
   constexpr bool GATHER = MODE != 0;      // rows of x gathered by slot; the activations go out as bfloat16
   constexpr int OWN = MT == 1 ? 1 : MT / 4;                  // x fragments this wave loads a k-block
   const int tile = blockIdx.x;
@@ -703,6 +710,7 @@ __global__ __launch_bounds__(256) void moe_gemm_bf16_kernel(
   for (int mt = 0; mt < MT; ++mt) {
     const int r = mt * 16 + r16;
     if (r >= rows) continue;
+    const float sw = MODE == 4 ? gp.slot_weights[slot_at[place0 + r]] : 1.f;
 #pragma unroll
     for (int nt = 0; nt < NT; ++nt) {
       const int c = col0 + nt * 16 + quad * 4;
@@ -711,7 +719,8 @@ __global__ __launch_bounds__(256) void moe_gemm_bf16_kernel(
       float v[4];
 #pragma unroll
       for (int i = 0; i < 4; ++i)
-        v[i] = MODE == 1   ? silu_f(acc_a[mt][nt][i]) * acc_b[mt][nt][i]
+        v[i] = MODE == 4   ? silu_f(sw * acc_a[mt][nt][i]) * (sw * acc_b[mt][nt][i])
+               : MODE == 1 ? silu_f(acc_a[mt][nt][i]) * acc_b[mt][nt][i]
                : MODE == 3 ? clipped_gate_f(acc_a[mt][nt][i], acc_b[mt][nt][i], gp)
                : MODE == 2 ? relu_squared_f(acc_a[mt][nt][i])
                            : acc_a[mt][nt][i];
@@ -745,18 +754,20 @@ extern "C" int tie_moe_bf16_tile_rows(int slots, int real) {
 // bfloat16 x and weights; gated = 1: out bfloat16 [slots][N] = silu(x Wa^T) * (x Wb^T) over gathered rows of x;
 // gated = 3: the same with clipped_gate (limit, slope, shift);
 // gated = 2: out bfloat16 [slots][N] = relu(x Wa^T)^2 over gathered rows of x;
+// gated = 4: as 1 with the sums times slot_weights [slots] first;
 // gated = 0: out float32 [slots][N] = x Wa^T over x [slots][K]. tile_rows (16, 64 or 128) as given to tie_moe_align.
 extern "C" int tie_moe_gemm_bf16(const void* x, const void* w_a, const void* w_b, void* out, int gated,
                                  const int* offsets, const int* slot_at, const int* tiles, const int* num_tiles,
                                  int max_tiles, int tile_rows, int top, int N, int K, float limit, float slope,
-                                 float shift, hipStream_t stream) {
-  if (max_tiles <= 0 || top <= 0 || N <= 0 || K <= 0 || K % 8 != 0 || gated < 0 || gated > 3 ||
-      (gated % 2 == 1 && w_b == nullptr) || (tile_rows != 16 && tile_rows != 64 && tile_rows != 128) || reinterpret_cast<uintptr_t>(x) % 16 != 0 ||
+                                 float shift, const float* slot_weights, hipStream_t stream) {
+  const bool two_weights = gated % 2 == 1 || gated == 4;
+  if (max_tiles <= 0 || top <= 0 || N <= 0 || K <= 0 || K % 8 != 0 || gated < 0 || gated > 4 ||
+      (two_weights && w_b == nullptr) || (gated == 4 && slot_weights == nullptr) || (tile_rows != 16 && tile_rows != 64 && tile_rows != 128) || reinterpret_cast<uintptr_t>(x) % 16 != 0 ||
       reinterpret_cast<uintptr_t>(w_a) % 16 != 0 || reinterpret_cast<uintptr_t>(w_b) % 16 != 0 ||
       reinterpret_cast<uintptr_t>(out) % 16 != 0)
     return TIE_BAD_ARGUMENT;
-  const int columns = tile_rows == 16 ? 16 : (tile_rows == 128 && gated % 2 == 1 ? 128 : 256);   // of a workgroup
-  const GateParams gp{limit, slope, shift};
+  const int columns = tile_rows == 16 ? 16 : (tile_rows == 128 && two_weights ? 128 : 256);   // of a workgroup
+  const GateParams gp{limit, slope, shift, slot_weights};
   const dim3 grid(max_tiles, (N + columns - 1) / columns);
   if (grid.y > 65535) return TIE_BAD_ARGUMENT;
 #define LAUNCH_B(MT, NT, G)                                                                                  \
@@ -765,11 +776,11 @@ extern "C" int tie_moe_gemm_bf16(const void* x, const void* w_a, const void* w_b
                                                             static_cast<const bf16_t*>(w_b), out, offsets,   \
                                                             slot_at, tiles, num_tiles, top, N, K, gp)
   if (tile_rows == 128) {
-    if (gated == 1) LAUNCH_B(8, 2, 1); else if (gated == 3) LAUNCH_B(8, 2, 3); else if (gated == 2) LAUNCH_B(8, 4, 2); else LAUNCH_B(8, 4, 0);
+    if (gated == 1) LAUNCH_B(8, 2, 1); else if (gated == 4) LAUNCH_B(8, 2, 4); else if (gated == 3) LAUNCH_B(8, 2, 3); else if (gated == 2) LAUNCH_B(8, 4, 2); else LAUNCH_B(8, 4, 0);
   } else if (tile_rows == 64) {
-    if (gated == 1) LAUNCH_B(4, 4, 1); else if (gated == 3) LAUNCH_B(4, 4, 3); else if (gated == 2) LAUNCH_B(4, 4, 2); else LAUNCH_B(4, 4, 0);
+    if (gated == 1) LAUNCH_B(4, 4, 1); else if (gated == 4) LAUNCH_B(4, 4, 4); else if (gated == 3) LAUNCH_B(4, 4, 3); else if (gated == 2) LAUNCH_B(4, 4, 2); else LAUNCH_B(4, 4, 0);
   } else {
-    if (gated == 1) LAUNCH_B(1, 1, 1); else if (gated == 3) LAUNCH_B(1, 1, 3); else if (gated == 2) LAUNCH_B(1, 1, 2); else LAUNCH_B(1, 1, 0);
+    if (gated == 1) LAUNCH_B(1, 1, 1); else if (gated == 4) LAUNCH_B(1, 1, 4); else if (gated == 3) LAUNCH_B(1, 1, 3); else if (gated == 2) LAUNCH_B(1, 1, 2); else LAUNCH_B(1, 1, 0);
   }
 #undef LAUNCH_B
   return tie_launch_status();
@@ -788,7 +799,7 @@ __global__ void moe_combine_kernel(const float* __restrict__ parts, const int* _
   for (int k = 0; k < top; ++k) {
     const int at = where[t * top + k];
     const float part = at >= 0 ? parts[static_cast<size_t>(at) * n + i] : load_as_float(self + t * n + i);
-    y = fmaf(weights[t * top + k], part, y);
+    y = fmaf(weights != nullptr ? weights[t * top + k] : 1.f, part, y);
   }
   out[t * n + i] = accumulate ? out[t * n + i] + y : y;
 }

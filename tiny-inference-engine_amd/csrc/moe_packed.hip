@@ -28,7 +28,7 @@ template <int MODE, int NT>
 __global__ __launch_bounds__(256) void moe_packed_few_rows_kernel(const bf16_t* __restrict__ x,
                                                                   const bf16_t* __restrict__ w, void* __restrict__ out,
                                                                   MoeRows rw, int N, int K, GateParams gp) {
-  constexpr bool GATED = MODE == 1 || MODE == 3;
+  constexpr bool GATED = MODE == 1 || MODE == 3 || MODE == 4;
   constexpr bool GATHER = MODE != 0;
   const int tile = blockIdx.x;
   if (tile >= *rw.num_tiles) return;                         // the whole workgroup leaves
@@ -81,6 +81,7 @@ __global__ __launch_bounds__(256) void moe_packed_few_rows_kernel(const bf16_t* 
     floatx4_t v = sums[nt][0][lane];
 #pragma unroll
     for (int p = 1; p < 4; ++p) v += sums[nt][p][lane];
+    if constexpr (MODE == 4) v *= gp.slot_weights[rw.slot_at[place]];
     if constexpr (GATED) {
       float u[4];
 #pragma unroll
@@ -112,7 +113,7 @@ __global__ __launch_bounds__(256) void moe_packed_many_rows_kernel(const bf16_t*
                                                                    MoeRows rw, int x_rows, int N, int K, int tiles_n,
                                                                    GateParams gp) {
 #if defined(__HIP_DEVICE_COMPILE__)
-  constexpr bool GATED = MODE == 1 || MODE == 3;
+  constexpr bool GATED = MODE == 1 || MODE == 3 || MODE == 4;
   constexpr bool GATHER = MODE != 0;
   constexpr int TN = BN / 64, TM = BM / 64;
   extern __shared__ bf16_t lds[];
@@ -154,16 +155,18 @@ __global__ __launch_bounds__(256) void moe_packed_many_rows_kernel(const bf16_t*
   for (int i = 0; i < TM; ++i) {
     const int m = wm * (BM / 2) + i * 32 + fr;
     if (m >= rows) continue;
+    const float sw = MODE == 4 ? gp.slot_weights[rw.slot_at[place0 + m]] : 1.f;
 #pragma unroll
     for (int j = 0; j < TN; ++j) {
 #pragma unroll
       for (int g = 0; g < 4; ++g) {
         const int n = col0 + wn * (BN / 2) + j * 32 + 8 * g + 4 * fk;
         if (n >= N) continue;
-        const float v0 = acc[i][j][4 * g], v1 = acc[i][j][4 * g + 1], v2 = acc[i][j][4 * g + 2], v3 = acc[i][j][4 * g + 3];
+        float v0 = acc[i][j][4 * g], v1 = acc[i][j][4 * g + 1], v2 = acc[i][j][4 * g + 2], v3 = acc[i][j][4 * g + 3];
         if constexpr (GATED) {
           if (g & 1) continue;                 // the ups of group g are register group g + 1
-          const float u0 = acc[i][j][4 * g + 4], u1 = acc[i][j][4 * g + 5], u2 = acc[i][j][4 * g + 6], u3 = acc[i][j][4 * g + 7];
+          float u0 = acc[i][j][4 * g + 4], u1 = acc[i][j][4 * g + 5], u2 = acc[i][j][4 * g + 6], u3 = acc[i][j][4 * g + 7];
+          if constexpr (MODE == 4) v0 *= sw, v1 *= sw, v2 *= sw, v3 *= sw, u0 *= sw, u1 *= sw, u2 *= sw, u3 *= sw;
           uint2 packed;
           packed.x = pack_bf16x2(gated_fast<MODE>(v0, u0, gp), gated_fast<MODE>(v1, u1, gp));
           packed.y = pack_bf16x2(gated_fast<MODE>(v2, u2, gp), gated_fast<MODE>(v3, u3, gp));
@@ -214,21 +217,21 @@ static int launch_many_rows(const void* x, const void* w, void* out, const MoeRo
   return tie_launch_status();
 }
 
-// x bfloat16 [x_rows][K]; w packed, [real * N][K] (N counts gate and up rows where gated); mode 1 or 3: out bfloat16
+// x bfloat16 [x_rows][K]; w packed, [real * N][K] (N counts gate and up rows where gated); mode 1, 3 or 4: out bfloat16
 // [slots][N / 2]; mode 2: out bfloat16 [slots][N]; mode 0: x_rows = slots, out float32 [slots][N]. tile_rows (16, 64,
 // 128 or 256) as given to tie_moe_align; columns: the columns a workgroup takes (128 or 256; tiles of 64 rows on), or 0
 // to choose.
 extern "C" int tie_moe_gemm_packed(const void* x, int x_rows, const void* w, void* out, int mode, const int* offsets,
                                    const int* slot_at, const int* tiles, const int* num_tiles, int max_tiles,
                                    int tile_rows, int columns, int top, int N, int K, float limit, float slope,
-                                   float shift, hipStream_t stream) {
-  if (x_rows <= 0 || max_tiles <= 0 || top <= 0 || N <= 0 || N % 16 || K < 96 || K % 32 || mode < 0 || mode > 3 ||
+                                   float shift, const float* slot_weights, hipStream_t stream) {
+  if ((mode == 4 && slot_weights == nullptr) || x_rows <= 0 || max_tiles <= 0 || top <= 0 || N <= 0 || N % 16 || K < 96 || K % 32 || mode < 0 || mode > 4 ||
       (columns != 0 && columns != 128 && columns != 256) || static_cast<size_t>(x_rows) * K * 2 > 0x7fffffffu ||
       static_cast<size_t>(K) * 512 > 0x7fffffffu || reinterpret_cast<uintptr_t>(x) % 16 ||
       reinterpret_cast<uintptr_t>(w) % 16 || reinterpret_cast<uintptr_t>(out) % 16)
     return TIE_BAD_ARGUMENT;
   const MoeRows rw{offsets, slot_at, tiles, num_tiles, top};
-  const GateParams gp{limit, slope, shift};
+  const GateParams gp{limit, slope, shift, slot_weights};
   if (tile_rows == 16) {
     const dim3 grid(max_tiles, (N / 16 + 1) / 2);
     if (grid.y > 65535) return TIE_BAD_ARGUMENT;
@@ -238,6 +241,7 @@ extern "C" int tie_moe_gemm_packed(const void* x, int x_rows, const void* w, voi
     if (mode == 0) FEW(0);
     else if (mode == 1) FEW(1);
     else if (mode == 2) FEW(2);
+    else if (mode == 4) FEW(4);
     else FEW(3);
 #undef FEW
     return tie_launch_status();
@@ -246,6 +250,7 @@ extern "C" int tie_moe_gemm_packed(const void* x, int x_rows, const void* w, voi
   (mode == 0   ? launch_many_rows<BM, BN, 0>(x, w, out, rw, max_tiles, x_rows, N, K, gp, stream)         \
    : mode == 1 ? launch_many_rows<BM, BN, 1>(x, w, out, rw, max_tiles, x_rows, N, K, gp, stream)         \
    : mode == 2 ? launch_many_rows<BM, BN, 2>(x, w, out, rw, max_tiles, x_rows, N, K, gp, stream)         \
+   : mode == 4 ? launch_many_rows<BM, BN, 4>(x, w, out, rw, max_tiles, x_rows, N, K, gp, stream)         \
                : launch_many_rows<BM, BN, 3>(x, w, out, rw, max_tiles, x_rows, N, K, gp, stream))
   if (columns == 0) columns = tile_rows == 64 ? 128 : 256;
   if (tile_rows == 64) return columns == 128 ? MANY(64, 128) : MANY(64, 256);

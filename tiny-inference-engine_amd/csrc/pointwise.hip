@@ -110,3 +110,33 @@ extern "C" int tie_token_gate(const float* gate, const int* tokens, const void* 
 #undef TG
   return tie_launch_status();
 }
+
+// ------------------------------------------------------------------ a gate on rows
+// rows[t][c] *= sigmoid(gate[t][c]) in float32, in place; gate rows are gate_row floats apart. VEC columns a thread.
+template <typename T, int VEC>
+__global__ void gate_rows_kernel(T* __restrict__ rows, const float* __restrict__ gate, int gate_row, int pieces) {
+  const int p = blockIdx.x * blockDim.x + threadIdx.x;
+  if (p >= pieces) return;
+  const size_t t = blockIdx.y;
+  T* r = rows + (t * pieces + p) * VEC;
+  const float* g = gate + t * gate_row + static_cast<size_t>(p) * VEC;
+  float v[VEC];
+#pragma unroll
+  for (int i = 0; i < VEC; ++i) v[i] = load_as_float(r + i) * (1.0f / (1.0f + expf(-g[i])));
+#pragma unroll
+  for (int i = 0; i < VEC; ++i) store_from_float(r + i, v[i]);
+}
+
+extern "C" int tie_gate_rows(void* rows, int dtype, const float* gate, int gate_row, int T, int n, hipStream_t stream) {
+  if (rows == nullptr || gate == nullptr || T <= 0 || T > 65535 || n <= 0 || gate_row < n) return TIE_BAD_ARGUMENT;
+  const int vec = n % 4 == 0 ? 4 : 1, pieces = n / vec;
+  const dim3 grid((pieces + 255) / 256, T);
+#define GATE(TYPE, VEC) gate_rows_kernel<TYPE, VEC><<<grid, 256, 0, stream>>>(static_cast<TYPE*>(rows), gate, gate_row, pieces)
+  if (dtype == TIE_F32 && vec == 4) GATE(float, 4);
+  else if (dtype == TIE_F32) GATE(float, 1);
+  else if (dtype == TIE_BF16 && vec == 4) GATE(bf16_t, 4);
+  else if (dtype == TIE_BF16) GATE(bf16_t, 1);
+  else return TIE_BAD_ARGUMENT;
+#undef GATE
+  return tie_launch_status();
+}

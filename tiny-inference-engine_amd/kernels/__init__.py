@@ -59,6 +59,7 @@ _SOURCES = {
     "moe": ("tie_moe", "moe.hip"),
     "moe_packed": ("tie_moe_packed", "moe_packed.hip"),
     "recurrent": ("tie_recurrent", "recurrent.hip"),
+    "matrix_state": ("tie_matrix_state", "matrix_state.hip"),
     "hyper": ("tie_hyper", "hyper.hip"),
     "delta_rule": ("tie_delta_rule", "delta_rule.hip"),
     "delta_chunks": ("tie_delta_chunks", "delta_chunks.hip"),
@@ -103,7 +104,7 @@ _SIGNATURES = {
                                       _c_void, _c_void, _c_int, _c_int, _c_int, _c_void, _c_void],
         "tie_norm_add_norm": [_c_void, _c_long, _c_int, _c_void, _c_void, _c_void, _c_void, _c_int, _c_int, _c_void,
                               _c_float, _c_void, _c_void, _c_float, _c_void, _c_int, _c_int, _c_int, _c_void],
-        "tie_gelu": [_c_void, _c_int, _c_void, _c_int, ctypes.c_longlong, _c_void],
+        "tie_gelu": [_c_void, _c_int, _c_void, _c_int, ctypes.c_longlong, _c_int, _c_void],
         "tie_add_partials_rms_norm": [_c_void, _c_void, _c_long, _c_int, _c_void, _c_float, _c_void, _c_int, _c_int,
                                       _c_int, _c_void],
         "tie_argmax": [_c_void, _c_void, _c_void, _c_void, _c_void, _c_int, _c_int, _c_void],
@@ -113,24 +114,24 @@ _SIGNATURES = {
     },
     "moe": {
         "tie_moe_route": [_c_void, _c_int, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
-                          _c_int, _c_float, _c_float, _c_int, _c_void, _c_void, _c_void],
+                          _c_int, _c_float, _c_float, _c_int, _c_int, _c_void, _c_void, _c_void],
         "tie_moe_route_align": [_c_void, _c_int, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
-                                _c_int, _c_float, _c_float, _c_int, _c_void, _c_void, _c_int, _c_int, _c_void, _c_void,
+                                _c_int, _c_float, _c_float, _c_int, _c_int, _c_void, _c_void, _c_int, _c_int, _c_void, _c_void,
                                 _c_void, _c_void, _c_int, _c_void, _c_void],
         "tie_moe_max_tiles": [_c_int, _c_int, _c_int],
         "tie_moe_align": [_c_void, _c_int, _c_int, _c_int, _c_void, _c_void, _c_void, _c_void, _c_int, _c_void, _c_void],
         "tie_moe_generic_tile_rows": [],
         "tie_moe_gemm_generic": [_c_void, _c_int, _c_void, _c_void, _c_int, _c_void, _c_int, _c_int, _c_void, _c_void,
-                                 _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_void],
+                                 _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_void, _c_void],
         "tie_moe_bf16_tile_rows": [_c_int, _c_int],
         "tie_moe_gemm_bf16": [_c_void, _c_void, _c_void, _c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_int,
-                              _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_void],
+                              _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_void, _c_void],
         "tie_moe_combine": [_c_void, _c_void, _c_void, _c_void, _c_int, _c_void, _c_int, _c_int, _c_int, _c_int, _c_void],
     },
     "moe_packed": {
         "tie_moe_packed_tile_rows": [_c_int, _c_int, _c_int],
         "tie_moe_gemm_packed": [_c_void, _c_int, _c_void, _c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_int,
-                                _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_void],
+                                _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_void, _c_void],
     },
     "gemm_generic": {
         "tie_gemm_generic": [_c_void, _c_int, _c_void, _c_int, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int,
@@ -148,6 +149,17 @@ _SIGNATURES = {
         "tie_min_gru_scan": [_c_void, _c_int, _c_void, _c_int, _c_void, _c_void, _c_void, _c_int, _c_int, _c_void,
                              _c_void, _c_int, _c_void, _c_void, _c_void],
     },
+    "matrix_state": {
+        "tie_matrix_state_walk_cols": [],
+        "tie_matrix_state_walk": [_c_int, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_void, _c_int, _c_void,
+                                  _c_void, _c_void, _c_int, _c_int, _c_float, _c_void, _c_void, _c_void, _c_void, _c_void,
+                                  _c_int, _c_int, _c_int, _c_int, _c_void],
+        "tie_matrix_state_chunks": [_c_int, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_void, _c_void,
+                                    _c_void, _c_int, _c_int, _c_float, _c_void, _c_void, _c_void, _c_void, _c_void, _c_void,
+                                    _c_int, _c_int, _c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
+                                    _c_void],
+        "tie_rotate_heads": [_c_void, _c_int, _c_int, _c_int, _c_void, _c_int, _c_int, _c_int, _c_int, _c_void],
+    },
     "hyper": {
         "tie_layer_norm": [_c_void, _c_int, _c_void, _c_float, _c_void, _c_int, _c_void, _c_int, _c_int, _c_void],
         "tie_hyper_connection": [_c_void, _c_long, _c_int, _c_int, _c_void, _c_int, _c_void, _c_long, _c_int, _c_void,
@@ -163,7 +175,7 @@ _SIGNATURES = {
                                  _c_int, _c_int, _c_int, _c_void],
         "tie_gated_delta_scan_chunked": [_c_void, _c_int, _c_void, _c_int, _c_void, _c_void, _c_int, _c_void, _c_void,
                                          _c_int, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_void],
-        "tie_grouped_gated_rms_norm": [_c_void, _c_int, _c_void, _c_float, _c_void, _c_int, _c_int, _c_void, _c_int,
+        "tie_grouped_gated_rms_norm": [_c_void, _c_int, _c_void, _c_int, _c_float, _c_void, _c_int, _c_int, _c_void, _c_int,
                                        _c_int, _c_int, _c_int, _c_void],
     },
     "delta_chunks": {
@@ -175,12 +187,15 @@ _SIGNATURES = {
     "pointwise": {
         "tie_dynamic_tanh": [_c_void, _c_void, _c_long, _c_int, _c_void, _c_void, _c_void, _c_void, _c_int, _c_void,
                              _c_int, _c_int, _c_int, _c_void],
+        "tie_gate_rows": [_c_void, _c_int, _c_void, _c_int, _c_int, _c_int, _c_void],
         "tie_token_gate": [_c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_void, _c_int, _c_int, _c_int, _c_void],
     },
     "residual": {
         "tie_add_results": [_c_void, _c_float, _c_void, _c_long, _c_int, _c_void, _c_long, _c_int, _c_void, _c_void,
                             _c_void, _c_void, _c_int, _c_int, _c_void, _c_float, _c_int, _c_void, _c_int, _c_int,
                             _c_int, _c_void],
+        "tie_add_normed_results": [_c_void] + 2 * [_c_void, _c_long, _c_int, _c_void, _c_float] +
+                                  [_c_void, _c_float, _c_void, _c_int, _c_int, _c_int, _c_void],
     },
     "latent": {
         "tie_rms_norm_columns": [_c_void, _c_int, _c_void, _c_float, _c_void, _c_int, _c_int, _c_int, _c_void],
@@ -485,14 +500,17 @@ def swiglu(gate_up: torch.Tensor, out: torch.Tensor, activation: str = "silu") -
                                           _stream())
 
 
-def gelu(x: torch.Tensor, out: torch.Tensor) -> None:
-    """out = 0.5 x (1 + erf(x / sqrt 2)), the exact gelu, element by element in float32."""
+def gelu(x: torch.Tensor, out: torch.Tensor, form: str = "erf") -> None:
+    """out = 0.5 x (1 + erf(x / sqrt 2)), the exact gelu, element by element in float32; ``form`` "tanh":
+    ``0.5 x (1 + tanh(sqrt(2 / pi) (x + 0.044715 x^3)))``."""
+    if form not in ("erf", "tanh"):
+        raise InvalidArgument(f"gelu has the forms 'erf' and 'tanh', not '{form}'")
     _gpu(x, "gelu input")
     _gpu(out, "gelu output")
     if x.numel() != out.numel():
         raise InvalidArgument("gelu: sizes differ")
     _call(_lib("elementwise").tie_gelu, "gelu", x.data_ptr(), _code(x, "gelu input"), out.data_ptr(),
-          _code(out, "gelu output"), x.numel(), _stream())
+          _code(out, "gelu output"), x.numel(), int(form == "tanh"), _stream())
 
 
 def poly_norm(z: torch.Tensor, coeff: torch.Tensor, eps: float, out: torch.Tensor) -> None:
@@ -517,7 +535,7 @@ def scale_softcap(x: torch.Tensor, scale: float = 1.0, cap: Optional[float] = No
 class RoutedParts:
     """A routed feed-forward's result before it is combined: the chosen experts' results by place
     (``parts`` float32 ``[slots, n]``), each row's places (``where`` int32 ``[T, top]``, -1 for an expert that returns
-    its input), weights (float32 ``[T, top]``) and the input rows themselves (``self_rows`` ``[T, n]``)."""
+    its input), weights (float32 ``[T, top]``, or None: all 1) and the input rows themselves (``self_rows`` ``[T, n]``)."""
 
     __slots__ = ("parts", "where", "weights", "self_rows")
 
@@ -542,10 +560,11 @@ def norm_add_norm(y, w_post: torch.Tensor, eps_post: float, x: torch.Tensor, w_n
         parts, where, weights, self_rows = y.parts, y.where, y.weights, y.self_rows
         _f32(parts, "the experts' results")
         _i32(where, "places")
-        _f32(weights, "routing weights")
         _gpu(self_rows, "the feed-forward's input rows")
         top = where.shape[1]
-        if parts.shape[-1] != n or tuple(where.shape) != (T, top) or tuple(weights.shape) != (T, top) or \
+        if weights is not None:
+            _f32(weights, "routing weights", (T, top))
+        if parts.shape[-1] != n or tuple(where.shape) != (T, top) or \
                 tuple(self_rows.shape) != (T, n):
             raise InvalidArgument("norm_add_norm: the routed parts do not fit the stream")
         self_code = _code(self_rows, "the feed-forward's input rows")
@@ -599,6 +618,18 @@ def add_bias(rows: torch.Tensor, bias: torch.Tensor) -> None:
     _f32(bias, "bias", (rows.shape[1],))
     _call(_lib("elementwise").tie_add_bias, "add_bias", rows.data_ptr(), _code(rows, "rows"), rows.shape[0],
           rows.shape[1], bias.data_ptr(), _stream())
+
+
+def gate_rows(rows: torch.Tensor, gate: torch.Tensor) -> None:
+    """rows *= sigmoid(gate), element by element in float32, in place; ``gate`` float32 rows that may lie further apart."""
+    _gpu(rows, "gated rows")
+    _gpu_strided(gate, "gate rows")
+    if gate.dtype != torch.float32 or rows.dim() != 2 or gate.shape != rows.shape or gate.stride(1) != 1:
+        raise InvalidArgument(f"gate rows {list(gate.shape)} {gate.dtype} do not fit float32 {list(rows.shape)}")
+    if rows.numel() == 0:
+        return
+    _call(_lib("pointwise").tie_gate_rows, "gate_rows", rows.data_ptr(), _code(rows, "gated rows"), gate.data_ptr(),
+          gate.stride(0), rows.shape[0], rows.shape[1], _stream())
 
 
 def scale_rows(rows: torch.Tensor, row_scale: "RowScale") -> None:
@@ -1679,7 +1710,6 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
 
 
 # ------------------------------------------------------------------ mixers with a state of fixed size
-DECAY_ATTENTION_MAX_DIM = 512      # rows of a head's state the scan kernel keeps in registers (a quarter of them a wave)
 SCAN_CHUNK_ROWS = 64               # rows of a chunk where a long portion's recurrence runs chunk beside chunk
 SCAN_CHUNKS_FROM = 128             # a step's longest portion from which the recurrences run in chunks
 
@@ -1719,45 +1749,111 @@ def scan_chunks(batch, device, rows: int = SCAN_CHUNK_ROWS, force: bool = False)
     return memo
 
 
-def decay_attention_scan(proj: torch.Tensor, out: torch.Tensor, state: torch.Tensor, query_start: torch.Tensor,
-                         state_slots: torch.Tensor, decay: torch.Tensor, num_seqs: int, heads: int, key_dim: int,
-                         value_dim: int, activation: str = "silu", chunks: Optional[ScanChunks] = None,
-                         scratch=None) -> None:
-    """Linear attention with a decay per head, token by token through each sequence's state.
+# ------------------------------------------------------- mixers that keep a matrix a head
+MATRIX_STATE_MAX_DIM = 512         # STATE_MAX_D of csrc/matrix_state.hip: rows of a head's matrix
+STATE_WALK_COLS = 32               # WALK_COLS there: value columns of a workgroup of the walk
+CHUNK_STATE_SCRATCH_MAX = 1 << 30  # bytes of chunk states above which the heads of a step run in several passes
 
-    ``S_t = decay[h] * S_(t-1) + k_t v_t^T``, ``out_t = S_t^T q_t`` with ``q, k, v = act(proj columns)``; ``proj``
-    float32 rows ``[q (heads * key_dim) | k (heads * key_dim) | v (heads * value_dim) | ...]``; ``state`` float32
-    ``[slots, heads, key_dim, value_dim]``, read at and written back to ``state_slots[s]`` for the rows
-    ``query_start[s] .. query_start[s + 1] - 1`` of every sequence s. ``out`` float32 ``[T, heads * value_dim]``.
 
-    With ``chunks`` (``scan_chunks``; ``scratch(name, shape, dtype)`` hands out the memory for the chunks' states)
-    the rows run chunk beside chunk in three launches: every chunk from zero, the chunks' states combined in
-    order, every chunk again from its true start. The same values up to rounding."""
+def memory_norm_shape(heads: int, key_dim: int, value_dim: int) -> tuple:
+    """The shape of the state a ``matrix_memory`` keeps beside its matrices: per head one copy of (n, m) for each block of
+    value columns the walk works on."""
+    return heads, -(-value_dim // STATE_WALK_COLS), key_dim + 1
+
+
+def _matrix_state(kind: int, proj: torch.Tensor, out: torch.Tensor, state: torch.Tensor, norm_state,
+                  query_start: torch.Tensor, state_slots: torch.Tensor, num_seqs: int, heads: int, key_dim: int, value_dim: int, activation: str, q_scale: float, factors: tuple, rotation, chunks, scratch,
+                  what: str) -> None:
+    """Both kinds of recurrence: ``factors`` are (decay, i_bias, f_bias, i_col, f_col, cap) as the kernels take them."""
     _gpu_strided(proj, "projection rows")
-    if proj.dtype != torch.float32:
+    if proj.dtype != torch.float32 or proj.stride(1) != 1:
         raise InvalidArgument(f"projection rows must be float32, got {proj.dtype}")
-    T = proj.shape[0]
-    _f32(out, "linear attention output", (T, heads * value_dim))
-    _f32(state, "linear attention state")
+    T, width = proj.shape
+    qk, v = heads * key_dim, heads * value_dim
+    _f32(out, f"{what} output", (T, v))
+    _f32(state, f"{what} state")
     if state.dim() != 4 or tuple(state.shape[1:]) != (heads, key_dim, value_dim):
         raise InvalidArgument(f"state {list(state.shape)} does not fit {heads} heads of {key_dim} x {value_dim}")
-    if key_dim > DECAY_ATTENTION_MAX_DIM:
-        raise InvalidArgument(f"a key size of {key_dim} exceeds the {DECAY_ATTENTION_MAX_DIM} this kernel takes")
-    if proj.shape[1] < heads * (2 * key_dim + value_dim):
-        raise InvalidArgument(f"projection rows hold {proj.shape[1]} values, {heads * (2 * key_dim + value_dim)} are needed")
+    if key_dim > MATRIX_STATE_MAX_DIM:
+        raise InvalidArgument(f"a key size of {key_dim} exceeds the {MATRIX_STATE_MAX_DIM} these kernels take")
+    if width < 2 * qk + v:
+        raise InvalidArgument(f"projection rows hold {width} values, {2 * qk + v} are needed")
     if activation not in ("silu", "none"):
         raise InvalidArgument(f"activation '{activation}' (supported: silu, none)")
     _i32(query_start, "query_start", num_seqs + 1)
     _i32(state_slots, "state slots", num_seqs)
+    angles, rot = None, 0
+    if rotation is not None:
+        angles, rot = rotation
+        _f32(angles, "rotation angles", (T, rot))
+        if rot % 2 or not 0 < rot <= key_dim:
+            raise InvalidArgument(f"{rot} rotated dimensions do not fit heads of {key_dim}")
+    decay, i_bias, f_bias, i_col, f_col, cap = factors
+    lib, silu = _lib("matrix_state"), int(activation == "silu")
+    if chunks is None:
+        _call(lib.tie_matrix_state_walk, what, kind, proj.data_ptr(), proj.stride(0), 0, qk, 2 * qk, silu, float(q_scale),
+              _ptr(angles), rot, _ptr(decay), _ptr(i_bias), _ptr(f_bias), i_col, f_col, float(cap), out.data_ptr(),
+              state.data_ptr(), _ptr(norm_state), query_start.data_ptr(), state_slots.data_ptr(),
+              num_seqs, heads, key_dim, value_dim, _stream())
+        return
+    if rotation is not None:
+        _call(lib.tie_rotate_heads, "rotate_heads", proj.data_ptr(), proj.stride(0), 0, qk, angles.data_ptr(), rot, T, heads,
+              key_dim, _stream())
+    per = key_dim * value_dim + (key_dim if kind else 0)
+    fit = max(1, min(heads, CHUNK_STATE_SCRATCH_MAX // (4 * per * chunks.count)))
+    states = scratch("scan.chunk_states", (chunks.count, fit, per), torch.float32)
+    sums = scratch("scan.chunk_sums", (chunks.count, fit, 2), torch.float64) if kind else None
+    starts = scratch("scan.chunk_starts", (chunks.count, fit), torch.float32) if kind else None
+    for first in range(0, heads, fit):
+        _call(lib.tie_matrix_state_chunks, what, kind, proj.data_ptr(), proj.stride(0), 0, qk, 2 * qk, silu,
+              float(q_scale), _ptr(decay), _ptr(i_bias), _ptr(f_bias), i_col, f_col, float(cap), out.data_ptr(),
+              state.data_ptr(), _ptr(norm_state), state_slots.data_ptr(), chunks.items.data_ptr(),
+              chunks.first_item.data_ptr(), chunks.count, chunks.longest, states.data_ptr(), _ptr(sums), _ptr(starts),
+              first, min(fit, heads - first), num_seqs, heads, key_dim, value_dim, _stream())
+
+
+def decay_attention_scan(proj: torch.Tensor, out: torch.Tensor, state: torch.Tensor, query_start: torch.Tensor,
+                         state_slots: torch.Tensor, decay: torch.Tensor, num_seqs: int, heads: int, key_dim: int,
+                         value_dim: int, activation: str = "silu", chunks: Optional[ScanChunks] = None, scratch=None,
+                         q_scale: float = 1.0, rotation=None) -> None:
+    """Linear attention with a decay per head through each sequence's state.
+
+    ``S_t = decay[h] * S_(t-1) + k_t v_t^T``, ``out_t = S_t^T q_t`` with ``q, k, v = act(proj columns)``, q then times
+    ``q_scale``; ``proj`` float32 rows ``[q (heads * key_dim) | k (heads * key_dim) | v (heads * value_dim) | ...]``;
+    ``state`` float32 ``[slots, heads, key_dim, value_dim]``, read at and written back to ``state_slots[s]`` for the rows
+    ``query_start[s] .. query_start[s + 1] - 1`` of every sequence s. ``out`` float32 ``[T, heads * value_dim]``.
+    ``rotation`` ``(angles, dims)``: the first ``dims`` dimensions of q and k turn by position, i paired with
+    ``i + dims / 2``, ``angles`` float32 ``[T, dims]`` from ``rope_angles`` (no activation beside it; with ``chunks`` the rows
+    of ``proj`` are rotated in place).
+
+    With ``chunks`` (``scan_chunks``; ``scratch(name, shape, dtype)`` hands out the memory for the chunks' states)
+    the rows run chunk beside chunk in three launches: every chunk from zero, the chunks' states combined in
+    order, every chunk's outputs from its true start. The same values up to rounding."""
     _f32(decay, "decay", (heads,))
-    chunk_states = None
-    if chunks is not None:
-        chunk_states = scratch("scan.chunk_states", (chunks.count, heads, key_dim, value_dim), torch.float32)
-    _call(_lib("recurrent").tie_decay_attention_scan, "decay_attention_scan", proj.data_ptr(), proj.stride(0),
-          out.data_ptr(), state.data_ptr(), query_start.data_ptr(), state_slots.data_ptr(), decay.data_ptr(),
-          num_seqs, heads, key_dim, value_dim, int(activation == "silu"),
-          _ptr(chunks.items) if chunks else None, _ptr(chunks.first_item) if chunks else None,
-          chunks.count if chunks else 0, _ptr(chunk_states), chunks.longest if chunks else 0, _stream())
+    if rotation is not None and activation != "none":
+        raise InvalidArgument("queries and keys are either rotated or activated")
+    _matrix_state(0, proj, out, state, None, query_start, state_slots, num_seqs, heads, key_dim, value_dim, activation, q_scale,
+                  (decay, None, None, 0, 0, 1.0), rotation, chunks, scratch, "decay_attention_scan")
+
+
+def matrix_memory_scan(proj: torch.Tensor, out: torch.Tensor, state: torch.Tensor, norm_state: torch.Tensor,
+                       query_start: torch.Tensor, state_slots: torch.Tensor, gate_column: int, i_bias: torch.Tensor,
+                       f_bias: torch.Tensor, cap: float, num_seqs: int, heads: int, key_dim: int, value_dim: int,
+                       q_scale: float = 1.0, chunks: Optional[ScanChunks] = None, scratch=None) -> None:
+    """A matrix memory with exponential gates through each sequence's state (``csrc/matrix_state.hip`` has the equations).
+
+    ``proj`` as for ``decay_attention_scan``; columns ``gate_column + h`` and ``gate_column + heads + h`` hold head h's input
+    and forget gate before their biases. ``state`` likewise, ``norm_state`` float32 ``[slots, *memory_norm_shape(...)]``."""
+    _f32(i_bias, "input gate bias", (heads,))
+    _f32(f_bias, "forget gate bias", (heads,))
+    _f32(norm_state, "the memory's normaliser")
+    if tuple(norm_state.shape[1:]) != memory_norm_shape(heads, key_dim, value_dim) or \
+            norm_state.shape[0] != state.shape[0]:
+        raise InvalidArgument(f"normaliser {list(norm_state.shape)} does not fit {heads} heads of {key_dim} x {value_dim}")
+    if gate_column < 0 or gate_column + 2 * heads > proj.shape[1] or not cap > 0:
+        raise InvalidArgument(f"gate columns from {gate_column} on (cap {cap}) do not fit rows of {proj.shape[1]}")
+    _matrix_state(1, proj, out, state, norm_state, query_start, state_slots, num_seqs, heads, key_dim, value_dim, "none", q_scale,
+                  (None, i_bias, f_bias, gate_column, gate_column + heads, cap), None, chunks, scratch, "matrix_memory_scan")
 
 
 def gated_rms_norm(o: torch.Tensor, weight: torch.Tensor, eps: float, gate: torch.Tensor, out: torch.Tensor) -> None:
@@ -1814,11 +1910,11 @@ MOE_MAX_GROUP_TOP = 8         # MOE_MAX_GROUP_TOP of csrc/moe.hip
 MOE_SCORINGS = {"softmax": 0, "sigmoid": 1, "softmax_chosen": 2}     # SCORE_* of csrc/moe.hip
 
 
-def _check_router(logits: torch.Tensor, top: int, shared: int):
+def _check_router(logits: torch.Tensor, top: int, shared: int, shared_gated: bool):
     _gpu_strided(logits, "router logits")
     if logits.dtype != torch.float32:
         raise InvalidArgument(f"router logits must be float32, got {logits.dtype}")
-    return logits.shape[0], logits.shape[1] - (1 if shared else 0), top + shared
+    return logits.shape[0], logits.shape[1] - (1 if shared and shared_gated else 0), top + shared
 
 
 # Up to here one workgroup routes all rows of a step and sorts their slots in the same launch (MOE_FEW_* of csrc/moe.hip).
@@ -1828,14 +1924,14 @@ MOE_FEW_ROWS, MOE_FEW_EXPERTS, MOE_FEW_SLOTS = 64, 256, 1024
 def moe_route_align(logits: torch.Tensor, correction: Optional[torch.Tensor], groups: int, keep: int, top: int,
                     ids: torch.Tensor, weights: torch.Tensor, real: int, tile_rows: int, scratch, scoring: str = "softmax",
                     group_top: int = 1, renormalize: bool = False, renorm_eps: float = 0.0, weight_scale: float = 1.0,
-                    shared: int = 0, bias: Optional[torch.Tensor] = None) -> "ExpertRows":
+                    shared: int = 0, bias: Optional[torch.Tensor] = None, shared_gated: bool = True) -> "ExpertRows":
     """``moe_route`` and then ``moe_align``; in steps of few rows as one launch."""
-    T, E, slots = _check_router(logits, top, shared)
+    T, E, slots = _check_router(logits, top, shared, shared_gated)
     few = T <= MOE_FEW_ROWS and E <= MOE_FEW_EXPERTS and T * slots <= MOE_FEW_SLOTS and \
         0 < real <= MOE_FEW_EXPERTS + MOE_MAX_GROUP_TOP
     if not few or T == 0:
         moe_route(logits, correction, groups, keep, top, ids, weights, scoring, group_top, renormalize, renorm_eps,
-                  weight_scale, shared, bias)
+                  weight_scale, shared, bias, shared_gated)
         return moe_align(ids, real, tile_rows, scratch)
     if correction is not None:
         _f32(correction, "the choice's correction", (E,))
@@ -1850,7 +1946,7 @@ def moe_route_align(logits: torch.Tensor, correction: Optional[torch.Tensor], gr
     rows = _expert_rows(T, slots, real, tile_rows, scratch)
     _call(_lib("moe").tie_moe_route_align, "moe_route_align", logits.data_ptr(), logits.stride(0), _ptr(bias),
           _ptr(correction), T, E, groups, keep, top, MOE_SCORINGS[scoring], int(group_top), int(bool(renormalize)),
-          float(renorm_eps), float(weight_scale), int(shared), ids.data_ptr(), weights.data_ptr(), real, tile_rows,
+          float(renorm_eps), float(weight_scale), int(shared), int(bool(shared_gated)), ids.data_ptr(), weights.data_ptr(), real, tile_rows,
           rows.offsets.data_ptr(), rows.slot_at.data_ptr(), rows.where.data_ptr(), rows.tiles.data_ptr(),
           rows.max_tiles, rows.num_tiles.data_ptr(), _stream())
     return rows
@@ -1859,7 +1955,7 @@ def moe_route_align(logits: torch.Tensor, correction: Optional[torch.Tensor], gr
 def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], groups: int, keep: int, top: int,
               ids: torch.Tensor, weights: torch.Tensor, scoring: str = "softmax", group_top: int = 1,
               renormalize: bool = False, renorm_eps: float = 0.0, weight_scale: float = 1.0, shared: int = 0,
-              bias: Optional[torch.Tensor] = None) -> None:
+              bias: Optional[torch.Tensor] = None, shared_gated: bool = True) -> None:
     """The router's choice for every row of float32 ``logits [T, E]`` (``[T, E + 1]`` with ``shared``), to which
     ``bias`` (float32 ``[E]``) is added first where there is one.
 
@@ -1869,10 +1965,11 @@ def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], groups: 
     eligible, and the ``top`` best of those are chosen (ties to the lower index) into ``ids`` int32; ``weights``
     float32 are ``s`` at the chosen, with ``renormalize`` divided by their sum + ``renorm_eps``, times
     ``weight_scale``. ``shared`` n: both arrays are ``[T, top + n]``, the last n slots of a row name the experts
-    ``E .. E + n - 1`` (experts every row uses) with the weight ``sigmoid(logits[:, E])``. ``scoring``
+    ``E .. E + n - 1`` (experts every row uses) with the weight ``sigmoid(logits[:, E])`` (without ``shared_gated``: 1, and the
+    logits have no such column). ``scoring``
     ``"softmax_chosen"``: ``s`` are the logits themselves and the weights the softmax over the chosen ones alone.
     """
-    T, E, slots = _check_router(logits, top, shared)
+    T, E, slots = _check_router(logits, top, shared, shared_gated)
     if correction is not None:
         _f32(correction, "the choice's correction", (E,))
     _i32(ids, "chosen experts")
@@ -1891,7 +1988,7 @@ def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], groups: 
         return
     _call(_lib("moe").tie_moe_route, "moe_route", logits.data_ptr(), logits.stride(0), _ptr(bias), _ptr(correction), T, E, groups,
           keep, top, MOE_SCORINGS[scoring], int(group_top), int(bool(renormalize)), float(renorm_eps), float(weight_scale),
-          int(shared), ids.data_ptr(), weights.data_ptr(), _stream())
+          int(shared), int(bool(shared_gated)), ids.data_ptr(), weights.data_ptr(), _stream())
 
 
 def pack_experts(w_gate: Optional[torch.Tensor], w_up: torch.Tensor, w_down: torch.Tensor):
@@ -1983,7 +2080,7 @@ def _moe_packed(x: torch.Tensor, w: PackedWeight, out: torch.Tensor, mode: int, 
     _gpu(out, "the experts' results")
     total, K = w.shape
     N = total // rows.real
-    width = N // 2 if mode in (1, 3) else N
+    width = N // 2 if mode in (1, 3, 4) else N
     if x.dtype != torch.bfloat16 or x.dim() != 2 or x.shape[1] != K or total % rows.real or N % 16 or \
             x.shape[0] * (rows.top if mode else 1) != rows.slots or tuple(out.shape) != (rows.slots, width) or \
             out.dtype != (torch.bfloat16 if mode else torch.float32):
@@ -1995,27 +2092,39 @@ def _moe_packed(x: torch.Tensor, w: PackedWeight, out: torch.Tensor, mode: int, 
 
 
 def moe_gate_up(x: torch.Tensor, w_gate: Optional[torch.Tensor], w_up: torch.Tensor, rows: ExpertRows,
-                act: torch.Tensor, clipped: Optional[tuple] = None) -> None:
+                act: torch.Tensor, clipped: Optional[tuple] = None,
+                slot_weights: Optional[torch.Tensor] = None) -> None:
     """``act[place] = silu(x[row] Wg_e^T) * (x[row] Wu_e^T)`` for every sorted slot: ``x [T, K]``, weights
     ``[real, F, K]``. Without gate weights (``w_gate`` None) the experts have no gate and the activation is the square
     of relu: ``act[place] = relu(x[row] Wu_e^T)^2``. ``clipped`` ``(limit, slope, shift)`` (with gate weights): the sums
     are cut off first, ``g = min(gate sum, limit)``, ``u = clamp(up sum, -limit, limit)``, and the activation is
-    ``g sigmoid(slope g) (u + shift)``. ``w_up`` may be the packed first matrices of ``pack_experts`` (gate weights then
+    ``g sigmoid(slope g) (u + shift)``. ``slot_weights`` (float32, one a (row, choice) slot; gated
+    silu only): the expert sees its row times the slot's weight w, ``act = silu(w * gate sum) * (w * up sum)``.
+    ``w_up`` may be the packed first matrices of ``pack_experts`` (gate weights then
     None; whether they hold gates follows from their rows)."""
+    if slot_weights is not None:
+        _f32(slot_weights, "slot weights")
+        if clipped is not None or slot_weights.numel() != rows.slots:
+            raise InvalidArgument(f"{slot_weights.numel()} slot weights for {rows.slots} slots, or beside clipped sums")
+    weights_ptr = _ptr(slot_weights)
     if isinstance(w_up, PackedWeight):
         gated = w_up.shape[0] == 2 * rows.real * act.shape[1]
+        if slot_weights is not None and not gated:
+            raise InvalidArgument("weights on the experts' input need experts with a gate")
         if clipped is not None and (not gated or not clipped[0] > 0):
             raise InvalidArgument(f"clipped sums need a gate and a positive limit, got {clipped}")
-        _moe_packed(x, w_up, act, (1 if clipped is None else 3) if gated else 2, rows,
-                    tuple(float(v) for v in clipped) if clipped is not None else (0.0, 0.0, 0.0), "moe_gate_up")
+        _moe_packed(x, w_up, act, (4 if slot_weights is not None else 1 if clipped is None else 3) if gated else 2, rows,
+                    (*(float(v) for v in clipped or (0.0, 0.0, 0.0)), weights_ptr), "moe_gate_up")
         return
     _gpu(x, "the experts' input rows")
     _gpu(act, "the experts' activations")
     F_, K = _moe_weights(w_up, rows.real, "up weights")
-    mode = 2 if w_gate is None else (1 if clipped is None else 3)
+    mode = 2 if w_gate is None else (4 if slot_weights is not None else 1 if clipped is None else 3)
+    if slot_weights is not None and w_gate is None:
+        raise InvalidArgument("weights on the experts' input need experts with a gate")
     if clipped is not None and (w_gate is None or not clipped[0] > 0):
         raise InvalidArgument(f"clipped sums need a gate and a positive limit, got {clipped}")
-    gate_params = tuple(float(v) for v in clipped) if clipped is not None else (0.0, 0.0, 0.0)
+    gate_params = (*(float(v) for v in clipped or (0.0, 0.0, 0.0)), weights_ptr)
     if w_gate is not None and (tuple(w_up.shape) != tuple(w_gate.shape) or w_up.dtype != w_gate.dtype or
                                not w_gate.is_contiguous() or not w_gate.is_cuda):
         raise InvalidArgument("gate and up weights must be alike")
@@ -2039,7 +2148,7 @@ def moe_down(act: torch.Tensor, w_down: torch.Tensor, rows: ExpertRows, parts: t
     """``parts[place] = act[place] Wd_e^T`` (float32 ``[slots, N]``) for every sorted slot; weights ``[real, N, F]`` or the
     packed ones of ``pack_experts``."""
     if isinstance(w_down, PackedWeight):
-        _moe_packed(act, w_down, parts, 0, rows, (0.0, 0.0, 0.0), "moe_down")
+        _moe_packed(act, w_down, parts, 0, rows, (0.0, 0.0, 0.0, None), "moe_down")
         return
     _gpu(act, "the experts' activations")
     _f32(parts, "the experts' results")
@@ -2049,12 +2158,12 @@ def moe_down(act: torch.Tensor, w_down: torch.Tensor, rows: ExpertRows, parts: t
     if _moe_on_matrix_cores(rows, act, w_down, parts, False):
         _call(_lib("moe").tie_moe_gemm_bf16, "moe_down", act.data_ptr(), w_down.data_ptr(), None, parts.data_ptr(), 0,
               rows.offsets.data_ptr(), rows.slot_at.data_ptr(), rows.tiles.data_ptr(), rows.num_tiles.data_ptr(),
-              rows.max_tiles, rows.tile_rows, rows.top, N, F_, 0.0, 0.0, 0.0, _stream())
+              rows.max_tiles, rows.tile_rows, rows.top, N, F_, 0.0, 0.0, 0.0, None, _stream())
         return
     _call(_lib("moe").tie_moe_gemm_generic, "moe_down", act.data_ptr(), _code(act, "activations"), w_down.data_ptr(),
           None, _code(w_down, "down weights"), parts.data_ptr(), F32, 0, rows.offsets.data_ptr(),
           rows.slot_at.data_ptr(), rows.tiles.data_ptr(), rows.num_tiles.data_ptr(), rows.max_tiles, rows.top, N, F_,
-          0.0, 0.0, 0.0, _stream())
+          0.0, 0.0, 0.0, None, _stream())
 
 
 def moe_combine(routed: RoutedParts, out: torch.Tensor, accumulate: bool = False) -> None:
@@ -2064,12 +2173,13 @@ def moe_combine(routed: RoutedParts, out: torch.Tensor, accumulate: bool = False
     top = routed.where.shape[1]
     _f32(routed.parts, "the experts' results")
     _i32(routed.where, "places", T * top)
-    _f32(routed.weights, "routing weights", (T, top))
+    if routed.weights is not None:
+        _f32(routed.weights, "routing weights", (T, top))
     _gpu(routed.self_rows, "input rows")
     if routed.parts.shape[-1] != n or tuple(routed.self_rows.shape) != (T, n):
         raise InvalidArgument("moe_combine: the parts do not fit the result")
     _call(_lib("moe").tie_moe_combine, "moe_combine", routed.parts.data_ptr(), routed.where.data_ptr(),
-          routed.weights.data_ptr(), routed.self_rows.data_ptr(), _code(routed.self_rows, "input rows"),
+          _ptr(routed.weights), routed.self_rows.data_ptr(), _code(routed.self_rows, "input rows"),
           out.data_ptr(), T, top, n, int(accumulate), _stream())
 
 
@@ -2179,7 +2289,8 @@ def add_results(x: torch.Tensor, results, scale: float = 1.0, norm: Optional[tup
         top = where.shape[1]
         _f32(parts, "the experts' results")
         _i32(where, "places", T * top)
-        _f32(weights, "routing weights", (T, top))
+        if weights is not None:
+            _f32(weights, "routing weights", (T, top))
         _gpu(self_rows, "the feed-forward's input rows")
         if parts.shape[-1] != n or tuple(self_rows.shape) != (T, n):
             raise InvalidArgument("add_results: the routed parts do not fit the stream")
@@ -2200,6 +2311,36 @@ def add_results(x: torch.Tensor, results, scale: float = 1.0, norm: Optional[tup
     _call(_lib("residual").tie_add_results, "add_results", x.data_ptr(), float(scale), *args, _ptr(parts), _ptr(where),
           _ptr(weights), _ptr(self_rows), self_code, top, _ptr(weight), float(eps), _NORM_KINDS[kind], _ptr(out),
           _code(out, "normed rows") if out is not None else F32, T, n, _stream())
+
+
+def add_normed_results(x: torch.Tensor, results, norm: Optional[tuple] = None) -> None:
+    """``x += sum of result / rms(result) * weight`` row by row, for one or two results of sub-layers that ran side by
+    side, one pass over the float32 stream ``x [T, n]``. ``results``: a list of ``(result, weight, eps)``, each result
+    float32 rows ``[T, n]`` or planes of partial sums ``[P, T, n]`` (added in plane order). ``norm`` ``(weight, eps,
+    out)``: also ``out = RMSNorm(x) * weight`` of the updated rows."""
+    _f32(x, "the stream")
+    T, n = x.shape
+    if not 1 <= len(results) <= 2 or n > ROW_IN_LDS_MAX:
+        raise InvalidArgument(f"add_normed_results takes one or two results, of rows of at most {ROW_IN_LDS_MAX}")
+    args = []
+    for y, weight, eps in results:
+        _f32(y, "a sub-layer's result")
+        if y.dim() not in (2, 3) or tuple(y.shape[-2:]) != (T, n):
+            raise InvalidArgument(f"add_normed_results: a result {list(y.shape)} does not fit the stream {[T, n]}")
+        _f32(weight, "a result's norm weight", (n,))
+        args += [y.data_ptr(), T * n, y.shape[0] if y.dim() == 3 else 1, weight.data_ptr(), float(eps)]
+    if len(results) == 1:
+        args += [None, 0, 0, None, 0.0]
+    weight, eps, out = norm if norm is not None else (None, 0.0, None)
+    if norm is not None:
+        _f32(weight, "norm weight", (n,))
+        _gpu(out, "normed rows")
+        if tuple(out.shape) != (T, n):
+            raise InvalidArgument(f"add_normed_results: normed rows {list(out.shape)} do not fit {[T, n]}")
+    if T == 0:
+        return
+    _call(_lib("residual").tie_add_normed_results, "add_normed_results", x.data_ptr(), *args, _ptr(weight), float(eps),
+          _ptr(out), _code(out, "normed rows") if out is not None else F32, T, n, _stream())
 
 
 def hyper_connection(streams: torch.Tensor, x: Optional[torch.Tensor] = None, from_x: bool = False, fold: bool = False,
@@ -2424,16 +2565,19 @@ def gated_delta_scan(tok: torch.Tensor, out: torch.Tensor, state: torch.Tensor, 
           G, H, d, e, int(head_decay), _stream())
 
 
-def grouped_gated_rms_norm(o: torch.Tensor, weight: torch.Tensor, eps: float, gate: torch.Tensor, out: torch.Tensor,
+def grouped_gated_rms_norm(o: torch.Tensor, weight: Optional[torch.Tensor], eps: float, gate: torch.Tensor, out: torch.Tensor,
                            groups: int, activation: str = "sigmoid") -> None:
     """out = o / rms(o over each of ``groups`` equal groups of columns) * weight[column in its group] * act(gate),
-    ``activation`` "sigmoid" or "silu".
+    ``activation`` "sigmoid" or "silu". ``weight`` may also hold a value for every column of a row, or be None (all 1).
     ``o`` float32 ``[T, n]``, ``gate`` float32 rows of n (a view whose rows may lie further apart)."""
     _f32(o, "gated norm input")
     T, n = o.shape
     if groups <= 0 or n % groups:
         raise InvalidArgument(f"{n} columns are not {groups} equal groups")
-    _f32(weight, "gated norm weight", (n // groups,))
+    group_stride = 0
+    if weight is not None:
+        group_stride = n // groups if groups > 1 and weight.numel() == n else 0
+        _f32(weight, "gated norm weight", (n if group_stride else n // groups,))
     _gpu_strided(gate, "gate rows")
     if gate.dtype != torch.float32 or tuple(gate.shape) != (T, n) or gate.stride(1) != 1:
         raise InvalidArgument(f"gate rows {list(gate.shape)} {gate.dtype} do not fit float32 {[T, n]}")
@@ -2445,8 +2589,8 @@ def grouped_gated_rms_norm(o: torch.Tensor, weight: torch.Tensor, eps: float, ga
     if T == 0:
         return
     _call(_lib("delta_rule").tie_grouped_gated_rms_norm, "grouped_gated_rms_norm", o.data_ptr(), o.stride(0),
-          weight.data_ptr(), float(eps), gate.data_ptr(), gate.stride(0), int(activation == "silu"), out.data_ptr(),
-          _code(out, "gated norm output"), T, groups, n // groups, _stream())
+          _ptr(weight), group_stride, float(eps), gate.data_ptr(), gate.stride(0), int(activation == "silu"),
+          out.data_ptr(), _code(out, "gated norm output"), T, groups, n // groups, _stream())
 
 
 # ------------------------------------------------- latent attention

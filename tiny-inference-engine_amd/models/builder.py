@@ -118,6 +118,7 @@ class Model:
         self.embedding = build_part("embedding", spec.embedding)
         self.layers: List[LayerParts] = [LayerParts(s) for s in spec.layers]
         self.head = build_part("head", spec.head)
+        self.stages = {i: build_part("stage", c.before) for i, c in enumerate(spec.order) if c.before is not None}
         self.cache_plan: CachePlan = plan_cache(
             [self.layers[c.layer].mixer.cache_need() if self.layers[c.layer].mixer is not None else None
              for c in spec.order],
@@ -137,6 +138,7 @@ class Model:
         out = [self.embedding]
         for layer in self.layers:
             out.extend(layer.parts())
+        out.extend(self.stages.values())
         out.append(self.head)
         return out
 
@@ -200,7 +202,7 @@ class Model:
             entry = self.cache_plan.calls[index]
             binding = None if entry is None else tuple((e.group, e.writes) for e in entry) \
                 if isinstance(entry, tuple) else (entry.group, entry.writes)
-            ok = all(getattr(c, "replayable", False) for c in classes)
+            ok = all(getattr(c, "replayable", False) for c in classes) and index not in self.stages
             names = {spec.name for part in layer_parts for spec in part.all_tensors()}
             signatures.append((tuple(classes), tuple(t[2:] for t in tensors), binding, _constants(scalars, names))
                               if ok else None)
@@ -330,6 +332,8 @@ class Model:
                 self._run_alike(ctx, x, index, alike_to)
                 index = alike_to
                 continue
+            if index in self.stages:
+                self.stages[index].forward(ctx, x)
             layer = self.layers[self.spec.order[index].layer]
             layer.block.forward(ctx, x, layer, ctx.cache_of(index))
             if self.layer_hook is not None:

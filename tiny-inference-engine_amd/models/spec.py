@@ -40,10 +40,13 @@ class LayerCall:
     call's mixer uses; by default every call owns a slot of its own (its index
     in the order). A call with ``reads_cache_of`` set to an earlier position in
     the order uses that call's slot read-only: it writes no keys or values.
+    ``before`` names a stage: a part that changes the residual stream right before the
+    call's layer runs (what a layer does every time it runs belongs into its block).
     """
 
     layer: int
     reads_cache_of: Optional[int] = None
+    before: Optional[PartSpec] = None
 
 
 @dataclasses.dataclass(frozen=True)

@@ -22,7 +22,9 @@ Further parameters, for architectures that have them (absent or None: not applie
   cache, and run through the attention kernels, at one common size (the larger of the two, in steps of 16):
   at load time the q, k and v weights get zero rows and the o weight zero columns for the dimensions a head
   lacks. Zero dimensions add nothing to a score, and zero values give zero outputs that meet zero columns,
-  so the arithmetic is unchanged. Such heads take no per-head norm and no rotation.
+  so the arithmetic is unchanged. A per-head norm over D stored of P padded dimensions is the kernels' norm over P with
+  ``eps D / P`` for eps and ``w sqrt(D / P)`` for w (the padding adds nothing to the sum of squares); a rotation may
+  cover stored dimensions only.
 * ``value_mix`` ``{"role", "weight", "share"}``: values blended across layers. The layer with role ``"keep"``
   keeps its values of the step's tokens (float32, in step scratch memory named by ``share``); a layer with role
   ``"blend"`` caches and attends to ``(1 - lam) * v + lam * v_kept`` with ``lam`` the one-element tensor
@@ -40,6 +42,8 @@ Further parameters, for architectures that have them (absent or None: not applie
 * ``values_are_keys``: there is no value projection; the values are the keys as projected (with their bias), before
   the per-head norm and the rotation. ``names`` then has no ``v`` and ``bias`` none for it.
 
+* ``gate`` (a tensor name, ``[num_heads * value size, hidden]``): the heads' outputs are multiplied element by element by
+  ``sigmoid(Wg h)`` before the output projection. The matrix is part of the first product.
 * ``conv`` ``{"taps", "q", "k", "v"}`` (tensor names, each ``[channels, taps]``): a short causal convolution over time
   on every channel of the projected q, k and v, directly behind the projection (before norm and rotation):
   ``y_t = sum_j w[:, j] * u_(t - taps + 1 + j)``, zeros before the sequence's start. The last ``taps - 1`` projected
@@ -55,6 +59,7 @@ adding it to a stream: for arrangements that norm a sub-layer's output first.
 
 from __future__ import annotations
 
+import math
 from typing import List, Optional
 
 import torch
@@ -104,8 +109,8 @@ class PagedAttention(Mixer):
             raise InvalidArgument(f"a convolution of {self.taps} taps: 1 to {kernels.CONV_MAX_TAPS} are supported")
         self.output_scale = float(params.get("output_scale", 1.0))
         self.conv_weight: torch.Tensor = None
-        plain_heads = not params.get("qk_norm") and (params.get("position") or PartSpec("none")).kind == "none" \
-            and not params.get("bias")
+        plain_heads = (params.get("position") or PartSpec("none")).kind == "none" and not self.norm_over_projection and \
+            not params.get("values_are_keys")
         self.padded = self.stored_value_dim != self.stored_key_dim or self.head_dim % 2 != 0 or \
             (plain_heads and self.head_dim % 16 != 0)
         if self.padded:
@@ -122,8 +127,10 @@ class PagedAttention(Mixer):
         inputs = "qk" if self.values_are_keys else "qkv"
         if any(k in bias for k in inputs) and not all(k in bias for k in inputs):
             raise InvalidArgument("the q, k and v projections run as one product: a bias for all of them or for none")
-        if self.padded and bias:
-            raise InvalidArgument("heads padded to a common size take no bias")
+        self.gate_name: Optional[str] = params.get("gate")
+        if self.gate_name and (self.conv or self.norm_over_projection):
+            raise InvalidArgument("a gate on the heads' outputs beside a convolution or a norm over the projection is not "
+                                  "supported")
         if (self.conv or self.norm_over_projection) and (self.values_are_keys or bias or self.value_mix is not None):
             raise InvalidArgument("a convolution or a norm over the whole projection goes with plain q, k and v "
                                   "projections: no bias, no blended values, no values that are the keys")
@@ -139,8 +146,14 @@ class PagedAttention(Mixer):
         self.bias_in_kernel = "q" in bias and build_part("position", position_spec).rotary_table() is not None
         self.qkv_bias_names = [bias[k] for k in inputs] if self.bias_in_kernel else None
         self.qkv_bias: torch.Tensor = None
-        self.qkv = Linear([names[k] for k in inputs], sizes[:len(inputs)], self.hidden,
-                          bias=[bias[k] for k in inputs] if "q" in bias and not self.bias_in_kernel else None)
+        if self.padded and "q" in bias and not self.bias_in_kernel:
+            raise InvalidArgument("heads padded to a common size take a bias only beside an encoding the fused kernel applies")
+        gate_names, gate_sizes = ([self.gate_name], [self.num_heads * self.stored_value_dim]) if self.gate_name else ([], [])
+        self.qkv = Linear([names[k] for k in inputs] + gate_names, sizes[:len(inputs)] + gate_sizes, self.hidden,
+                          bias=[bias[k] for k in inputs] + [None] * len(gate_names)
+                          if "q" in bias and not self.bias_in_kernel else None)
+        self.joinable = not (self.conv or self.norm_over_projection) and self.qkv.bias_names is None and \
+            build_part("position", position_spec).rotary_table() is not None
         self.out = Linear([names["o"]], [self.hidden], self.num_heads * self.stored_value_dim if self.padded else q_dim,
                           bias=[bias["o"]] if "o" in bias else None)
         self.q_norm_weight: torch.Tensor = None
@@ -152,13 +165,18 @@ class PagedAttention(Mixer):
                                   "other changes the projected keys in place before they are cached as values")
         table = self.position.rotary_table()
         rotates_only = table is not None and int(table[1] or 0) <= self.stored_key_dim
-        if self.padded and ((self.qk_norm and not self.norm_over_projection) or
-                            (position.kind != "none" and not rotates_only)):
-            raise InvalidArgument("heads whose key and value sizes differ take no per-head norm, and a rotation only "
-                                  "of dimensions the stored keys have")
+        if self.padded and position.kind != "none" and not rotates_only:
+            raise InvalidArgument("heads whose key and value sizes differ take a rotation only of dimensions the stored "
+                                  "keys have")
+        # What the kernels' norm over a padded head divides by (see above).
+        self.norm_share = self.stored_key_dim / self.head_dim if self.padded and not self.norm_over_projection else 1.0
+        self.qk_eps = float(self.qk_norm["eps"]) * self.norm_share if self.qk_norm else 0.0
 
     def children(self) -> List[Part]:
         return [self.position]
+
+    def first_product(self):
+        return self.qkv if self.joinable else None
 
     def cache_need(self):
         pages = PagedKV(self.num_kv_heads, self.head_dim, self.window, self.chunk, self.keep_first)
@@ -170,11 +188,11 @@ class PagedAttention(Mixer):
         specs = self.qkv.tensors() + self.out.tensors()
         if self.qkv_bias_names is not None:
             specs += [TensorSpec(b, (o,), "vector", ("normal", 0.02))
-                      for b, o in zip(self.qkv_bias_names, self.qkv.out_features)]
+                      for b, o in zip(self.qkv_bias_names, self.qkv.out_features)]      # a gate's columns have none
         if self.qk_norm:
             init = ("one_plus_uniform", 0.1)
             sizes = (self.num_heads * self.stored_key_dim, self.num_kv_heads * self.stored_key_dim) \
-                if self.norm_over_projection else (self.head_dim, self.head_dim)
+                if self.norm_over_projection else (self.stored_key_dim, self.stored_key_dim)
             specs.append(TensorSpec(self.qk_norm["q_weight"], (sizes[0],), "vector", init))
             specs.append(TensorSpec(self.qk_norm["k_weight"], (sizes[1],), "vector", init))
         if self.conv:
@@ -196,9 +214,12 @@ class PagedAttention(Mixer):
             out[:, :stored] = w.view(heads, stored, self.hidden)
             return out.view(heads * self.head_dim, self.hidden)
 
-        q, k, v = self.qkv.names
+        q, k, v = self.qkv.names[:3]
         parts = [rows(q, self.num_heads, self.stored_key_dim), rows(k, self.num_kv_heads, self.stored_key_dim),
                  rows(v, self.num_kv_heads, self.stored_value_dim)]
+        if self.gate_name:
+            parts.append(rows(self.gate_name, self.num_heads, self.stored_value_dim))
+        self.qkv.out_features = [p.shape[0] for p in parts]
         self.qkv.set_weight(torch.cat(parts, dim=0).contiguous())
         w = fetch(self.out.names[0], "matrix")
         o = w.new_zeros((self.hidden, self.num_heads, self.head_dim))
@@ -240,10 +261,18 @@ class PagedAttention(Mixer):
             if self.norm_over_projection:
                 self.q_norm_weight = self._per_channel(self.q_norm_weight, H, self.stored_key_dim).reshape(-1).contiguous()
                 self.k_norm_weight = self._per_channel(self.k_norm_weight, KVH, self.stored_key_dim).reshape(-1).contiguous()
+            elif self.padded:
+                self.q_norm_weight, self.k_norm_weight = (
+                    (self._per_channel(w, 1, self.stored_key_dim) * math.sqrt(self.norm_share)).reshape(-1).contiguous()
+                    for w in (self.q_norm_weight, self.k_norm_weight))
         if self.sink_name:
             self.sinks = fetch(self.sink_name, "vector").to(torch.float32).contiguous()
         if self.qkv_bias_names is not None:
-            self.qkv_bias = torch.cat([fetch(b, "vector").to(torch.float32) for b in self.qkv_bias_names]).contiguous()
+            vectors = [fetch(b, "vector").to(torch.float32) for b in self.qkv_bias_names]
+            if self.padded:
+                vectors = [self._per_channel(v, heads, stored).reshape(-1) for v, heads, stored in
+                           zip(vectors, (H, KVH, KVH), (self.stored_key_dim, self.stored_key_dim, self.stored_value_dim))]
+            self.qkv_bias = torch.cat(vectors).contiguous()
 
     def _finish(self, ctx: StepContext, attn: torch.Tensor, residual: Optional[torch.Tensor]):
         """The output projection: added to ``residual``, or (``residual`` None) returned for the caller to place."""
@@ -286,7 +315,7 @@ class PagedAttention(Mixer):
         if isinstance(cache, tuple):          # pages, and the convolution's last inputs
             cache, conv_state = cache[0], cache[1].state
         step = cache.step
-        eps = float(self.qk_norm["eps"]) if self.qk_norm else 0.0
+        eps = self.qk_eps
         q_weight, k_weight = (self.q_norm_weight, self.k_norm_weight) if self.qk_norm else (None, None)
 
         width = self.q_dim + (1 if self.values_are_keys else 2) * self.kv_dim
@@ -294,12 +323,12 @@ class PagedAttention(Mixer):
         table = self.position.rotary_table()
         # Decode-size steps: the projection comes as planes of partial sums, added by the kernel that reads them.
         rows_first = self.conv is not None or self.norm_over_projection
-        planes = self.qkv.partial_planes(ctx, h, "attention.qkv") if table is not None and not rows_first else None
+        own = self.qkv.weight is not None and not self.gate_name     # neither joined with another part's product nor gated
+        planes = self.qkv.partial_planes(ctx, h, "attention.qkv") if table is not None and not rows_first and own else None
         if planes is not None:
             qkv = planes[0]
         else:
-            qkv = ctx.scratch("attention.qkv", (T, width), torch.float32)
-            self.qkv(h, qkv, ctx=ctx)
+            qkv = ctx.product(self.qkv, h, "attention.qkv")
         if rows_first:
             # The convolution over time (from the rows as projected and the sequence's state) and the norms over a
             # whole projection, one kernel; the kernels below then neither norm nor see the raw rows.
@@ -317,7 +346,7 @@ class PagedAttention(Mixer):
             inv_freq, rotary_dim, pairing = table
             if (inv_freq is not None and not rows_first and rotary_dim == Dh and pairing == "rotate_half" and self.softcap is None
                     and self.value_mix is None and not self.values_are_keys and not self.chunk and self.sinks is None
-                    and self.qkv_bias is None and not self.keep_first
+                    and self.qkv_bias is None and not self.keep_first and own
                     and kernels.decode_attention_prepares(ctx.batch, q.dtype, cache.k_cache, H)):
                 # A step of single decoded tokens: the attention kernel sums the planes, norms and rotates its own
                 # queries and writes the newest keys and values itself: one kernel less.
@@ -356,4 +385,6 @@ class PagedAttention(Mixer):
         kernels.paged_attention(q, cache.k_cache, cache.v_cache, attn, step, ctx.batch, H, self.scale, self.window,
                                 scratch=ctx.scratch, softcap=self.softcap, chunk=self.chunk, sinks=self.sinks,
                                 keep_first=self.keep_first)
+        if self.gate_name:
+            kernels.gate_rows(attn, qkv[:, width:width + self.q_dim])
         return self._finish(ctx, attn, residual)

@@ -8,7 +8,8 @@ Five kinds of part exist, each with a registry from a kind name to a class:
 * feed_forward  ``forward(ctx, h, residual)``
 * block         ``forward(ctx, x, layer, cache)``: the arrangement of the above
 
-plus the two ends of a model, ``embedding`` and ``head``. A part is built from
+plus the two ends of a model, ``embedding`` and ``head``, and ``stage`` (``forward(ctx, x)``), a change of the
+residual stream before one entry of the run order. A part is built from
 the parameters of its PartSpec (sizes, constants, tensor names) and never looks
 at the model around it. It declares the tensors it expects (``tensors()``),
 takes them at load time (``load``) and runs on a StepContext.
@@ -43,7 +44,7 @@ class PartSpec:
     params: Mapping[str, Any] = dataclasses.field(default_factory=dict)
 
 
-_KINDS = ("norm", "position", "mixer", "feed_forward", "block", "embedding", "head")
+_KINDS = ("norm", "position", "mixer", "feed_forward", "block", "embedding", "head", "stage")
 _REGISTRIES: Dict[str, Dict[str, type]] = {k: {} for k in _KINDS}
 
 
@@ -349,6 +350,9 @@ class Norm(Part):
     leaves_row_scale = False
     # True: forward() takes ``results`` = (sub-layers' results, scale), adds them to x in its own pass and norms the sum.
     adds_results = False
+    # True: forward() takes ``normed_results`` = [(a sub-layer's result, norm weight, eps), ...] and adds them to x, each
+    # RMS-normed, in its own pass.
+    adds_normed_results = False
     reads_either_type = False   # True: forward() also reads bfloat16 rows (an embedding table's, gathered by ``rows``)
 
     def forward(self, ctx: StepContext, x: torch.Tensor, rows: Optional[torch.Tensor] = None,
@@ -402,7 +406,8 @@ class Block(Part):
 
     An arrangement settles what is owed to the residual stream before it hands the stream to a part
     that does not add the debt itself (``normed`` does so for norms). ``consumer``: the part the normed rows
-    go to and to nothing else; if it says ``takes_row_scale`` (every product it forms from the rows goes through
+    go to and to nothing else. Results that a part left for the next pass over the stream (``StepContext.leave_late`` with
+    the key ``("results", rows, width)`` or ``("normed_results", rows, width)``) go to a norm that adds them itself. If the consumer says ``takes_row_scale`` (every product it forms from the rows goes through
     ``parts.Linear`` with the step context, or asks ``ctx.row_scale_of`` itself), a norm that can may hand it the
     rows without their 1 / rms.
     """
@@ -412,6 +417,14 @@ class Block(Part):
 
     @staticmethod
     def normed(ctx: StepContext, norm, x: torch.Tensor, consumer=None) -> torch.Tensor:
+        if getattr(norm, "adds_normed_results", False):
+            left = ctx.take_late(("normed_results",) + tuple(x.shape))
+            if left is not None:
+                return norm.forward(ctx, x, normed_results=left)
+        if norm.adds_results:
+            left = ctx.take_late(("results",) + tuple(x.shape))
+            if left is not None:
+                return norm.forward(ctx, x, results=(left, 1.0))
         if norm.adds_owed:
             ctx.run_late()
         else:
@@ -421,6 +434,14 @@ class Block(Part):
         return norm.forward(ctx, x)
 
     def forward(self, ctx: StepContext, x: torch.Tensor, layer, cache) -> None:
+        raise NotImplementedError
+
+
+class Stage(Part):
+    """A change of the residual stream before one entry of the run order. What is owed to the stream may stay owed where
+    the change commutes with adding it (``ctx.run_late()`` is called first); otherwise the stage settles."""
+
+    def forward(self, ctx: StepContext, x: torch.Tensor) -> None:
         raise NotImplementedError
 
 
@@ -436,6 +457,6 @@ class Head(Part):
 
 __all__ = [
     "BFLOAT16", "FLOAT32", "Block", "Embedding", "FeedForward", "Head", "Mixer", "Norm", "PagedBinding",
-    "Part", "PartSpec", "Position", "StateBinding", "StepContext", "TensorSpec", "Workspace", "build_part",
+    "Part", "PartSpec", "Position", "Stage", "StateBinding", "StepContext", "TensorSpec", "Workspace", "build_part",
     "register_part", "registered_parts", "unregister_part",
 ]

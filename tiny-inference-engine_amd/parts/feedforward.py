@@ -12,7 +12,7 @@ through another function, ``activation``: ``silu`` (the default) or ``gelu_tanh`
 ``0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)))``.
 
 ``mlp`` is ``down(act(up(h)))`` without a gate; ``activation`` names the function (``gelu``: the exact form,
-``0.5 z (1 + erf(z / sqrt 2))``; ``poly_norm``: ``a N(z) + b N(z^2) + c N(z^3) + e`` with powers taken element by
+``0.5 z (1 + erf(z / sqrt 2))``; ``gelu_tanh`` as above; ``poly_norm``: ``a N(z) + b N(z^2) + c N(z^3) + e`` with powers taken element by
 element, ``N(y) = y / sqrt(mean(y^2) + eps)`` over the row, and the four numbers a stored tensor, named by
 ``activation_weight``, with ``activation_eps``). Parameters: ``hidden``, ``intermediate``, ``activation``, ``names``
 (``up``, ``down``).
@@ -36,10 +36,13 @@ named, and the weights are the softmax over the chosen logits alone); ``expert_a
 ``activation_params`` (limit, slope, shift), ``g = min(gate_e h, limit)``, ``u = clamp(up_e h, -limit, limit)``,
 ``down_e(g sigmoid(slope g) (u + shift))``;
 ``expert_activation`` ``relu_squared`` with no ``gate`` names (experts without a gate, ``down_e(relu(up_e h)^2)``);
+``weight_on`` "input" (the default: "output"): a chosen expert sees the row times its weight and the results are added as
+they are; the products are linear, so the factor meets their float32 sums, ``down_e(silu(w g) (w u))``;
 ``shared`` ``{"intermediate", "up", "down", "gate_logit"}`` (and ``"gate"`` for gated experts): one more expert of the
 same form that every row uses, its result multiplied by ``sigmoid(w_gate_logit . h)``, one number a row. It runs as
 pieces of the routed experts' size among them (further experts that every row chooses, all with that weight), so
-the same launches carry it; its gate's logit is one more column of the router's product.
+the same launches carry it; its gate's logit is one more column of the router's product. With ``gate_logit`` None its
+result is added as it is.
 
 Nothing of a step is read on the host: the rows are sorted by expert on the device and the experts' products
 run over a tile list that lives there (``kernels.moe_align``), so routed layers are recorded and replayed like
@@ -126,7 +129,7 @@ class Mlp(FeedForward):
     capturable = True
     replayable = True
     returns_result = True
-    ACTIVATIONS = ("gelu", "poly_norm")
+    ACTIVATIONS = ("gelu", "gelu_tanh", "poly_norm")
 
     def __init__(self, params):
         super().__init__(params)
@@ -164,7 +167,7 @@ class Mlp(FeedForward):
         if self.activation == "poly_norm":
             kernels.poly_norm(pre, self.activation_weight, self.activation_eps, act)
         else:
-            kernels.gelu(pre, act)
+            kernels.gelu(pre, act, form="tanh" if self.activation == "gelu_tanh" else "erf")
         return _finish(ctx, self.down, act, residual, "feed_forward.result")
 
 
@@ -204,6 +207,10 @@ class RoutedExperts(FeedForward):
             self.clipped = tuple(float(p[k]) for k in ("limit", "slope", "shift"))
             if not self.clipped[0] > 0:
                 raise InvalidArgument(f"the limit of an expert's sums must be positive, got {self.clipped[0]}")
+        self.weight_on = params.get("weight_on") or "output"
+        if self.weight_on not in ("output", "input") or (self.weight_on == "input" and self.activation != "silu"):
+            raise UnsupportedError(f"routing weights on an expert's '{self.weight_on}' with the activation "
+                                   f"'{self.activation}' (supported: output; input with silu)")
         if self.experts <= 0 or self.identity < 0 or self.outputs > kernels.MOE_MAX_EXPERTS:
             raise InvalidArgument(f"a routed feed-forward takes 1 to {kernels.MOE_MAX_EXPERTS} experts, got "
                                   f"{self.experts} + {self.identity}")
@@ -220,14 +227,17 @@ class RoutedExperts(FeedForward):
         self.shared = dict(params["shared"]) if params.get("shared") else None
         self.shared_intermediate = int(self.shared["intermediate"]) if self.shared else 0
         self.shared_pieces = -(-self.shared_intermediate // self.intermediate) if self.shared else 0
+        self.shared_gated = bool(self.shared) and bool(self.shared.get("gate_logit"))
+        if self.weight_on == "input" and self.identity:
+            raise InvalidArgument("weights on the experts' input beside experts that return it are not supported")
         if self.shared:
             if self.identity:
                 raise InvalidArgument("a shared expert beside experts that return their input is not supported")
             if self.shared_intermediate <= 0 or self.experts + self.shared_pieces > kernels.MOE_MAX_EXPERTS:
                 raise InvalidArgument(f"a shared expert of inner size {self.shared_intermediate} does not fit")
-            router_names, router_sizes = [names["router"], self.shared["gate_logit"]], [self.outputs, 1]
-        else:
-            router_names, router_sizes = [names["router"]], [self.outputs]
+        router_names, router_sizes = [names["router"]], [self.outputs]
+        if self.shared_gated:
+            router_names, router_sizes = router_names + [self.shared["gate_logit"]], router_sizes + [1]
         self.router = Linear(router_names, router_sizes, self.hidden)
         self.correction: torch.Tensor = None
         self.router_bias: torch.Tensor = None
@@ -296,14 +306,17 @@ class RoutedExperts(FeedForward):
         rows = kernels.moe_route_align(logits, self.correction, self.groups, self.keep_groups, self.top, ids, weights, real,
                                        tile_rows, ctx.scratch, scoring=self.scoring, group_top=self.group_top,
                                        renormalize=self.renormalize, renorm_eps=self.renorm_eps,
-                                       weight_scale=self.weight_scale, shared=self.shared_pieces, bias=self.router_bias)
+                                       weight_scale=self.weight_scale, shared=self.shared_pieces, bias=self.router_bias,
+                                       shared_gated=self.shared_gated)
+        on_input = self.weight_on == "input"
         act = ctx.scratch("moe.act", (T * slots, self.intermediate))
-        kernels.moe_gate_up(h, self.gate, self.up, rows, act, clipped=self.clipped)
+        kernels.moe_gate_up(h, self.gate, self.up, rows, act, clipped=self.clipped,
+                            slot_weights=weights if on_input else None)
         parts = ctx.scratch("moe.parts", (T * slots, self.hidden), torch.float32)
         kernels.moe_down(act, self.down, rows, parts)
-        routed = kernels.RoutedParts(parts, rows.where, weights, h)
+        routed = kernels.RoutedParts(parts, rows.where, None if on_input else weights, h)
         if residual is None:
             return routed
-        ctx.settle()
-        kernels.moe_combine(routed, residual, accumulate=True)
+        # what is added rides in the next norm's pass over the stream
+        ctx.leave_late(("results",) + tuple(residual.shape), lambda results: kernels.add_results(residual, results), [routed])
         return None

@@ -34,6 +34,8 @@ class RMSNorm(Norm):
     replayable = True
     adds_owed = True
     leaves_row_scale = True
+    adds_results = True
+    adds_normed_results = True
     reads_either_type = True
 
     def __init__(self, params):
@@ -54,8 +56,10 @@ class RMSNorm(Norm):
             self.weight = (self.weight.to(torch.float32) + 1.0).contiguous()
 
     def forward(self, ctx: StepContext, x: torch.Tensor, rows: Optional[torch.Tensor] = None,
-                out_name: str = "norm.out", out_dtype: torch.dtype = None, lazy: bool = False) -> torch.Tensor:
-        """``lazy``: the caller's consumer applies a row scale (``Block.normed``). If the product that ends the
+                out_name: str = "norm.out", out_dtype: torch.dtype = None, lazy: bool = False, results=None,
+                normed_results=None) -> torch.Tensor:
+        """``results`` (without ``rows``): ``(sub-layers' results, scale)`` that are added to ``x`` in the same pass;
+        ``normed_results``: ``[(result, weight, eps), ...]`` added each RMS-normed. ``lazy``: the caller's consumer applies a row scale (``Block.normed``). If the product that ends the
         sub-layer before is still pending, it is launched here with an epilogue that adds it to ``x`` and leaves
         ``x * weight`` and the rows' sums of squares: the result lacks its ``1 / rms``, which the consumer's
         products apply (``ctx.row_scale_of``), and no norm kernel runs."""
@@ -70,6 +74,12 @@ class RMSNorm(Norm):
                 ctx.set_row_scale(out, kernels.RowScale(squares, self.dim, self.eps))
                 return out
         ctx.set_row_scale(out, None)
+        if results is not None:
+            kernels.add_results(x, *results, norm=("rms_norm", self.weight, self.eps, out))
+            return out
+        if normed_results is not None:
+            kernels.add_normed_results(x, normed_results, norm=(self.weight, self.eps, out))
+            return out
         owed = ctx.take_owed(x)
         if owed is not None and rows is None:
             kernels.add_partials(x, owed, self.weight, self.eps, out)   # x += owed sums; out = norm(x), one pass

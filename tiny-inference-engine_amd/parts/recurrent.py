@@ -6,6 +6,21 @@
     per head   S_t = decay[head] * S_(t-1) + k_t v_t^T ,   o_t = S_t^T q_t          (no other scale)
     y = Wo ( RMSNorm(o_t, all heads side by side; weight ``norm``) * sigmoid(Wg h) )
 
+For designs that have them: ``key_scale`` (a factor on k), ``position`` (a PartSpec of a rotation whose pairs are dimension
+halves: q and k turn by position; no activation beside it), ``norm_per`` "head" (every head's output is divided by its own
+root mean square; ``norm`` then names one weight a dimension of all heads, or None), ``gate_activation`` "silu".
+
+``matrix_memory`` keeps a matrix a head with exponential gates and a normaliser (mLSTM):
+
+    q = key_dim^(-1/2) Wq h,  k = Wk h   (heads x key_dim)        v = Wv h   (heads x value_dim)
+    per head   i = cap tanh((Wi h + bi) / cap),   f = log sigmoid(cap tanh((Wf h + bf) / cap))
+    m_t = max(f + m_(t-1), i);  S_t = exp(f + m_(t-1) - m_t) S_(t-1) + exp(i - m_t) k v^T;  n_t alike with k alone
+    o = S_t^T q / (max(|n_t . q|, exp(-m_t)) + 1e-6)
+    y = Wo ( o / rms(o over value_dim) * norm (all heads side by side) * sigmoid(Wg h) )
+
+Its states are S and, as a second need, (n, m). Parameters: ``hidden``, ``heads``, ``key_dim``, ``value_dim``, ``gate_cap``,
+``eps``, ``names`` (``q``, ``k``, ``v``, ``g``, ``o``, ``norm``, ``i``, ``f``, ``i_bias``, ``f_bias``).
+
 ``min_gru`` is a gated recurrence whose gates read the current token only:
 
     z = sigmoid(Wz h + bz),   u = Wx h + bx,   candidate = u + 1/2 for u >= 0, sigmoid(u) below
@@ -52,16 +67,21 @@ import torch
 from .. import kernels
 from ..cache.spec import FixedState
 from ..errors import InvalidArgument
-from .base import Mixer, StepContext, TensorSpec, register_part
+from .base import Mixer, Part, StepContext, TensorSpec, build_part, register_part
 from .linear import Linear
 
 
-def _finish(ctx: StepContext, out: Linear, rows: torch.Tensor, residual: Optional[torch.Tensor], name: str):
-    """The output projection: added to ``residual``, or (None) returned as float32 rows."""
+def _finish(ctx: StepContext, out: Linear, rows: torch.Tensor, residual: Optional[torch.Tensor], name: str,
+            planes: bool = False):
+    """The output projection: added to ``residual``, or (None) returned as float32 rows (or, with ``planes``, as planes of
+    partial sums where that is the faster way)."""
     if residual is not None:
         out(rows, residual, accumulate=True, ctx=ctx)
         return None
     ctx.settle()
+    partial = out.partial_planes(ctx, rows, name + "_planes") if planes else None
+    if partial is not None:
+        return partial
     result = ctx.scratch(name, (rows.shape[0], out.total_out), torch.float32)
     out(rows, result, accumulate=False, ctx=ctx)
     return result
@@ -81,44 +101,133 @@ class DecayAttention(Mixer):
         self.value_dim = int(params.get("value_dim") or self.key_dim)
         self.decay_values = [float(d) for d in params["decay"]]
         self.activation = params.get("activation", "silu")
+        self.key_scale = float(params.get("key_scale") or 1.0)
+        self.norm_per = params.get("norm_per") or "row"
+        self.gate_activation = params.get("gate_activation") or "sigmoid"
+        self.position = build_part("position", params["position"]) if params.get("position") else None
         self.eps = float(params["eps"])
+        if self.norm_per not in ("row", "head") or self.gate_activation not in ("sigmoid", "silu") or \
+                (self.norm_per == "row" and self.gate_activation != "sigmoid"):
+            raise InvalidArgument(f"a decay attention norms its output per 'row' with a sigmoid gate or per 'head', not per "
+                                  f"'{self.norm_per}' with '{self.gate_activation}'")
+        if self.position is not None:
+            table = self.position.rotary_table()
+            if table is None or table[2] != "rotate_half" or self.activation != "none" or table[1] > self.key_dim:
+                raise InvalidArgument("a decay attention rotates halves of its (not activated) queries and keys only")
         if len(self.decay_values) != self.heads:
             raise InvalidArgument(f"{self.heads} heads need {self.heads} decays, got {len(self.decay_values)}")
-        if self.key_dim > kernels.DECAY_ATTENTION_MAX_DIM:
-            raise InvalidArgument(f"a key size of {self.key_dim} exceeds {kernels.DECAY_ATTENTION_MAX_DIM}")
+        if self.key_dim > kernels.MATRIX_STATE_MAX_DIM:
+            raise InvalidArgument(f"a key size of {self.key_dim} exceeds {kernels.MATRIX_STATE_MAX_DIM}")
         names = params["names"]
         self.qk_width, self.v_width = self.heads * self.key_dim, self.heads * self.value_dim
         self.inputs = Linear([names["q"], names["k"], names["v"], names["g"]],
                              [self.qk_width, self.qk_width, self.v_width, self.v_width], self.hidden)
         self.out = Linear([names["o"]], [self.hidden], self.v_width)
         self.norm_name = names["norm"]
+        if self.norm_name is None and self.norm_per == "row":
+            raise InvalidArgument("the norm over all heads has a weight")
         self.norm_weight: torch.Tensor = None
         self.decay: torch.Tensor = None
+
+    def children(self) -> List[Part]:
+        return [self.position] if self.position is not None else []
+
+    def first_product(self):
+        return self.inputs
 
     def cache_need(self):
         return FixedState((self.heads, self.key_dim, self.value_dim))
 
     def tensors(self) -> List[TensorSpec]:
-        return self.inputs.tensors() + self.out.tensors() + \
-            [TensorSpec(self.norm_name, (self.v_width,), "vector", ("one_plus_uniform", 0.1))]
+        weight = [TensorSpec(self.norm_name, (self.v_width,), "vector", ("one_plus_uniform", 0.1))] if self.norm_name else []
+        return self.inputs.tensors() + self.out.tensors() + weight
 
     def load(self, fetch, mode, device) -> None:
         self.inputs.load(fetch)
         self.out.load(fetch)
-        self.norm_weight = fetch(self.norm_name, "vector")
+        self.norm_weight = fetch(self.norm_name, "vector") if self.norm_name else None
         self.decay = torch.tensor(self.decay_values, dtype=torch.float32).to(device)
 
     def forward(self, ctx: StepContext, h: torch.Tensor, cache, residual: Optional[torch.Tensor]):
         T = h.shape[0]
-        proj = ctx.scratch("decay_attention.proj", (T, self.inputs.total_out), torch.float32)
-        self.inputs(h, proj, ctx=ctx)
+        proj = ctx.product(self.inputs, h, "decay_attention.proj")
+        rotation = None
+        if self.position is not None:
+            rotation = (self.position.angles(ctx), self.position.rotary_table()[1])
         o = ctx.scratch("decay_attention.o", (T, self.v_width), torch.float32)
         kernels.decay_attention_scan(proj, o, cache.state, ctx.batch.query_start, cache.state_slots, self.decay,
                                      ctx.batch.num_seqs, self.heads, self.key_dim, self.value_dim, self.activation,
-                                     chunks=kernels.scan_chunks(ctx.batch, ctx.device), scratch=ctx.scratch)
+                                     chunks=kernels.scan_chunks(ctx.batch, ctx.device), scratch=ctx.scratch,
+                                     q_scale=self.key_scale, rotation=rotation)      # o is linear in k: the same factor
         gated = ctx.scratch("decay_attention.gated", (T, self.v_width))
-        kernels.gated_rms_norm(o, self.norm_weight, self.eps, proj[:, 2 * self.qk_width + self.v_width:], gated)
+        gate = proj[:, 2 * self.qk_width + self.v_width:]
+        if self.norm_per == "head":
+            kernels.grouped_gated_rms_norm(o, self.norm_weight, self.eps, gate, gated, self.heads,
+                                           activation=self.gate_activation)
+        else:
+            kernels.gated_rms_norm(o, self.norm_weight, self.eps, gate, gated)
         return _finish(ctx, self.out, gated, residual, "decay_attention.result")
+
+
+@register_part("mixer", "matrix_memory")
+class MatrixMemory(Mixer):
+    capturable = True
+    takes_row_scale = True
+    returns_result = True
+
+    def __init__(self, params):
+        super().__init__(params)
+        self.hidden = int(params["hidden"])
+        self.heads = int(params["heads"])
+        self.key_dim = int(params["key_dim"])
+        self.value_dim = int(params.get("value_dim") or self.key_dim)
+        self.gate_cap = float(params["gate_cap"])
+        self.eps = float(params["eps"])
+        if not self.gate_cap > 0:
+            raise InvalidArgument(f"the gates' cap must be positive, got {self.gate_cap}")
+        if self.key_dim > kernels.MATRIX_STATE_MAX_DIM:
+            raise InvalidArgument(f"a key size of {self.key_dim} exceeds {kernels.MATRIX_STATE_MAX_DIM}")
+        n = self.names = dict(params["names"])
+        self.qk_width, self.v_width = self.heads * self.key_dim, self.heads * self.value_dim
+        self.gate_column = 2 * self.qk_width + 2 * self.v_width
+        self.inputs = Linear([n[k] for k in ("q", "k", "v", "g", "i", "f")],
+                             [self.qk_width, self.qk_width, self.v_width, self.v_width, self.heads, self.heads], self.hidden)
+        self.out = Linear([n["o"]], [self.hidden], self.v_width)
+        self.i_bias = self.f_bias = self.norm_weight = None
+
+    def first_product(self):
+        return self.inputs
+
+    def cache_need(self):
+        return (FixedState((self.heads, self.key_dim, self.value_dim)),
+                FixedState(kernels.memory_norm_shape(self.heads, self.key_dim, self.value_dim)))
+
+    def tensors(self) -> List[TensorSpec]:
+        n = self.names
+        return self.inputs.tensors() + self.out.tensors() + [
+            TensorSpec(n["norm"], (self.v_width,), "vector", ("one_plus_uniform", 0.1)),
+            TensorSpec(n["i_bias"], (self.heads,), "vector", ("normal", 0.5)),
+            TensorSpec(n["f_bias"], (self.heads,), "vector", ("one_plus_uniform", 4.0))]
+
+    def load(self, fetch, mode, device) -> None:
+        self.inputs.load(fetch)
+        self.out.load(fetch)
+        self.norm_weight, self.i_bias, self.f_bias = (fetch(self.names[k], "vector").to(torch.float32).contiguous()
+                                                      for k in ("norm", "i_bias", "f_bias"))
+
+    def forward(self, ctx: StepContext, h: torch.Tensor, cache, residual: Optional[torch.Tensor]):
+        T = h.shape[0]
+        memory, normaliser = cache
+        proj = ctx.product(self.inputs, h, "matrix_memory.proj")
+        o = ctx.scratch("matrix_memory.o", (T, self.v_width), torch.float32)
+        kernels.matrix_memory_scan(proj, o, memory.state, normaliser.state, ctx.batch.query_start, memory.state_slots,
+                                   self.gate_column, self.i_bias, self.f_bias, self.gate_cap, ctx.batch.num_seqs, self.heads,
+                                   self.key_dim, self.value_dim, q_scale=self.key_dim ** -0.5,
+                                   chunks=kernels.scan_chunks(ctx.batch, ctx.device), scratch=ctx.scratch)
+        gated = ctx.scratch("matrix_memory.gated", (T, self.v_width))
+        gate = proj[:, 2 * self.qk_width + self.v_width:self.gate_column]
+        kernels.grouped_gated_rms_norm(o, self.norm_weight, self.eps, gate, gated, self.heads)
+        return _finish(ctx, self.out, gated, residual, "matrix_memory.result", planes=True)
 
 
 @register_part("mixer", "min_gru")
