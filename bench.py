@@ -4,7 +4,7 @@
     python bench.py --shape 32b                 the same measurements at the Qwen3-32B sizes
     python bench.py --sweep [--shape 32b]       decode at contexts 4096 / 16384 / 32768 x batch 1 / 8 / 32, a line a point
     python bench.py --workload stress           64 requests through the scheduler at the Qwen3-1.7B sizes
-    python bench.py --workload minerax          another design beside Qwen3 at equal sizes (also duzozen, topapel, vipalorn, zovudra): prefill, decode
+    python bench.py --workload minerax          another design beside Qwen3 at equal sizes (also duzozen, topapel, vipalorn, vosurax, zovudra): prefill, decode
 
 Prints ONE JSON line. A "step" is one decode step of the engine (schedule, build the batch, run
 the model, sample greedily) at the default batch of 8 with every sequence near the benchmark
@@ -220,12 +220,44 @@ def vipalorn_config(size):
             "layers": [pattern[i % len(pattern)] for i in range(size["layers"])]}
 
 
+# ``--workload vosurax``: the Vosurax design at sizes that resemble a real model's layers, beside Qwen3 with the same
+# stream, as many heads of the same size and a gated feed-forward with as many weights as the two matrices of Vosurax's
+# dense one (2/3 of ff). Two of the layers run twice, "layers" counts the runs (Qwen3 has as many layers): attention in chunks beside
+# a matrix memory, with a dense feed-forward or with experts, and retention with experts. A token uses four experts and a
+# shared one.
+VOSURAX_SIZES = {
+    "2k": {"width": 2048, "heads": 16, "kv_heads": 4, "dim": 128, "chunk": 1024, "memory_heads": 16, "memory_dim": 128,
+           "ff": 6144, "experts": 32, "expert_ff": 768, "top": 4, "shared_ff": 1536, "layers": 8, "vocab": 32000},
+    "4k": {"width": 4096, "heads": 32, "kv_heads": 8, "dim": 128, "chunk": 2048, "memory_heads": 32, "memory_dim": 128,
+           "ff": 12288, "experts": 64, "expert_ff": 1536, "top": 4, "shared_ff": 3072, "layers": 6, "vocab": 32000},
+}
+
+
+def vosurax_config(size):
+    dense = {"kind": "dense", "ff": size["ff"]}
+    moe = {"kind": "moe", "expert": {"ff": size["expert_ff"]}, "shared": {"ff": size["shared_ff"]},
+           "router": {"experts": size["experts"], "top": size["top"]}}
+    heads, dim = size["memory_heads"], size["memory_dim"]
+    parallel = {"left": {"heads": size["heads"], "kv_heads": size["kv_heads"], "dim": size["dim"], "vdim": size["dim"],
+                         "scale": size["dim"] ** -0.5, "mask": {"size": size["chunk"]}},
+                "right": {"heads": heads, "dim": dim, "vdim": dim, "gate_cap": 15.0}}
+    retention = {"heads": heads, "dim": dim, "vdim": dim, "rot": {"dims": dim, "base": 10000.0},
+                 "decay": [1.0 - 2.0 ** (-5 - 3 * h / heads) for h in range(heads)]}
+    layers = [{"type": "parallel", "mixer": parallel, "mlp": dense}, {"type": "parallel", "mixer": parallel, "mlp": moe},
+              {"type": "retention", "mixer": retention, "mlp": moe}, {"type": "parallel", "mixer": parallel, "mlp": dense},
+              {"type": "retention", "mixer": retention, "mlp": moe}, {"type": "parallel", "mixer": parallel, "mlp": moe}]
+    loop = {"start": 1, "stop": 3, "times": 2}
+    return {"architecture": "Vosurax", "vocab": size["vocab"], "width": size["width"], "norm": {"eps": 1e-6}, "loop": loop,
+            "layers": layers[:size["layers"] - (loop["stop"] - loop["start"]) * (loop["times"] - 1)]}
+
+
 # design -> (sizes, its config at a size, Qwen3 at that size, the context a decode step may reach)
 DESIGNS = {
     "duzozen": (DUZOZEN_SIZES, duzozen_config, qwen3_beside, lambda size: 2 * size["window"]),
     "topapel": (TOPAPEL_SIZES, topapel_config, qwen3_beside_topapel, lambda size: 2 * size["chunk"]),
     "minerax": (MINERAX_SIZES, minerax_config, qwen3_beside_minerax, lambda size: 4 * size["window"]),
     "vipalorn": (VIPALORN_SIZES, vipalorn_config, qwen3_beside, lambda size: size["context"]),
+    "vosurax": (VOSURAX_SIZES, vosurax_config, qwen3_beside_topapel, lambda size: 2 * size["chunk"]),
     "zovudra": (ZOVUDRA_SIZES, zovudra_config, qwen3_beside_zovudra, lambda size: 4 * size["window"]),
 }
 BLOCK_SIZE = 16
@@ -485,9 +517,9 @@ def main():
     parser.add_argument("--layers", type=int, default=0, help="run fewer layers than the shape has (0 = all)")
     parser.add_argument("--shape", choices=sorted(SHAPES), default=None,
                         help="layer sizes: 8b (default), 32b, or 1.7b (the default of --workload stress)")
-    parser.add_argument("--workload", choices=["decode", "stress", "long-prompt", "duzozen", "topapel", "minerax", "vipalorn", "zovudra"], default="decode",
+    parser.add_argument("--workload", choices=["decode", "stress", "long-prompt", "duzozen", "topapel", "minerax", "vipalorn", "vosurax", "zovudra"], default="decode",
                         help="decode: the headline measurement; stress: many requests through a small cache; "
-                             "long-prompt: one long prompt in portions; duzozen, topapel, minerax, vipalorn, zovudra: that design "
+                             "long-prompt: one long prompt in portions; duzozen, topapel, minerax, vipalorn, vosurax, zovudra: that design "
                              "beside Qwen3 at equal sizes (--sizes), prefill and decode")
     parser.add_argument("--design-models", default="design,qwen3",
                         help="a design's workload: which of the two models to run (design: the workload's own; or its name)")

@@ -21,7 +21,7 @@ def stream_norm(x, w, eps):
 
 def rotate(x, rot, first_position=0):
     """x ``[T, heads, width]``: the first rot.dims dimensions of a head turn by position, i paired with i + dims / 2."""
-    dims = rot["dims"]
+    dims = rot.get("dims", x.shape[-1])
     half = dims // 2
     freq = rot["base"] ** (-2.0 * torch.arange(half, dtype=torch.float64) / dims)
     positions = torch.arange(first_position, first_position + x.shape[0], dtype=torch.float64)
@@ -40,7 +40,8 @@ def seen_in_chunks(T, size):
 
 def chunked_attention(w, p, m, h, eps):
     T = h.shape[0]
-    H, G, d, e = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    H, d = m["heads"], m["dim"]
+    G, e = m.get("kv_heads", H), m.get("vdim", d)
     q = (h @ w[p + "q"].T + w[p + "q.b"]).view(T, H, d)
     k = (h @ w[p + "k"].T + w[p + "k.b"]).view(T, G, d)
     v = (h @ w[p + "v"].T + w[p + "v.b"]).view(T, G, e)
@@ -81,7 +82,7 @@ def capped(z, cap):
 
 def matrix_memory(w, p, m, h, eps):
     T = h.shape[0]
-    H, d, e, cap = m["heads"], m["dim"], m["vdim"], m["gate_cap"]
+    H, d, e, cap = m["heads"], m["dim"], m.get("vdim", m["dim"]), m["gate_cap"]
     q = (h @ w[p + "q"].T).view(T, H, d) * d ** -0.5
     k = (h @ w[p + "k"].T).view(T, H, d)
     v = (h @ w[p + "v"].T).view(T, H, e)
@@ -110,7 +111,8 @@ def retention_scan(q, k, v, decay, state=None):
 
 def retention_mixer(w, p, m, h, eps):
     T = h.shape[0]
-    H, d, e = m["heads"], m["dim"], m["vdim"]
+    H, d = m["heads"], m["dim"]
+    e = m.get("vdim", d)
     q = rotate((h @ w[p + "q"].T).view(T, H, d), m["rot"])
     k = rotate((h @ w[p + "k"].T).view(T, H, d), m["rot"]) * d ** -0.5
     v = (h @ w[p + "v"].T).view(T, H, e)

@@ -753,11 +753,65 @@ __global__ void grouped_gated_rms_norm_kernel(const float* __restrict__ o, int o
     store_from_float(d + c, (r[c] * inv) * (w ? w[static_cast<size_t>(g) * w_group + c] : 1.f) * (silu_gate ? silu_f(gt[c]) : sigmoid_f(gt[c])));
 }
 
+// The same for groups of up to 4 LANES columns in whole aligned pieces of four: LANES lanes a group, four columns a lane, the
+// groups of all rows one behind the other.
+template <typename TO, int LANES>
+__global__ __launch_bounds__(256) void grouped_gated_rms_norm_piece_kernel(
+    const float* __restrict__ o, int o_row, const float* __restrict__ w, int w_group, float eps,
+    const float* __restrict__ gate, int gate_row, int silu_gate, TO* __restrict__ out, int groups, int group, long total) {
+  const long at = static_cast<long>(blockIdx.x) * (256 / LANES) + threadIdx.x / LANES;
+  const int c = (threadIdx.x % LANES) * 4;
+  const bool in = at < total && c < group;
+  const long t = in ? at / groups : 0;
+  const int g = in ? static_cast<int>(at - t * groups) : 0;
+  float4 v = make_float4(0.f, 0.f, 0.f, 0.f), z = v, s = make_float4(1.f, 1.f, 1.f, 1.f);
+  if (in) {
+    v = *reinterpret_cast<const float4*>(o + t * o_row + static_cast<size_t>(g) * group + c);
+    z = *reinterpret_cast<const float4*>(gate + t * gate_row + static_cast<size_t>(g) * group + c);
+    if (w) s = *reinterpret_cast<const float4*>(w + static_cast<size_t>(g) * w_group + c);
+  }
+  float ss = (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
+#pragma unroll
+  for (int off = LANES / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off, TIE_WAVE);
+  if (!in) return;
+  const float inv = 1.0f / sqrtf(ss / static_cast<float>(group) + eps);
+  auto act = [&](float x) { return silu_gate ? silu_f(x) : sigmoid_f(x); };
+  const float r0 = (v.x * inv) * s.x * act(z.x), r1 = (v.y * inv) * s.y * act(z.y);
+  const float r2 = (v.z * inv) * s.z * act(z.z), r3 = (v.w * inv) * s.w * act(z.w);
+  TO* d = out + (t * groups + g) * group + c;
+  if constexpr (sizeof(TO) == 2)
+    *reinterpret_cast<uint2*>(d) = make_uint2(pack_bf16x2(r0, r1), pack_bf16x2(r2, r3));
+  else
+    *reinterpret_cast<float4*>(d) = make_float4(r0, r1, r2, r3);
+}
+
 extern "C" int tie_grouped_gated_rms_norm(const float* o, int o_row, const float* w, int w_group, float eps, const float* gate,
                                           int gate_row, int silu_gate, void* out, int out_dtype, int T, int groups,
                                           int group, hipStream_t stream) {
   if (T <= 0 || groups <= 0 || group <= 0 || o_row < groups * group || gate_row < groups * group)
     return TIE_BAD_ARGUMENT;
+  if (group % 4 == 0 && group <= 256 && o_row % 4 == 0 && gate_row % 4 == 0 && w_group % 4 == 0 &&
+      (out_dtype == TIE_F32 || out_dtype == TIE_BF16) &&
+      (reinterpret_cast<uintptr_t>(o) | reinterpret_cast<uintptr_t>(w) | reinterpret_cast<uintptr_t>(gate) |
+       reinterpret_cast<uintptr_t>(out)) % 16 == 0) {
+    const long total = static_cast<long>(T) * groups;
+#define PIECE(TO, LANES)                                                                                              \
+  grouped_gated_rms_norm_piece_kernel<TO, LANES>                                                                      \
+      <<<static_cast<unsigned>((total + 256 / LANES - 1) / (256 / LANES)), 256, 0, stream>>>(                         \
+          o, o_row, w, w_group, eps, gate, gate_row, silu_gate, static_cast<TO*>(out), groups, group, total)
+#define PIECES(LANES)                              \
+  {                                                \
+    if (out_dtype == TIE_F32) PIECE(float, LANES); \
+    else PIECE(bf16_t, LANES);                     \
+  }
+    if (group <= 32) PIECES(8)
+    else if (group <= 64) PIECES(16)
+    else if (group <= 128) PIECES(32)
+    else PIECES(64)
+#undef PIECES
+#undef PIECE
+    return tie_launch_status();
+  }
   const int waves = groups >= 4 ? 4 : groups;
   const dim3 grid(T, (groups + waves - 1) / waves);
   if (out_dtype == TIE_F32)

@@ -233,6 +233,134 @@ __global__ __launch_bounds__(256) void state_walk_kernel(StateInputs in, StateFa
   if (KIND == KIND_MEMORY && tid == 0) nm[d] = m;
 }
 
+// One token a sequence (decode steps): the same layout, keys, queries and values straight from memory into the threads that
+// need them, everything asked for before the first use, one barrier.
+template <int KIND, int RPT>
+__global__ __launch_bounds__(256) void state_step_kernel(StateInputs in, StateFactors fa, float* __restrict__ out,
+                                                         float* __restrict__ state, float* __restrict__ norm_state,
+                                                         const int* __restrict__ query_start,
+                                                         const int* __restrict__ state_slots) {
+  __shared__ __attribute__((aligned(16))) float o_s[4][WALK_COLS];
+  __shared__ float nq_s[4];
+  const int tid = threadIdx.x, wave = tid / TIE_WAVE, lane = tid & (TIE_WAVE - 1);
+  const int quad = tid & 7, group = tid >> 3;
+  const int block = blockIdx.x, h = blockIdx.y, s = blockIdx.z;
+  const int H = in.H, d = in.d, e = in.e;
+  const int first = block * WALK_COLS, col = first + quad * 4;
+  const size_t slot = state_slots[s];
+  const size_t t = query_start[s];
+  float* S = state + (slot * H + h) * d * e;
+  float* nm = KIND == KIND_MEMORY ? norm_state + ((slot * H + h) * gridDim.x + block) * (d + 1) : nullptr;
+  const float* p = in.proj + t * in.row;
+  const bool whole = (e & 3) == 0;
+  float st[RPT][4], nst[RPT], k[RPT], q[RPT], v[4];
+  float m = 0.f, zi = 0.f, zf = 0.f;
+  if (KIND == KIND_MEMORY) {
+    m = nm[d];
+    zi = p[fa.i_col + h] + fa.i_bias[h];
+    zf = p[fa.f_col + h] + fa.f_bias[h];
+  }
+#pragma unroll
+  for (int c = 0; c < 4; ++c) v[c] = col + c < e ? p[in.v_col + h * e + col + c] : 0.f;
+#pragma unroll
+  for (int i = 0; i < RPT; ++i) {
+    const int r = i * 32 + group;
+    const bool has = r < d;
+    k[i] = has ? p[in.k_col + h * d + r] : 0.f;
+    q[i] = has ? p[in.q_col + h * d + r] : 0.f;
+    nst[i] = (KIND == KIND_MEMORY && has) ? nm[r] : 0.f;
+    float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (has && col < e) {
+      const float* at = S + static_cast<size_t>(r) * e + col;
+      if (whole) {
+        x = *reinterpret_cast<const float4*>(at);
+      } else {
+        x.x = at[0];
+        if (col + 1 < e) x.y = at[1];
+        if (col + 2 < e) x.z = at[2];
+        if (col + 3 < e) x.w = at[3];
+      }
+    }
+    st[i][0] = x.x, st[i][1] = x.y, st[i][2] = x.z, st[i][3] = x.w;
+  }
+  if (KIND == KIND_DECAY && in.angles != nullptr) {     // dimension r turns with r + rot / 2 (or r - rot / 2)
+    const int half = in.rot / 2;
+    const float* a = in.angles + t * in.rot;
+#pragma unroll
+    for (int i = 0; i < RPT; ++i) {
+      const int r = i * 32 + group;
+      if (r >= in.rot) continue;
+      const bool low = r < half;
+      const int other = low ? r + half : r - half, pair = low ? r : r - half;
+      const float cs = a[pair], sn = low ? -a[half + pair] : a[half + pair];
+      k[i] = k[i] * cs + p[in.k_col + h * d + other] * sn;
+      q[i] = q[i] * cs + p[in.q_col + h * d + other] * sn;
+    }
+  }
+  if (in.activation) {
+#pragma unroll
+    for (int c = 0; c < 4; ++c) v[c] = state_silu(v[c]);
+#pragma unroll
+    for (int i = 0; i < RPT; ++i) k[i] = state_silu(k[i]), q[i] = state_silu(q[i]);
+  }
+  float keep = 1.f, take = 1.f;
+  if (KIND == KIND_MEMORY) {
+    const float li = gate_in(zi, fa.cap), lf = gate_forget(zf, fa.cap) + m;
+    m = fmaxf(lf, li);
+    keep = expf(lf - m);
+    take = expf(li - m);
+#pragma unroll
+    for (int c = 0; c < 4; ++c) v[c] *= take;
+  } else {
+    keep = fa.decay[h];
+  }
+  float o[4] = {0.f, 0.f, 0.f, 0.f}, nq = 0.f;
+#pragma unroll
+  for (int i = 0; i < RPT; ++i) {
+    const float qs = q[i] * in.q_scale;
+#pragma unroll
+    for (int c = 0; c < 4; ++c) {
+      st[i][c] = fmaf(keep, st[i][c], k[i] * v[c]);
+      o[c] = fmaf(st[i][c], qs, o[c]);
+    }
+    if (KIND == KIND_MEMORY) {
+      nst[i] = fmaf(keep, nst[i], take * k[i]);
+      nq = fmaf(nst[i], qs, nq);
+    }
+  }
+#pragma unroll
+  for (int off = 8; off < TIE_WAVE; off *= 2) {
+#pragma unroll
+    for (int c = 0; c < 4; ++c) o[c] += __shfl_xor(o[c], off, TIE_WAVE);
+    if (KIND == KIND_MEMORY) nq += __shfl_xor(nq, off, TIE_WAVE);
+  }
+  if (lane < 8) *reinterpret_cast<float4*>(&o_s[wave][quad * 4]) = make_float4(o[0], o[1], o[2], o[3]);
+  if (KIND == KIND_MEMORY && lane == 0) nq_s[wave] = nq;
+#pragma unroll
+  for (int i = 0; i < RPT; ++i) {
+    const int r = i * 32 + group;
+    if (r < d && col < e) {
+      float* at = S + static_cast<size_t>(r) * e + col;
+      if (whole) {
+        *reinterpret_cast<float4*>(at) = make_float4(st[i][0], st[i][1], st[i][2], st[i][3]);
+      } else {
+        at[0] = st[i][0];
+        if (col + 1 < e) at[1] = st[i][1];
+        if (col + 2 < e) at[2] = st[i][2];
+        if (col + 3 < e) at[3] = st[i][3];
+      }
+    }
+    if (KIND == KIND_MEMORY && quad == 0 && r < d) nm[r] = nst[i];
+  }
+  __syncthreads();                                      // every thread has read nm[d] by now
+  if (tid < WALK_COLS && first + tid < e) {
+    float x = ((o_s[0][tid] + o_s[1][tid]) + o_s[2][tid]) + o_s[3][tid];
+    if (KIND == KIND_MEMORY) x /= fmaxf(fabsf(((nq_s[0] + nq_s[1]) + nq_s[2]) + nq_s[3]), expf(-m)) + 1e-6f;
+    out[(t * H + h) * e + first + tid] = x;
+  }
+  if (KIND == KIND_MEMORY && tid == 0) nm[d] = m;
+}
+
 // ------------------------------------------------------------------ chunks
 typedef float state_f16_t __attribute__((ext_vector_type(16)));
 
@@ -291,31 +419,50 @@ __device__ __forceinline__ float decay_power(float log2_lam, int m) {   // m = 0
   return m > 0 ? exp2f(static_cast<float>(m) * log2_lam) : 1.f;
 }
 
+__device__ __forceinline__ float4 f4_map(float4 v, bool silu, float scale) {
+  if (silu) v = make_float4(state_silu(v.x), state_silu(v.y), state_silu(v.z), state_silu(v.w));
+  return make_float4(v.x * scale, v.y * scale, v.z * scale, v.w * scale);
+}
+
+// Four columns c .. c + 3 of a row of n values: one 16-byte load where rows are made of whole aligned pieces (WHOLE).
+template <bool WHOLE>
+__device__ __forceinline__ float4 load_piece(const float* row, int c, int n, bool in) {
+  float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+  if (!in || c >= n) return v;
+  if (WHOLE) return *reinterpret_cast<const float4*>(row + c);
+  v.x = row[c];
+  if (c + 1 < n) v.y = row[c + 1];
+  if (c + 2 < n) v.z = row[c + 2];
+  if (c + 3 < n) v.w = row[c + 3];
+  return v;
+}
+
 // Launch 1. A workgroup owns 128 rows x 128 columns of one (chunk, head): 32 tokens of keys and values at a time in LDS, wave
 // w the rows 32 w .. of four tiles of 32 columns, two tokens an instruction (lane l hands over token l / 32). The
 // accumulators hold, in lane l, column l % 32 and the rows 8 (r / 4) + 4 (l / 32) + r % 4 of register r.
-template <int KIND>
+template <int KIND, bool WHOLE>
 __global__ __launch_bounds__(256) void chunk_state_kernel(StateInputs in, StateFactors fa, ChunkPlan plan,
                                                           const float* __restrict__ norm_state,
                                                           const int* __restrict__ state_slots, int blocks_e, int copies) {
-  __shared__ float k_s[32][128];
-  __shared__ float v_s[32][128];
+  __shared__ __attribute__((aligned(16))) float k_s[32][128];
+  __shared__ __attribute__((aligned(16))) float v_s[32][128];
   __shared__ float weight_s[CHUNK_ROWS];
   const int tid = threadIdx.x, wave = tid / TIE_WAVE, lane = tid & (TIE_WAVE - 1);
   const int hl = blockIdx.y, h = plan.h_first + hl, item = blockIdx.z;
   const int d = in.d, e = in.e;
   const int d_first = (blockIdx.x / blocks_e) * 128, e_first = (blockIdx.x % blocks_e) * 128;
   const int t0 = plan.items[item * 3 + 1], n = plan.items[item * 3 + 2] - t0;
-  const float* kp = in.proj + static_cast<size_t>(t0) * in.row + in.k_col + h * d + d_first;
-  const float* vp = in.proj + static_cast<size_t>(t0) * in.row + in.v_col + h * e + e_first;
-  float kr[16], vr[16];
+  const float* kp = in.proj + static_cast<size_t>(t0) * in.row + in.k_col + h * d;
+  const float* vp = in.proj + static_cast<size_t>(t0) * in.row + in.v_col + h * e;
+  float4 kr[4], vr[4];
+  const int i4 = (tid & 31) * 4;                         // the four columns a thread stages, of the tokens tid / 32 + 8 u
   auto fetch = [&](int from) {
 #pragma unroll
-    for (int u = 0; u < 16; ++u) {
-      const int idx = tid + u * 256, j = from + (idx >> 7), i = idx & 127;
-      const size_t at = static_cast<size_t>(min(j, n - 1)) * in.row + i;
-      kr[u] = (j < n && d_first + i < d) ? kp[at] : 0.f;
-      vr[u] = (j < n && e_first + i < e) ? vp[at] : 0.f;
+    for (int u = 0; u < 4; ++u) {
+      const int j = from + (tid >> 5) + 8 * u;
+      const size_t at = static_cast<size_t>(min(j, n - 1)) * in.row;
+      kr[u] = load_piece<WHOLE>(kp + at, d_first + i4, d, j < n);
+      vr[u] = load_piece<WHOLE>(vp + at, e_first + i4, e, j < n);
     }
   };
   fetch(0);
@@ -348,11 +495,10 @@ __global__ __launch_bounds__(256) void chunk_state_kernel(StateInputs in, StateF
   float n_sum = 0.f;
   for (int from = 0; from < n; from += 32) {            // uniform for the workgroup
 #pragma unroll
-    for (int u = 0; u < 16; ++u) {
-      const int idx = tid + u * 256, j = idx >> 7, i = idx & 127;
-      const float k = in.activation ? state_silu(kr[u]) : kr[u];
-      k_s[j][i] = k * weight_s[from + j];
-      v_s[j][i] = in.activation ? state_silu(vr[u]) : vr[u];
+    for (int u = 0; u < 4; ++u) {
+      const int j = (tid >> 5) + 8 * u;
+      *reinterpret_cast<float4*>(&k_s[j][i4]) = f4_map(kr[u], in.activation, weight_s[from + j]);
+      *reinterpret_cast<float4*>(&v_s[j][i4]) = f4_map(vr[u], in.activation, 1.f);
     }
     __syncthreads();
     if (from + 32 < n) fetch(from + 32);                // in flight during the products
@@ -465,12 +611,13 @@ __global__ __launch_bounds__(256) void combine_chunks_kernel(ChunkPlan plan, Sta
 // lane l takes the words 8 u + 4 (l / 32) + t, and instruction t pairs the two halves' words t; the other operand follows.
 #define CO_K 36            // words of a staged row of 32 query or key dimensions
 #define CO_P 68            // words of a row of 64 scores
-template <int KIND, int NT>
+template <int KIND, int NT, bool WHOLE>
 __global__ __launch_bounds__(256) void chunk_output_kernel(StateInputs in, StateFactors fa, ChunkPlan plan,
                                                            float* __restrict__ out) {
   constexpr int COLS = 64 * NT;
   constexpr int CO_S = COLS + 8;                        // words of a row of state or value columns
-  constexpr int SV = 32 * COLS / 256;                   // values a thread stages of those
+  constexpr int SV = 32 * COLS / 1024;                  // pieces of four values a thread stages of those
+  constexpr int PIECES = COLS / 4;                      // ... of a row
   __shared__ __attribute__((aligned(16))) float qk_s[2 * CHUNK_ROWS * CO_K];    // queries | keys, later the scores
   __shared__ __attribute__((aligned(16))) float sv_s[32 * CO_S];
   __shared__ float n_s[32], left_s[CHUNK_ROWS], floor_s[CHUNK_ROWS], scale_s[CHUNK_ROWS];
@@ -488,23 +635,25 @@ __global__ __launch_bounds__(256) void chunk_output_kernel(StateInputs in, State
   const float* S = plan.states + (static_cast<size_t>(item) * plan.heads + hl) * plan.per;
   const float* qp = in.proj + static_cast<size_t>(t0) * in.row + in.q_col + h * d;
   const float* kp = in.proj + static_cast<size_t>(t0) * in.row + in.k_col + h * d;
-  const float* vp = in.proj + static_cast<size_t>(t0) * in.row + in.v_col + h * e + e_first;
+  const float* vp = in.proj + static_cast<size_t>(t0) * in.row + in.v_col + h * e;
   const float log2_lam = KIND == KIND_DECAY ? log2f(fa.decay[h]) : 0.f;
 
-  float qr[8], kr[8], sr[SV], nr = 0.f;
+  float4 qr[2], kr[2], sr[SV];
+  float nr = 0.f;
+  const int qj = tid >> 3, qi = (tid & 7) * 4;          // of queries and keys a thread stages the tokens qj and qj + 32
+  const int sj = tid / PIECES, sc = (tid % PIECES) * 4; // of state or values the rows sj + u 256 / PIECES
   auto fetch = [&](int k0) {
 #pragma unroll
-    for (int u = 0; u < 8; ++u) {
-      const int idx = tid + u * 256, j = idx >> 5, i = k0 + (idx & 31);
-      const size_t at = static_cast<size_t>(min(j, n - 1)) * in.row + i;
-      const bool has = j < n && i < d;
-      qr[u] = has ? qp[at] : 0.f;
-      kr[u] = has ? kp[at] : 0.f;
+    for (int u = 0; u < 2; ++u) {
+      const int j = qj + 32 * u;
+      const size_t at = static_cast<size_t>(min(j, n - 1)) * in.row;
+      qr[u] = load_piece<WHOLE>(qp + at, k0 + qi, d, j < n);
+      kr[u] = load_piece<WHOLE>(kp + at, k0 + qi, d, j < n);
     }
 #pragma unroll
     for (int u = 0; u < SV; ++u) {
-      const int idx = tid + u * 256, i = k0 + idx / COLS, c = idx % COLS;
-      sr[u] = (i < d && e_first + c < e) ? S[static_cast<size_t>(i) * e + e_first + c] : 0.f;
+      const int i = k0 + sj + u * (256 / PIECES);
+      sr[u] = load_piece<WHOLE>(S + static_cast<size_t>(min(i, d - 1)) * e, e_first + sc, e, i < d);
     }
     if (KIND == KIND_MEMORY && tid < 32) nr = k0 + tid < d ? S[static_cast<size_t>(d) * e + k0 + tid] : 0.f;
   };
@@ -535,16 +684,12 @@ __global__ __launch_bounds__(256) void chunk_output_kernel(StateInputs in, State
   for (int k0 = 0; k0 < d; k0 += 32) {                  // uniform for the workgroup
     if (k0 > 0) __syncthreads();
 #pragma unroll
-    for (int u = 0; u < 8; ++u) {
-      const int idx = tid + u * 256, j = idx >> 5, i = idx & 31;
-      q_s[j * CO_K + i] = (in.activation ? state_silu(qr[u]) : qr[u]) * in.q_scale;
-      k_s[j * CO_K + i] = in.activation ? state_silu(kr[u]) : kr[u];
+    for (int u = 0; u < 2; ++u) {
+      *reinterpret_cast<float4*>(&q_s[(qj + 32 * u) * CO_K + qi]) = f4_map(qr[u], in.activation, in.q_scale);
+      *reinterpret_cast<float4*>(&k_s[(qj + 32 * u) * CO_K + qi]) = f4_map(kr[u], in.activation, 1.f);
     }
 #pragma unroll
-    for (int u = 0; u < SV; ++u) {
-      const int idx = tid + u * 256;
-      sv_s[(idx / COLS) * CO_S + idx % COLS] = sr[u];
-    }
+    for (int u = 0; u < SV; ++u) *reinterpret_cast<float4*>(&sv_s[(sj + u * (256 / PIECES)) * CO_S + sc]) = sr[u];
     if (KIND == KIND_MEMORY && tid < 32) n_s[tid] = nr;
     __syncthreads();
     if (k0 + 32 < d) fetch(k0 + 32);
@@ -574,20 +719,18 @@ __global__ __launch_bounds__(256) void chunk_output_kernel(StateInputs in, State
     }
   }
   // values of the first 32 tokens on their way while the scores are finished
-  float vr[SV];
+  float4 vr[SV];
   auto fetch_values = [&](int from) {
 #pragma unroll
     for (int u = 0; u < SV; ++u) {
-      const int idx = tid + u * 256, j = from + idx / COLS, c = idx % COLS;
-      vr[u] = (j < n && e_first + c < e) ? vp[static_cast<size_t>(j) * in.row + c] : 0.f;
+      const int j = from + sj + u * (256 / PIECES);
+      vr[u] = load_piece<WHOLE>(vp + static_cast<size_t>(min(j, n - 1)) * in.row, e_first + sc, e, j < n);
     }
   };
   auto publish_values = [&]() {
 #pragma unroll
-    for (int u = 0; u < SV; ++u) {
-      const int idx = tid + u * 256;
-      sv_s[(idx / COLS) * CO_S + idx % COLS] = in.activation ? state_silu(vr[u]) : vr[u];
-    }
+    for (int u = 0; u < SV; ++u)
+      *reinterpret_cast<float4*>(&sv_s[(sj + u * (256 / PIECES)) * CO_S + sc]) = f4_map(vr[u], in.activation, 1.f);
   };
   fetch_values(0);
   __syncthreads();                                      // queries, keys and state have been read
@@ -666,24 +809,30 @@ static bool bad_inputs(const StateInputs& in, const StateFactors& fa, int kind) 
 }
 
 // kind 0: decay [H], angles [T][rot] or null; kind 1: biases [H], norm_state [slots][H][ceil(e / WALK_COLS)][d + 1].
-// proj rows query_start[0] .. query_start[S] - 1; out [T][H][e]; state [slots][H][d][e].
+// proj rows query_start[0] .. query_start[S] - 1; out [T][H][e]; state [slots][H][d][e]. single: every sequence brings one
+// row.
 extern "C" int tie_matrix_state_walk(int kind, const float* proj, int row, int q_col, int k_col, int v_col, int activation,
                                      float q_scale, const float* angles, int rot, const float* decay, const float* i_bias,
                                      const float* f_bias, int i_col, int f_col, float cap, float* out, float* state,
-                                     float* norm_state, const int* query_start, const int* state_slots, int S, int H, int d,
-                                     int e, hipStream_t stream) {
+                                     float* norm_state, const int* query_start, const int* state_slots, int single, int S,
+                                     int H, int d, int e, hipStream_t stream) {
   const StateInputs in{proj, row, q_col, k_col, v_col, activation, q_scale, angles, rot, H, d, e};
   const StateFactors fa{decay, i_bias, f_bias, i_col, f_col, cap};
   if (bad_inputs(in, fa, kind) || S <= 0 || S > 65535 || out == nullptr || state == nullptr ||
       (kind == KIND_MEMORY && norm_state == nullptr))
     return TIE_BAD_ARGUMENT;
   const dim3 grid((e + WALK_COLS - 1) / WALK_COLS, H, S);
-#define WALK(KIND, RPT) \
-  state_walk_kernel<KIND, RPT><<<grid, 256, 0, stream>>>(in, fa, out, state, norm_state, query_start, state_slots)
+#define WALK(KIND, RPT)                                                                                                    \
+  {                                                                                                                       \
+    if (single)                                                                                                           \
+      state_step_kernel<KIND, RPT><<<grid, 256, 0, stream>>>(in, fa, out, state, norm_state, query_start, state_slots);   \
+    else                                                                                                                  \
+      state_walk_kernel<KIND, RPT><<<grid, 256, 0, stream>>>(in, fa, out, state, norm_state, query_start, state_slots);   \
+  }
 #define WALKS(RPT)                              \
   {                                             \
-    if (kind == KIND_DECAY) WALK(KIND_DECAY, RPT); \
-    else WALK(KIND_MEMORY, RPT);                \
+    if (kind == KIND_DECAY) WALK(KIND_DECAY, RPT) \
+    else WALK(KIND_MEMORY, RPT)                 \
   }
   if (d <= 32) WALKS(1)
   else if (d <= 64) WALKS(2)
@@ -717,19 +866,28 @@ extern "C" int tie_matrix_state_chunks(int kind, const float* proj, int row, int
   const int blocks_e = (e + 127) / 128, blocks_d = (d + 127) / 128;
   const int per_head = (per + 255) / 256;
   const dim3 grid1(blocks_d * blocks_e, heads, count), grid2(per_head * heads, S);
-#define PASSES(KIND)                                                                                                  \
+  // rows of whole aligned pieces of four: keys, queries, values of every head, the chunks' states
+  const bool whole = row % 4 == 0 && q_col % 4 == 0 && k_col % 4 == 0 && v_col % 4 == 0 && d % 4 == 0 && e % 4 == 0 &&
+                     reinterpret_cast<uintptr_t>(proj) % 16 == 0 && reinterpret_cast<uintptr_t>(states) % 16 == 0;
+#define PASSES_W(KIND, WHOLE)                                                                                         \
   {                                                                                                                   \
-    chunk_state_kernel<KIND><<<grid1, 256, 0, stream>>>(in, fa, plan, norm_state, state_slots, blocks_e, copies);     \
+    chunk_state_kernel<KIND, WHOLE><<<grid1, 256, 0, stream>>>(in, fa, plan, norm_state, state_slots, blocks_e, copies); \
     combine_chunks_kernel<KIND><<<grid2, 256, 0, stream>>>(plan, fa, state, norm_state, state_slots, H, d, e,         \
                                                            per_head, copies);                                         \
     if (e <= 64)                                                                                                      \
-      chunk_output_kernel<KIND, 1><<<dim3(1, heads, count), 256, 0, stream>>>(in, fa, plan, out);                     \
+      chunk_output_kernel<KIND, 1, WHOLE><<<dim3(1, heads, count), 256, 0, stream>>>(in, fa, plan, out);              \
     else                                                                                                              \
-      chunk_output_kernel<KIND, 2><<<dim3(blocks_e, heads, count), 256, 0, stream>>>(in, fa, plan, out);              \
+      chunk_output_kernel<KIND, 2, WHOLE><<<dim3(blocks_e, heads, count), 256, 0, stream>>>(in, fa, plan, out);       \
+  }
+#define PASSES(KIND)                   \
+  {                                    \
+    if (whole) PASSES_W(KIND, true)    \
+    else PASSES_W(KIND, false)         \
   }
   if (kind == KIND_DECAY) PASSES(KIND_DECAY)
   else PASSES(KIND_MEMORY)
 #undef PASSES
+#undef PASSES_W
   return tie_launch_status();
 }
 

@@ -143,8 +143,6 @@ _SIGNATURES = {
                                         _c_float, _c_int, _c_int, _c_int, _c_void, _c_void],
     },
     "recurrent": {
-        "tie_decay_attention_scan": [_c_void, _c_int, _c_void, _c_void, _c_void, _c_void, _c_void, _c_int, _c_int,
-                                     _c_int, _c_int, _c_int, _c_void, _c_void, _c_int, _c_void, _c_int, _c_void],
         "tie_gated_rms_norm": [_c_void, _c_void, _c_float, _c_void, _c_int, _c_void, _c_int, _c_int, _c_int, _c_void],
         "tie_min_gru_scan": [_c_void, _c_int, _c_void, _c_int, _c_void, _c_void, _c_void, _c_int, _c_int, _c_void,
                              _c_void, _c_int, _c_void, _c_void, _c_void],
@@ -153,7 +151,7 @@ _SIGNATURES = {
         "tie_matrix_state_walk_cols": [],
         "tie_matrix_state_walk": [_c_int, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_void, _c_int, _c_void,
                                   _c_void, _c_void, _c_int, _c_int, _c_float, _c_void, _c_void, _c_void, _c_void, _c_void,
-                                  _c_int, _c_int, _c_int, _c_int, _c_void],
+                                  _c_int, _c_int, _c_int, _c_int, _c_int, _c_void],
         "tie_matrix_state_chunks": [_c_int, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_void, _c_void,
                                     _c_void, _c_int, _c_int, _c_float, _c_void, _c_void, _c_void, _c_void, _c_void, _c_void,
                                     _c_int, _c_int, _c_void, _c_void, _c_void, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
@@ -1794,7 +1792,7 @@ def _matrix_state(kind: int, proj: torch.Tensor, out: torch.Tensor, state: torch
         _call(lib.tie_matrix_state_walk, what, kind, proj.data_ptr(), proj.stride(0), 0, qk, 2 * qk, silu, float(q_scale),
               _ptr(angles), rot, _ptr(decay), _ptr(i_bias), _ptr(f_bias), i_col, f_col, float(cap), out.data_ptr(),
               state.data_ptr(), _ptr(norm_state), query_start.data_ptr(), state_slots.data_ptr(),
-              num_seqs, heads, key_dim, value_dim, _stream())
+              int(T == num_seqs), num_seqs, heads, key_dim, value_dim, _stream())      # as many rows: one each
         return
     if rotation is not None:
         _call(lib.tie_rotate_heads, "rotate_heads", proj.data_ptr(), proj.stride(0), 0, qk, angles.data_ptr(), rot, T, heads,

@@ -33,6 +33,7 @@ def _needs_of(mixer) -> tuple:
 @register_part("mixer", "parallel")
 class ParallelMixer(Mixer):
     capturable = True
+    replayable = True
     returns_result = True
 
     def __init__(self, params):

@@ -90,6 +90,7 @@ def _finish(ctx: StepContext, out: Linear, rows: torch.Tensor, residual: Optiona
 @register_part("mixer", "decay_attention")
 class DecayAttention(Mixer):
     capturable = True      # reads the step on the device only: may be recorded into a HIP graph
+    replayable = True        # the chunks of a long step and the angles are made once a step and kept
     takes_row_scale = True   # h goes into the one projection only, through Linear with the step context
     returns_result = True
 
@@ -172,6 +173,7 @@ class DecayAttention(Mixer):
 @register_part("mixer", "matrix_memory")
 class MatrixMemory(Mixer):
     capturable = True
+    replayable = True
     takes_row_scale = True
     returns_result = True
 
